@@ -4,3 +4,4 @@ from . import vivevik  # noqa: F401
 from . import ruvalorn  # noqa: F401
 from . import minodra  # noqa: F401
 from . import ninisun  # noqa: F401
+from . import mazanex  # noqa: F401

@@ -57,7 +57,9 @@ def group_page_need(window: Optional[int], page_size: int, total_tokens: int, ma
                     keep_first: int = 0) -> int:
     """Most pages of one group a request holds at any time when it grows to
     ``total_tokens`` in steps of at most ``max_step_tokens``.  The pages of the first
-    ``keep_first`` positions are held throughout."""
+    ``keep_first`` positions are held throughout.  (A group that reads by chunks of ``c``
+    positions needs what a window of ``c`` needs: the current chunk's positions before the
+    step's are at most ``c - 1``.)"""
     full = pages_for_tokens(total_tokens, page_size)
     if window is None:
         return full
@@ -142,7 +144,7 @@ class CacheManager:
         return {
             "page_size": self.page_size,
             "rows_total": self.max_requests, "rows_used": self.live_requests,
-            "groups": [{"window": g.window, "layers": len(g.entries), "pages_total": p.num_pages,
+            "groups": [{"window": g.window, "chunk": g.spec.chunk, "layers": len(g.entries), "pages_total": p.num_pages,
                         "pages_free": p.free_count, "pages_used": p.used_count,
                         "pages_high_water": p.high_water}
                        for g, p in zip(self.groups, self.pools)],
@@ -163,7 +165,7 @@ class CacheManager:
         return [st.get("v") for st in self.storage]
 
     def page_need(self, total_tokens: int, max_step_tokens: int) -> List[int]:
-        return [group_page_need(g.window, self.page_size, total_tokens, max_step_tokens, g.spec.keep_first)
+        return [group_page_need(g.spec.reach, self.page_size, total_tokens, max_step_tokens, g.spec.keep_first)
                 for g in self.groups]
 
     # -------------------------------------------------------------- lifecycle
@@ -222,14 +224,14 @@ class CacheManager:
 
     def commit(self, req: RequestCache) -> None:
         """The step that wrote the reserved positions is done: they count, and
-        pages that every later query's window has passed are given back."""
+        pages that every later query's window (or chunk) has passed are given back."""
         req.computed_len = req.reserved_len
         for gi, g in enumerate(self.groups):
-            if g.window is None:
+            if not g.spec.bounded:
                 continue
-            # A later query sits at position >= computed_len and reads keys from
-            # position - window + 1 on: nothing below this bound is read again.
-            lowest_needed = max(0, req.computed_len - g.window + 1)
+            # A later query sits at position >= computed_len: nothing below this bound is
+            # read again.
+            lowest_needed = g.spec.lowest_read(req.computed_len)
             first_needed_page = lowest_needed // self.page_size
             pages = req.pages[gi]
             # (pages that hold any of the first ``keep_first`` positions stay for good)

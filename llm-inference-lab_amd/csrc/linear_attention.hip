@@ -1,6 +1,10 @@
 // Gated linear attention: a matrix-valued recurrent state per head,
 //   S_t = diag(a_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t,
-// with a decay a_t in (0, 1) per key channel.  The state [D, E] per head lives in float32 in
+// with a decay a_t in (0, 1) per key channel.  Two relatives go through the same kernels:
+//   bonus      o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t: the current token through a learned vector u
+//   memory     S_t = keep_t S_(t-1) + take_t k_t v_t^T,  n_t = keep_t n_(t-1) + take_t k_t, with one number
+//              keep_t and take_t per head from exponential gates and a running maximum (below)
+// The state [D, E] per head lives in float32 in
 // a slot per request and is carried from step to step; everything here is float32.  gfx950.
 //
 // Three kernels: the decays from their low-rank projection; the scan over the tokens of every
@@ -16,29 +20,126 @@ constexpr int SLICE = 16;      // key channels of the state that one thread keep
 // a[r, c] = sigmoid(z)^(1 / tau), z = bias[c] + sum_j w2[c, j] * low[r, j]  (c over heads * D
 // key channels, j over the rank of the projection).  sigmoid(z)^(1/tau) = exp(-softplus(-z) / tau),
 // with softplus(u) = max(u, 0) + log1p(exp(-|u|)), so that neither end overflows.
+// kind 1 (DECAY_DOUBLE_EXP): a[r, c] = exp(-exp(z)), z = bias[c] + sum_j w2[c, j] * tanh(low[r, j]).
+constexpr int DECAY_SIGMOID = 0, DECAY_DOUBLE_EXP = 1;
+__device__ __forceinline__ float decay_of(float z, int kind, float inv_tau) {
+  if (kind == DECAY_DOUBLE_EXP) return expf(-expf(z));
+  const float u = -z;
+  const float sp = fmaxf(u, 0.f) + log1pf(expf(-fabsf(u)));
+  return expf(-sp * inv_tau);
+}
 __global__ __launch_bounds__(256) void gla_decay_kernel(const float* __restrict__ low, int ld, int rank,
                                                         const float* __restrict__ w2, const float* __restrict__ bias,
-                                                        float inv_tau, float* __restrict__ decay, int channels) {
+                                                        int kind, float inv_tau, float* __restrict__ decay, int channels) {
+  extern __shared__ float s_low[];
   const int r = blockIdx.x;
   const float* t = low + (size_t)r * ld;
+  for (int j = threadIdx.x; j < rank; j += blockDim.x) s_low[j] = kind == DECAY_DOUBLE_EXP ? tanhf(t[j]) : t[j];
+  __syncthreads();
   for (int c = threadIdx.x; c < channels; c += blockDim.x) {
     float z = bias ? bias[c] : 0.f;
     const float* w = w2 + (size_t)c * rank;
-    for (int j = 0; j < rank; ++j) z = fmaf(w[j], t[j], z);
-    const float u = -z;
-    const float sp = fmaxf(u, 0.f) + log1pf(expf(-fabsf(u)));
-    decay[(size_t)r * channels + c] = expf(-sp * inv_tau);
+    if ((rank & 3) == 0) {                       // (a row of the second factor 16 bytes a load, all on their way together)
+      for (int j = 0; j < rank; j += 4) {
+        const floatx4 w4 = *(const floatx4*)(w + j);
+        z = fmaf(w4[0], s_low[j], z);
+        z = fmaf(w4[1], s_low[j + 1], z);
+        z = fmaf(w4[2], s_low[j + 2], z);
+        z = fmaf(w4[3], s_low[j + 3], z);
+      }
+    } else {
+      for (int j = 0; j < rank; ++j) z = fmaf(w[j], s_low[j], z);
+    }
+    decay[(size_t)r * channels + c] = decay_of(z, kind, inv_tau);
   }
 }
 
 extern "C" int llmlab_gla_decay(const float* low, int ld, int rows, int rank, const float* w2, const float* bias,
-                                float tau, float* decay, int channels, hipStream_t stream) {
-  LLMLAB_REQUIRE(rows >= 0 && rank > 0 && channels > 0 && ld >= rank && tau > 0.f,
-                 "gla_decay: bad sizes rows=%d rank=%d channels=%d ld=%d tau=%g", rows, rank, channels, ld, (double)tau);
+                                int kind, float tau, float* decay, int channels, hipStream_t stream) {
+  LLMLAB_REQUIRE(rows >= 0 && rank > 0 && rank <= 8192 && channels > 0 && ld >= rank && tau > 0.f &&
+                     (kind == DECAY_SIGMOID || kind == DECAY_DOUBLE_EXP),
+                 "gla_decay: bad sizes rows=%d rank=%d channels=%d ld=%d kind=%d tau=%g", rows, rank, channels, ld, kind,
+                 (double)tau);
   if (rows == 0) return 0;
-  hipLaunchKernelGGL(gla_decay_kernel, dim3(rows), dim3(256), 0, stream, low, ld, rank, w2, bias, 1.0f / tau, decay,
-                     channels);
+  hipLaunchKernelGGL(gla_decay_kernel, dim3(rows), dim3(256), rank * sizeof(float), stream, low, ld, rank, w2, bias, kind,
+                     1.0f / tau, decay, channels);
   LLMLAB_LAUNCH_CHECK("gla_decay");
+  return 0;
+}
+
+// ---------------------------------------------------------- gates of a matrix memory
+// Per head and row the log gates i = cap * tanh((proj_i + bias_i) / cap) and f = logsigmoid(cap *
+// tanh((proj_f + bias_f) / cap)), the running maximum m_t = max(f_t + m_(t-1), i_t) from the slot's (0 at
+// a sequence's start), and what the recurrence multiplies by: keep = exp(f_t + m_(t-1) - m_t), take =
+// exp(i_t - m_t).  All float32.  Block (request, head): the rows MEMORY_TILE at a time, a thread a
+// row; the maxima of a tile by a scan over (sum of f, maximum so far) pairs, (F1, M1) then (F2, M2) =
+// (F1 + F2, max(M1 + F2, M2)).  Whatever rounding the scan adds to an m, keep and take of all rows
+// are taken from the same m's, so the state stays exact in them.
+constexpr int MEMORY_TILE = 256;
+__global__ __launch_bounds__(MEMORY_TILE) void memory_gates_kernel(
+    const float* __restrict__ proj, int ld, int off_i, int off_f, const float* __restrict__ bias_i,
+    const float* __restrict__ bias_f, float cap, int n_heads, float* __restrict__ max_state, const int* __restrict__ q_start,
+    const int* __restrict__ req_rows, float* __restrict__ keep, float* __restrict__ take, float* __restrict__ maxima) {
+  __shared__ float s_f[MEMORY_TILE / 64], s_m[MEMORY_TILE / 64], s_max[MEMORY_TILE + 1];
+  const int b = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int first = q_start[b], last = q_start[b + 1];
+  if (first >= last) return;
+  float* slot = max_state + (size_t)req_rows[b] * n_heads + h;
+  float carry = *slot;
+  const float bi = bias_i ? bias_i[h] : 0.f, bf = bias_f ? bias_f[h] : 0.f;
+  for (int t0 = first; t0 < last; t0 += MEMORY_TILE) {
+    const int t = t0 + (int)threadIdx.x;
+    const bool in = t < last;
+    float i = -__builtin_huge_valf(), f = 0.f;      // (rows past the end leave the maximum as it is)
+    if (in) {
+      const float* row = proj + (size_t)t * ld;
+      i = cap * tanhf((row[off_i + h] + bi) / cap);
+      const float z = cap * tanhf((row[off_f + h] + bf) / cap);
+      f = -(fmaxf(-z, 0.f) + log1pf(expf(-fabsf(z))));
+    }
+    float F = f, M = i;
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const float F1 = __shfl_up(F, off, WAVE), M1 = __shfl_up(M, off, WAVE);
+      if (lane >= off) {
+        M = fmaxf(M1 + F, M);
+        F = F1 + F;
+      }
+    }
+    if (lane == 63) {
+      s_f[wave] = F;
+      s_m[wave] = M;
+    }
+    if (threadIdx.x == 0) s_max[0] = carry;
+    __syncthreads();
+    float m0 = carry;                               // the maximum before this wave's rows
+    for (int w = 0; w < wave; ++w) m0 = fmaxf(s_f[w] + m0, s_m[w]);
+    const float m = fmaxf(F + m0, M);
+    s_max[threadIdx.x + 1] = m;
+    __syncthreads();
+    if (in) {
+      const size_t at = (size_t)t * n_heads + h;
+      keep[at] = expf(f + s_max[threadIdx.x] - m);
+      take[at] = expf(i - m);
+      maxima[at] = m;
+    }
+    carry = s_max[MEMORY_TILE];
+    __syncthreads();
+  }
+  if (threadIdx.x == 0) *slot = carry;
+}
+
+extern "C" int llmlab_memory_gates(const float* proj, int ld, int off_i, int off_f, const float* bias_i, const float* bias_f,
+                                   float cap, int n_heads, float* max_state, const int* q_start, const int* req_rows,
+                                   int n_reqs, float* keep, float* take, float* maxima, hipStream_t stream) {
+  LLMLAB_REQUIRE(n_reqs >= 0 && n_heads > 0 && n_heads <= 65535 && cap > 0.f && off_i >= 0 && off_f >= 0 &&
+                     ld >= off_i + n_heads && ld >= off_f + n_heads,
+                 "memory_gates: bad sizes requests=%d heads=%d cap=%g ld=%d", n_reqs, n_heads, (double)cap, ld);
+  LLMLAB_REQUIRE(proj && max_state && q_start && req_rows && keep && take && maxima, "memory_gates: an operand is missing");
+  if (n_reqs == 0) return 0;
+  hipLaunchKernelGGL(memory_gates_kernel, dim3(n_reqs, n_heads), dim3(MEMORY_TILE), 0, stream, proj, ld, off_i, off_f, bias_i,
+                     bias_f, cap, n_heads, max_state, q_start, req_rows, keep, take, maxima);
+  LLMLAB_LAUNCH_CHECK("memory_gates");
   return 0;
 }
 
@@ -61,12 +162,20 @@ extern "C" int llmlab_gla_decay(const float* low, int ld, int rows, int rank, co
 //   FINISH per chunk: the rows again from S_start[c], now with outputs.
 // All of it in float32; the result differs from the row-by-row recurrence by rounding only.
 enum { SCAN_WHOLE = 0, SCAN_LOCAL = 1, SCAN_FINISH = 2 };
+// KIND: DECAY and BONUS take a decay per key channel (and the bonus u [heads, D]); MEMORY one
+// number keep_t and one take_t per head.  MEMORY's normaliser n (key channels only, no values) is
+// the business of one more block per head (blockIdx.z past the columns): lane c < SLICE of slice s
+// keeps n[d0 + c] and leaves the slice's part of n_t . q_t in norm_parts[row, h, s].
+enum { KIND_DECAY = 0, KIND_BONUS = 1, KIND_MEMORY = 2 };
 
 struct ScanArgs {
   const float* proj; int ld, off_q, off_k, off_v;
   const float* decay; float q_scale; int n_heads, D, E, cols, slices;
   float* state; const int* q_start; const int* req_rows; float* parts;
   int n_reqs, chunk; float* chunk_state; float* chunk_decay;      // [chunks, heads, D, E] and [chunks, heads, D]
+  const float* bonus;                                              // BONUS: u [heads, D]
+  const float* keep; const float* take;                            // MEMORY: [rows, heads]
+  float* norm_state; float* norm_parts; float* chunk_norm;         // MEMORY: [slots, heads, D], [rows, heads, slices], [chunks, heads, D]
 };
 
 // Which request and which rows the chunk `index` of the step covers (chunks are counted
@@ -86,7 +195,67 @@ __device__ __forceinline__ bool find_chunk(const ScanArgs& a, int index, int& fi
   return false;
 }
 
-template <int MODE, bool UNIFORM, int THREADS>
+// The normaliser of one head over the rows [first, last): see KIND_MEMORY above.
+template <int MODE>
+__device__ __forceinline__ void scan_normaliser(const ScanArgs& a, int h, int first, int last) {
+  const int c = threadIdx.x % a.cols, s = threadIdx.x / a.cols;
+  const int D = a.D, d = s * SLICE + c;
+  const bool mine = c < SLICE && s < a.slices && d < D;
+  if (a.cols % SLICE != 0) {      // (a slice's lanes are no whole groups of 16 then: one lane a slice walks all its channels)
+    if (c != 0 || s >= a.slices) return;
+    float* st = (MODE == SCAN_WHOLE ? a.norm_state + ((size_t)a.req_rows[blockIdx.x] * a.n_heads + h) * D
+                                    : a.chunk_norm + ((size_t)blockIdx.x * a.n_heads + h) * D) + s * SLICE;
+    const int n = D - s * SLICE < SLICE ? D - s * SLICE : SLICE;
+    float N[SLICE];
+    for (int i = 0; i < SLICE; ++i) N[i] = (MODE != SCAN_LOCAL && i < n) ? st[i] : 0.f;
+    for (int t = first; t < last; ++t) {
+      const float* row = a.proj + (size_t)t * a.ld + h * D + s * SLICE;
+      const float keep = a.keep[(size_t)t * a.n_heads + h], take = a.take[(size_t)t * a.n_heads + h];
+      float acc = 0.f;
+#pragma unroll
+      for (int i = 0; i < SLICE; ++i) {
+        N[i] = fmaf(keep, N[i], i < n ? take * row[a.off_k + i] : 0.f);
+        if (MODE != SCAN_LOCAL) acc = fmaf(N[i], i < n ? row[a.off_q + i] : 0.f, acc);
+      }
+      if (MODE != SCAN_LOCAL) a.norm_parts[((size_t)t * a.n_heads + h) * a.slices + s] = acc * a.q_scale;
+    }
+    if (MODE == SCAN_FINISH) return;
+    for (int i = 0; i < n; ++i) st[i] = N[i];
+    return;
+  }
+  float* st = MODE == SCAN_WHOLE ? a.norm_state + ((size_t)a.req_rows[blockIdx.x] * a.n_heads + h) * D + d
+                                 : a.chunk_norm + ((size_t)blockIdx.x * a.n_heads + h) * D + d;
+  if (c >= SLICE || s >= a.slices) return;      // (whole quarters of a wave leave or stay: the sum below is over 16 lanes)
+  float N = (MODE != SCAN_LOCAL && mine) ? *st : 0.f;
+  struct Row { float keep, take, k, q; } r0, r1;
+  auto fetch = [&](Row& r, int t) {
+    const float* row = a.proj + (size_t)t * a.ld + h * D + d;
+    r.keep = a.keep[(size_t)t * a.n_heads + h];
+    r.take = a.take[(size_t)t * a.n_heads + h];
+    r.k = mine ? row[a.off_k] : 0.f;
+    if (MODE != SCAN_LOCAL) r.q = mine ? row[a.off_q] : 0.f;
+  };
+  auto step = [&](const Row& r, int t) {
+    N = fmaf(r.keep, N, r.take * r.k);
+    if (MODE == SCAN_LOCAL) return;
+    float x = N * r.q;
+#pragma unroll
+    for (int off = 8; off > 0; off >>= 1) x += __shfl_xor(x, off, SLICE);
+    if (c == 0) a.norm_parts[((size_t)t * a.n_heads + h) * a.slices + s] = x * a.q_scale;
+  };
+  if (first < last) fetch(r0, first);
+  for (int t = first; t < last; t += 2) {
+    if (t + 1 < last) fetch(r1, t + 1);
+    step(r0, t);
+    if (t + 1 < last) {
+      if (t + 2 < last) fetch(r0, t + 2);
+      step(r1, t + 1);
+    }
+  }
+  if (MODE != SCAN_FINISH && mine) *st = N;
+}
+
+template <int MODE, int KIND, bool UNIFORM, int THREADS>
 __global__ __launch_bounds__(THREADS) void gla_scan_kernel(ScanArgs a) {
   const int h = blockIdx.y;
   const int e = blockIdx.z * a.cols + (int)(threadIdx.x % a.cols);
@@ -100,9 +269,18 @@ __global__ __launch_bounds__(THREADS) void gla_scan_kernel(ScanArgs a) {
   } else if (!find_chunk(a, blockIdx.x, first, last)) {
     return;
   }
+  if (KIND == KIND_MEMORY && (int)blockIdx.z * a.cols >= a.E) {
+    scan_normaliser<MODE>(a, h, first, last);
+    return;
+  }
   if (e >= a.E || s >= a.slices) return;
   const int D = a.D, E = a.E, d0 = s * SLICE;
   float S[SLICE], P[SLICE];
+  float U[KIND == KIND_BONUS ? SLICE : 1];
+  if (KIND == KIND_BONUS) {
+#pragma unroll
+    for (int i = 0; i < SLICE; ++i) U[i] = d0 + i < D ? a.bonus[h * D + d0 + i] : 0.f;
+  }
   float* st = MODE == SCAN_WHOLE ? a.state + (((size_t)a.req_rows[blockIdx.x] * a.n_heads + h) * D + d0) * E + e
                                  : a.chunk_state + (((size_t)blockIdx.x * a.n_heads + h) * D + d0) * E + e;
 #pragma unroll
@@ -115,18 +293,22 @@ __global__ __launch_bounds__(THREADS) void gla_scan_kernel(ScanArgs a) {
   // nothing is copied.
   const bool whole = d0 + SLICE <= D;
   struct Row {
-    float a[SLICE], k[SLICE], q[SLICE], v;
+    float a[KIND == KIND_MEMORY ? 1 : SLICE], k[SLICE], q[SLICE], v;
   };
   auto fetch = [&](Row& r, int t) {
     const float* row = a.proj + (size_t)t * a.ld;
     const float* qp = row + a.off_q + h * D + d0;
     const float* kp = row + a.off_k + h * D + d0;
-    const float* ap = a.decay + ((size_t)t * a.n_heads + h) * D + d0;
+    const float* ap = KIND == KIND_MEMORY ? a.keep : a.decay + ((size_t)t * a.n_heads + h) * D + d0;
     r.v = row[a.off_v + h * E + e];
+    if (KIND == KIND_MEMORY) {
+      r.a[0] = a.keep[(size_t)t * a.n_heads + h];
+      r.v *= a.take[(size_t)t * a.n_heads + h];
+    }
 #pragma unroll
     for (int i = 0; i < SLICE; ++i) {
       const bool in = whole || d0 + i < D;
-      r.a[i] = in ? ap[i] : 1.f;
+      if (KIND != KIND_MEMORY) r.a[i] = in ? ap[i] : 1.f;
       r.k[i] = in ? kp[i] : 0.f;
       if (MODE != SCAN_LOCAL) r.q[i] = in ? qp[i] : 0.f;
     }
@@ -135,9 +317,11 @@ __global__ __launch_bounds__(THREADS) void gla_scan_kernel(ScanArgs a) {
     float acc = 0.f;
 #pragma unroll
     for (int i = 0; i < SLICE; ++i) {
-      S[i] = fmaf(r.a[i], S[i], r.k[i] * r.v);
-      if (MODE == SCAN_LOCAL) P[i] *= r.a[i];
-      else acc = fmaf(S[i], r.q[i], acc);
+      const float decay = r.a[KIND == KIND_MEMORY ? 0 : i], kv = r.k[i] * r.v;
+      if (KIND == KIND_BONUS && MODE != SCAN_LOCAL) acc = fmaf(fmaf(U[i], kv, S[i]), r.q[i], acc);
+      S[i] = fmaf(decay, S[i], kv);
+      if (MODE == SCAN_LOCAL) P[i] *= decay;
+      else if (KIND != KIND_BONUS) acc = fmaf(S[i], r.q[i], acc);
     }
     if (MODE != SCAN_LOCAL) a.parts[(((size_t)t * a.n_heads + h) * a.slices + s) * E + e] = acc * a.q_scale;
   };
@@ -168,8 +352,25 @@ __global__ __launch_bounds__(THREADS) void gla_scan_kernel(ScanArgs a) {
 __global__ __launch_bounds__(256) void gla_carry_kernel(ScanArgs a) {
   const int b = blockIdx.y;
   const size_t per = (size_t)a.n_heads * a.D * a.E;
-  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i >= per) return;
+  size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= per) {              // (behind the states' numbers the normalisers', if there are any)
+    i -= per;
+    const size_t hd_all = (size_t)a.n_heads * a.D;
+    if (!a.norm_state || i >= hd_all) return;
+    int c = 0;
+    for (int r = 0; r < b; ++r) c += (a.q_start[r + 1] - a.q_start[r] + a.chunk - 1) / a.chunk;
+    const int last = c + (a.q_start[b + 1] - a.q_start[b] + a.chunk - 1) / a.chunk;
+    float* slot = a.norm_state + (size_t)a.req_rows[b] * hd_all + i;
+    float N = *slot;
+    for (; c < last; ++c) {
+      float* l = a.chunk_norm + (size_t)c * hd_all + i;
+      const float built = *l;
+      *l = N;
+      N = fmaf(a.chunk_decay[(size_t)c * hd_all + i], N, built);
+    }
+    *slot = N;
+    return;
+  }
   int before = 0;
   for (int r = 0; r < b; ++r) before += (a.q_start[r + 1] - a.q_start[r] + a.chunk - 1) / a.chunk;
   const int n = (a.q_start[b + 1] - a.q_start[b] + a.chunk - 1) / a.chunk;
@@ -188,14 +389,22 @@ __global__ __launch_bounds__(256) void gla_carry_kernel(ScanArgs a) {
 extern "C" int llmlab_gla_slices(int D) { return (D + SLICE - 1) / SLICE; }
 
 // proj [rows, ld] float32 holds q at off_q (heads * D), k at off_k, v at off_v (heads * E);
-// decay [rows, heads * D]; state [slots, heads, D, E]; parts [rows, heads, slices, E].
+// decay [rows, heads * D]; state [slots, heads, D, E]; parts [rows, heads, slices, E].  kind: 0 decays per
+// key channel, 1 the same with a bonus [heads * D] for the current row, 2 keep and take [rows, heads]
+// in place of the decays, with the normaliser's state, pieces and (in chunks) chunk_norm.
 // chunk > 0: the three-pass form over chunks of so many rows; chunk_state then holds
 // max_chunks * heads * D * E floats and chunk_decay max_chunks * heads * D, with max_chunks >=
 // rows / chunk + n_reqs.
 extern "C" int llmlab_gla_scan(const float* proj, int ld, int off_q, int off_k, int off_v, const float* decay,
                                float q_scale, int n_heads, int D, int E, float* state, const int* q_start,
                                const int* req_rows, int n_reqs, float* parts, int rows, int chunk,
-                               float* chunk_state, float* chunk_decay, int max_chunks, hipStream_t stream) {
+                               float* chunk_state, float* chunk_decay, int max_chunks, int kind, const float* bonus,
+                               const float* keep, const float* take, float* norm_state, float* norm_parts,
+                               float* chunk_norm, hipStream_t stream) {
+  LLMLAB_REQUIRE(kind >= KIND_DECAY && kind <= KIND_MEMORY && (kind == KIND_MEMORY || decay) &&
+                     (kind != KIND_BONUS || bonus) &&
+                     (kind != KIND_MEMORY || (keep && take && norm_state && norm_parts && (chunk <= 0 || chunk_norm))),
+                 "gla_scan: an operand of kind %d is missing", kind);
   LLMLAB_REQUIRE(n_reqs >= 0 && n_heads > 0 && D > 0 && E > 0, "gla_scan: bad sizes reqs=%d heads=%d D=%d E=%d", n_reqs,
                  n_heads, D, E);
   const int slices = (D + SLICE - 1) / SLICE;
@@ -206,20 +415,27 @@ extern "C" int llmlab_gla_scan(const float* proj, int ld, int off_q, int off_k, 
                  "gla_scan: too many heads, columns or requests");
   if (n_reqs == 0) return 0;
   ScanArgs a{proj, ld, off_q, off_k, off_v, decay, q_scale, n_heads, D, E, cols, slices, state, q_start, req_rows, parts,
-             n_reqs, chunk, chunk_state, chunk_decay};
+             n_reqs, chunk, chunk_state, chunk_decay, bonus, keep, take, kind == KIND_MEMORY ? norm_state : nullptr, norm_parts,
+             chunk_norm};
   const bool uniform = cols == 64;
   dim3 block(slices * cols);
-  const unsigned slabs = (E + cols - 1) / cols;
+  const unsigned slabs = (E + cols - 1) / cols + (kind == KIND_MEMORY ? 1 : 0);
   // (blocks of up to 256 threads, heads of up to 64 key channels, are compiled with the
   // registers that leaves them: the rows fetched ahead stay in registers then)
   const bool small = slices * cols <= 256;
-#define LLMLAB_SCAN(MODE, GRIDX)                                                                                  \
-  do {                                                                                                            \
-    const dim3 grid_(GRIDX, n_heads, slabs);                                                                      \
-    if (uniform && small) hipLaunchKernelGGL((gla_scan_kernel<MODE, true, 256>), grid_, block, 0, stream, a);     \
-    else if (uniform) hipLaunchKernelGGL((gla_scan_kernel<MODE, true, 1024>), grid_, block, 0, stream, a);        \
-    else if (small) hipLaunchKernelGGL((gla_scan_kernel<MODE, false, 256>), grid_, block, 0, stream, a);          \
-    else hipLaunchKernelGGL((gla_scan_kernel<MODE, false, 1024>), grid_, block, 0, stream, a);                    \
+#define LLMLAB_SCAN_KIND(MODE, KIND, GRIDX)                                                                           \
+  do {                                                                                                               \
+    const dim3 grid_(GRIDX, n_heads, slabs);                                                                         \
+    if (uniform && small) hipLaunchKernelGGL((gla_scan_kernel<MODE, KIND, true, 256>), grid_, block, 0, stream, a);  \
+    else if (uniform) hipLaunchKernelGGL((gla_scan_kernel<MODE, KIND, true, 1024>), grid_, block, 0, stream, a);     \
+    else if (small) hipLaunchKernelGGL((gla_scan_kernel<MODE, KIND, false, 256>), grid_, block, 0, stream, a);       \
+    else hipLaunchKernelGGL((gla_scan_kernel<MODE, KIND, false, 1024>), grid_, block, 0, stream, a);                 \
+  } while (0)
+#define LLMLAB_SCAN(MODE, GRIDX)                                              \
+  do {                                                                        \
+    if (kind == KIND_DECAY) LLMLAB_SCAN_KIND(MODE, KIND_DECAY, GRIDX);        \
+    else if (kind == KIND_BONUS) LLMLAB_SCAN_KIND(MODE, KIND_BONUS, GRIDX);   \
+    else LLMLAB_SCAN_KIND(MODE, KIND_MEMORY, GRIDX);                          \
   } while (0)
   if (chunk <= 0) {
     LLMLAB_SCAN(SCAN_WHOLE, n_reqs);
@@ -229,11 +445,12 @@ extern "C" int llmlab_gla_scan(const float* proj, int ld, int off_q, int off_k, 
                    "gla_scan: %d rows of %d requests in chunks of %d need room for %d chunks, got %d", rows, n_reqs,
                    chunk, chunks, max_chunks);
     LLMLAB_SCAN(SCAN_LOCAL, chunks);
-    const size_t per = (size_t)n_heads * D * E;
+    const size_t per = (size_t)n_heads * D * E + (kind == KIND_MEMORY ? (size_t)n_heads * D : 0);
     hipLaunchKernelGGL(gla_carry_kernel, dim3((unsigned)((per + 255) / 256), n_reqs), dim3(256), 0, stream, a);
     LLMLAB_SCAN(SCAN_FINISH, chunks);
   }
 #undef LLMLAB_SCAN
+#undef LLMLAB_SCAN_KIND
   LLMLAB_LAUNCH_CHECK("gla_scan");
   return 0;
 }
@@ -242,19 +459,29 @@ extern "C" int llmlab_gla_scan(const float* proj, int ld, int off_q, int off_k, 
 // Block (row, head): o = sum over slices of parts; y = o / sqrt(mean(o^2) + eps) * w[e]
 // (the weight has one entry per value channel, the same for every head; w_per_head: one per
 // head and channel, w[h * E + e]); out = T(y * silu(gate)), silu(g) = g / (1 + exp(-g))
-// (gate_kind 1: y * sigmoid(gate)); gate [rows, ld] float32 at column off_g.
+// (gate_kind 1: y * sigmoid(gate)); gate [rows, ld] float32 at column off_g.  norm_parts [rows, heads,
+// slices] and maxima [rows, heads] (a memory with a normaliser): o is first divided by max(|n . q|,
+// exp(-m)) + 1e-6, n . q the sum of its parts.
+__device__ __forceinline__ float memory_size(float nq, float m) { return fmaxf(fabsf(nq), expf(-m)) + 1e-6f; }
 template <typename T>
 __global__ __launch_bounds__(1024) void gla_output_kernel(const float* __restrict__ parts, int slices, int n_heads, int E,
                                                           const float* __restrict__ w, float eps,
                                                           const float* __restrict__ proj, int ld, int off_g,
                                                           T* __restrict__ out, int w_per_head, int gate_kind,
-                                                          int count) {
+                                                          int count, const float* __restrict__ norm_parts,
+                                                          const float* __restrict__ maxima) {
   __shared__ float red[17];
   const int r = blockIdx.x, h = blockIdx.y, e = threadIdx.x;
   float o = 0.f;
   if (e < E) {
     const float* p = parts + (((size_t)r * n_heads + h) * slices) * E + e;
     for (int s = 0; s < slices; ++s) o += p[(size_t)s * E];
+  }
+  if (norm_parts) {
+    const float* n = norm_parts + ((size_t)r * n_heads + h) * slices;
+    float nq = 0.f;
+    for (int s = 0; s < slices; ++s) nq += n[s];
+    o = o / memory_size(nq, maxima[(size_t)r * n_heads + h]);
   }
   const float ms = block_sum(o * o, red) / (float)count;      // (count < E: the channels behind it are zeros)
   if (e < E) {
@@ -269,7 +496,9 @@ __global__ __launch_bounds__(1024) void gla_output_kernel(const float* __restric
 // norm_count > 0: the mean of the squares is taken over so many channels (the others are zeros)
 extern "C" int llmlab_gla_output(const float* parts, int rows, int n_heads, int D, int E, const float* w, float eps,
                                  const float* proj, int ld, int off_g, void* out, int dtype, int slices_given,
-                                 int w_per_head, int gate_kind, int norm_count, hipStream_t stream) {
+                                 int w_per_head, int gate_kind, int norm_count, const float* norm_parts,
+                                 const float* maxima, hipStream_t stream) {
+  LLMLAB_REQUIRE((norm_parts == nullptr) == (maxima == nullptr), "gla_output: a normaliser comes with its maxima");
   LLMLAB_REQUIRE(rows >= 0 && n_heads > 0 && n_heads <= 65535 && E > 0 && E <= 1024,
                  "gla_output: bad sizes rows=%d heads=%d E=%d", rows, n_heads, E);
   LLMLAB_REQUIRE(gate_kind == 0 || gate_kind == 1, "gla_output: unknown gate %d", gate_kind);
@@ -280,10 +509,10 @@ extern "C" int llmlab_gla_output(const float* parts, int rows, int n_heads, int 
   dim3 grid(rows, n_heads), block((E + 63) / 64 * 64);
   if (dtype == DT_BF16)
     hipLaunchKernelGGL(gla_output_kernel<bf16_t>, grid, block, 0, stream, parts, slices, n_heads, E, w, eps, proj, ld,
-                       off_g, (bf16_t*)out, w_per_head, gate_kind, count);
+                       off_g, (bf16_t*)out, w_per_head, gate_kind, count, norm_parts, maxima);
   else
     hipLaunchKernelGGL(gla_output_kernel<float>, grid, block, 0, stream, parts, slices, n_heads, E, w, eps, proj, ld,
-                       off_g, (float*)out, w_per_head, gate_kind, count);
+                       off_g, (float*)out, w_per_head, gate_kind, count, norm_parts, maxima);
   LLMLAB_LAUNCH_CHECK("gla_output");
   return 0;
 }

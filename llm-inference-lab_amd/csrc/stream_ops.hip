@@ -5,8 +5,11 @@
 //   gated_add       x += y * sigmoid(gate + bias)
 //   softcap         x = cap * tanh(x / cap)
 //   rmsnorm_add     x += y / sqrt(mean(y^2) + eps) * w   (a norm on a sublayer's result, before the sum;
-//                   the norm that reads the stream next may run in the same launch)
+//                   the norm that reads the stream next, or a rounded copy, may come out of the same launch)
 //   scaled_sum      out = a * y1 + b * y2
+//   normed_sum      out = a * norm1(y1) + b * norm2(y2)
+//   shift_mix       out_m = h + (previous row's h - h) * mix_m, for one or several mixes
+//   poly_norm       out = a N(z) + b N(z^2) + c N(z^3) + e, N(v) = v / sqrt(mean(v^2) + eps)
 // What a request's earlier steps left (its last token, the last inputs of a convolution) lives in
 // per-request slots; a step's rows of one request are adjacent.
 #include "common.h"
@@ -410,9 +413,10 @@ extern "C" int llmlab_gated_add(float* x, const float* y, int pieces, size_t pie
 // pieces, in the pieces' order).  All float32.  A thread keeps up to NORM_ADD_KEEP of the row's numbers
 // in registers between the two passes; wider rows are read again.
 constexpr int NORM_ADD_KEEP = 8;
-// NEXT: the norm that reads the stream next runs in the same launch on the row's new numbers:
-// next_out[r, c] = T(x[r, c] / sqrt(mean(x[r]^2) + next_eps) * next_w[c]).
-template <typename T, bool NEXT>
+// NEXT 1: the norm that reads the stream next runs in the same launch on the row's new numbers:
+// next_out[r, c] = T(x[r, c] / sqrt(mean(x[r]^2) + next_eps) * next_w[c]).  NEXT 2: a copy of them,
+// next_out[r, c] = T(x[r, c]).
+template <typename T, int NEXT>
 __global__ __launch_bounds__(256) void rmsnorm_add_kernel(float* __restrict__ x, const float* __restrict__ y, int pieces,
                                                           size_t piece_stride, const float* __restrict__ w, float eps,
                                                           int width, const float* __restrict__ next_w, float next_eps,
@@ -448,15 +452,17 @@ __global__ __launch_bounds__(256) void rmsnorm_add_kernel(float* __restrict__ x,
     if (c < width) {
       keep[n] = xs[n] + keep[n] * inv * ws[n];
       x[row + c] = keep[n];
+      if (NEXT == 2) next_out[row + c] = from_float<T>(keep[n]);
       ss2 = fmaf(keep[n], keep[n], ss2);
     }
   }
   for (int c = threadIdx.x + 256 * NORM_ADD_KEEP; c < width; c += 256) {
     const float v = x[row + c] + value(c) * inv * w[c];
     x[row + c] = v;
+    if (NEXT == 2) next_out[row + c] = from_float<T>(v);
     ss2 = fmaf(v, v, ss2);
   }
-  if (!NEXT) return;
+  if (NEXT != 1) return;
   const float inv2 = 1.0f / sqrtf(block_sum(ss2, red) / (float)width + next_eps);
 #pragma unroll
   for (int n = 0; n < NORM_ADD_KEEP; ++n) {
@@ -472,17 +478,17 @@ extern "C" int llmlab_rmsnorm_add(float* x, const float* y, int pieces, size_t p
                                   int next_dtype, hipStream_t stream) {
   LLMLAB_REQUIRE(rows >= 0 && width > 0 && pieces >= 1 && x && y && w, "rmsnorm_add: bad arguments rows=%d width=%d pieces=%d",
                  rows, width, pieces);
-  LLMLAB_REQUIRE((next_w == nullptr) == (next_out == nullptr), "rmsnorm_add: the next norm needs its weight and its output");
+  LLMLAB_REQUIRE(next_w == nullptr || next_out, "rmsnorm_add: the next norm needs an output");
   if (rows == 0) return 0;
-  if (!next_out)
-    hipLaunchKernelGGL((rmsnorm_add_kernel<float, false>), dim3(rows), dim3(256), 0, stream, x, y, pieces, piece_stride, w,
-                       eps, width, nullptr, 0.f, nullptr);
-  else if (next_dtype == DT_BF16)
-    hipLaunchKernelGGL((rmsnorm_add_kernel<bf16_t, true>), dim3(rows), dim3(256), 0, stream, x, y, pieces, piece_stride, w,
-                       eps, width, next_w, next_eps, (bf16_t*)next_out);
-  else
-    hipLaunchKernelGGL((rmsnorm_add_kernel<float, true>), dim3(rows), dim3(256), 0, stream, x, y, pieces, piece_stride, w,
-                       eps, width, next_w, next_eps, (float*)next_out);
+#define LLMLAB_NORM_ADD(T, NEXT)                                                                                           \
+  hipLaunchKernelGGL((rmsnorm_add_kernel<T, NEXT>), dim3(rows), dim3(256), 0, stream, x, y, pieces, piece_stride, w, eps, \
+                     width, next_w, next_eps, (T*)next_out)
+  if (!next_out) LLMLAB_NORM_ADD(float, 0);
+  else if (next_w && next_dtype == DT_BF16) LLMLAB_NORM_ADD(bf16_t, 1);
+  else if (next_w) LLMLAB_NORM_ADD(float, 1);
+  else if (next_dtype == DT_BF16) LLMLAB_NORM_ADD(bf16_t, 2);
+  else LLMLAB_NORM_ADD(float, 2);
+#undef LLMLAB_NORM_ADD
   LLMLAB_LAUNCH_CHECK("rmsnorm_add");
   return 0;
 }
@@ -501,6 +507,205 @@ extern "C" int llmlab_scaled_sum(float* out, const float* y1, float a, const flo
   const int blocks = (int)((n + 255) / 256 < 65535 ? (n + 255) / 256 : 65535);
   hipLaunchKernelGGL(scaled_sum_kernel, dim3(blocks), dim3(256), 0, stream, out, y1, a, y2, b, n);
   LLMLAB_LAUNCH_CHECK("scaled_sum");
+  return 0;
+}
+
+// out[r] = a * norm(y1[r]) * w1 + b * norm(y2[r]) * w2, each row over its own root mean square (eps
+// inside the root).  One block a row, all float32.
+__global__ __launch_bounds__(256) void normed_sum_kernel(float* __restrict__ out, const float* __restrict__ y1,
+                                                         const float* __restrict__ w1, float a, const float* __restrict__ y2,
+                                                         const float* __restrict__ w2, float b, float eps, int width) {
+  __shared__ float red1[17], red2[17];
+  const size_t row = (size_t)blockIdx.x * width;
+  float k1[NORM_ADD_KEEP], k2[NORM_ADD_KEEP];
+  float s1 = 0.f, s2 = 0.f;
+#pragma unroll
+  for (int n = 0; n < NORM_ADD_KEEP; ++n) {
+    const int c = threadIdx.x + 256 * n;
+    k1[n] = c < width ? y1[row + c] : 0.f;
+    k2[n] = c < width ? y2[row + c] : 0.f;
+    s1 = fmaf(k1[n], k1[n], s1);
+    s2 = fmaf(k2[n], k2[n], s2);
+  }
+  for (int c = threadIdx.x + 256 * NORM_ADD_KEEP; c < width; c += 256) {
+    const float v1 = y1[row + c], v2 = y2[row + c];
+    s1 = fmaf(v1, v1, s1);
+    s2 = fmaf(v2, v2, s2);
+  }
+  const float i1 = a / sqrtf(block_sum(s1, red1) / (float)width + eps);
+  const float i2 = b / sqrtf(block_sum(s2, red2) / (float)width + eps);
+#pragma unroll
+  for (int n = 0; n < NORM_ADD_KEEP; ++n) {
+    const int c = threadIdx.x + 256 * n;
+    if (c < width) out[row + c] = k1[n] * i1 * w1[c] + k2[n] * i2 * w2[c];
+  }
+  for (int c = threadIdx.x + 256 * NORM_ADD_KEEP; c < width; c += 256)
+    out[row + c] = y1[row + c] * i1 * w1[c] + y2[row + c] * i2 * w2[c];
+}
+
+extern "C" int llmlab_normed_sum(float* out, const float* y1, const float* w1, float a, const float* y2, const float* w2,
+                                 float b, float eps, int rows, int width, hipStream_t stream) {
+  LLMLAB_REQUIRE(rows >= 0 && width > 0 && out && y1 && y2 && w1 && w2, "normed_sum: bad arguments rows=%d width=%d", rows,
+                 width);
+  if (rows == 0) return 0;
+  hipLaunchKernelGGL(normed_sum_kernel, dim3(rows), dim3(256), 0, stream, out, y1, w1, a, y2, w2, b, eps, width);
+  LLMLAB_LAUNCH_CHECK("normed_sum");
+  return 0;
+}
+
+// ------------------------------------------------------------------ a row mixed with the one before it
+// out[m][r, c] = TO(h[r, c] + (p - h[r, c]) * mix[m, c]) for m < n_mix, p the same channel of the row
+// before r in its request: row r - 1 of the step, or, for the request's first row of the step,
+// state[slot] (zeros before a sequence's start: a slot is zeroed when a request is admitted).  The
+// request's first row's block then stores the request's LAST row there, after it has read the old
+// one (a thread owns its channels, no other block touches the slot).  h, state: TI.  One block a row.
+__device__ __forceinline__ floatx4 load4(const float* p) { return *(const floatx4*)p; }
+__device__ __forceinline__ floatx4 load4(const bf16_t* p) {
+  const bf16x4 t = *(const bf16x4*)p;
+  return floatx4{(float)t[0], (float)t[1], (float)t[2], (float)t[3]};
+}
+__device__ __forceinline__ void store4(float* p, floatx4 v) { *(floatx4*)p = v; }
+__device__ __forceinline__ void store4(bf16_t* p, floatx4 v) {
+  *(bf16x4*)p = bf16x4{(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
+}
+
+template <typename TI, typename TO, bool VEC>
+__global__ __launch_bounds__(256) void shift_mix_kernel(const TI* __restrict__ h, const float* __restrict__ mix, int n_mix,
+                                                        TI* __restrict__ state, const int* __restrict__ row_req,
+                                                        const int* __restrict__ q_start, const int* __restrict__ req_rows,
+                                                        TO* __restrict__ out, size_t out_stride, int width) {
+  const int r = blockIdx.x, b = row_req[r], first = q_start[b];
+  const bool lead = r == first;
+  TI* st = state + (size_t)req_rows[b] * width;
+  const TI* own_row = h + (size_t)r * width;
+  const TI* before = lead ? st : own_row - width;
+  const TI* latest = h + (size_t)(q_start[b + 1] - 1) * width;
+  if (VEC) {
+    for (int c = threadIdx.x * 4; c < width; c += blockDim.x * 4) {
+      const floatx4 own = load4(own_row + c), d = load4(before + c) - own;
+      for (int m = 0; m < n_mix; ++m)
+        store4(out + m * out_stride + (size_t)r * width + c, own + d * load4(mix + (size_t)m * width + c));
+      if (lead) store4(st + c, load4(latest + c));
+    }
+  } else {
+    for (int c = threadIdx.x; c < width; c += blockDim.x) {
+      const float own = to_float(own_row[c]), d = to_float(before[c]) - own;
+      for (int m = 0; m < n_mix; ++m)
+        out[m * out_stride + (size_t)r * width + c] = from_float<TO>(fmaf(d, mix[(size_t)m * width + c], own));
+      if (lead) st[c] = latest[c];
+    }
+  }
+}
+
+extern "C" int llmlab_shift_mix(const void* h, int h_dtype, const float* mix, int n_mix, void* state, const int* row_req,
+                                const int* q_start, const int* req_rows, void* out, int out_dtype, int rows, int width,
+                                hipStream_t stream) {
+  LLMLAB_REQUIRE(rows >= 0 && width > 0 && n_mix > 0 && h && mix && state && row_req && q_start && req_rows && out,
+                 "shift_mix: bad arguments rows=%d width=%d mixes=%d", rows, width, n_mix);
+  if (rows == 0) return 0;
+  const bool vec = width % 4 == 0 && (((uintptr_t)h | (uintptr_t)mix | (uintptr_t)state | (uintptr_t)out) & 15) == 0;
+  const size_t stride = (size_t)rows * width;
+#define LLMLAB_SHIFT(TI, TO, VEC)                                                                                          \
+  hipLaunchKernelGGL((shift_mix_kernel<TI, TO, VEC>), dim3(rows), dim3(256), 0, stream, (const TI*)h, mix, n_mix,         \
+                     (TI*)state, row_req, q_start, req_rows, (TO*)out, stride, width)
+#define LLMLAB_SHIFT_ANY(TI, TO)        \
+  do {                                  \
+    if (vec) LLMLAB_SHIFT(TI, TO, true); \
+    else LLMLAB_SHIFT(TI, TO, false);   \
+  } while (0)
+  if (h_dtype == DT_F32 && out_dtype == DT_F32) LLMLAB_SHIFT_ANY(float, float);
+  else if (h_dtype == DT_F32) LLMLAB_SHIFT_ANY(float, bf16_t);
+  else {
+    LLMLAB_REQUIRE(out_dtype == DT_BF16, "shift_mix: bfloat16 rows give bfloat16 mixes");
+    LLMLAB_SHIFT_ANY(bf16_t, bf16_t);
+  }
+#undef LLMLAB_SHIFT_ANY
+#undef LLMLAB_SHIFT
+  LLMLAB_LAUNCH_CHECK("shift_mix");
+  return 0;
+}
+
+// ------------------------------------------------------------------ norms of a row's powers
+// out[r, c] = T(a N(z) + b N(z^2) + c N(z^3) + e), powers element by element, N(v) = v / sqrt(mean(v^2) +
+// eps) over the row's first `count` numbers (the ones behind them are zeros of padded products);
+// a, b, c, e = coef[0 .. 3].  One block a row; a thread keeps up to POLY_KEEP quads of the row in
+// registers between the sums and the result, wider rows are read again.  columns: a multiple of 4.
+constexpr int POLY_KEEP = 5;
+template <typename T>
+__global__ __launch_bounds__(1024) void poly_norm_kernel(const float* __restrict__ z, const float* __restrict__ coef, float eps,
+                                                         int count, int columns, T* __restrict__ out) {
+  __shared__ float red[16][3];
+  __shared__ float s_inv[3];
+  const size_t row = (size_t)blockIdx.x * columns;
+  const int threads = blockDim.x, quads = columns >> 2;
+  const float a = coef[0], b = coef[1], c3 = coef[2], e = coef[3];
+  floatx4 keep[POLY_KEEP];
+  float s[3] = {0.f, 0.f, 0.f};
+  auto sums = [&](const floatx4& v) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float v2 = v[i] * v[i], v4 = v2 * v2;
+      s[0] += v2;
+      s[1] += v4;
+      s[2] = fmaf(v4, v2, s[2]);
+    }
+  };
+#pragma unroll
+  for (int n = 0; n < POLY_KEEP; ++n) {
+    const int i = threadIdx.x + threads * n;
+    keep[n] = i < quads ? load4(z + row + 4 * (size_t)i) : floatx4{0.f, 0.f, 0.f, 0.f};
+  }
+#pragma unroll
+  for (int n = 0; n < POLY_KEEP; ++n) sums(keep[n]);
+  for (int i = threadIdx.x + threads * POLY_KEEP; i < quads; i += threads) sums(load4(z + row + 4 * (size_t)i));
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = threads >> 6;
+#pragma unroll
+  for (int k = 0; k < 3; ++k) {
+    s[k] = wave_sum(s[k]);
+    if (lane == 0) red[wave][k] = s[k];
+  }
+  __syncthreads();
+  if (threadIdx.x < 3) {
+    float t = 0.f;
+    for (int i = 0; i < waves; ++i) t += red[i][threadIdx.x];
+    s_inv[threadIdx.x] = 1.0f / sqrtf(t / (float)count + eps);
+  }
+  __syncthreads();
+  const float ka = a * s_inv[0], kb = b * s_inv[1], kc = c3 * s_inv[2];
+  auto result = [&](const floatx4& v) {
+    floatx4 o;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[i] = fmaf(fmaf(fmaf(kc, v[i], kb), v[i], ka), v[i], e);
+    return o;
+  };
+#pragma unroll
+  for (int n = 0; n < POLY_KEEP; ++n) {
+    const int i = threadIdx.x + threads * n;
+    if (i < quads) store4(out + row + 4 * (size_t)i, result(keep[n]));
+  }
+  for (int i = threadIdx.x + threads * POLY_KEEP; i < quads; i += threads)
+    store4(out + row + 4 * (size_t)i, result(load4(z + row + 4 * (size_t)i)));
+}
+
+extern "C" int llmlab_poly_norm(const float* z, const float* coef, float eps, int rows, int count, int columns, void* out,
+                                int dtype, hipStream_t stream) {
+  LLMLAB_REQUIRE(rows >= 0 && count > 0 && columns >= count && columns % 4 == 0 && z && coef && out,
+                 "poly_norm: bad arguments rows=%d count=%d columns=%d", rows, count, columns);
+  LLMLAB_REQUIRE((((uintptr_t)z | (uintptr_t)out) & 15) == 0, "poly_norm: rows are 16-byte aligned");
+  if (rows == 0) return 0;
+  // few rows: as many threads as keep a row in registers; many rows: blocks of which several share a unit
+  const int quads = columns / 4, most = rows <= 256 ? 1024 : 256;
+  int threads = (quads + 63) / 64 * 64;
+  if (threads > most) threads = most;
+  while (threads < 1024 && quads > threads * POLY_KEEP) threads *= 2;
+  if (threads > 1024) threads = 1024;
+  if (dtype == DT_BF16)
+    hipLaunchKernelGGL(poly_norm_kernel<bf16_t>, dim3(rows), dim3(threads), 0, stream, z, coef, eps, count, columns,
+                       (bf16_t*)out);
+  else
+    hipLaunchKernelGGL(poly_norm_kernel<float>, dim3(rows), dim3(threads), 0, stream, z, coef, eps, count, columns,
+                       (float*)out);
+  LLMLAB_LAUNCH_CHECK("poly_norm");
   return 0;
 }
 

@@ -188,6 +188,185 @@ extern "C" int llmlab_project_rotate_write(const float* proj, int ld, int rows, 
   return 0;
 }
 
+// The same for layers whose projections pass a short causal convolution, turn, and are brought to
+// unit root mean square head by head.  proj[r, :] = q | k | v (float32 sums; heads of D, D and E
+// channels).  Channel by channel: `bias` is added (null: none); with taps > 0 the convolution over
+// the positions of the row's request, y_t = sum_j w[c, j] u_(t - taps + 1 + j), u the biased
+// projection, inputs from before the step from state [slots, taps - 1, channels] float32 (zeros before
+// a sequence's start).  Of every query and key head the first rot_dims channels turn by positions[r] *
+// freq[i]: channel i with i + rot_dims / 2, or (neighbours) channel 2i with 2i + 1.  unit: the head is
+// then divided by its root mean square over D.  Queries and keys are laid out DK >= D channels wide
+// (zeros behind), values E.  A wave a head; the head's numbers lie in LDS between the steps.
+// own_state: every request brings one row, and the row's block moves its slot on after it has read
+// it (a thread owns its channels); else conv_slots_kernel does.
+struct ConvArgs {
+  const float* proj; int ld, n_heads, n_kv, D, DK, E; const float* bias; const float* w; int taps;
+  float* state; const int* q_start; const int* req_rows; const float* freq; int rot_dims, neighbours, unit; float eps;
+  int page_size; const int* positions; const int* row_req; const int* table; int max_pages, own_state;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void project_conv_write_kernel(ConvArgs a, T* __restrict__ q_out,
+                                                                 T* __restrict__ k_cache, T* __restrict__ v_cache) {
+  extern __shared__ float conv_lds[];           // cos [half], sin [half], then D numbers a wave
+  const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
+  const int half = a.rot_dims >> 1, D = a.D, E = a.E, keep = a.taps - 1;
+  float* s_cos = conv_lds;
+  float* s_sin = conv_lds + half;
+  float* s_head = conv_lds + 2 * half + wave * (D > E ? D : E);
+  const float* src = a.proj + (size_t)r * a.ld;
+  const int pos = a.positions[r], b = a.row_req[r];
+  const int inside = r - a.q_start[b];          // rows of this request before r in the step
+  const int q_size = a.n_heads * D, k_size = a.n_kv * D, channels = q_size + k_size + a.n_kv * E;
+  float* st = keep > 0 ? a.state + (size_t)a.req_rows[b] * keep * channels : nullptr;
+  for (int i = threadIdx.x; i < half; i += blockDim.x) {
+    float sn, cs;
+    sincosf((float)pos * a.freq[i], &sn, &cs);
+    s_cos[i] = cs;
+    s_sin[i] = sn;
+  }
+  __syncthreads();
+  const int page = a.table[(size_t)b * a.max_pages + pos / a.page_size];
+  const int slot = pos % a.page_size;
+  // channel c of the row after bias and convolution
+  auto channel = [&](int c) {
+    const float bias = a.bias ? a.bias[c] : 0.f;
+    const float own = src[c] + bias;
+    if (a.taps <= 0) return own;
+    const float* w = a.w + (size_t)c * a.taps;
+    float acc = 0.f;
+    for (int j = 0; j < keep; ++j) {
+      const int back = keep - j;
+      const float u = back <= inside ? src[c - (ptrdiff_t)back * a.ld] + bias
+                                     : st[(size_t)(keep - (back - inside)) * channels + c];
+      acc = fmaf(w[j], u, acc);
+    }
+    acc = fmaf(w[keep], own, acc);
+    if (a.own_state && keep > 0) {
+      for (int j = 0; j + 1 < keep; ++j) st[(size_t)j * channels + c] = st[(size_t)(j + 1) * channels + c];
+      st[(size_t)(keep - 1) * channels + c] = own;
+    }
+    return acc;
+  };
+  const int heads = a.n_heads + 2 * a.n_kv;     // query heads, key heads, value heads
+  for (int h0 = 0; h0 < heads; h0 += waves) {   // (every wave takes part in the barriers)
+    const int h = h0 + wave;
+    const bool turns = h < a.n_heads + a.n_kv, live = h < heads;
+    const int width = turns ? D : E;
+    const int c0 = turns ? h * D : q_size + k_size + (h - a.n_heads - a.n_kv) * E;
+    if (live)
+      for (int d = lane; d < width; d += 64) s_head[d] = channel(c0 + d);
+    __syncthreads();
+    if (live && turns) {
+      float ss = 0.f;
+      auto turned = [&](int d) {
+        float x = s_head[d];
+        if (d < a.rot_dims) {
+          const int i = a.neighbours ? d >> 1 : (d < half ? d : d - half);
+          const bool first = a.neighbours ? (d & 1) == 0 : d < half;
+          const float other = s_head[a.neighbours ? d ^ 1 : (first ? d + half : d - half)];
+          x = first ? x * s_cos[i] - other * s_sin[i] : x * s_cos[i] + other * s_sin[i];
+        }
+        return x;
+      };
+      float inv = 1.f;
+      if (a.unit) {
+        for (int d = lane; d < D; d += 64) {
+          const float x = turned(d);
+          ss = fmaf(x, x, ss);
+        }
+        inv = 1.0f / sqrtf(wave_sum(ss) / (float)D + a.eps);
+      }
+      T* dst = h < a.n_heads ? q_out + ((size_t)r * a.n_heads + h) * a.DK
+                             : k_cache + (((size_t)page * a.n_kv + (h - a.n_heads)) * a.page_size + slot) * a.DK;
+      for (int d = lane; d < a.DK; d += 64) dst[d] = from_float<T>(d < D ? turned(d) * inv : 0.f);
+    } else if (live) {
+      const int g = h - a.n_heads - a.n_kv;
+      for (int e = lane; e < E; e += 64)
+        v_cache[((size_t)page * a.n_kv + g) * a.page_size * E + value_index(slot, e, E)] = from_float<T>(s_head[e]);
+    }
+    __syncthreads();
+  }
+}
+
+// The slots after the step: the last taps - 1 inputs (biased projections) of every request.  The
+// block of a request's first row does it for the request; a thread reads place n + s before it
+// writes place s, in rising order, so nothing is read after it changed.
+__global__ __launch_bounds__(256) void conv_slots_kernel(ConvArgs a) {
+  const int r = blockIdx.x, b = a.row_req[r], first = a.q_start[b];
+  if (r != first) return;
+  const int n = a.q_start[b + 1] - first, keep = a.taps - 1;
+  const int channels = (a.n_heads + a.n_kv) * a.D + a.n_kv * a.E;
+  float* st = a.state + (size_t)a.req_rows[b] * keep * channels;
+  for (int c = threadIdx.x; c < channels; c += blockDim.x) {
+    const float bias = a.bias ? a.bias[c] : 0.f;
+    for (int s = 0; s < keep; ++s) {
+      const int at = n + s;                    // place in [what the slot held | the step's rows]
+      st[(size_t)s * channels + c] =
+          at < keep ? st[(size_t)at * channels + c] : a.proj[(size_t)(first + at - keep) * a.ld + c] + bias;
+    }
+  }
+}
+
+extern "C" int llmlab_project_conv_write(const float* proj, int ld, int rows, int n_heads, int n_kv, int D, int DK, int E,
+                                         const float* bias, const float* w, int taps, float* state, const int* q_start,
+                                         const int* req_rows, const float* freq, int rot_dims, int neighbours, int unit,
+                                         float eps, void* q_out, void* k_cache, void* v_cache, int dtype, int page_size,
+                                         const int* positions, const int* row_req, const int* table, int max_pages,
+                                         int one_row_each, hipStream_t stream) {
+  LLMLAB_REQUIRE(rows >= 0 && n_heads > 0 && n_kv > 0 && D > 0 && DK >= D && E > 0 && page_size > 0 && page_size % 4 == 0 &&
+                     D <= 2048 && E <= 2048,
+                 "project_conv_write: bad sizes rows=%d heads=%d kv=%d D=%d/%d E=%d page=%d", rows, n_heads, n_kv, D, DK, E,
+                 page_size);
+  LLMLAB_REQUIRE(ld >= (n_heads + n_kv) * D + n_kv * E, "project_conv_write: rows of %d numbers do not hold the projections",
+                 ld);
+  LLMLAB_REQUIRE(taps >= 0 && (taps == 0 || w) && (taps <= 1 || (state && req_rows)),
+                 "project_conv_write: %d taps need their weights and the requests' slots", taps);
+  LLMLAB_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= D && (rot_dims == 0 || freq),
+                 "project_conv_write: %d of %d channels cannot turn in pairs", rot_dims, D);
+  LLMLAB_REQUIRE(q_out && k_cache && v_cache && positions && row_req && table && q_start,
+                 "project_conv_write: queries, pages and the step's description are needed");
+  if (rows == 0) return 0;
+  ConvArgs a{proj, ld, n_heads, n_kv, D, DK, E, bias, w, taps, state, q_start, req_rows, freq, rot_dims, neighbours, unit, eps,
+             page_size, positions, row_req, table, max_pages, one_row_each};
+  const size_t lds = (size_t)(rot_dims + 4 * (D > E ? D : E)) * sizeof(float);
+  if (dtype == DT_BF16)
+    hipLaunchKernelGGL(project_conv_write_kernel<bf16_t>, dim3(rows), dim3(256), lds, stream, a, (bf16_t*)q_out,
+                       (bf16_t*)k_cache, (bf16_t*)v_cache);
+  else
+    hipLaunchKernelGGL(project_conv_write_kernel<float>, dim3(rows), dim3(256), lds, stream, a, (float*)q_out,
+                       (float*)k_cache, (float*)v_cache);
+  if (taps > 1 && !one_row_each) hipLaunchKernelGGL(conv_slots_kernel, dim3(rows), dim3(256), 0, stream, a);
+  LLMLAB_LAUNCH_CHECK("project_conv_write");
+  return 0;
+}
+
+// out[r, c] = T(out[r, c] * sigmoid(gate[r, c])): a gate per channel of the heads' outputs, read
+// from the float32 projections (row stride ld).
+template <typename T>
+__global__ void gate_channels_kernel(T* __restrict__ out, const float* __restrict__ gate, int ld, int width, size_t n) {
+  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
+    const size_t r = i / width;
+    const float g = gate[r * ld + (i - r * width)];
+    out[i] = from_float<T>(to_float(out[i]) / (1.f + __expf(-g)));
+  }
+}
+
+extern "C" int llmlab_gate_channels(void* out, const float* gate, int ld, int rows, int width, int dtype,
+                                    hipStream_t stream) {
+  LLMLAB_REQUIRE(rows >= 0 && width > 0 && ld >= width && out && gate, "gate_channels: bad arguments rows=%d width=%d ld=%d",
+                 rows, width, ld);
+  const size_t n = (size_t)rows * width;
+  if (n == 0) return 0;
+  const int blocks = (int)((n + 255) / 256 < 65535 ? (n + 255) / 256 : 65535);
+  if (dtype == DT_BF16)
+    hipLaunchKernelGGL(gate_channels_kernel<bf16_t>, dim3(blocks), dim3(256), 0, stream, (bf16_t*)out, gate, ld, width, n);
+  else
+    hipLaunchKernelGGL(gate_channels_kernel<float>, dim3(blocks), dim3(256), 0, stream, (float*)out, gate, ld, width, n);
+  LLMLAB_LAUNCH_CHECK("gate_channels");
+  return 0;
+}
+
 static int g_force_plain = 0;      // tests and measurements: no matrix-core kernel
 extern "C" void llmlab_debug_windowed_attention_plain(int on) { g_force_plain = on; }
 static int g_private_tiles = 0;    // tests and measurements: prompts by the kernel whose waves fetch their own tiles
@@ -195,7 +374,8 @@ extern "C" void llmlab_debug_windowed_attention_private_tiles(int on) { g_privat
 
 // ------------------------------------------------------------------ attention
 // The query at position i of its request attends to the keys i - window < j <= i and to the
-// kept prefix j < min(keep_first, i + 1); window <= 0: every j <= i.  Scores, the running maximum, the denominator
+// kept prefix j < min(keep_first, i + 1); window <= 0: every j <= i, or, with chunk > 0, the keys
+// of its own chunk of positions, i - i % chunk <= j <= i.  Scores, the running maximum, the denominator
 // and the weighted sum of values are float32.  With a sink the running maximum starts at
 // sink[h] and the denominator at 1 = exp(sink - sink), and nothing is added to the weighted sum.
 // mode 1 (MODE_SIGMOID): no softmax; the weight of a visible key is sigmoid(score + sink[h])
@@ -208,9 +388,16 @@ __device__ __forceinline__ float sigmoid_weight(float s) { return 1.0f / (1.0f +
 // Both kernels walk the keys in two runs, each from an aligned start, and mask key by key:
 // the kept prefix [0, min(keep_first, B)) and [B, i], where B is the window's first key
 // rounded down (to a quad of keys here, to 16 in the matrix-core kernel).
-__device__ __forceinline__ bool sees(int i, int j, int window, int keep_first) {
-  return j <= i && (window <= 0 || i - j < window || j < keep_first);
-}
+struct Mask {
+  int window, keep_first, chunk;
+  // the lowest key that the query at position i sees beside the kept prefix (it never falls as i rises)
+  __device__ __forceinline__ int low(int i) const {
+    if (window > 0) return i - window + 1 > 0 ? i - window + 1 : 0;
+    return chunk > 0 ? i - i % chunk : 0;
+  }
+};
+// (lo: the mask's low(i), taken once per query)
+__device__ __forceinline__ bool sees(int i, int j, int lo, int keep_first) { return j <= i && (j >= lo || j < keep_first); }
 
 // ---- plain kernel: one wave per (row, head); float32 products.  Keys are taken 64 at a
 // time: lane n scores one key (its own row of D numbers), the weights go through LDS, then
@@ -265,7 +452,7 @@ template <typename T>
 __global__ __launch_bounds__(64) void sink_window_attention_kernel(
     const T* __restrict__ q, int n_heads, int n_kv, int D, int E, const T* __restrict__ k_cache,
     const T* __restrict__ v_cache, const int* __restrict__ table, int max_pages, int page_size,
-    const int* __restrict__ positions, const int* __restrict__ row_req, int window, int keep_first,
+    const int* __restrict__ positions, const int* __restrict__ row_req, Mask mask,
     const float* __restrict__ sink, float scale, T* __restrict__ out, const int* __restrict__ q_start, int long_from,
     int mode) {
   if (long_from > 0) {      // (rows of requests that bring many rows are the other kernel's)
@@ -282,9 +469,9 @@ __global__ __launch_bounds__(64) void sink_window_attention_kernel(
   const int* pages = table + (size_t)row_req[r] * max_pages;
   for (int d = lane; d < D; d += 64) qs[d] = to_float(q[((size_t)r * n_heads + h) * D + d]) * scale;
   __syncthreads();
-  const int lo = window > 0 ? (i - window + 1 > 0 ? i - window + 1 : 0) : 0;
+  const int lo = mask.low(i);
   const int b_start = lo & ~3;
-  const int a_end = keep_first < b_start ? keep_first : b_start;
+  const int a_end = mask.keep_first < b_start ? mask.keep_first : b_start;
   const bool sig = mode == MODE_SIGMOID;
   const float bias = (sig && sink) ? sink[h] : 0.f;
   float m = sig ? 0.f : (sink ? sink[h] : NEG_INF);
@@ -297,7 +484,7 @@ __global__ __launch_bounds__(64) void sink_window_attention_kernel(
     const int end = run == 0 ? a_end : i + 1;          // keys [first, end)
     for (int base = first; base < end; base += 64) {
       const int j = base + lane;
-      const bool valid = j < end && sees(i, j, window, keep_first);
+      const bool valid = j < end && sees(i, j, lo, mask.keep_first);
       float s = NEG_INF;
       if (j < end) {
         const int page = pages[j / page_size];
@@ -364,10 +551,11 @@ struct Running {
 // the queries; b_start: the lowest window's first key rounded down to 16).
 struct KeyTiles {
   int a_end, b_start, end_b, tiles_a, tiles, p_lo, p_hi;
-  __device__ KeyTiles(int p_lo_, int p_hi_, int window, int keep_first) : p_lo(p_lo_), p_hi(p_hi_) {
-    const int lo = window > 0 ? (p_lo - window + 1 > 0 ? p_lo - window + 1 : 0) : 0;
-    b_start = lo & ~15;
-    a_end = keep_first < b_start ? keep_first : b_start;
+  int full_from;      // keys from here on are within every one of the queries' windows (or chunks)
+  __device__ KeyTiles(int p_lo_, int p_hi_, const Mask& mask) : p_lo(p_lo_), p_hi(p_hi_) {
+    b_start = mask.low(p_lo) & ~15;
+    full_from = mask.low(p_hi);
+    a_end = mask.keep_first < b_start ? mask.keep_first : b_start;
     end_b = p_hi + 1;
     tiles_a = (a_end + 31) >> 5;
     tiles = tiles_a + ((end_b - b_start + 31) >> 5);
@@ -421,11 +609,11 @@ template <int DC, int EB>
 __device__ __forceinline__ void attend_tiles(const KeyTiles& kt, int t_begin, int t_end, const bf16x8 (&qf)[DC], bool seen,
                                              int pos, const int* __restrict__ pages, int page_size, int n_kv, int g,
                                              const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
-                                             int window, int keep_first, float scale, Running<EB>& run,
-                                             int mode, float bias) {
+                                             const Mask& mask, float scale, Running<EB>& run, int mode, float bias) {
   constexpr int E = 16 * EB;
   const int lane = threadIdx.x & 63, c = lane & 15, g4 = lane >> 4;
   if (t_begin >= t_end) return;
+  const int lo = mask.low(pos);
   KeyFrags<DC> cur, nxt;
   load_keys<DC, E>(cur, kt, t_begin, pages, page_size, n_kv, g, k_cache);
   for (int t = t_begin; t < t_end; ++t) {
@@ -452,7 +640,7 @@ __device__ __forceinline__ void attend_tiles(const KeyTiles& kt, int t_begin, in
     // a whole tile that every query of the wave sees (behind the lowest position, inside the
     // window of the highest or the kept prefix) needs no mask key by key: most tiles of a long window
     const bool interior = cur.have[1] && cur.j0 + 31 < cur.end && cur.j0 + 31 <= kt.p_lo &&
-                          (window <= 0 || kt.p_hi - cur.j0 < window || cur.j0 + 31 < keep_first);
+                          (cur.j0 >= kt.full_from || cur.j0 + 31 < mask.keep_first);
     if (interior) {
 #pragma unroll
       for (int u = 0; u < 2; ++u)
@@ -467,7 +655,7 @@ __device__ __forceinline__ void attend_tiles(const KeyTiles& kt, int t_begin, in
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int j = cur.j0 + 16 * u + 4 * g4 + i;
-          const bool ok = cur.have[u] && seen && j < cur.end && sees(pos, j, window, keep_first);
+          const bool ok = cur.have[u] && seen && j < cur.end && sees(pos, j, lo, mask.keep_first);
           s[u][i] = ok ? s[u][i] * scale : NEG_INF;
           tmax = fmaxf(tmax, s[u][i]);
         }
@@ -514,7 +702,7 @@ __device__ __forceinline__ void attend_tiles(const KeyTiles& kt, int t_begin, in
 struct MfmaArgs {
   const bf16_t* q; int n_rows, n_heads, n_kv;
   const bf16_t* k_cache; const bf16_t* v_cache; const int* table; int max_pages, page_size;
-  const int* positions; const int* row_req; int window, keep_first; const float* sink; float scale;
+  const int* positions; const int* row_req; Mask mask; const float* sink; float scale;
   bf16_t* out; const int* q_start; int long_from;
   int splits; float* part_o; float* part_ml;      // (decoding) [rows, heads, splits, E] and [rows, heads, splits, 2]
   int mode;                                       // MODE_SOFTMAX, or MODE_SIGMOID (sink: the bias of the scores)
@@ -560,9 +748,9 @@ __global__ __launch_bounds__(256) void sink_window_attention_mfma_kernel(MfmaArg
       p_hi = max(p_hi, __shfl_xor(p_hi, off, WAVE));
     }
     if (p_hi < 0) continue;
-    const KeyTiles kt(p_lo, p_hi, a.window, a.keep_first);
+    const KeyTiles kt(p_lo, p_hi, a.mask);
     attend_tiles<DC, EB>(kt, 0, kt.tiles, qf, mine, pos, a.table + (size_t)b * a.max_pages, a.page_size, a.n_kv, g,
-                         a.k_cache, a.v_cache, a.window, a.keep_first, a.scale, run, a.mode, bias);
+                         a.k_cache, a.v_cache, a.mask, a.scale, run, a.mode, bias);
   }
   if (!row_ok) return;
   if (a.long_from > 0 && a.q_start[req + 1] - a.q_start[req] < a.long_from) return;
@@ -603,6 +791,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
   const int r = r0 + c;
   const bool row_ok = r < a.n_rows;
   const int pos = row_ok ? a.positions[r] : 0;
+  const int low = a.mask.low(pos);
   const int req = row_ok ? a.row_req[r] : -1;
   bf16x8 zero8;
 #pragma unroll
@@ -630,7 +819,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
       p_hi = max(p_hi, __shfl_xor(p_hi, off, WAVE));
     }
     if (p_hi < 0) continue;
-    const KeyTiles kt(p_lo, p_hi, a.window, a.keep_first);
+    const KeyTiles kt(p_lo, p_hi, a.mask);
     const int* pages = a.table + (size_t)b * a.max_pages;
     // Two sets of staging registers: a tile's pieces are asked for TWO tiles ahead and stored one
     // tile ahead, so that their way from memory lies behind the products of a whole tile and
@@ -705,7 +894,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
       }
       float tmax = NEG_INF;
       const bool interior = have1 && j0 + 31 < end && j0 + 31 <= kt.p_lo &&
-                            (a.window <= 0 || kt.p_hi - j0 < a.window || j0 + 31 < a.keep_first);
+                            (j0 >= kt.full_from || j0 + 31 < a.mask.keep_first);
       if (interior) {
 #pragma unroll
         for (int u = 0; u < 2; ++u)
@@ -720,7 +909,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
             const int j = j0 + 16 * u + 4 * g4 + i;
-            const bool ok = mine && j < end && sees(pos, j, a.window, a.keep_first);
+            const bool ok = mine && j < end && sees(pos, j, low, a.mask.keep_first);
             s[u][i] = ok ? s[u][i] * a.scale : NEG_INF;
             tmax = fmaxf(tmax, s[u][i]);
           }
@@ -834,11 +1023,11 @@ __global__ __launch_bounds__(64) void sink_window_attention_grouped_kernel(MfmaA
   run.l = sig ? (z == 0 ? 1.f : 0.f) : ((a.sink && head_ok && z == 0) ? 1.f : 0.f);
 #pragma unroll
   for (int eb = 0; eb < EB; ++eb) run.o[eb] = floatx4{0.f, 0.f, 0.f, 0.f};
-  const KeyTiles kt(pos, pos, a.window, a.keep_first);
+  const KeyTiles kt(pos, pos, a.mask);
   const int per = (kt.tiles + a.splits - 1) / a.splits;
   const int t_begin = z * per, t_end = (z + 1) * per < kt.tiles ? (z + 1) * per : kt.tiles;
   attend_tiles<DC, EB>(kt, t_begin, t_end, qf, head_ok, pos, a.table + (size_t)b * a.max_pages, a.page_size, a.n_kv, g,
-                       a.k_cache, a.v_cache, a.window, a.keep_first, a.scale, run, a.mode, bias);
+                       a.k_cache, a.v_cache, a.mask, a.scale, run, a.mode, bias);
   if (!head_ok) return;
   if (a.splits == 1) {
     const float inv = 1.0f / run.l;
@@ -968,7 +1157,7 @@ static void launch_mfma_any(int D, int E, int which, dim3 grid, dim3 block, hipS
 extern "C" int llmlab_sink_window_attention(const void* q, int dtype, int rows, int n_heads, int n_kv, int D, int E,
                                             const void* k_cache, const void* v_cache, const int* table, int max_pages,
                                             int page_size, const int* positions, const int* row_req, int window,
-                                            int keep_first, const float* sink, float scale, void* out,
+                                            int keep_first, int chunk, const float* sink, float scale, void* out,
                                             const int* q_start, int long_from, int launches, int max_keys,
                                             float* workspace, size_t workspace_floats, int num_cus, int mode,
                                             hipStream_t stream) {
@@ -977,6 +1166,8 @@ extern "C" int llmlab_sink_window_attention(const void* q, int dtype, int rows, 
                  "sink_window_attention: bad sizes rows=%d heads=%d kv=%d D=%d E=%d", rows, n_heads, n_kv, D, E);
   LLMLAB_REQUIRE(E <= 64 * MAX_E_PER_LANE, "sink_window_attention: values up to %d wide, got %d", 64 * MAX_E_PER_LANE, E);
   LLMLAB_REQUIRE(D <= 4096 && n_heads <= 65535, "sink_window_attention: keys up to 4096 wide and 65535 heads");
+  LLMLAB_REQUIRE(chunk >= 0 && (chunk == 0 || window <= 0), "sink_window_attention: a window or chunks, not both");
+  const Mask mask{window, keep_first, chunk};
   LLMLAB_REQUIRE(keep_first >= 0 && page_size > 0 && page_size % 4 == 0 && max_pages > 0,
                  "sink_window_attention: bad window or page arguments");
   if (rows == 0) return 0;
@@ -987,7 +1178,7 @@ extern "C" int llmlab_sink_window_attention(const void* q, int dtype, int rows, 
   }
   if (long_from > 0) {
     MfmaArgs a{(const bf16_t*)q, rows, n_heads, n_kv, (const bf16_t*)k_cache, (const bf16_t*)v_cache, table, max_pages,
-               page_size, positions, row_req, window, keep_first, sink, scale, (bf16_t*)out, q_start, long_from, 1,
+               page_size, positions, row_req, mask, sink, scale, (bf16_t*)out, q_start, long_from, 1,
                nullptr, nullptr, mode};
     if (launches & 2) {
       // heads that read the same keys and values share the tiles a block stages in LDS
@@ -1029,11 +1220,11 @@ extern "C" int llmlab_sink_window_attention(const void* q, int dtype, int rows, 
   if (dtype == DT_BF16)
     hipLaunchKernelGGL(sink_window_attention_kernel<bf16_t>, grid, block, lds, stream, (const bf16_t*)q, n_heads, n_kv, D,
                        E, (const bf16_t*)k_cache, (const bf16_t*)v_cache, table, max_pages, page_size, positions,
-                       row_req, window, keep_first, sink, scale, (bf16_t*)out, q_start, long_from, mode);
+                       row_req, mask, sink, scale, (bf16_t*)out, q_start, long_from, mode);
   else
     hipLaunchKernelGGL(sink_window_attention_kernel<float>, grid, block, lds, stream, (const float*)q, n_heads, n_kv, D,
                        E, (const float*)k_cache, (const float*)v_cache, table, max_pages, page_size, positions,
-                       row_req, window, keep_first, sink, scale, (float*)out, q_start, long_from, mode);
+                       row_req, mask, sink, scale, (float*)out, q_start, long_from, mode);
   LLMLAB_LAUNCH_CHECK("sink_window_attention");
   return 0;
 }

@@ -351,12 +351,12 @@ class StepFunction:
         seen_all = sum(ctx.host_start_pos[:ctx.n_reqs]) + ctx.n_rows      # (without a window: one sum for all requests)
         for g in self.cache.groups:
             per_token = len(g.entries) * g.spec.bytes_per_token(self.cache.dtype)
-            if not g.window:
+            if not g.spec.bounded:
                 total += per_token * seen_all
                 continue
             for b in range(ctx.n_reqs):
                 seen = ctx.host_start_pos[b] + ctx.host_q_start[b + 1] - ctx.host_q_start[b]
-                total += per_token * min(seen, g.window + g.spec.keep_first)
+                total += per_token * min(seen, seen - g.spec.lowest_read(seen - 1) + g.spec.keep_first)
         return total
 
     def _decode_auto(self) -> torch.Tensor:

@@ -531,8 +531,8 @@ class HipOps:
         """``resid += x w^T (+ bias)``, and the pending pieces of ``resid`` with it."""
         self._linear(x, w, resid, bias, EPI_RESID, w.shape[0], pending)
 
-    def linear_logits(self, x, w, out) -> None:
-        self._linear(x, w, out, None, EPI_F32, w.shape[0])
+    def linear_logits(self, x, w, out, bias=None) -> None:
+        self._linear(x, w, out, bias, EPI_F32, w.shape[0])
 
     def linear_swiglu(self, x, w_gate_up, out, activation: str = "silu") -> None:
         """``out = act(x Wg^T) * (x Wu^T)`` with the rows of gate and up interleaved in runs of 16;
@@ -1061,9 +1061,16 @@ class HipOps:
                 lib.llmlab_project_norm_write.restype = _c_int
                 lib.llmlab_sink_window_attention.argtypes = [
                     _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
-                    _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr,
-                    _c_size, _c_int, _c_int, _c_ptr]
+                    _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_int, _c_int, _c_int,
+                    _c_ptr, _c_size, _c_int, _c_int, _c_ptr]
                 lib.llmlab_sink_window_attention.restype = _c_int
+                lib.llmlab_project_conv_write.argtypes = [
+                    _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr,
+                    _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
+                    _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr]
+                lib.llmlab_project_conv_write.restype = _c_int
+                lib.llmlab_gate_channels.argtypes = [_c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr]
+                lib.llmlab_gate_channels.restype = _c_int
                 lib.llmlab_project_rotate_write.argtypes = [
                     _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_float, _c_int,
                     _c_float, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
@@ -1103,18 +1110,31 @@ class HipOps:
                 lib.llmlab_rmsnorm_add.restype = _c_int
                 lib.llmlab_scaled_sum.argtypes = [_c_ptr, _c_ptr, _c_float, _c_ptr, _c_float, _c_size, _c_ptr]
                 lib.llmlab_scaled_sum.restype = _c_int
+                lib.llmlab_normed_sum.argtypes = [_c_ptr, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_float,
+                                                  _c_int, _c_int, _c_ptr]
+                lib.llmlab_normed_sum.restype = _c_int
+                lib.llmlab_shift_mix.argtypes = [_c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
+                                                 _c_int, _c_int, _c_int, _c_ptr]
+                lib.llmlab_shift_mix.restype = _c_int
+                lib.llmlab_poly_norm.argtypes = [_c_ptr, _c_ptr, _c_float, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_ptr]
+                lib.llmlab_poly_norm.restype = _c_int
             elif kind == "linear_attention":
-                lib.llmlab_gla_decay.argtypes = [_c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_float, _c_ptr,
+                lib.llmlab_gla_decay.argtypes = [_c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_float, _c_ptr,
                                                  _c_int, _c_ptr]
+                lib.llmlab_memory_gates.argtypes = [_c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_float, _c_int,
+                                                    _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr]
+                lib.llmlab_memory_gates.restype = _c_int
                 lib.llmlab_gla_decay.restype = _c_int
                 lib.llmlab_gla_slices.argtypes = [_c_int]
                 lib.llmlab_gla_slices.restype = _c_int
                 lib.llmlab_gla_scan.argtypes = [_c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_float, _c_int, _c_int,
                                                 _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr,
-                                                _c_ptr, _c_int, _c_ptr]
+                                                _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
+                                                _c_ptr]
                 lib.llmlab_gla_scan.restype = _c_int
                 lib.llmlab_gla_output.argtypes = [_c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_float, _c_ptr,
-                                                  _c_int, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr]
+                                                  _c_int, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int,
+                                                  _c_ptr, _c_ptr, _c_ptr]
                 lib.llmlab_gla_output.restype = _c_int
                 lib.llmlab_delta_gates.argtypes = [_c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr,
                                                    _c_ptr, _c_float, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
@@ -1402,12 +1422,15 @@ class HipOps:
 
     def sink_window_attention(self, q, num_heads, num_kv_heads, key_dim, value_dim, k_cache, v_cache, block_table,
                               page_size, positions, row_req, window, keep_first, sink, scale, out,
-                              q_start=None, long_from=0, launches=3, max_keys=0, weights: str = "softmax") -> None:
+                              q_start=None, long_from=0, launches=3, max_keys=0, weights: str = "softmax",
+                              chunk=None) -> None:
         """The query of row ``r`` at position ``i = positions[r]`` of request ``row_req[r]`` attends
         to the cached keys ``j <= i`` with ``i - j < window`` or ``j < keep_first`` (``window`` None:
         all); ``sink`` (float32 per head, or None) adds ``exp(sink)`` to the softmax's denominator.
         ``weights="sigmoid"``: no softmax; a visible key weighs ``sigmoid(score + sink[h])``
         (``sink``: then a bias per head on every score, None for none), not normalised over the keys.
+        ``chunk`` (with ``window`` None): the keys of the query's own chunk of so many positions, ``j <=
+        i`` with ``j // chunk == i // chunk`` (or ``j < keep_first``).
         ``long_from > 0`` (``windowed_attention_long_rows``: sizes that the matrix cores take):
         requests that bring at least so many rows (by ``q_start``) are served in tiles of 16 rows
         of a head, the others a row and a group of heads at a time with the row's keys cut into
@@ -1441,7 +1464,7 @@ class HipOps:
         self._call(lib.llmlab_sink_window_attention, self._ptr(q), _dt(q), rows, num_heads, num_kv_heads, key_dim,
                    value_dim, self._ptr(k_cache), self._ptr(v_cache), self._ptr(block_table), block_table.stride(0),
                    page_size, self._ptr(positions), self._ptr(row_req), int(window) if window else 0,
-                   int(keep_first or 0), self._ptr(sink), float(scale), self._ptr(out),
+                   int(keep_first or 0), int(chunk or 0), self._ptr(sink), float(scale), self._ptr(out),
                    self._ptr(q_start) if long_from else None, int(long_from), int(launches), int(max_keys),
                    self._ptr(self.workspace), self.workspace.numel(), self.num_cus, self.ATTENTION_WEIGHTS[weights],
                    self._stream(), lib=lib)
@@ -1499,12 +1522,86 @@ class HipOps:
                    self._ptr(positions), self._ptr(row_req), self._ptr(block_table), block_table.stride(0),
                    self._stream(), lib=lib)
 
+    def project_conv_write(self, proj, num_heads, num_kv_heads, key_dim, value_dim, bias, conv, state, q_start, req_rows,
+                           freq, rot_dims, pairing: str, unit_eps, q_out, k_cache, v_cache, page_size, positions, row_req,
+                           block_table, one_row_each: bool) -> None:
+        """From the float32 projections ``proj [rows, q | k | v (| ...)]`` (heads of ``key_dim``, ``key_dim``
+        and ``value_dim`` channels): ``bias`` (float32, the same order, or None) is added; ``conv [q + k +
+        v, taps]`` float32 (or None): a causal convolution channel by channel over the positions of each
+        request, ``y_t = sum_j conv[:, j] u_(t - taps + 1 + j)`` of the biased projections ``u``, whose last
+        ``taps - 1`` rows live in ``state [slots, taps - 1, q + k + v]`` float32; the first ``rot_dims``
+        channels of every query and key head turn by ``positions[r] * freq[i]``, channel ``i`` with ``i +
+        rot_dims / 2`` (``pairing="halves"``) or ``2i`` with ``2i + 1`` (``"neighbours"``); ``unit_eps`` (None:
+        no norm): every query and key head is divided by its root mean square.  Queries go to ``q_out
+        [rows, heads * DK]``, keys and values to the rows' places in the pages; ``DK >= key_dim`` is the
+        pages' key width, zeros behind a head's channels.  ``one_row_each``: every request of the step
+        brings exactly one row."""
+        lib = self._mixer_lib("windowed_attention")
+        self._need(proj, "projections", torch.float32)
+        self._need(q_out, "queries")
+        rows, laid = q_out.shape[0], k_cache.shape[-1]
+        sizes = (num_heads + num_kv_heads) * key_dim + num_kv_heads * value_dim
+        if (proj.shape[0] != rows or proj.shape[1] < sizes or tuple(q_out.shape) != (rows, num_heads * laid)
+                or laid < key_dim):
+            raise ValueError(f"project_conv_write: projections {tuple(proj.shape)}, queries {tuple(q_out.shape)} do not "
+                             f"fit {sizes} numbers a row and key heads of {key_dim} laid out in {laid}")
+        self._paged(k_cache, v_cache, num_kv_heads, page_size, laid, value_dim, q_out.dtype)
+        if bias is not None:
+            self._need(bias, "projection bias", torch.float32)
+            if bias.numel() < sizes:
+                raise ValueError(f"project_conv_write: a bias of {bias.numel()} numbers for {sizes} projections")
+        taps = 0
+        if conv is not None:
+            self._need(conv, "convolution taps", torch.float32)
+            taps = conv.shape[1]
+            if conv.shape[0] != sizes:
+                raise ValueError(f"project_conv_write: taps {tuple(conv.shape)} for {sizes} channels")
+        if taps > 1:
+            self._need(state, "convolution state", torch.float32)
+            if tuple(state.shape[1:]) != (taps - 1, sizes):
+                raise ValueError(f"project_conv_write: state {tuple(state.shape)} does not hold {taps - 1} rows of {sizes}")
+        rot_dims = int(rot_dims or 0)
+        if rot_dims:
+            self._need(freq, "rotation frequencies", torch.float32)
+            if rot_dims % 2 or rot_dims > key_dim or freq.numel() != rot_dims // 2:
+                raise ValueError(f"project_conv_write: {rot_dims} of {key_dim} channels with {freq.numel()} frequencies")
+        for t, name, least in ((positions, "positions", rows), (row_req, "row -> request map", rows),
+                               (q_start, "request row starts", 2), (req_rows, "request slots", 1)):
+            self._need(t, name, torch.int32)
+            if t.numel() < least:
+                raise ValueError(f"project_conv_write: {name} is too short")
+        self._need(block_table, "block table", torch.int32, contiguous=False)
+        if block_table.stride(1) != 1:
+            raise ValueError("project_conv_write: block table rows are contiguous")
+        self._call(lib.llmlab_project_conv_write, self._ptr(proj), proj.stride(0), rows, num_heads, num_kv_heads, key_dim,
+                   laid, value_dim, self._ptr(bias), self._ptr(conv), taps, self._ptr(state) if taps > 1 else None,
+                   self._ptr(q_start), self._ptr(req_rows), self._ptr(freq) if rot_dims else None, rot_dims,
+                   {"halves": 0, "neighbours": 1}[pairing], 0 if unit_eps is None else 1, float(unit_eps or 0.0),
+                   self._ptr(q_out), self._ptr(k_cache), self._ptr(v_cache), _dt(q_out), page_size,
+                   self._ptr(positions), self._ptr(row_req), self._ptr(block_table), block_table.stride(0),
+                   1 if one_row_each else 0, self._stream(), lib=lib)
+
+    def gate_channels(self, out, proj, off_gate: int) -> None:
+        """``out[r, c] *= sigmoid(proj[r, off_gate + c])`` with the product in float32 (``out`` in a kernel
+        dtype, ``proj`` float32)."""
+        lib = self._mixer_lib("windowed_attention")
+        self._need(out, "heads' outputs")
+        self._need(proj, "projections", torch.float32)
+        rows, width = out.shape
+        if proj.shape[0] != rows or off_gate < 0 or off_gate + width > proj.shape[1]:
+            raise ValueError(f"gate_channels: gates at {off_gate} of {tuple(proj.shape)} for outputs {tuple(out.shape)}")
+        self._call(lib.llmlab_gate_channels, self._ptr(out), proj.data_ptr() + 4 * int(off_gate), proj.stride(0), rows, width,
+                   _dt(out), self._stream(), lib=lib)
+
     def gla_slices(self, key_dim: int) -> int:
         """Into how many pieces the scan leaves each output (one per slice of key channels)."""
         return int(self._mixer_lib("linear_attention").llmlab_gla_slices(int(key_dim)))
 
-    def gla_decay(self, low, rank, w2, bias, tau, decay) -> None:
-        """``decay[r, c] = sigmoid(bias[c] + w2[c] . low[r, :rank]) ** (1 / tau)``, all float32."""
+    DECAY_KINDS = {"sigmoid": 0, "double_exp": 1}
+
+    def gla_decay(self, low, rank, w2, bias, tau, decay, kind: str = "sigmoid") -> None:
+        """``decay[r, c] = sigmoid(bias[c] + w2[c] . low[r, :rank]) ** (1 / tau)``, all float32;
+        ``kind="double_exp"``: ``exp(-exp(bias[c] + w2[c] . tanh(low[r, :rank])))`` (no ``tau``)."""
         lib = self._mixer_lib("linear_attention")
         for t, name in ((low, "low-rank projection"), (w2, "decay weight"), (decay, "decays")):
             self._need(t, name, torch.float32, contiguous=name != "low-rank projection")
@@ -1517,7 +1614,37 @@ class HipOps:
             if bias.numel() != channels:
                 raise ValueError("gla_decay: one bias per channel")
         self._call(lib.llmlab_gla_decay, self._ptr(low), low.stride(0), rows, int(rank), self._ptr(w2),
-                   self._ptr(bias), float(tau), self._ptr(decay), channels, self._stream(), lib=lib)
+                   self._ptr(bias), self.DECAY_KINDS[kind], float(tau), self._ptr(decay), channels, self._stream(),
+                   lib=lib)
+
+    def memory_gates(self, proj, off_i, off_f, bias_i, bias_f, cap: float, num_heads: int, max_state, q_start, req_rows,
+                     n_reqs, keep, take, maxima) -> None:
+        """The gates of a matrix memory for the rows of every request: log gates ``i = cap * tanh((proj[:,
+        off_i + h] + bias_i) / cap)`` and ``f = logsigmoid(cap * tanh((proj[:, off_f + h] + bias_f) / cap))``,
+        the running maximum ``m_t = max(f_t + m_(t-1), i_t)`` from ``max_state [slots, heads]`` (left at the
+        last row's), ``keep = exp(f_t + m_(t-1) - m_t)``, ``take = exp(i_t - m_t)`` and ``maxima = m_t``, each
+        ``[rows, heads]``; all float32."""
+        lib = self._mixer_lib("linear_attention")
+        for t, name in ((proj, "projections"), (max_state, "maxima of the slots"), (keep, "keep"), (take, "take"),
+                        (maxima, "maxima")):
+            self._need(t, name, torch.float32)
+        rows = proj.shape[0]
+        for t in (keep, take, maxima):
+            if tuple(t.shape) != (rows, num_heads):
+                raise ValueError("memory_gates: one number per row and head")
+        for t in (bias_i, bias_f):
+            if t is not None:
+                self._need(t, "gate bias", torch.float32)
+                if t.numel() != num_heads:
+                    raise ValueError("memory_gates: one bias per head")
+        self._need(q_start, "request row starts", torch.int32)
+        self._need(req_rows, "state slots", torch.int32)
+        if (tuple(max_state.shape[1:]) != (num_heads,) or min(off_i, off_f) < 0
+                or max(off_i, off_f) + num_heads > proj.shape[1] or q_start.numel() < n_reqs + 1 or req_rows.numel() < n_reqs):
+            raise ValueError("memory_gates: the operands do not fit each other")
+        self._call(lib.llmlab_memory_gates, self._ptr(proj), proj.stride(0), int(off_i), int(off_f), self._ptr(bias_i),
+                   self._ptr(bias_f), float(cap), num_heads, self._ptr(max_state), self._ptr(q_start), self._ptr(req_rows),
+                   int(n_reqs), self._ptr(keep), self._ptr(take), self._ptr(maxima), self._stream(), lib=lib)
 
     def gla_scan_chunk(self, rows: int, longest: int, num_heads: int, value_dim: int) -> int:
         """Into chunks of how many rows the scan cuts a step whose longest request brings
@@ -1533,7 +1660,7 @@ class HipOps:
         return chunk
 
     def gla_scan(self, proj, off_q, off_k, off_v, decay, q_scale, num_heads, key_dim, value_dim, state, q_start,
-                 req_rows, n_reqs, parts, chunk=0, chunk_state=None, chunk_decay=None) -> None:
+                 req_rows, n_reqs, parts, chunk=0, chunk_state=None, chunk_decay=None, bonus=None, memory=None) -> None:
         """The recurrence ``S = decay_t * S + k_t v_t^T; o_t = S^T (q_scale q_t)`` over the rows
         ``q_start[b] .. q_start[b + 1]`` of each of the step's ``n_reqs`` requests, on the float32
         state ``state[req_rows[b]]`` ``[heads, key_dim, value_dim]``, which is left updated;
@@ -1541,16 +1668,41 @@ class HipOps:
         ``chunk > 0``: every request's rows in chunks of so many that run side by side, their
         states joined afterwards (``chunk_state [chunks, heads, key_dim, value_dim]`` and
         ``chunk_decay [chunks, heads, key_dim]`` float32 scratch, ``chunks >= rows // chunk +
-        n_reqs``)."""
+        n_reqs``).
+
+        ``bonus [heads * key_dim]`` float32: the outputs are ``o_t = (S_(t-1) + diag(bonus) k_t v_t^T)^T
+        (q_scale q_t)`` instead.  ``memory = (keep, take, norm_state, norm_parts, chunk_norm)`` (``decay`` is
+        then None): ``S = keep_t S + take_t k_t v_t^T`` with ``keep``, ``take [rows, heads]``, and beside it the
+        normaliser ``n = keep_t n + take_t k_t`` on ``norm_state [slots, heads, key_dim]``, whose products ``n .
+        (q_scale q_t)`` go to ``norm_parts [rows, heads, slices]`` in pieces (``chunk_norm [chunks, heads,
+        key_dim]``: scratch of the chunks, else None)."""
         lib = self._mixer_lib("linear_attention")
-        for t, name in ((proj, "projections"), (decay, "decays"), (state, "recurrent state"), (parts, "output pieces")):
+        for t, name in ((proj, "projections"), (state, "recurrent state"), (parts, "output pieces")):
             self._need(t, name, torch.float32)
         self._need(q_start, "request row starts", torch.int32)
         self._need(req_rows, "state slots", torch.int32)
         rows = proj.shape[0]
         slices = self.gla_slices(key_dim)
-        if (tuple(decay.shape) != (rows, num_heads * key_dim)
-                or tuple(parts.shape) != (rows, num_heads, slices, value_dim)
+        kind, keep, take, norm_state, norm_parts, chunk_norm = 0, None, None, None, None, None
+        if memory is not None:
+            kind = 2
+            keep, take, norm_state, norm_parts, chunk_norm = memory
+            for t, name in ((keep, "keep"), (take, "take"), (norm_state, "normaliser"), (norm_parts, "normaliser's pieces")):
+                self._need(t, name, torch.float32)
+            if (bonus is not None or tuple(keep.shape) != (rows, num_heads) or tuple(take.shape) != (rows, num_heads)
+                    or tuple(norm_state.shape) != (state.shape[0], num_heads, key_dim)
+                    or tuple(norm_parts.shape) != (rows, num_heads, slices)):
+                raise ValueError("gla_scan: the memory's operands do not fit each other")
+        else:
+            self._need(decay, "decays", torch.float32)
+            if tuple(decay.shape) != (rows, num_heads * key_dim):
+                raise ValueError("gla_scan: one decay per row, head and key channel")
+            if bonus is not None:
+                kind = 1
+                self._need(bonus, "bonus", torch.float32)
+                if bonus.numel() != num_heads * key_dim:
+                    raise ValueError("gla_scan: one bonus per head and key channel")
+        if (tuple(parts.shape) != (rows, num_heads, slices, value_dim)
                 or tuple(state.shape[1:]) != (num_heads, key_dim, value_dim)
                 or q_start.numel() < n_reqs + 1 or req_rows.numel() < n_reqs
                 or min(off_q, off_k, off_v) < 0
@@ -1566,22 +1718,34 @@ class HipOps:
                     or max_chunks < rows // chunk + n_reqs):
                 raise ValueError(f"gla_scan: the scratch of the chunks does not fit {rows} rows of {n_reqs} requests "
                                  f"in chunks of {chunk}")
+            if kind == 2:
+                self._need(chunk_norm, "chunk normalisers", torch.float32)
+                if tuple(chunk_norm.shape) != (max_chunks, num_heads, key_dim):
+                    raise ValueError("gla_scan: the normalisers' scratch does not fit the chunks")
         self._call(lib.llmlab_gla_scan, self._ptr(proj), proj.stride(0), int(off_q), int(off_k), int(off_v),
                    self._ptr(decay), float(q_scale), num_heads, key_dim, value_dim, self._ptr(state),
                    self._ptr(q_start), self._ptr(req_rows), int(n_reqs), self._ptr(parts), rows, int(chunk),
                    self._ptr(chunk_state) if chunk else None, self._ptr(chunk_decay) if chunk else None, max_chunks,
-                   self._stream(), lib=lib)
+                   kind, self._ptr(bonus), self._ptr(keep), self._ptr(take), self._ptr(norm_state), self._ptr(norm_parts),
+                   self._ptr(chunk_norm) if chunk else None, self._stream(), lib=lib)
 
     OUTPUT_GATES = {"silu": 0, "sigmoid": 1}
 
     def gla_output(self, parts, num_heads, key_dim, value_dim, weight, eps, proj, off_gate, out, gate: str = "silu",
-                   norm_count: int = 0) -> None:
+                   norm_count: int = 0, norm_parts=None, maxima=None) -> None:
         """``out[r, h] = rmsnorm(sum of parts[r, h]) * weight * silu(gate[r, h])`` with the gate at
         column ``off_gate`` of the float32 ``proj``; ``out`` in the compute dtype.  ``parts [rows, heads,
         pieces, value_dim]`` with any number of pieces; ``weight`` of ``value_dim`` numbers (the same for
         every head) or of ``heads * value_dim``; ``gate="sigmoid"``: ``... * sigmoid(gate[r, h])``; ``norm_count``:
-        the mean of the squares is taken over so many channels of a head (the ones behind them are zeros)."""
+        the mean of the squares is taken over so many channels of a head (the ones behind them are zeros).
+        ``norm_parts [rows, heads, pieces]`` with ``maxima [rows, heads]`` (a matrix memory): a head's sum is
+        first divided by ``max(|sum of norm_parts|, exp(-maxima)) + 1e-6``."""
         lib = self._mixer_lib("linear_attention")
+        if norm_parts is not None:
+            self._need(norm_parts, "normaliser's pieces", torch.float32)
+            self._need(maxima, "maxima", torch.float32)
+            if tuple(norm_parts.shape) != tuple(parts.shape[:3]) or tuple(maxima.shape) != tuple(parts.shape[:2]):
+                raise ValueError("gla_output: the normaliser's pieces do not fit the outputs'")
         self._need(parts, "output pieces", torch.float32)
         self._need(proj, "projections", torch.float32)
         self._need(weight, "output norm weight", torch.float32)
@@ -1595,7 +1759,8 @@ class HipOps:
         per_head = 1 if weight.numel() == num_heads * value_dim and num_heads > 1 else 0
         self._call(lib.llmlab_gla_output, self._ptr(parts), rows, num_heads, key_dim, value_dim, self._ptr(weight),
                    float(eps), self._ptr(proj), proj.stride(0), int(off_gate), self._ptr(out), _dt(out),
-                   int(parts.shape[2]), per_head, self.OUTPUT_GATES[gate], int(norm_count or 0), self._stream(), lib=lib)
+                   int(parts.shape[2]), per_head, self.OUTPUT_GATES[gate], int(norm_count or 0), self._ptr(norm_parts),
+                   self._ptr(maxima), self._stream(), lib=lib)
 
     def delta_gates(self, proj, off_low, rank, off_rate, off_k, w2, w0, rate_bias, decay_scale, key_eps, num_heads,
                     key_dim, decay, unit, removal) -> None:
@@ -1812,12 +1977,13 @@ class HipOps:
         self._call(lib.llmlab_gated_add, self._ptr(x), self._ptr(y), pieces, piece_stride, self._ptr(gate), cols,
                    self._ptr(bias), rows, width, self._stream(), lib=lib)
 
-    def rmsnorm_add(self, y, weight, eps: float, x, next_norm=None) -> None:
+    def rmsnorm_add(self, y, weight, eps: float, x, next_norm=None, copy=None) -> None:
         """``x += y / sqrt(mean(y^2) + eps) * weight`` row by row, all float32: the norm of a sublayer's
         result on its way into the stream.  ``y [rows, width]``, or a product left in pieces
         (``PendingSums``), which are summed on the way.  ``next_norm = (weight, eps, out)``: the RMS norm
         that reads the stream next, in the same launch: ``out = norm(x)`` of the new rows (float32
-        weight, ``out`` in a kernel dtype)."""
+        weight, ``out`` in a kernel dtype).  ``copy``: a tensor of a kernel dtype that receives the new rows
+        rounded (instead of a next norm)."""
         lib = self._mixer_lib("stream_ops")
         self._need(x, "stream", torch.float32)
         self._need(weight, "norm weight", torch.float32)
@@ -1837,6 +2003,11 @@ class HipOps:
             raise ValueError("rmsnorm_add: one weight per column")
         next_w = next_out = None
         next_eps = 0.0
+        if copy is not None:
+            self._need(copy, "stream copy")
+            if next_norm is not None or tuple(copy.shape) != (rows, width):
+                raise ValueError("rmsnorm_add: a next norm or a copy of the stream's shape, not both")
+            next_out = copy
         if next_norm is not None:
             next_w, next_eps, next_out = next_norm
             self._need(next_w, "next norm's weight", torch.float32)
@@ -1856,6 +2027,62 @@ class HipOps:
             raise ValueError("scaled_sum: three tensors of one shape")
         self._call(lib.llmlab_scaled_sum, self._ptr(out), self._ptr(y1), float(a), self._ptr(y2), float(b), out.numel(),
                    self._stream(), lib=lib)
+
+    def normed_sum(self, out, y1, w1, a: float, y2, w2, b: float, eps: float) -> None:
+        """``out = a * rms(y1) * w1 + b * rms(y2) * w2`` row by row, ``rms(v) = v / sqrt(mean(v^2) + eps)``;
+        all float32."""
+        lib = self._mixer_lib("stream_ops")
+        for t, name in ((out, "sum"), (y1, "first term"), (y2, "second term"), (w1, "first weight"), (w2, "second weight")):
+            self._need(t, name, torch.float32)
+        rows, width = out.shape
+        if tuple(out.shape) != tuple(y1.shape) or tuple(out.shape) != tuple(y2.shape):
+            raise ValueError("normed_sum: three tensors of one shape")
+        if w1.numel() != width or w2.numel() != width:
+            raise ValueError("normed_sum: weights of the rows' width")
+        self._call(lib.llmlab_normed_sum, self._ptr(out), self._ptr(y1), self._ptr(w1), float(a),
+                   self._ptr(y2), self._ptr(w2), float(b), float(eps), rows, width, self._stream(), lib=lib)
+
+    def shift_mix(self, h, mix, state, row_req, q_start, req_rows, out) -> None:
+        """``out[m] = h + (p - h) * mix[m]`` for every row of ``mix [mixes, width]`` float32, ``p`` the row
+        before in the same request: the step's, or, for a request's first row, ``state [slots, width]``
+        (zeros before a sequence's start), which then takes the request's last row.  ``h [rows, width]``
+        and ``state`` share a dtype; ``out [mixes, rows, width]``: float32 or bfloat16 from float32 rows,
+        bfloat16 from bfloat16 rows."""
+        lib = self._mixer_lib("stream_ops")
+        self._need(h, "rows")
+        self._need(state, "rows before", h.dtype)
+        self._need(mix, "mixes", torch.float32)
+        self._need(out, "mixed rows")
+        rows, width = h.shape
+        n_mix = mix.shape[0]
+        if (mix.dim() != 2 or mix.shape[1] != width or tuple(out.shape) != (n_mix, rows, width)
+                or tuple(state.shape[1:]) != (width,)):
+            raise ValueError(f"shift_mix: rows {tuple(h.shape)}, mixes {tuple(mix.shape)}, state {tuple(state.shape)}, output "
+                             f"{tuple(out.shape)} do not fit each other")
+        for t, name, least in ((row_req, "row -> request map", rows), (q_start, "request row starts", 2),
+                               (req_rows, "request slots", 1)):
+            self._need(t, name, torch.int32)
+            if t.numel() < least:
+                raise ValueError(f"shift_mix: {name} is too short")
+        self._call(lib.llmlab_shift_mix, self._ptr(h), _dt(h), self._ptr(mix), n_mix, self._ptr(state), self._ptr(row_req),
+                   self._ptr(q_start), self._ptr(req_rows), self._ptr(out), _dt(out), rows, width, self._stream(), lib=lib)
+
+    def poly_norm(self, z, coef, eps: float, count: int, out) -> None:
+        """``out = a N(z) + b N(z^2) + c N(z^3) + e`` with ``(a, b, c, e) = coef`` (float32 on the GPU), powers
+        element by element and ``N`` the division of a row by the root mean square of its first ``count``
+        numbers (``eps`` inside the root; the numbers behind are padding and zero in ``z``).  ``z`` float32,
+        ``out`` in a kernel dtype."""
+        lib = self._mixer_lib("stream_ops")
+        self._need(z, "sums", torch.float32)
+        self._need(coef, "coefficients", torch.float32)
+        self._need(out, "activations")
+        rows, columns = z.shape
+        if coef.numel() != 4 or tuple(out.shape) != (rows, columns) or not 0 < count <= columns:
+            raise ValueError(f"poly_norm: sums {tuple(z.shape)}, {coef.numel()} coefficients, output {tuple(out.shape)}")
+        if columns % 4:
+            raise UnsupportedSizeError(f"poly_norm takes rows of a multiple of 4 numbers, got {columns}")
+        self._call(lib.llmlab_poly_norm, self._ptr(z), self._ptr(coef), float(eps), rows, int(count), columns, self._ptr(out),
+                   _dt(out), self._stream(), lib=lib)
 
     def softcap(self, x, cap: float) -> None:
         """``x = cap * tanh(x / cap)`` in place, float32."""

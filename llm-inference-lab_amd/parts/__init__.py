@@ -4,7 +4,7 @@ from .base import (Part, Norm, NormedInput, PendingSums, PositionEncoding, Mixer
 from .norms import RMSNorm, LayerNorm
 from .positions import RotaryEmbedding, PairRotary, NoPosition
 from .attention import GQAAttention, WindowedSinkAttention
-from .linear_attention import GatedLinearAttention, DeltaRuleAttention
+from .linear_attention import GatedLinearAttention, DeltaRuleAttention, TimeMixAttention, MatrixMemoryAttention
 from .parallel import ParallelMixers
 from .latent_attention import LatentAttention
 from .feed_forward import SwiGLU, DenseFeedForward, interleave_gate_up

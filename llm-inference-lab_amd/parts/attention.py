@@ -321,6 +321,20 @@ class WindowedSinkAttention(Mixer):
     ``(1 - lambda) v + lambda v_first`` with ``v_first`` what the ``"first"`` layer left for the same
     token and ``lambda`` one learned number (role ``value_mix``); the mixed values are what is cached.
 
+    ``chunk`` (in place of a window): the query at position i attends to the keys ``j <= i`` of its own
+    chunk of positions, ``j // chunk == i // chunk``, counted from the sequence's start.
+    ``conv_taps``: every channel of the (biased) projections q, k and v passes a causal convolution over
+    the positions, ``y_t = sum_j w[:, j] u_(t - taps + 1 + j)``, nothing before the sequence's start (roles
+    ``q_conv``, ``k_conv``, ``v_conv``, ``[channels, taps]``); the last ``taps - 1`` projected rows are
+    per-request state in float32.  A position encoding with a ``half_table()`` (``rope``) turns channel
+    ``i`` with ``i + dims / 2``.  ``qk_norm="head"``: after the convolution and the rotation every query and
+    key head is divided by its root mean square over ``key_dim`` (``norm_eps`` inside the root, no weight).
+    ``output_gate="channels"``: a gate per channel of the heads' outputs (``gate_weight [heads * value_dim,
+    hidden]``), through a sigmoid.  ``out_bias``: the output projection has a bias (role ``o_bias``).  Such
+    layers go through one kernel between the projections and the pages, float32 throughout; their key
+    heads are laid out in multiples of 32 channels and their value heads of 16 (zeros behind), the
+    sizes of the matrix cores.
+
     Pages: keys ``[kv_heads, P, key_dim]``, values ``[kv_heads, P, value_dim]``.  The products'
     inner sizes are multiples of 8: a value head of another width is laid out with zeros behind
     its channels (zero rows of the value projection, zero columns of the output projection), which
@@ -330,32 +344,44 @@ class WindowedSinkAttention(Mixer):
     takes_normed_input = True      # (few rows: the norm in front of the mixer runs inside its first product)
     WEIGHTS = ("softmax", "sigmoid")
     VALUE_MIX = (None, "first", "mix")
+    OUTPUT_GATES = (None, "sigmoid", "channels")
 
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, key_dim: int, value_dim: int,
                  scale: float, tensors: Dict[str, str], window: Optional[int] = None, keep_first: int = 0,
                  sink: bool = True, qk_norm: Optional[str] = "whole", norm_eps: float = 1e-6,
                  own_kv: bool = True, position: Optional[PartSpec] = None, qkv_bias: bool = False,
                  weights: str = "softmax", score_bias: bool = False, output_gate: Optional[str] = None,
-                 value_mix: Optional[str] = None):
+                 value_mix: Optional[str] = None, chunk: Optional[int] = None, conv_taps: int = 0,
+                 out_bias: bool = False):
         super().__init__(tensors)
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads are not a multiple of {num_kv_heads} kv heads")
-        if qk_norm not in (None, "whole"):
-            raise ValueError(f"qk_norm is None or 'whole', got {qk_norm!r}")
-        if weights not in self.WEIGHTS or value_mix not in self.VALUE_MIX or output_gate not in (None, "sigmoid"):
-            raise ValueError(f"weights is one of {self.WEIGHTS}, value_mix of {self.VALUE_MIX}, output_gate None or "
-                             f"'sigmoid'; got {weights!r}, {value_mix!r}, {output_gate!r}")
+        if qk_norm not in (None, "whole", "head"):
+            raise ValueError(f"qk_norm is None, 'whole' or 'head', got {qk_norm!r}")
+        if weights not in self.WEIGHTS or value_mix not in self.VALUE_MIX or output_gate not in self.OUTPUT_GATES:
+            raise ValueError(f"weights is one of {self.WEIGHTS}, value_mix of {self.VALUE_MIX}, output_gate of "
+                             f"{self.OUTPUT_GATES}; got {weights!r}, {value_mix!r}, {output_gate!r}")
+        if chunk is not None and (window is not None or int(chunk) <= 0):
+            raise ValueError(f"a chunk of positive size stands in place of a window, got {chunk} and {window}")
+        self.chunk = None if chunk is None else int(chunk)
+        self.conv_taps, self.out_bias = int(conv_taps or 0), bool(out_bias)
         self.weights, self.value_mix, self.output_gate = weights, value_mix, output_gate
         self.qkv_bias, self.has_score_bias = bool(qkv_bias), bool(score_bias)
         self.position = build_part("position", position) if position is not None else None
         # the projections that turn, carry biases, mix values or gate heads go through one kernel
         # of their own, which knows no norm over the whole projection and writes keys and values
-        self.rotates = bool(self.position is not None or qkv_bias or value_mix or output_gate)
+        self.shaped = bool(self.conv_taps or qk_norm == "head" or output_gate == "channels"
+                           or (self.position is not None and not hasattr(self.position, "pair_table")))
+        self.rotates = not self.shaped and bool(self.position is not None or qkv_bias or value_mix or output_gate)
+        if self.shaped and (qk_norm == "whole" or not own_kv or value_mix or output_gate == "sigmoid"):
+            raise ValueError("convolutions, norms head by head, halves that turn and gates per channel go with keys and "
+                             "values of the layer's own, without a norm over the whole projection, mixed values or a "
+                             "gate per head")
         if self.rotates and (qk_norm or not own_kv):
             raise ValueError("a position encoding, biases, mixed values or an output gate go with keys and values "
                              "of the layer's own and without a norm over the whole projection")
-        if self.position is not None and not hasattr(self.position, "pair_table"):
-            raise ValueError(f"{type(self.position).__name__} has no pair_table(): this mixer turns neighbouring channels")
+        if self.position is not None and not (hasattr(self.position, "pair_table") or hasattr(self.position, "half_table")):
+            raise ValueError(f"{type(self.position).__name__} has neither a pair_table() nor a half_table()")
         if weights == "sigmoid" and sink:
             raise ValueError("a sink belongs to a softmax's denominator; sigmoid weights have none")
         if score_bias and weights != "sigmoid":
@@ -366,12 +392,14 @@ class WindowedSinkAttention(Mixer):
         self.hidden_size, self.num_heads, self.num_kv_heads = int(hidden_size), int(num_heads), int(num_kv_heads)
         self.key_dim = int(key_dim)
         self.file_value_dim = int(value_dim)                       # a value head as the model file has it
-        self.value_dim = (self.file_value_dim + 7) // 8 * 8        # and as the kernels and the pages see it
+        unit = 16 if self.shaped else 8
+        self.value_dim = (self.file_value_dim + unit - 1) // unit * unit      # and as the kernels and the pages see it
+        self.laid_dim = (self.key_dim + 31) // 32 * 32 if self.shaped else self.key_dim      # a key head in the pages
         self.scale = float(scale)
         self.window = None if window is None else int(window)
         self.keep_first = int(keep_first or 0)
         self.has_sink, self.qk_norm, self.norm_eps, self.own_kv = bool(sink), qk_norm, float(norm_eps), bool(own_kv)
-        self.w_in = self.w_o = self.q_norm = self.k_norm = self.sink = None
+        self.w_in = self.w_o = self.b_o = self.conv = self.q_norm = self.k_norm = self.sink = None
 
     @property
     def q_size(self):
@@ -386,9 +414,12 @@ class WindowedSinkAttention(Mixer):
         return self.num_kv_heads * self.value_dim
 
     @property
+    def gate_size(self):
+        return {None: 0, "sigmoid": self.num_heads, "channels": self.num_heads * self.value_dim}[self.output_gate]
+
+    @property
     def in_size(self):
-        return (self.q_size + (self.k_size + self.v_size if self.own_kv else 0)
-                + (self.num_heads if self.output_gate else 0))
+        return self.q_size + (self.k_size + self.v_size if self.own_kv else 0) + self.gate_size
 
     def tensor_specs(self):
         t, w = self.tensor_names, self.hidden_size
@@ -405,12 +436,18 @@ class WindowedSinkAttention(Mixer):
         if self.has_score_bias:
             specs[t["score_bias"]] = TensorSpec((self.num_heads,), VECTOR)
         if self.output_gate:
-            specs[t["gate_weight"]] = TensorSpec((self.num_heads, w), MATRIX)
+            gates = self.num_heads * (self.file_value_dim if self.output_gate == "channels" else 1)
+            specs[t["gate_weight"]] = TensorSpec((gates, w), MATRIX)
+        if self.out_bias:
+            specs[t["o_bias"]] = TensorSpec((w,), VECTOR)
+        if self.conv_taps:
+            for role, channels in (("q_conv", self.q_size), ("k_conv", self.k_size), ("v_conv", file_v)):
+                specs[t[role]] = TensorSpec((channels, self.conv_taps), MATRIX)
         if self.value_mix and "value_mix" in t:       # (every mixing layer of a model file may carry the number)
             specs[t["value_mix"]] = TensorSpec((), VECTOR)
         if self.position is not None:
             specs.update(self.position.tensor_specs())
-        if self.qk_norm:
+        if self.qk_norm == "whole":
             specs[t["q_norm"]] = TensorSpec((self.q_size,), VECTOR, INIT_NORM)
             if self.own_kv:
                 specs[t["k_norm"]] = TensorSpec((self.k_size,), VECTOR, INIT_NORM)
@@ -420,7 +457,7 @@ class WindowedSinkAttention(Mixer):
 
     def bind(self, tensors, ops, dtype):
         super().bind(tensors, ops, dtype)
-        ops.check_windowed_attention_sizes(self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim, dtype)
+        ops.check_windowed_attention_sizes(self.num_heads, self.num_kv_heads, self.laid_dim, self.value_dim, dtype)
         ops.check_product_sizes(self.hidden_size, dtype, "attention projections (hidden size)")
         ops.check_product_sizes(self.num_heads * self.value_dim, dtype, "attention output projection (heads * value size)")
         t = self.tensor_names
@@ -436,15 +473,22 @@ class WindowedSinkAttention(Mixer):
         rows = [tensors[t["q_weight"]]]
         if self.own_kv:
             rows += [tensors[t["k_weight"]], value_heads(tensors[t["v_weight"]], self.num_kv_heads)]
-        if self.output_gate:
+        if self.output_gate == "channels":
+            rows.append(value_heads(tensors[t["gate_weight"]], self.num_heads))
+        elif self.output_gate:
             rows.append(tensors[t["gate_weight"]])
         self.w_in = ops.prepare_weight(torch.cat(rows, dim=0).contiguous())       # one product for q (, k, v, gates)
         if self.qkv_bias:
             bias = [tensors[t["q_bias"]].float(), tensors[t["k_bias"]].float(),
                     value_heads(tensors[t["v_bias"]].float(), self.num_kv_heads)]
             if self.output_gate:
-                bias.append(torch.zeros(self.num_heads, dtype=torch.float32, device=bias[0].device))
+                bias.append(torch.zeros(self.gate_size, dtype=torch.float32, device=bias[0].device))
             self.b_in = torch.cat(bias).contiguous()
+        if self.conv_taps:
+            self.conv = torch.cat([tensors[t["q_conv"]].float(), tensors[t["k_conv"]].float(),
+                                   value_heads(tensors[t["v_conv"]].float(), self.num_kv_heads)]).contiguous()
+        if self.out_bias:
+            self.b_o = tensors[t["o_bias"]].contiguous()
         if self.has_score_bias:
             self.score_bias = tensors[t["score_bias"]].float().contiguous()
         if self.value_mix == "mix":
@@ -452,16 +496,46 @@ class WindowedSinkAttention(Mixer):
         if self.position is not None:
             self.position.bind(tensors, ops, dtype)
         self.w_o = ops.prepare_weight(value_heads(tensors[t["o_weight"]].t(), self.num_heads).t().contiguous())
-        if self.qk_norm:
+        if self.qk_norm == "whole":
             self.q_norm = tensors[t["q_norm"]].float().contiguous()
             self.k_norm = tensors[t["k_norm"]].float().contiguous() if self.own_kv else None
         if self.has_sink:
             self.sink = tensors[t["sink"]].float().contiguous()
 
     def cache_spec(self):
-        return CacheSpec((("k", PageTensor((self.num_kv_heads, self.key_dim), 1)),
+        return CacheSpec((("k", PageTensor((self.num_kv_heads, self.laid_dim), 1)),
                           ("v", PageTensor((self.num_kv_heads, self.value_dim), 1))),
-                         self.window, self.keep_first if self.window is not None else 0)
+                         self.window, self.keep_first if self.window is not None or self.chunk is not None else 0, self.chunk)
+
+    def state_spec(self):
+        if self.conv_taps <= 1:
+            return {}
+        return {"conv": ((self.conv_taps - 1, self.q_size + self.k_size + self.v_size), torch.float32)}
+
+    def _shape_and_write(self, proj, q, ctx, entry, group):
+        """Convolution, rotation and norms of the projections; queries out, keys and values to the pages."""
+        ops = self.ops
+        freq, rot_dims, pairing = None, 0, "halves"
+        if self.position is not None and hasattr(self.position, "half_table"):
+            freq, rot_dims = self.position.half_table()
+        elif self.position is not None:
+            freq, rot_dims, magnitude = self.position.pair_table()
+            pairing = "neighbours"
+            if magnitude != 1.0:
+                raise ValueError("this mixer's kernel turns channels without a magnitude")
+
+        def launch():
+            # (whether every request brings one row is not a matter of the number of rows)
+            ops.project_conv_write(proj, self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim, self.b_in,
+                                   self.conv, entry.state.get("conv"), ctx.all_q_start, ctx.all_req_rows, freq, rot_dims,
+                                   pairing, self.norm_eps if self.qk_norm == "head" else None, q, entry.k_cache,
+                                   entry.v_cache, group.page_size, ctx.positions, ctx.row_req, group.block_table,
+                                   ctx.n_rows == ctx.n_reqs)
+        live = getattr(ops, "live", None)
+        if live is not None:
+            live(launch)
+        else:
+            launch()
 
     def forward_into(self, h, out, ctx, entry):
         ops, rows = self.ops, h.shape[0]
@@ -471,9 +545,11 @@ class WindowedSinkAttention(Mixer):
         group = ctx.group(entry.group)
         proj = ctx.scratch("windowed_attention.proj", (rows, self.in_size), torch.float32)
         project_normed(ops, h, self.w_in, proj, self.dtype, self.hidden_size)
-        q = ctx.scratch("windowed_attention.q", (rows, self.q_size), self.dtype)
+        q = ctx.scratch("windowed_attention.q", (rows, self.num_heads * self.laid_dim), self.dtype)
         gate = None
-        if self.rotates:
+        if self.shaped:
+            self._shape_and_write(proj, q, ctx, entry, group)
+        elif self.rotates:
             freq, rot_dims, magnitude = self.position.pair_table() if self.position is not None else (None, 0, 1.0)
             if self.output_gate:
                 gate = ctx.scratch("windowed_attention.gate", (rows, self.num_heads), torch.float32)
@@ -491,18 +567,21 @@ class WindowedSinkAttention(Mixer):
         mixed = ctx.scratch("windowed_attention.out", (rows, self.num_heads * self.value_dim), self.dtype)
         sigmoid = self.weights == "sigmoid"
         kind = dict(weights="sigmoid") if sigmoid else {}
+        if self.chunk is not None:
+            kind["chunk"] = self.chunk
+        reach = self.window if self.window is not None else self.chunk
 
         def attend():
             # (which requests bring many rows is read from the step's description when the launch
             # is made, also when it is made again from a kept sequence of calls)
             long_from, launches = self._split(ctx, group.page_size)
-            ops.sink_window_attention(q, self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim,
+            ops.sink_window_attention(q, self.num_heads, self.num_kv_heads, self.laid_dim, self.value_dim,
                                       entry.k_cache, entry.v_cache, group.block_table, group.page_size,
                                       ctx.positions, ctx.row_req, self.window, self.keep_first,
                                       self.score_bias if sigmoid else self.sink,
                                       self.scale, mixed, ctx.all_q_start, long_from, launches,
-                                      ctx.max_ctx_len if self.window is None
-                                      else min(ctx.max_ctx_len, self.window + self.keep_first), **kind)
+                                      ctx.max_ctx_len if reach is None
+                                      else min(ctx.max_ctx_len, reach + self.keep_first), **kind)
         live = getattr(ops, "live", None)
         if live is not None:
             live(attend)
@@ -510,7 +589,12 @@ class WindowedSinkAttention(Mixer):
             attend()
         if gate is not None:
             ops.gate_heads(mixed, gate, self.num_heads, self.value_dim, self.output_gate)
-        ops.linear_logits(mixed, self.w_o, out)
+        if self.output_gate == "channels":
+            ops.gate_channels(mixed, proj, self.q_size + self.k_size + self.v_size)
+        if self.b_o is not None:
+            ops.linear_logits(mixed, self.w_o, out, self.b_o)
+        else:
+            ops.linear_logits(mixed, self.w_o, out)
 
     def forward(self, h, residual, ctx, entry):
         y = ctx.scratch("windowed_attention.sum", (1,) + tuple(residual.shape), torch.float32)
@@ -518,7 +602,7 @@ class WindowedSinkAttention(Mixer):
         self.ops.add_pending(residual, PendingSums(y, 1))
 
     def _split(self, ctx, page_size):
-        return rows_by_kernel(self.ops, ctx, self.dtype, self.key_dim, self.value_dim, page_size)
+        return rows_by_kernel(self.ops, ctx, self.dtype, self.laid_dim, self.value_dim, page_size)
 
     keeps_launches = True      # (what depends on the step beyond its rows is asked for at the launch)
 
@@ -527,7 +611,7 @@ class WindowedSinkAttention(Mixer):
 
     def weight_bytes(self):
         total = 0
-        for w in (self.w_in, self.w_o, self.q_norm, self.k_norm, self.sink, self.b_in, self.score_bias):
+        for w in (self.w_in, self.w_o, self.q_norm, self.k_norm, self.sink, self.b_in, self.score_bias, self.conv, self.b_o):
             if w is not None:
                 total += w.numel() * w.element_size()
         return total

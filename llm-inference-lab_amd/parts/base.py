@@ -52,6 +52,8 @@ class CacheSpec:
     of the latest positions (the current one included) it ever reads, or ``None`` for
     all; ``keep_first``: how many of a sequence's first positions it goes on reading after
     the window has passed them (their pages are never given back while the request lives).
+    ``chunk`` (in place of a window): the mixer reads the positions of the current one's own chunk
+    only, chunks of so many positions counted from the sequence's start.
     Mixers with equal specs share one group of pages and one block table; the cache
     manager allocates ``[runs, pages, *page_shape]`` per name and a run of the mixer finds
     its slices in ``entry.cache[name]``."""
@@ -59,6 +61,7 @@ class CacheSpec:
     tensors: Tuple[Tuple[str, PageTensor], ...]
     window: Optional[int] = None
     keep_first: int = 0
+    chunk: Optional[int] = None
 
     def __post_init__(self):
         names = [n for n, _ in self.tensors]
@@ -68,12 +71,32 @@ class CacheSpec:
             raise ValueError(f"a window holds at least the current position, got {self.window}")
         if self.keep_first < 0:
             raise ValueError(f"keep_first counts positions, got {self.keep_first}")
+        if self.chunk is not None and (self.chunk <= 0 or self.window is not None):
+            raise ValueError(f"a chunk holds at least one position and stands in place of a window, got {self.chunk}")
+
+    def lowest_read(self, position: int) -> int:
+        """The lowest position (the kept first ones aside) that the query at ``position``, or at any
+        later one, reads."""
+        if self.window is not None:
+            return max(0, position - self.window + 1)
+        return position // self.chunk * self.chunk if self.chunk is not None else 0
+
+    @property
+    def bounded(self) -> bool:
+        """Whether positions fall out of sight as a sequence grows."""
+        return self.window is not None or self.chunk is not None
+
+    @property
+    def reach(self) -> Optional[int]:
+        """The most positions a query sees beside the kept first ones (None: all)."""
+        return self.window if self.window is not None else self.chunk
 
     def widened_by(self, other: "CacheSpec") -> "CacheSpec":
         """The same tensors kept long enough for ``other``'s reads as well (a run that reads
         another run's cache through a window of its own)."""
         window = None if self.window is None or other.window is None else max(self.window, other.window)
-        return dataclasses.replace(self, window=window, keep_first=max(self.keep_first, other.keep_first))
+        chunk = self.chunk if window is None and self.chunk == other.chunk else None      # (else: everything is kept)
+        return dataclasses.replace(self, window=window, chunk=chunk, keep_first=max(self.keep_first, other.keep_first))
 
     def bytes_per_token(self, dtype: torch.dtype) -> int:
         return sum(t.token_elements() * torch.empty((), dtype=t.dtype or dtype).element_size()

@@ -68,11 +68,18 @@ class SublayerNormBlock(Block):
 
     A part that ``writes_output`` writes its float32 result into a scratch buffer
     (``forward_into``); any other part (made for blocks that add the sublayer's result
-    straight into the stream) is handed a zeroed buffer in the stream's place."""
+    straight into the stream) is handed a zeroed buffer in the stream's place.
+
+    ``token_shift``: what the mixer reads is the stream's row mixed with the row before it in the
+    sequence, ``h_t = x_t + (x_(t-1) - x_t) * shift`` element by element (``shift [width]``: tensor role
+    ``shift``; zeros before the sequence's start), taken in float32 and rounded once.  The last row is
+    per-request state, so a sequence may be cut anywhere.  The feed-forward reads ``x`` itself."""
 
     def __init__(self, hidden_size: int, mixer: PartSpec, norm1: PartSpec, feed_forward: PartSpec = None,
-                 norm2: PartSpec = None, tensors: Dict[str, str] = None):
+                 norm2: PartSpec = None, tensors: Dict[str, str] = None, token_shift: bool = False):
         super().__init__(tensors)
+        self.token_shift = bool(token_shift)
+        self.shift = None
         if (feed_forward is None) != (norm2 is None):
             raise ValueError("a feed-forward and its norm come together")
         self.hidden_size = int(hidden_size)
@@ -94,12 +101,25 @@ class SublayerNormBlock(Block):
         specs = {}
         for p in self.parts():
             specs.update(p.tensor_specs())
+        if self.token_shift:
+            specs[self.tensor_names["shift"]] = TensorSpec((self.hidden_size,), VECTOR)
         return specs
+
+    def state_spec(self):
+        spec = dict(self.mixer.state_spec())
+        if self.token_shift:
+            spec["shifted_row"] = ((self.hidden_size,), torch.float32)
+        return spec
 
     def bind(self, tensors, ops, dtype):
         super().bind(tensors, ops, dtype)
         for p in self.parts():
             p.bind(tensors, ops, dtype)
+        if self.token_shift:
+            self.shift = tensors[self.tensor_names["shift"]].float().view(1, -1).contiguous()
+
+    def kernel_libraries(self):
+        return [("stream_ops", None)] + super().kernel_libraries()
 
     def _fold(self, residual, ctx):
         pending = getattr(ctx, "pending", None)
@@ -121,8 +141,18 @@ class SublayerNormBlock(Block):
         self.ops.activation(residual, h, "cast")
         return h
 
-    def _sublayer(self, part, h, residual, ctx, *entry):
+    def _shifted(self, residual, ctx, entry):
+        """The mixer's input where tokens are shifted: every row of the stream mixed with the one before."""
+        h = ctx.scratch("block.shifted", (1,) + tuple(residual.shape), self.dtype)
+        self.ops.shift_mix(residual, self.shift, entry.state["shifted_row"], ctx.row_req, ctx.all_q_start,
+                           ctx.all_req_rows, h)
+        return h[0]
+
+    def _sublayer(self, part, norm, h, residual, ctx, *entry):
         y = ctx.scratch("block.sublayer_out", tuple(residual.shape), torch.float32)
+        if hasattr(part, "forward_pending") and getattr(norm, "adds_pieces", False):
+            pieces = part.forward_pending(h, y, ctx, *entry)      # (a product left in pieces is summed by the norm)
+            return y if pieces is None else pieces
         if part.writes_output:
             part.forward_into(h, y, ctx, *entry)
         else:
@@ -133,16 +163,22 @@ class SublayerNormBlock(Block):
 
     def forward(self, residual, ctx, entry):
         self._fold(residual, ctx)
-        h = self._input(residual, ctx, entry)
         # every sum's new rows go to the next reader of the stream in the same pass
+        if self.token_shift:
+            # (the next reader of the last sum is a kernel that takes the float32 rows)
+            mixed = self._shifted(residual, ctx, entry)
+            h = (residual if self.dtype == torch.float32
+                 else ctx.scratch("block.stream_copy", tuple(residual.shape), self.dtype))
+        else:
+            mixed = h = self._input(residual, ctx, entry)
         copy = h if self.dtype != torch.float32 else None
-        y = self._sublayer(self.mixer, h, residual, ctx, entry)
-        self.norm1.add_into(y, residual, copy)
+        y = self._sublayer(self.mixer, self.norm1, mixed, residual, ctx, entry)
+        self.norm1.add_into(y, residual, copy if self.feed_forward is not None or not self.token_shift else None)
         if self.feed_forward is not None:
-            y = self._sublayer(self.feed_forward, h, residual, ctx)
-            self.norm2.add_into(y, residual, copy)
+            y = self._sublayer(self.feed_forward, self.norm2, h, residual, ctx)
+            self.norm2.add_into(y, residual, None if self.token_shift else copy)
         memo = getattr(ctx, "memo", None)
-        if memo is not None and copy is not None:
+        if memo is not None and copy is not None and not self.token_shift:
             memo[self.NOTE] = entry.index
 
     def weight_bytes(self):

@@ -5,7 +5,7 @@ from typing import Dict
 
 import torch
 
-from ..weights.loader import TensorSpec, MATRIX
+from ..weights.loader import TensorSpec, MATRIX, VECTOR, INIT_NORM
 from .base import FeedForward, NormedInput
 from .registry import register_part
 
@@ -143,15 +143,22 @@ class SwiGLU(FeedForward):
 
 class DenseFeedForward(FeedForward):
     """``W_down act(W_up h)`` with no gate and no biases; ``activation="relu2"``: ``act(z) =
-    max(z, 0) ** 2``, taken on the float32 sums of the first product and rounded once."""
+    max(z, 0) ** 2``, taken on the float32 sums of the first product and rounded once.
+
+    ``activation="poly_norm"``: ``act(z) = a N(z) + b N(z^2) + c N(z^3) + e`` with four learned numbers
+    (tensor role ``act_coef [4]``: a, b, c, e), powers element by element and ``N`` the division of a
+    row by its root mean square over the feed-forward's width (``norm_eps`` inside the root); float32
+    from the sums of the first product on, rounded once."""
 
     writes_output = True
     keeps_launches = True
-    ACTIVATIONS = ("relu2",)
+    ACTIVATIONS = ("relu2", "poly_norm")
 
     def __init__(self, hidden_size: int, intermediate_size: int, tensors: Dict[str, str],
-                 activation: str = "relu2"):
+                 activation: str = "relu2", norm_eps: float = 1e-6):
         super().__init__(tensors)
+        self.norm_eps = float(norm_eps)
+        self.coef = None
         if activation not in self.ACTIVATIONS:
             raise ValueError(f"a dense feed-forward takes the activations {self.ACTIVATIONS}, got '{activation}'")
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
@@ -161,7 +168,10 @@ class DenseFeedForward(FeedForward):
 
     def tensor_specs(self):
         t, h, i = self.tensor_names, self.hidden_size, self.intermediate_size
-        return {t["up_weight"]: TensorSpec((i, h), MATRIX), t["down_weight"]: TensorSpec((h, i), MATRIX)}
+        specs = {t["up_weight"]: TensorSpec((i, h), MATRIX), t["down_weight"]: TensorSpec((h, i), MATRIX)}
+        if self.activation == "poly_norm":
+            specs[t["act_coef"]] = TensorSpec((4,), VECTOR, INIT_NORM)
+        return specs
 
     def bind(self, tensors, ops, dtype):
         super().bind(tensors, ops, dtype)
@@ -169,6 +179,11 @@ class DenseFeedForward(FeedForward):
         t = self.tensor_names
         self.w_up = ops.prepare_weight(pad_rows(tensors[t["up_weight"]], self.kernel_size))
         self.w_down = ops.prepare_weight(pad_columns(tensors[t["down_weight"]], self.kernel_size))
+        if self.activation == "poly_norm":
+            self.coef = tensors[t["act_coef"]].float().contiguous()
+
+    def kernel_libraries(self):
+        return [("stream_ops", None)] if self.activation == "poly_norm" else []
 
     def _activated(self, h, ctx):
         rows = h.shape[0]
@@ -179,8 +194,23 @@ class DenseFeedForward(FeedForward):
             return act
         sums = ctx.scratch("dense_ffn.sums", (rows, self.kernel_size), torch.float32)
         self.ops.linear_logits(h, self.w_up, sums)
-        self.ops.activation(sums, act, self.activation)
+        if self.activation == "poly_norm":
+            self.ops.poly_norm(sums, self.coef, self.norm_eps, self.intermediate_size, act)
+        else:
+            self.ops.activation(sums, act, self.activation)
         return act
+
+    def forward_pending(self, h, out, ctx):
+        """As ``SwiGLU.forward_pending``: into ``out``, or the pieces of the down product."""
+        if isinstance(h, NormedInput):
+            h = h.tensor()
+        rows, act = h.shape[0], self._activated(h, ctx)
+        splits = self.ops.split_count(rows, self.dtype, self.hidden_size, self.kernel_size)
+        if splits > 1:
+            parts = ctx.scratch("dense_ffn.pieces", (splits, rows, self.hidden_size), torch.float32)
+            return self.ops.linear_partials(act, self.w_down, parts, splits)
+        self.ops.linear_logits(act, self.w_down, out)
+        return None
 
     def forward_into(self, h, out, ctx):
         self.ops.linear_logits(self._activated(h, ctx), self.w_down, out)

@@ -10,7 +10,107 @@ from .base import Mixer, NormedInput, PendingSums, project_normed
 from .registry import register_part
 
 
-class GatedLinearAttention(Mixer):
+def pad_heads(x, heads: int, channels: int, laid: int):
+    """Rows (or entries) of ``heads`` heads of ``channels`` channels -> of ``laid``, zeros behind."""
+    if channels == laid:
+        return x
+    per_head = x.unflatten(0, (heads, channels))
+    zeros = torch.zeros((heads, laid - channels) + tuple(x.shape[1:]), dtype=x.dtype, device=x.device)
+    return torch.cat([per_head, zeros], dim=1).flatten(0, 1)
+
+
+class ScanMixer(Mixer):
+    """What the mixers share whose state ``S [key_dim, value_dim]`` per head follows ``S_t = decay_t * S_(t-1) + k_t
+    v_t^T``: the state's slots, the scan over a step's rows (whole, or long portions in chunks side by
+    side) and room for it.  ``value_dim`` is a value head as the kernels see it: a multiple of 8 (the
+    products' inner sizes), zeros behind the file's ``file_value_dim`` channels."""
+
+    writes_output = True
+    keeps_launches = True
+
+    def _set_sizes(self, hidden_size, num_heads, key_dim, value_dim):
+        self.hidden_size, self.num_heads, self.key_dim = int(hidden_size), int(num_heads), int(key_dim)
+        self.file_value_dim = int(value_dim)
+        self.value_dim = (self.file_value_dim + 7) // 8 * 8
+
+    @property
+    def qk_size(self):
+        return self.num_heads * self.key_dim
+
+    @property
+    def v_size(self):
+        return self.num_heads * self.value_dim
+
+    def _values(self, x):
+        return pad_heads(x, self.num_heads, self.file_value_dim, self.value_dim)
+
+    def _check_sizes(self, ops, dtype, name):
+        ops.check_linear_attention_sizes(self.num_heads, self.key_dim, self.value_dim)
+        ops.check_product_sizes(self.hidden_size, dtype, f"{name} projections (hidden size)")
+        ops.check_product_sizes(self.v_size, dtype, f"{name} output projection (heads * value size)")
+
+    def state_spec(self):
+        return {"s": ((self.num_heads, self.key_dim, self.value_dim), torch.float32)}
+
+    def _min_chunk(self) -> int:
+        rules = getattr(self.ops, "rules", None)
+        return int(getattr(rules, "scan_min_chunk", 16))
+
+    def _scan(self, proj, off_q, off_k, off_v, decay, q_scale, state, ctx, bonus=None, memory=None):
+        """The outputs of this step's rows in pieces ``[rows, heads, slices, value_dim]``.  ``memory``: ``(keep,
+        take, normaliser's state)``; the normaliser's pieces ``[rows, heads, slices]`` come back beside them."""
+        ops, rows = self.ops, proj.shape[0]
+        heads, d, e = self.num_heads, self.key_dim, self.value_dim
+        slices = ops.gla_slices(d)
+        parts = ctx.scratch("linear_attention.parts", (rows, heads, slices, e), torch.float32)
+        # room for the chunks of a long portion: at most rows / (smallest chunk) + requests
+        most = rows // max(1, self._min_chunk()) + ctx.max_reqs
+        chunk_state = ctx.scratch("linear_attention.chunk_state", (most, heads, d, e), torch.float32)
+        chunk_decay = ctx.scratch("linear_attention.chunk_decay", (most, heads, d), torch.float32)
+        norm_parts = chunk_norm = None
+        if memory is not None:
+            norm_parts = ctx.scratch("linear_attention.norm_parts", (rows, heads, slices), torch.float32)
+            chunk_norm = ctx.scratch("linear_attention.chunk_norm", (most, heads, d), torch.float32)
+
+        def scan():
+            # (how many requests the step has and how long the longest portion is are read when
+            # the launch is made, also when it is made again from a kept sequence of calls)
+            pick = getattr(ops, "gla_scan_chunk", None)
+            chunk = pick(rows, ctx.max_q_len, heads, e) if pick is not None else 0
+            kind = {}
+            if bonus is not None:
+                kind["bonus"] = bonus
+            if memory is not None:
+                kind["memory"] = tuple(memory) + (norm_parts, chunk_norm if chunk else None)
+            ops.gla_scan(proj, off_q, off_k, off_v, decay, q_scale, heads, d, e, state, ctx.all_q_start, ctx.all_req_rows,
+                         ctx.n_reqs, parts, chunk, chunk_state if chunk else None, chunk_decay if chunk else None, **kind)
+        live = getattr(ops, "live", None)
+        if live is not None:
+            live(scan)
+        else:
+            scan()
+        return parts if memory is None else (parts, norm_parts)
+
+    def _output(self, parts, weight, eps, proj, off_gate, gate, ctx, **memory):
+        mixed = ctx.scratch("linear_attention.out", (proj.shape[0], self.v_size), self.dtype)
+        if self.file_value_dim != self.value_dim:      # (the heads' norm is over the file's channels)
+            memory["norm_count"] = self.file_value_dim
+        self.ops.gla_output(parts, self.num_heads, self.key_dim, self.value_dim, weight, eps, proj, off_gate, mixed, gate,
+                            **memory)
+        return mixed
+
+    def forward(self, h, residual, ctx, entry):
+        if isinstance(h, NormedInput) and not self.takes_normed_input:
+            h = h.tensor()
+        y = ctx.scratch("linear_attention.sum", (1,) + tuple(residual.shape), torch.float32)
+        self.forward_into(h, y[0], ctx, entry)
+        self.ops.add_pending(residual, PendingSums(y, 1))
+
+    def kernel_libraries(self):
+        return [("linear_attention", None)]
+
+
+class GatedLinearAttention(ScanMixer):
     """Linear attention with a decay per key channel and a matrix-valued state per head.
 
     With ``D = key_dim`` and ``E = value_dim``: ``q = Wq h * q_scale`` (``q_scale`` defaults to
@@ -29,13 +129,10 @@ class GatedLinearAttention(Mixer):
     step to step; the decays, the recurrence and the norm are float32 throughout, and the
     projections reach them unrounded (32-bit sums of the matrix products)."""
 
-    writes_output = True
-
     def __init__(self, hidden_size: int, num_heads: int, key_dim: int, value_dim: int, decay_rank: int,
                  tau: float, tensors: Dict[str, str], norm_eps: float = 1e-6, q_scale: Optional[float] = None):
         super().__init__(tensors)
-        self.hidden_size, self.num_heads = int(hidden_size), int(num_heads)
-        self.key_dim, self.value_dim = int(key_dim), int(value_dim)
+        self._set_sizes(hidden_size, num_heads, key_dim, value_dim)
         # (None: the rank is whatever the model file's decay tensors have)
         self.decay_rank = None if decay_rank is None else int(decay_rank)
         self.tau, self.norm_eps = float(tau), float(norm_eps)
@@ -44,23 +141,15 @@ class GatedLinearAttention(Mixer):
         self.q_scale = float(q_scale) if q_scale is not None else self.key_dim ** -0.5
         self.w_in = self.w_o = self.w_decay = self.b_decay = self.norm_weight = None
 
-    @property
-    def qk_size(self):
-        return self.num_heads * self.key_dim
-
-    @property
-    def v_size(self):
-        return self.num_heads * self.value_dim
-
     def tensor_specs(self):
         t, w = self.tensor_names, self.hidden_size
         return {
             t["q_weight"]: TensorSpec((self.qk_size, w), MATRIX),
             t["k_weight"]: TensorSpec((self.qk_size, w), MATRIX),
-            t["v_weight"]: TensorSpec((self.v_size, w), MATRIX),
-            t["gate_weight"]: TensorSpec((self.v_size, w), MATRIX),
-            t["o_weight"]: TensorSpec((w, self.v_size), MATRIX),
-            t["out_norm"]: TensorSpec((self.value_dim,), VECTOR, INIT_NORM),
+            t["v_weight"]: TensorSpec((self.num_heads * self.file_value_dim, w), MATRIX),
+            t["gate_weight"]: TensorSpec((self.num_heads * self.file_value_dim, w), MATRIX),
+            t["o_weight"]: TensorSpec((w, self.num_heads * self.file_value_dim), MATRIX),
+            t["out_norm"]: TensorSpec((self.file_value_dim,), VECTOR, INIT_NORM),
             t["decay_down"]: TensorSpec((self.decay_rank, w), MATRIX),
             t["decay_up"]: TensorSpec((self.qk_size, self.decay_rank), MATRIX),
             t["decay_bias"]: TensorSpec((self.qk_size,), VECTOR),
@@ -68,9 +157,7 @@ class GatedLinearAttention(Mixer):
 
     def bind(self, tensors, ops, dtype):
         super().bind(tensors, ops, dtype)
-        ops.check_linear_attention_sizes(self.num_heads, self.key_dim, self.value_dim)
-        ops.check_product_sizes(self.hidden_size, dtype, "linear attention projections (hidden size)")
-        ops.check_product_sizes(self.v_size, dtype, "linear attention output projection (heads * value size)")
+        self._check_sizes(ops, dtype, "linear attention")
         t = self.tensor_names
         rank = int(tensors[t["decay_down"]].shape[0])
         if int(tensors[t["decay_up"]].shape[1]) != rank:
@@ -84,22 +171,15 @@ class GatedLinearAttention(Mixer):
         rows = []
         for role in ("q_weight", "k_weight", "v_weight", "gate_weight", "decay_down"):
             self.offsets[role] = at
-            rows.append(tensors[t[role]])
+            rows.append(self._values(tensors[t[role]]) if role in ("v_weight", "gate_weight") else tensors[t[role]])
             at += rows[-1].shape[0]
         self.in_size = at
         self.w_in = ops.prepare_weight(torch.cat(rows, dim=0).contiguous())
-        self.w_o = ops.prepare_weight(tensors[t["o_weight"]].contiguous())
+        self.w_o = ops.prepare_weight(self._values(tensors[t["o_weight"]].t()).t().contiguous())
         # the second factor of the decays is applied in float32, inside the decay kernel
         self.w_decay = tensors[t["decay_up"]].float().contiguous()
         self.b_decay = tensors[t["decay_bias"]].float().contiguous()
-        self.norm_weight = tensors[t["out_norm"]].float().contiguous()
-
-    def _min_chunk(self) -> int:
-        rules = getattr(self.ops, "rules", None)
-        return int(getattr(rules, "scan_min_chunk", 16))
-
-    def state_spec(self):
-        return {"s": ((self.num_heads, self.key_dim, self.value_dim), torch.float32)}
+        self.norm_weight = pad_heads(tensors[t["out_norm"]].float(), 1, self.file_value_dim, self.value_dim).contiguous()
 
     def forward_into(self, h, out, ctx, entry):
         ops, rows, o = self.ops, h.shape[0], self.offsets
@@ -107,44 +187,9 @@ class GatedLinearAttention(Mixer):
         ops.linear_logits(h, self.w_in, proj)
         decay = ctx.scratch("linear_attention.decay", (rows, self.qk_size), torch.float32)
         ops.gla_decay(proj[:, o["decay_down"]:], self.decay_rank, self.w_decay, self.b_decay, self.tau, decay)
-        parts = ctx.scratch("linear_attention.parts",
-                            (rows, self.num_heads, ops.gla_slices(self.key_dim), self.value_dim), torch.float32)
-        state = entry.state["s"]
-        # room for the chunks of a long portion: at most rows / (smallest chunk) + requests
-        most = rows // max(1, self._min_chunk()) + ctx.max_reqs
-        chunk_state = ctx.scratch("linear_attention.chunk_state",
-                                  (most, self.num_heads, self.key_dim, self.value_dim), torch.float32)
-        chunk_decay = ctx.scratch("linear_attention.chunk_decay", (most, self.num_heads, self.key_dim), torch.float32)
-
-        def scan():
-            # (how many requests the step has and how long the longest portion is are read when
-            # the launch is made, also when it is made again from a kept sequence of calls)
-            pick = getattr(ops, "gla_scan_chunk", None)
-            chunk = pick(rows, ctx.max_q_len, self.num_heads, self.value_dim) if pick is not None else 0
-            ops.gla_scan(proj, o["q_weight"], o["k_weight"], o["v_weight"], decay, self.q_scale, self.num_heads,
-                         self.key_dim, self.value_dim, state, ctx.all_q_start, ctx.all_req_rows, ctx.n_reqs, parts,
-                         chunk, chunk_state if chunk else None, chunk_decay if chunk else None)
-        live = getattr(ops, "live", None)
-        if live is not None:
-            live(scan)
-        else:
-            scan()
-        mixed = ctx.scratch("linear_attention.out", (rows, self.v_size), self.dtype)
-        ops.gla_output(parts, self.num_heads, self.key_dim, self.value_dim, self.norm_weight, self.norm_eps, proj,
-                       o["gate_weight"], mixed)
+        parts = self._scan(proj, o["q_weight"], o["k_weight"], o["v_weight"], decay, self.q_scale, entry.state["s"], ctx)
+        mixed = self._output(parts, self.norm_weight, self.norm_eps, proj, o["gate_weight"], "silu", ctx)
         ops.linear_logits(mixed, self.w_o, out)
-
-    def forward(self, h, residual, ctx, entry):
-        if isinstance(h, NormedInput):
-            h = h.tensor()
-        y = ctx.scratch("linear_attention.sum", (1,) + tuple(residual.shape), torch.float32)
-        self.forward_into(h, y[0], ctx, entry)
-        self.ops.add_pending(residual, PendingSums(y, 1))
-
-    keeps_launches = True
-
-    def kernel_libraries(self):
-        return [("linear_attention", None)]
 
     def weight_bytes(self):
         return sum(w.numel() * w.element_size()
@@ -236,15 +281,9 @@ class DeltaRuleAttention(Mixer):
                              f"{int(tensors[t['decay_up']].shape[1])} columns: the two factors of the decay "
                              f"projection do not fit")
         self.decay_rank = rank
-        e, ek = self.file_value_dim, self.value_dim
 
         def value_heads(x):
-            """Rows (or entries) of the heads' ``e`` value channels -> of ``ek``, zeros behind."""
-            if e == ek:
-                return x
-            per_head = x.unflatten(0, (self.num_heads, e))
-            zeros = torch.zeros((self.num_heads, ek - e) + tuple(x.shape[1:]), dtype=x.dtype, device=x.device)
-            return torch.cat([per_head, zeros], dim=1).flatten(0, 1)
+            return pad_heads(x, self.num_heads, self.file_value_dim, self.value_dim)
         # one product for r, k, v, the gate, the rates and the low-rank input of the decays
         self.offsets, at, rows = {}, 0, []
         for role in ("r_weight", "k_weight", "v_weight", "gate_weight", "rate_weight", "decay_down"):
@@ -321,5 +360,214 @@ class DeltaRuleAttention(Mixer):
                                                           self.norm_weight) if w is not None)
 
 
+class TimeMixAttention(ScanMixer):
+    """A recurrent mixer whose projections each read their own mix of the current token and the one
+    before it, with a decay per key channel and a bonus for the current token.
+
+    With ``h'`` the previous token's input (zeros for a sequence's first): each ``s`` of ``r, k, v, g, w``
+    reads ``h + (h' - h) * mix_s``.  ``r, k`` (``heads x D``) and ``v`` (``heads x E``, default ``E = D``) are
+    products with their mixes, the decays ``w = exp(-exp(W2 tanh(W1 mix_w) + w0))`` per head and key channel;
+    per head, token by token, with the learned bonus ``u``::
+
+        o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t
+        S_t = diag(w_t) S_(t-1) + k_t v_t^T                  (S is D x E, zero at a sequence's start)
+
+    then every head's ``o_t`` is divided by its root mean square over ``E`` (``norm_eps`` inside the root), the
+    heads are put side by side, multiplied by a weight of all heads' size and by ``silu`` of the product
+    of the ``g`` mix (``gate="sigmoid"``: its sigmoid), and projected by ``Wo``.
+
+    State per request: ``S`` in float32 and the last input row (compute dtype).  Decays, bonus, the
+    recurrence and the norm are float32, and the projections reach them unrounded; the mixes are
+    rounded once.  The rank of the decay projection is whatever the model file's tensors have.
+
+    Tensor roles: ``mix_r, mix_k, mix_v, mix_g, mix_w, r_weight, k_weight, v_weight, gate_weight, decay_down,
+    decay_up, decay_bias, bonus, out_norm, o_weight``."""
+
+    MIXES = (("mix_r", "r_weight"), ("mix_k", "k_weight"), ("mix_v", "v_weight"), ("mix_g", "gate_weight"),
+             ("mix_w", "decay_down"))
+
+    def __init__(self, hidden_size: int, num_heads: int, key_dim: int, tensors: Dict[str, str],
+                 value_dim: Optional[int] = None, norm_eps: float = 1e-6, gate: str = "silu"):
+        super().__init__(tensors)
+        self._set_sizes(hidden_size, num_heads, key_dim, key_dim if value_dim is None else value_dim)
+        self.norm_eps = float(norm_eps)
+        if gate not in ("sigmoid", "silu"):
+            raise ValueError(f"the output gate is 'sigmoid' or 'silu', got {gate!r}")
+        self.gate = gate
+        self.decay_rank = None
+        self.mix = self.w_o = self.w_decay = self.b_decay = self.bonus = self.norm_weight = None
+        self.w_mixed, self.offsets, self.in_size = {}, {}, 0
+
+    def tensor_specs(self):
+        t, w = self.tensor_names, self.hidden_size
+        file_v = self.num_heads * self.file_value_dim
+        specs = {t[role]: TensorSpec((w,), VECTOR) for role, _ in self.MIXES}
+        specs.update({
+            t["r_weight"]: TensorSpec((self.qk_size, w), MATRIX),
+            t["k_weight"]: TensorSpec((self.qk_size, w), MATRIX),
+            t["v_weight"]: TensorSpec((file_v, w), MATRIX),
+            t["gate_weight"]: TensorSpec((file_v, w), MATRIX),
+            t["decay_down"]: TensorSpec((None, w), MATRIX),
+            t["decay_up"]: TensorSpec((self.qk_size, None), MATRIX),
+            t["decay_bias"]: TensorSpec((self.qk_size,), VECTOR),
+            t["bonus"]: TensorSpec((self.num_heads, self.key_dim), VECTOR),
+            t["out_norm"]: TensorSpec((file_v,), VECTOR, INIT_NORM),
+            t["o_weight"]: TensorSpec((w, file_v), MATRIX),
+        })
+        return specs
+
+    def bind(self, tensors, ops, dtype):
+        super().bind(tensors, ops, dtype)
+        self._check_sizes(ops, dtype, "time mixing")
+        t = self.tensor_names
+        rank = int(tensors[t["decay_down"]].shape[0])
+        if int(tensors[t["decay_up"]].shape[1]) != rank:
+            raise ValueError(f"{t['decay_down']} has {rank} rows but {t['decay_up']} has "
+                             f"{int(tensors[t['decay_up']].shape[1])} columns: the two factors of the decay "
+                             f"projection do not fit")
+        self.decay_rank = rank
+        self.mix = torch.stack([tensors[t[role]].float() for role, _ in self.MIXES]).contiguous()
+        at = 0
+        for _, role in self.MIXES:
+            w = self._values(tensors[t[role]]) if role in ("v_weight", "gate_weight") else tensors[t[role]]
+            self.w_mixed[role] = ops.prepare_weight(w.contiguous())
+            self.offsets[role] = at
+            at += (w.shape[0] + 31) // 32 * 32       # (every product's columns start on a boundary of 128 bytes)
+        self.in_size = at
+        self.w_o = ops.prepare_weight(self._values(tensors[t["o_weight"]].t()).t().contiguous())
+        # the second factor of the decays is applied in float32, inside the decay kernel
+        self.w_decay = tensors[t["decay_up"]].float().contiguous()
+        self.b_decay = tensors[t["decay_bias"]].float().contiguous()
+        self.bonus = tensors[t["bonus"]].float().reshape(-1).contiguous()
+        self.norm_weight = self._values(tensors[t["out_norm"]].float()).contiguous()
+
+    def state_spec(self):
+        return dict(super().state_spec(), previous_row=((self.hidden_size,), None))
+
+    def forward_into(self, h, out, ctx, entry):
+        ops, rows, o = self.ops, h.shape[0], self.offsets
+        mixed = ctx.scratch("time_mix.mixed", (len(self.MIXES), rows, self.hidden_size), self.dtype)
+        ops.shift_mix(h, self.mix, entry.state["previous_row"], ctx.row_req, ctx.all_q_start, ctx.all_req_rows, mixed)
+        proj = ctx.scratch("time_mix.proj", (rows, self.in_size), torch.float32)
+        for i, (_, role) in enumerate(self.MIXES):
+            w = self.w_mixed[role]
+            ops.linear_logits(mixed[i], w, proj[:, o[role]:o[role] + w.shape[0]])
+        decay = ctx.scratch("linear_attention.decay", (rows, self.qk_size), torch.float32)
+        ops.gla_decay(proj[:, o["decay_down"]:], self.decay_rank, self.w_decay, self.b_decay, 1.0, decay, "double_exp")
+        parts = self._scan(proj, o["r_weight"], o["k_weight"], o["v_weight"], decay, 1.0, entry.state["s"], ctx,
+                           bonus=self.bonus)
+        gated = self._output(parts, self.norm_weight, self.norm_eps, proj, o["gate_weight"], self.gate, ctx)
+        ops.linear_logits(gated, self.w_o, out)
+
+    def kernel_libraries(self):
+        return [("stream_ops", None), ("linear_attention", None)]
+
+    def weight_bytes(self):
+        return sum(w.numel() * w.element_size() for w in (*self.w_mixed.values(), self.mix, self.w_o, self.w_decay,
+                                                          self.b_decay, self.bonus, self.norm_weight) if w is not None)
+
+
+class MatrixMemoryAttention(ScanMixer):
+    """A matrix memory with exponential gates: one log input gate and one log forget gate per head, a
+    running maximum that keeps the exponentials in range, and a normaliser.
+
+    With ``D = key_dim`` and ``E = value_dim``: ``q = Wq h * q_scale`` (``q_scale`` defaults to ``D ** -0.5``), ``k = Wk
+    h`` (``heads x D``), ``v = Wv h`` (``heads x E``); per head ``i = cap * tanh((Wi h + bi) / cap)`` and ``f =
+    logsigmoid(cap * tanh((Wf h + bf) / cap))``; token by token, all of ``S``, ``n`` and ``m`` zero at a
+    sequence's start::
+
+        m_t = max(f_t + m_(t-1), i_t)
+        S_t = exp(f_t + m_(t-1) - m_t) S_(t-1) + exp(i_t - m_t) k_t v_t^T        (S is D x E)
+        n_t = exp(f_t + m_(t-1) - m_t) n_(t-1) + exp(i_t - m_t) k_t
+        o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6)
+
+    then every head's ``o_t`` is divided by its root mean square over ``E`` (``norm_eps`` inside the root), the
+    heads are put side by side, multiplied by a weight of all heads' size and by ``sigmoid(Wg h)``
+    (``gate="silu"``: by ``silu``), and projected by ``Wo``.
+
+    State per request, float32: ``S``, ``n`` and ``m``.  Gates, maximum, recurrence, normaliser and norm are
+    float32, and the projections reach them unrounded (32-bit sums of the matrix products).
+
+    Tensor roles: ``q_weight, k_weight, v_weight, gate_weight, i_weight, i_bias, f_weight, f_bias, out_norm,
+    o_weight``."""
+
+    def __init__(self, hidden_size: int, num_heads: int, key_dim: int, value_dim: int, gate_cap: float,
+                 tensors: Dict[str, str], norm_eps: float = 1e-6, q_scale: Optional[float] = None, gate: str = "sigmoid"):
+        super().__init__(tensors)
+        self._set_sizes(hidden_size, num_heads, key_dim, value_dim)
+        self.gate_cap, self.norm_eps = float(gate_cap), float(norm_eps)
+        if self.gate_cap <= 0:
+            raise ValueError(f"the gates' cap must be positive, got {gate_cap}")
+        if gate not in ("sigmoid", "silu"):
+            raise ValueError(f"the output gate is 'sigmoid' or 'silu', got {gate!r}")
+        self.gate = gate
+        self.q_scale = float(q_scale) if q_scale is not None else self.key_dim ** -0.5
+        self.w_in = self.w_o = self.b_i = self.b_f = self.norm_weight = None
+        self.offsets, self.in_size = {}, 0
+
+    def tensor_specs(self):
+        t, w = self.tensor_names, self.hidden_size
+        file_v = self.num_heads * self.file_value_dim
+        return {
+            t["q_weight"]: TensorSpec((self.qk_size, w), MATRIX),
+            t["k_weight"]: TensorSpec((self.qk_size, w), MATRIX),
+            t["v_weight"]: TensorSpec((file_v, w), MATRIX),
+            t["gate_weight"]: TensorSpec((file_v, w), MATRIX),
+            t["i_weight"]: TensorSpec((self.num_heads, w), MATRIX),
+            t["i_bias"]: TensorSpec((self.num_heads,), VECTOR),
+            t["f_weight"]: TensorSpec((self.num_heads, w), MATRIX),
+            t["f_bias"]: TensorSpec((self.num_heads,), VECTOR),
+            t["out_norm"]: TensorSpec((file_v,), VECTOR, INIT_NORM),
+            t["o_weight"]: TensorSpec((w, file_v), MATRIX),
+        }
+
+    def bind(self, tensors, ops, dtype):
+        super().bind(tensors, ops, dtype)
+        self._check_sizes(ops, dtype, "matrix memory")
+        t = self.tensor_names
+        at, rows = 0, []
+        for role in ("q_weight", "k_weight", "v_weight", "gate_weight", "i_weight", "f_weight"):      # (one product)
+            self.offsets[role] = at
+            rows.append(self._values(tensors[t[role]]) if role in ("v_weight", "gate_weight") else tensors[t[role]])
+            at += rows[-1].shape[0]
+        self.in_size = at
+        self.w_in = ops.prepare_weight(torch.cat(rows, dim=0).contiguous())
+        self.w_o = ops.prepare_weight(self._values(tensors[t["o_weight"]].t()).t().contiguous())
+        self.b_i = tensors[t["i_bias"]].float().contiguous()
+        self.b_f = tensors[t["f_bias"]].float().contiguous()
+        self.norm_weight = self._values(tensors[t["out_norm"]].float()).contiguous()
+
+    def state_spec(self):
+        return dict(super().state_spec(), n=((self.num_heads, self.key_dim), torch.float32),
+                    m=((self.num_heads,), torch.float32))
+
+    def forward_into(self, h, out, ctx, entry):
+        ops, rows, o = self.ops, h.shape[0], self.offsets
+        proj = ctx.scratch("linear_attention.proj", (rows, self.in_size), torch.float32)
+        ops.linear_logits(h, self.w_in, proj)
+        keep, take, maxima = (ctx.scratch("matrix_memory." + name, (rows, self.num_heads), torch.float32)
+                              for name in ("keep", "take", "maxima"))
+
+        def gates():        # (how many requests the step has is read when the launch is made)
+            ops.memory_gates(proj, o["i_weight"], o["f_weight"], self.b_i, self.b_f, self.gate_cap, self.num_heads,
+                             entry.state["m"], ctx.all_q_start, ctx.all_req_rows, ctx.n_reqs, keep, take, maxima)
+        live = getattr(ops, "live", None)
+        if live is not None:
+            live(gates)
+        else:
+            gates()
+        parts, norm_parts = self._scan(proj, o["q_weight"], o["k_weight"], o["v_weight"], None, self.q_scale,
+                                       entry.state["s"], ctx, memory=(keep, take, entry.state["n"]))
+        mixed = self._output(parts, self.norm_weight, self.norm_eps, proj, o["gate_weight"], self.gate, ctx,
+                             norm_parts=norm_parts, maxima=maxima)
+        ops.linear_logits(mixed, self.w_o, out)
+
+    def weight_bytes(self):
+        return sum(w.numel() * w.element_size() for w in (self.w_in, self.w_o, self.b_i, self.b_f, self.norm_weight)
+                   if w is not None)
+
+
 register_part("mixer", "gated_linear_attention", GatedLinearAttention)
+register_part("mixer", "time_mix_attention", TimeMixAttention)
+register_part("mixer", "matrix_memory_attention", MatrixMemoryAttention)
 register_part("mixer", "delta_rule_attention", DeltaRuleAttention)

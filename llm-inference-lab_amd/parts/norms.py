@@ -33,6 +33,7 @@ class RMSNorm(Norm):
         self.weight_offset = float(weight_offset)
         self.scalar = bool(scalar)
         self.weight: Optional[torch.Tensor] = None
+        self.weight_f32: Optional[torch.Tensor] = None      # made when a result is first normed into the stream
 
     def tensor_specs(self):
         return {self.tensor_names["weight"]: TensorSpec(() if self.scalar else (self.size,), VECTOR,
@@ -40,6 +41,7 @@ class RMSNorm(Norm):
 
     def bind(self, tensors, ops, dtype):
         super().bind(tensors, ops, dtype)
+        self.weight_f32 = None
         self.weight = tensors[self.tensor_names["weight"]].contiguous()
         if self.scalar:
             self.weight = self.weight.reshape(1).expand(self.size).contiguous()
@@ -54,6 +56,15 @@ class RMSNorm(Norm):
 
     def rms_params(self):
         return self.weight, self.eps
+
+    adds_pieces = True      # ``add_into`` takes a result left in pieces as well
+
+    def add_into(self, y, stream, copy=None):
+        """``stream += norm(y)`` (``y`` float32, or ``PendingSums``); ``copy`` (compute dtype) receives the
+        stream's new rows.  (The kernel takes its weight in float32.)"""
+        if self.weight_f32 is None:
+            self.weight_f32 = self.weight.float().contiguous()
+        self.ops.rmsnorm_add(y, self.weight_f32, self.eps, stream, copy=copy)
 
     def weight_bytes(self):
         return self.weight.numel() * self.weight.element_size()

@@ -38,6 +38,12 @@ class RotaryEmbedding(PositionEncoding):
             raise ValueError(f"heads of {dim} channels do not fit an even {self.padded_dim}")
         self.theta = float(theta)
         self.inv_freq: Optional[torch.Tensor] = None
+        self.half_freq: Optional[torch.Tensor] = None
+
+    def half_table(self):
+        """``(f [rotary_dim / 2], rotary_dim)`` for a mixer whose kernel turns channel ``i`` with channel ``i +
+        rotary_dim / 2`` in the file's own order."""
+        return self.half_freq, self.rotary_dim
 
     def bind(self, tensors, ops, dtype):
         super().bind(tensors, ops, dtype)
@@ -45,6 +51,7 @@ class RotaryEmbedding(PositionEncoding):
         freq = torch.zeros(self.padded_dim // 2, dtype=torch.float64)
         freq[:self.rotary_dim // 2] = 1.0 / (torch.tensor(self.theta, dtype=torch.float64) ** exponent)
         self.inv_freq = freq.to(torch.float32).to(ops.device)
+        self.half_freq = self.inv_freq[:self.rotary_dim // 2].contiguous()
 
     def channel_order(self):
         """``order[j]``: which channel of a head, as the model file has it, goes to place ``j`` (-1: a

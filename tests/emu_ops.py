@@ -55,7 +55,8 @@ class EmuRecord:
 class EmuOps:
     # the operations that do work on tensors: written down while a part is recorded, as the
     # product's kernel set writes down its calls into the kernel libraries
-    RECORDED = ("embed", "gather_tokens", "rmsnorm", "linear", "linear_relu2", "linear_residual", "linear_partials",
+    RECORDED = ("shift_mix", "poly_norm", "normed_sum", "project_conv_write", "gate_channels", "memory_gates",
+                "embed", "gather_tokens", "rmsnorm", "linear", "linear_relu2", "linear_residual", "linear_partials",
                 "add_pending", "linear_logits", "linear_swiglu", "fused_norm_qkv", "qkv_rope_cache",
                 "fused_norm_swiglu", "fused_norm_logits", "rope_inplace", "rope_kv_write",
                 "paged_attention", "argmax", "sample", "layernorm", "layernorm_add", "activation",
@@ -216,9 +217,9 @@ class EmuOps:
         self._count("add_pending")
         x.add_(self._owed(pending))
 
-    def linear_logits(self, x, w, out):
+    def linear_logits(self, x, w, out, bias=None):
         self._count("linear_logits")
-        out.copy_(x.float() @ w.float().t())
+        out.copy_(x.float() @ w.float().t() + (0.0 if bias is None else bias.float()))
 
     def linear_swiglu(self, x, w_gu, out, activation="silu"):
         """w_gu rows alternate in runs of 16: gate rows of 16 outputs, then the
@@ -289,7 +290,7 @@ class EmuOps:
 
     def sink_window_attention(self, q, num_heads, num_kv_heads, key_dim, value_dim, k_cache, v_cache, block_table,
                               page_size, positions, row_req, window, keep_first, sink, scale, out,
-                              q_start=None, long_from=0, launches=3, max_keys=0, weights="softmax"):
+                              q_start=None, long_from=0, launches=3, max_keys=0, weights="softmax", chunk=None):
         """(``long_from``, ``launches``: how the kernels share the rows; the result is the same.)"""
         self._count("sink_window_attention")
         rows = q.shape[0]
@@ -297,7 +298,7 @@ class EmuOps:
         group = num_heads // num_kv_heads
         for r in range(rows):
             i, b = int(positions[r]), int(row_req[r])
-            lo = max(0, i - window + 1) if window else 0
+            lo = max(0, i - window + 1) if window else i // chunk * chunk if chunk else 0
             js = list(range(min(int(keep_first or 0), lo))) + list(range(lo, i + 1))
             pages = torch.tensor([int(block_table[b, j // page_size]) for j in js])
             offs = torch.tensor([j % page_size for j in js])
@@ -395,10 +396,83 @@ class EmuOps:
                 st.copy_(new)
                 o[t] = torch.einsum("hde,hd->he", st, r)
 
-    def rmsnorm_add(self, y, weight, eps, x, next_norm=None):
+    def normed_sum(self, out, y1, w1, a, y2, w2, b, eps):
+        self._count("normed_sum")
+        rms = lambda y: y / torch.sqrt((y * y).mean(-1, keepdim=True) + eps)
+        out.copy_(a * rms(y1) * w1 + b * rms(y2) * w2)
+
+    def shift_mix(self, h, mix, state, row_req, q_start, req_rows, out):
+        self._count("shift_mix")
+        hf = h.float()
+        for b in sorted({int(x) for x in row_req[:h.shape[0]]}):
+            lo, hi, slot = int(q_start[b]), int(q_start[b + 1]), int(req_rows[b])
+            before = torch.cat([state[slot].float().view(1, -1), hf[lo:hi - 1]], dim=0)
+            for m in range(mix.shape[0]):
+                out[m, lo:hi] = (hf[lo:hi] + (before - hf[lo:hi]) * mix[m]).to(out.dtype)
+            state[slot] = h[hi - 1]
+
+    def poly_norm(self, z, coef, eps, count, out):
+        self._count("poly_norm")
+        n = lambda v: v / torch.sqrt((v * v).sum(-1, keepdim=True) / count + eps)
+        a, b, c, e = (coef[i] for i in range(4))
+        out.copy_((a * n(z) + b * n(z * z) + c * n(z * z * z) + e).to(out.dtype))
+
+    def project_conv_write(self, proj, num_heads, num_kv_heads, key_dim, value_dim, bias, conv, state, q_start, req_rows,
+                           freq, rot_dims, pairing, unit_eps, q_out, k_cache, v_cache, page_size, positions, row_req,
+                           block_table, one_row_each):
+        self._count("project_conv_write")
+        rows, laid = q_out.shape[0], k_cache.shape[-1]
+        qs, ks, vs = num_heads * key_dim, num_kv_heads * key_dim, num_kv_heads * value_dim
+        u = proj[:, :qs + ks + vs].float()
+        if bias is not None:
+            u = u + bias[:qs + ks + vs]
+        reqs = sorted({int(x) for x in row_req[:rows]})
+        assert not one_row_each or rows == len(reqs)
+        y = u
+        if conv is not None:
+            taps, y = conv.shape[1], torch.zeros_like(u)
+            for b in reqs:
+                lo, hi, slot = int(q_start[b]), int(q_start[b + 1]), int(req_rows[b])
+                joined = torch.cat([state[slot], u[lo:hi]], dim=0) if taps > 1 else u[lo:hi]
+                for j in range(taps):
+                    y[lo:hi] += conv[:, j] * joined[j:j + hi - lo]
+                if taps > 1:
+                    state[slot] = joined[-(taps - 1):]
+
+        def shaped(x, heads):
+            x = x.reshape(rows, heads, key_dim).clone()
+            if rot_dims:
+                half = rot_dims // 2
+                ang = positions[:rows].float().unsqueeze(-1) * freq.float()
+                cos, sin = torch.cos(ang).unsqueeze(1), torch.sin(ang).unsqueeze(1)
+                first, second = ((slice(0, half), slice(half, rot_dims)) if pairing == "halves"
+                                 else (slice(0, rot_dims, 2), slice(1, rot_dims, 2)))
+                a, b = x[..., first].clone(), x[..., second].clone()
+                x[..., first], x[..., second] = a * cos - b * sin, b * cos + a * sin
+            if unit_eps is not None:
+                x = x / torch.sqrt((x * x).mean(-1, keepdim=True) + unit_eps)
+            return torch.nn.functional.pad(x, (0, laid - key_dim))
+        q_out.copy_(shaped(y[:, :qs], num_heads).reshape(rows, -1).to(q_out.dtype))
+        k = shaped(y[:, qs:qs + ks], num_kv_heads).to(k_cache.dtype)
+        v = y[:, qs + ks:].to(v_cache.dtype).view(rows, num_kv_heads, value_dim)
+        for r in range(rows):
+            at = int(positions[r])
+            page = int(block_table[int(row_req[r]), at // page_size])
+            o = at % page_size
+            k_cache[page, :, o] = k[r]
+            cache_layout.value_quads(v_cache[page])[:, o >> 2, :, o & 3] = v[r]
+
+    def gate_channels(self, out, proj, off_gate):
+        self._count("gate_channels")
+        g = torch.sigmoid(proj[:, off_gate:off_gate + out.shape[1]].float())
+        out.copy_((out.float() * g).to(out.dtype))
+
+    def rmsnorm_add(self, y, weight, eps, x, next_norm=None, copy=None):
         self._count("rmsnorm_add")
         v = self._owed(y) if isinstance(y, PendingSums) else y.float()
         x.add_(v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * weight.float())
+        if copy is not None:
+            copy.copy_(x.to(copy.dtype))
         if next_norm is not None:
             w, e, out = next_norm
             out.copy_((x / torch.sqrt((x * x).mean(-1, keepdim=True) + e) * w.float()).to(out.dtype))
@@ -412,18 +486,32 @@ class EmuOps:
     def gla_slices(self, key_dim):
         return (key_dim + self.SCAN_SLICE - 1) // self.SCAN_SLICE
 
-    def gla_decay(self, low, rank, w2, bias, tau, decay):
+    def gla_decay(self, low, rank, w2, bias, tau, decay, kind="sigmoid"):
         self._count("gla_decay")
-        z = low[:, :rank].float() @ w2.float().t()
+        x = low[:, :rank].float()
+        z = (torch.tanh(x) if kind == "double_exp" else x) @ w2.float().t()
         if bias is not None:
             z = z + bias.float()
-        decay.copy_(torch.exp(torch.nn.functional.logsigmoid(z) / tau))
+        decay.copy_(torch.exp(-torch.exp(z)) if kind == "double_exp"
+                    else torch.exp(torch.nn.functional.logsigmoid(z) / tau))
+
+    def memory_gates(self, proj, off_i, off_f, bias_i, bias_f, cap, num_heads, max_state, q_start, req_rows, n_reqs, keep,
+                     take, maxima):
+        self._count("memory_gates")
+        z = lambda at, b: cap * torch.tanh((proj[:, at:at + num_heads] + (0.0 if b is None else b)) / cap)
+        i, f = z(off_i, bias_i), torch.nn.functional.logsigmoid(z(off_f, bias_f))
+        for b in range(n_reqs):
+            m = max_state[int(req_rows[b])]
+            for t in range(int(q_start[b]), int(q_start[b + 1])):
+                new = torch.maximum(f[t] + m, i[t])
+                keep[t], take[t], maxima[t] = torch.exp(f[t] + m - new), torch.exp(i[t] - new), new
+                m.copy_(new)
 
     def gla_scan_chunk(self, rows, longest, num_heads, value_dim):
         return 16 if longest >= 32 else 0
 
     def gla_scan(self, proj, off_q, off_k, off_v, decay, q_scale, num_heads, key_dim, value_dim, state, q_start,
-                 req_rows, n_reqs, parts, chunk=0, chunk_state=None, chunk_decay=None):
+                 req_rows, n_reqs, parts, chunk=0, chunk_state=None, chunk_decay=None, bonus=None, memory=None):
         """(``chunk``: how the kernel spreads the work; the recurrence is the same.)"""
         self._count("gla_scan")
         if chunk:
@@ -436,15 +524,30 @@ class EmuOps:
                 q = proj[t, off_q:off_q + H * D].view(H, D) * q_scale
                 k = proj[t, off_k:off_k + H * D].view(H, D)
                 v = proj[t, off_v:off_v + H * E].view(H, E)
-                st.mul_(decay[t].view(H, D, 1)).add_(k.unsqueeze(-1) * v.unsqueeze(-2))
-                o = st * q.unsqueeze(-1)                        # [H, D, E]
+                kv = k.unsqueeze(-1) * v.unsqueeze(-2)
+                if memory is not None:
+                    keep, take, n, norm_parts, _ = memory
+                    st.mul_(keep[t].view(H, 1, 1)).add_(take[t].view(H, 1, 1) * kv)
+                    n[slot].mul_(keep[t].view(H, 1)).add_(take[t].view(H, 1) * k)
+                    nq = n[slot] * q
+                    for s in range(norm_parts.shape[2]):
+                        norm_parts[t, :, s] = nq[:, s * S:(s + 1) * S].sum(1)
+                    o = st * q.unsqueeze(-1)
+                elif bonus is not None:
+                    o = (st + bonus.view(H, D, 1) * kv) * q.unsqueeze(-1)
+                    st.mul_(decay[t].view(H, D, 1)).add_(kv)
+                else:
+                    st.mul_(decay[t].view(H, D, 1)).add_(kv)
+                    o = st * q.unsqueeze(-1)                        # [H, D, E]
                 for s in range(parts.shape[2]):
                     parts[t, :, s] = o[:, s * S:(s + 1) * S].sum(1)
 
     def gla_output(self, parts, num_heads, key_dim, value_dim, weight, eps, proj, off_gate, out, gate="silu",
-                   norm_count=0):
+                   norm_count=0, norm_parts=None, maxima=None):
         self._count("gla_output")
         o = parts.sum(2)                                        # [rows, H, E]
+        if norm_parts is not None:
+            o = o / (torch.maximum(norm_parts.sum(2).abs(), torch.exp(-maxima)) + 1e-6).unsqueeze(-1)
         w = weight.float().view(num_heads, value_dim) if weight.numel() == num_heads * value_dim else weight.float()
         y = o / torch.sqrt((o * o).sum(-1, keepdim=True) / (norm_count or value_dim) + eps) * w
         g = proj[:, off_gate:off_gate + num_heads * value_dim].float().view(-1, num_heads, value_dim)
