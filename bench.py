@@ -3,7 +3,7 @@
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--context S]
                     [--shape 0.5b|7b|32b] [--layers L] [--dtype bf16|f32]
     python bench.py --mixed [--shape 7b] [--requests 64] [--chunk 512] [--outputs 64]
-    python bench.py --design vivevik|ruvalorn|minodra|ninisun [--size small|medium|large] [--context 2048]
+    python bench.py --design vivevik|ruvalorn|minodra|ninisun|mazanex [--size small|medium|large] [--context 2048]
 
 Default: the layer sizes of the Qwen2.5-0.5B shape with seeded random weights,
 batch 8, context 4096, bfloat16.  A "step" is one decode step of the whole
@@ -53,6 +53,11 @@ attention with turned neighbouring channels and values mixed with the first laye
 layer attention with sigmoid weights beside a delta-rule state, gelu-gated feed-forwards), beside
 the Vivevik design of equal size (the closest one: the same attention kernels, a recurrent layer in
 every three) and the Qwen2 decoder.
+
+``--design mazanex``: the same for the Mazanex design (a token shift in front of every mixer, norms on the
+sublayers' results, feed-forwards of normed powers; in turn attention over chunks beside time mixing,
+gated linear attention and a matrix memory with exponential gates), beside the Vivevik design of equal
+size (the closest one: the same attention and scan kernels) and the Qwen2 decoder.
 
 ``--mixed``: many requests with prompts of different lengths go through the
 scheduler with a small token budget, so that portions of prompts run beside the
@@ -293,6 +298,51 @@ def ninisun_flops(cfg, tokens):
     return total + 2 * w * cfg.vocab
 
 
+# ``--design mazanex``: layers in threes: a parallel layer (attention over chunks of 1,024 positions beside
+# time mixing with width / 64 heads of 64 x 64), gated linear attention with Vivevik's sizes, a matrix
+# memory of the same state; every layer has the feed-forward of normed powers (two matrices).
+def mazanex_config(size):
+    import llm_inference_lab_amd as lab
+    width, heads, kv, dim, ff, layers = DESIGN_SIZES[size]
+    listed = []
+    for i in range(layers):
+        mlp = dict(kind="dense", ff=ff)
+        if i % 3 == 0:
+            left = dict(heads=heads, kv_heads=kv, dim=dim, vdim=dim, scale=dim ** -0.5, conv=4, rot=dict(dims=dim, base=1e4),
+                        mask=dict(size=DESIGN_WINDOW))
+            listed.append(dict(type="parallel", mixer=dict(left=left, right=dict(heads=width // 64, dim=64)), mlp=mlp))
+        elif i % 3 == 1:
+            listed.append(dict(type="gla", mixer=dict(heads=width // 128, dim=64, vdim=128, tau=8.0), mlp=mlp))
+        else:
+            listed.append(dict(type="mlstm", mixer=dict(heads=width // 128, dim=64, vdim=128, gate_cap=12.0), mlp=mlp))
+    return lab.MazanexConfig.from_dict(dict(architecture="Mazanex", vocab=DESIGN_VOCAB, width=width,
+                                            norm=dict(eps=1e-6), layers=listed))
+
+
+def mazanex_flops(cfg, tokens):
+    """Multiply-adds times two of one prompt of ``tokens`` positions (products and attention; a recurrence
+    counts its state update and its read-out)."""
+    w, total = cfg.width, 0
+    rank = cfg.DEFAULT_DECAY_RANK
+    for l in cfg.layers:
+        if l.type == "parallel":
+            a, r = l.left, l.right
+            q, k, v, e = a.heads * a.dim, a.kv_heads * a.dim, a.kv_heads * a.vdim, a.heads * a.vdim
+            total += tokens * 2 * (w * (q + k + v + e) + e * w)
+            chunk = a.chunk or tokens
+            total += 2 * sum(i % chunk + 1 for i in range(tokens)) * a.heads * (a.dim + a.vdim)
+            n = r.heads * r.dim
+            total += tokens * (2 * (w * (4 * n + rank) + rank * n + n * w) + 4 * n * r.dim)
+        else:
+            r = l.recurrent
+            qk, v = r.heads * r.dim, r.heads * r.vdim
+            low = rank * (w + qk) if l.type == "gla" else 2 * r.heads * w
+            total += tokens * (2 * (w * (2 * qk + 2 * v) + v * w + low) + 4 * r.heads * r.dim * r.vdim)
+        if l.mlp is not None:
+            total += tokens * 4 * w * l.mlp.ff
+    return total + 2 * w * cfg.vocab
+
+
 def design_run(args, bracket=None):
     """``--design vivevik``: both models at each size, one after the other on the same GPU.
     ``--only-model``, ``--only-prefill`` / ``--only-decode`` and ``--batch`` narrow the run (for
@@ -313,9 +363,9 @@ def design_run(args, bracket=None):
         record[size] = {"width": width, "heads": heads, "kv_heads": kv, "head_dim": dim, "ff": ff, "layers": layers,
                         "context": context, "window": DESIGN_WINDOW}
         design = {"ruvalorn": ruvalorn_config, "minodra": minodra_config, "vivevik": vivevik_config,
-                  "ninisun": ninisun_config}[args.design](size)
+                  "ninisun": ninisun_config, "mazanex": mazanex_config}[args.design](size)
         beside = [("qwen2", qwen)]
-        if args.design == "ninisun":         # (the closest design first)
+        if args.design in ("ninisun", "mazanex"):         # (the closest design first)
             beside.insert(0, ("vivevik", vivevik_config(size)))
         for label, cfg in [(args.design, design)] + beside:
             if args.only_model and label != args.only_model:
@@ -335,6 +385,7 @@ def design_run(args, bracket=None):
                      ruvalorn_flops(cfg, args.prefill_tokens) if label == "ruvalorn" else
                      minodra_flops(cfg, args.prefill_tokens) if label == "minodra" else
                      ninisun_flops(cfg, args.prefill_tokens) if label == "ninisun" else
+                     mazanex_flops(cfg, args.prefill_tokens) if label == "mazanex" else
                      prefill_flops(cfg, args.prefill_tokens))
             out = {"weight_bytes_per_step": engine.weight_bytes_per_step()}
             if not args.only_decode:
@@ -356,7 +407,7 @@ def design_run(args, bracket=None):
             torch.cuda.empty_cache()
         print(f"[bench] {size}: {json.dumps(record[size])}", file=sys.stderr, flush=True)
     print(json.dumps({"metric": "design_throughput", "design": args.design,
-                      "beside": "vivevik, qwen2" if args.design == "ninisun" else "qwen2", "dtype": args.dtype,
+                      "beside": "vivevik, qwen2" if args.design in ("ninisun", "mazanex") else "qwen2", "dtype": args.dtype,
                       "data": "synthetic", "unit": "tokens/s", "prefill_tokens": args.prefill_tokens,
                       "sizes": record}))
 
@@ -867,10 +918,10 @@ def main():
                     help="fix a choice of the kernels for the whole run, to compare variants: a keyword of "
                          "engine.ops.debug.force, values separated by ':' (attention_splits=64:8, "
                          "attention_merge_kernel=64, gemm_tile=129)")
-    ap.add_argument("--design", choices=["vivevik", "ruvalorn", "minodra", "ninisun"], default=None,
+    ap.add_argument("--design", choices=["vivevik", "ruvalorn", "minodra", "ninisun", "mazanex"], default=None,
                     help="throughput of another design beside the Qwen2 decoder of equal size")
     ap.add_argument("--size", choices=sorted(DESIGN_SIZES), default=None, help="--design: one size only")
-    ap.add_argument("--only-model", choices=["vivevik", "ruvalorn", "minodra", "ninisun", "qwen2"], default=None, help="--design: one of the two models only")
+    ap.add_argument("--only-model", choices=["vivevik", "ruvalorn", "minodra", "ninisun", "mazanex", "qwen2"], default=None, help="--design: one of the two models only")
     ap.add_argument("--only-decode", action="store_true", help="--design: decode at --batch only, no prefill")
     ap.add_argument("--side", choices=["7b", "32b", "f32", "peaks"], help=argparse.SUPPRESS)
     args = ap.parse_args()
