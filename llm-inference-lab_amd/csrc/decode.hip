@@ -90,6 +90,11 @@ struct SkinnyArgs {
   int ksplit;
   size_t part_stride;
   int act;         // SK_STORE: 1 = max(z, 0)^2 before the rounding; SK_SWIGLU: 2 = gelu (tanh form) gate
+  // SK_PART: segments of the columns may read inputs of their own: the strips from seg_end[s - 1] to
+  // seg_end[s] - 1 multiply the rows x + s * seg_stride (segs <= 1: all strips read x).
+  int segs;
+  int seg_end[7];
+  size_t seg_stride;
   int tiles;       // tiles of 16 MB rows
   int col_blocks;  // blocks that a tile of rows takes (sets of columns, times ksplit)
 };
@@ -412,8 +417,15 @@ __global__ __launch_bounds__(MB >= 4 ? 512 : 1024) void skinny_block_kernel(Skin
     // piece past K or a row past M reads a valid piece instead: it meets zeros of
     // the padded W, or lands in a row of the result that nobody reads
     const bf16_t* xb[MB];
+    const bf16_t* x_rows = (const bf16_t*)a.x;
+    if constexpr (EPI == SK_PART) {
+      int seg = 0;
 #pragma unroll
-    for (int mb = 0; mb < MB; ++mb) xb[mb] = (const bf16_t*)a.x + (size_t)min(mb * 16 + c, M - 1) * K;
+      for (int i = 0; i < 7; ++i) seg += (i + 1 < a.segs && wstrip >= a.seg_end[i]) ? 1 : 0;
+      x_rows += seg * a.seg_stride;
+    }
+#pragma unroll
+    for (int mb = 0; mb < MB; ++mb) xb[mb] = x_rows + (size_t)min(mb * 16 + c, M - 1) * K;
     auto xload = [&](int st, int mb) {
       return *(const bf16x8*)(xb[mb] + min(max(0, min(st, steps - 1)) * 32 + g * 8, K - 8));
     };
@@ -720,6 +732,8 @@ extern "C" void llmlab_skinny_shape(int epilogue, int norm, int M, int N, int K,
 //   pend / pend_splits / pend_ld / pend_stride: pieces that a former SK_PART call left and
 //     that belong to the rows of x (norm != 0: added while the rows are read) or to the
 //     rows of out (SK_RESID: added with the product, which folds them into the stream)
+//   segs > 1 (SK_PART): the strips of 16 rows of W below seg_ends[0] multiply x, the ones from there to
+//     below seg_ends[1] x + seg_stride, and so on (seg_ends: segs - 1 numbers in host memory)
 extern "C" int llmlab_skinny_linear(const void* x, int norm, const int* x_rows, const void* norm_w,
                                     int norm_w_dtype, float eps, const void* w, const void* bias,
                                     int bias_dtype, int epilogue, void* out, int M, int N, int K,
@@ -727,8 +741,10 @@ extern "C" int llmlab_skinny_linear(const void* x, int norm, const int* x_rows, 
                                     const int* row_req, const int* table, int table_stride,
                                     int page_size, void* kcache, void* vcache, int nq, int nkv, int d,
                                     int num_cus, const float* pend, int pend_splits, int pend_ld,
-                                    size_t pend_stride, int ksplit, size_t part_stride,
-                                    hipStream_t stream) {
+                                    size_t pend_stride, int ksplit, size_t part_stride, int segs,
+                                    const int* seg_ends, size_t seg_stride, hipStream_t stream) {
+  LLMLAB_REQUIRE(segs <= 1 || (segs <= 8 && seg_ends && epilogue == SK_PART && seg_stride % 8 == 0),
+                 "skinny_linear: up to 8 segments with inputs of their own, in pieces, got %d", segs);
   LLMLAB_REQUIRE(M >= 0 && M <= SK_MAX_ROWS, "skinny_linear: takes at most %d rows, got %d", SK_MAX_ROWS, M);
   LLMLAB_REQUIRE(N > 0 && K > 0 && K % 8 == 0, "skinny_linear: bad sizes N=%d K=%d (K must be a multiple of 8)", N, K);
   // (6 at this interface: STORE through the squared relu; 7: the paired product with a gelu gate)
@@ -787,6 +803,9 @@ extern "C" int llmlab_skinny_linear(const void* x, int norm, const int* x_rows, 
   const int blocks = (N + 16 * shape.nsb - 1) / (16 * shape.nsb) * ksplit;
   SkinnyArgs a;
   a.pend = pend; a.pend_splits = pend_splits; a.pend_ld = pend_ld; a.pend_stride = pend_stride;
+  a.segs = segs;
+  for (int i = 0; i < 7; ++i) a.seg_end[i] = i + 1 < segs ? seg_ends[i] : 0;
+  a.seg_stride = seg_stride;
   a.ksplit = ksplit; a.part_stride = part_stride; a.tiles = tiles; a.col_blocks = blocks;
   a.qsplit = shape.qsplit;
   a.act = act;

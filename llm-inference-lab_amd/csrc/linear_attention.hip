@@ -518,6 +518,197 @@ extern "C" int llmlab_gla_output(const float* parts, int rows, int n_heads, int 
 }
 
 
+// ------------------------------------------------------------------ one row, whole
+// Decoding: every request brings ONE row.  A block takes a request's row for one head and does what
+// the decays (or gates), the scan and the output do in three launches: the state [D, E] comes from the
+// slot into registers (a group of E / 4 lanes a key channel, four value channels a lane, the loads
+// asked for before anything else), meanwhile the decays of the head's key channels (or its gates) are worked
+// out, then the update, the read-out, the sum over the groups through LDS, the head's norm and its gate.
+// The same numbers as the three kernels up to the order of the sums over key channels.
+struct RowArgs {
+  const float* proj; int ld, off_q, off_k, off_v, off_g; float q_scale; int n_heads, D, E, groups;
+  float* state; const int* q_start; const int* req_rows;
+  const float* w; float eps; int w_per_head, gate_kind, count;
+  int off_low, rank; const float* w2; const float* bias; int decay_kind; float inv_tau;      // DECAY, BONUS
+  const float* bonus;                                                                         // BONUS
+  int off_i, off_f; const float* bias_i; const float* bias_f; float cap; float* norm_state; float* max_state;      // MEMORY
+};
+constexpr int ROW_MAX_RANK = 512;
+template <int KIND, typename T, int ROWS>      // ROWS: key channels a group of lanes takes at most
+__global__ __launch_bounds__(1024) void recurrent_row_kernel(RowArgs a, T* __restrict__ out) {
+  extern __shared__ float row_lds[];           // low [rank] | q, k, decay, bonus [D each] | sums [groups, E]
+  __shared__ float red[17];
+  const int b = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, D = a.D, E = a.E;
+  const int r = a.q_start[b], slot = a.req_rows[b];
+  const float* row = a.proj + (size_t)r * a.ld;
+  float* s_low = row_lds;
+  float* s_q = row_lds + (KIND == KIND_MEMORY ? 0 : a.rank);
+  float* s_k = s_q + D;
+  float* s_a = s_k + D;
+  float* s_u = s_a + D;
+  float* s_sum = s_u + D;
+  const int lanes = E >> 2, g = tid / lanes, j = tid - g * lanes;
+  const bool active = g < a.groups;
+  float* st = a.state + ((size_t)slot * a.n_heads + h) * D * E + 4 * j;
+  floatx4 S[ROWS];
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {             // (past the end: the last channel again, dropped below)
+    const int d = min(g + a.groups * i, D - 1);
+    S[i] = active ? *(const floatx4*)(st + (size_t)d * E) : floatx4{0.f, 0.f, 0.f, 0.f};
+  }
+  floatx4 v = floatx4{0.f, 0.f, 0.f, 0.f};
+  if (active)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = row[a.off_v + h * E + 4 * j + i];
+  const float gate = tid < E ? row[a.off_g + h * E + tid] : 0.f;
+  const float w = tid < E ? a.w[a.w_per_head ? h * E + tid : tid] : 0.f;
+  for (int d = tid; d < D; d += blockDim.x) {
+    s_q[d] = row[a.off_q + h * D + d];
+    s_k[d] = row[a.off_k + h * D + d];
+    if (KIND == KIND_BONUS) s_u[d] = a.bonus[h * D + d];
+  }
+  float keep = 0.f, m = 0.f;
+  if (KIND == KIND_MEMORY) {                   // (a head's two gates: every thread for itself)
+    const float before = a.max_state[(size_t)slot * a.n_heads + h];
+    const float in = a.cap * tanhf((row[a.off_i + h] + (a.bias_i ? a.bias_i[h] : 0.f)) / a.cap);
+    const float z = a.cap * tanhf((row[a.off_f + h] + (a.bias_f ? a.bias_f[h] : 0.f)) / a.cap);
+    const float f = -(fmaxf(-z, 0.f) + log1pf(expf(-fabsf(z))));
+    m = fmaxf(f + before, in);
+    keep = expf(f + before - m);
+    const float take = expf(in - m);
+    v *= take;
+    float part = 0.f;
+    float* n = a.norm_state + ((size_t)slot * a.n_heads + h) * D;
+    for (int d = tid; d < D; d += blockDim.x) {
+      const float x = fmaf(keep, n[d], take * s_k[d]);      // (this thread's own s_k, s_q)
+      n[d] = x;
+      part = fmaf(x, s_q[d], part);
+    }
+    const float nq = block_sum(part, red) * a.q_scale;      // (also the barrier behind s_q and s_k)
+    if (tid == 0) a.max_state[(size_t)slot * a.n_heads + h] = m;
+    m = memory_size(nq, m);
+  } else {
+    for (int i = tid; i < a.rank; i += blockDim.x) {
+      const float x = row[a.off_low + i];
+      s_low[i] = a.decay_kind == DECAY_DOUBLE_EXP ? tanhf(x) : x;
+    }
+    __syncthreads();
+    for (int d = tid; d < D; d += blockDim.x) {
+      const int c = h * D + d;
+      float z = a.bias ? a.bias[c] : 0.f;
+      const float* w2 = a.w2 + (size_t)c * a.rank;
+      if ((a.rank & 3) == 0) {
+        for (int i = 0; i < a.rank; i += 4) {
+          const floatx4 w4 = *(const floatx4*)(w2 + i);
+#pragma unroll
+          for (int q = 0; q < 4; ++q) z = fmaf(w4[q], s_low[i + q], z);
+        }
+      } else {
+        for (int i = 0; i < a.rank; ++i) z = fmaf(w2[i], s_low[i], z);
+      }
+      s_a[d] = decay_of(z, a.decay_kind, a.inv_tau);
+    }
+    __syncthreads();
+  }
+  floatx4 acc = floatx4{0.f, 0.f, 0.f, 0.f};
+  if (active) {
+#pragma unroll
+    for (int i = 0; i < ROWS; ++i) {
+      const int d = g + a.groups * i;
+      if (d < D) {
+        const float k = s_k[d], q = s_q[d], decay = KIND == KIND_MEMORY ? keep : s_a[d];
+        const float u = KIND == KIND_BONUS ? s_u[d] : 0.f;
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+          const float kv = k * v[c];
+          if (KIND == KIND_BONUS) acc[c] = fmaf(fmaf(u, kv, S[i][c]), q, acc[c]);
+          S[i][c] = fmaf(decay, S[i][c], kv);
+          if (KIND != KIND_BONUS) acc[c] = fmaf(S[i][c], q, acc[c]);
+        }
+        *(floatx4*)(st + (size_t)d * E) = S[i];
+      }
+    }
+#pragma unroll
+    for (int c = 0; c < 4; ++c) s_sum[g * E + 4 * j + c] = acc[c];
+  }
+  __syncthreads();
+  float o = 0.f;
+  if (tid < E) {
+    for (int i = 0; i < a.groups; ++i) o += s_sum[i * E + tid];
+    o *= a.q_scale;
+    if (KIND == KIND_MEMORY) o = o / m;
+  }
+  const float ms = block_sum(o * o, red) / (float)a.count;
+  if (tid < E) {
+    const float y = o * (1.0f / sqrtf(ms + a.eps)) * w;
+    const float sg = 1.0f / (1.0f + expf(-gate));
+    out[((size_t)r * a.n_heads + h) * E + tid] = from_float<T>(y * (a.gate_kind == 1 ? sg : gate * sg));
+  }
+}
+
+constexpr int ROW_MAX_ROWS = 8;
+// threads of a block (0: these sizes are not taken)
+extern "C" int llmlab_recurrent_row_threads(int D, int E) {
+  if (D <= 0 || E <= 0 || E % 4 != 0 || E > 1024 || D > 1024) return 0;
+  for (int threads = (E + 63) / 64 * 64 < 256 ? 256 : (E + 63) / 64 * 64; threads <= 1024; threads += 64) {
+    const int groups = threads / (E / 4);
+    if ((D + groups - 1) / groups <= (threads < 512 ? 4 : ROW_MAX_ROWS)) return threads;
+  }
+  return 0;
+}
+
+extern "C" int llmlab_recurrent_row(const float* proj, int ld, int off_q, int off_k, int off_v, int off_g, float q_scale,
+                                    int n_heads, int D, int E, float* state, const int* q_start, const int* req_rows,
+                                    int n_reqs, const float* w, float eps, int w_per_head, int gate_kind, int norm_count,
+                                    int kind, int off_low, int rank, const float* w2, const float* bias, int decay_kind,
+                                    float tau, const float* bonus, int off_i, int off_f, const float* bias_i,
+                                    const float* bias_f, float cap, float* norm_state, float* max_state, void* out, int dtype,
+                                    hipStream_t stream) {
+  const int threads = llmlab_recurrent_row_threads(D, E);
+  LLMLAB_REQUIRE(threads > 0 && n_reqs >= 0 && n_heads > 0 && n_heads <= 65535, "recurrent_row: sizes D=%d E=%d heads=%d are not taken",
+                 D, E, n_heads);
+  LLMLAB_REQUIRE(proj && state && q_start && req_rows && w && out && norm_count >= 0 && norm_count <= E &&
+                     (gate_kind == 0 || gate_kind == 1), "recurrent_row: an operand is missing");
+  LLMLAB_REQUIRE(ld >= off_q + n_heads * D && ld >= off_k + n_heads * D && ld >= off_v + n_heads * E &&
+                     ld >= off_g + n_heads * E && off_q >= 0 && off_k >= 0 && off_v >= 0 && off_g >= 0,
+                 "recurrent_row: rows of %d numbers do not hold the projections", ld);
+  LLMLAB_REQUIRE(kind >= KIND_DECAY && kind <= KIND_MEMORY, "recurrent_row: unknown kind %d", kind);
+  if (kind == KIND_MEMORY) {
+    LLMLAB_REQUIRE(norm_state && max_state && cap > 0.f && off_i >= 0 && off_f >= 0 && ld >= off_i + n_heads &&
+                       ld >= off_f + n_heads, "recurrent_row: the memory's operands");
+    rank = 0;
+  } else {
+    LLMLAB_REQUIRE(w2 && rank > 0 && rank <= ROW_MAX_RANK && off_low >= 0 && ld >= off_low + rank && tau > 0.f &&
+                       (kind != KIND_BONUS || bonus), "recurrent_row: the decays' operands, a rank of up to %d", ROW_MAX_RANK);
+  }
+  if (n_reqs == 0) return 0;
+  int groups = threads / (E / 4);
+  if (groups > D) groups = D;
+  const int rows = (D + groups - 1) / groups;
+  const RowArgs a{proj, ld, off_q, off_k, off_v, off_g, q_scale, n_heads, D, E, groups, state, q_start, req_rows, w, eps,
+                  w_per_head, gate_kind, norm_count > 0 ? norm_count : E, off_low, rank, w2, bias, decay_kind, 1.0f / tau,
+                  bonus, off_i, off_f, bias_i, bias_f, cap, norm_state, max_state};
+  const size_t lds = (size_t)(rank + 4 * D + groups * E) * sizeof(float);
+  const dim3 grid(n_reqs, n_heads), block(threads);
+#define LLMLAB_ROW(KIND, T, ROWS) \
+  hipLaunchKernelGGL((recurrent_row_kernel<KIND, T, ROWS>), grid, block, lds, stream, a, (T*)out)
+#define LLMLAB_ROW_ANY(KIND)                                    \
+  do {                                                          \
+    if (dtype == DT_BF16 && rows <= 4) LLMLAB_ROW(KIND, bf16_t, 4); \
+    else if (dtype == DT_BF16) LLMLAB_ROW(KIND, bf16_t, ROW_MAX_ROWS); \
+    else if (rows <= 4) LLMLAB_ROW(KIND, float, 4);             \
+    else LLMLAB_ROW(KIND, float, ROW_MAX_ROWS);                 \
+  } while (0)
+  if (kind == KIND_DECAY) LLMLAB_ROW_ANY(KIND_DECAY);
+  else if (kind == KIND_BONUS) LLMLAB_ROW_ANY(KIND_BONUS);
+  else LLMLAB_ROW_ANY(KIND_MEMORY);
+#undef LLMLAB_ROW_ANY
+#undef LLMLAB_ROW
+  LLMLAB_LAUNCH_CHECK("recurrent_row");
+  return 0;
+}
+
+
 // ================================================================== generalised delta rule
 // A matrix-valued state per head whose transition is a decay per key channel less a rank-one
 // removal along the unit key, before the new key/value pair is written:

@@ -415,15 +415,20 @@ extern "C" int llmlab_gated_add(float* x, const float* y, int pieces, size_t pie
 constexpr int NORM_ADD_KEEP = 8;
 // NEXT 1: the norm that reads the stream next runs in the same launch on the row's new numbers:
 // next_out[r, c] = T(x[r, c] / sqrt(mean(x[r]^2) + next_eps) * next_w[c]).  NEXT 2: a copy of them,
-// next_out[r, c] = T(x[r, c]).
+// next_out[r, c] = T(x[r, c]).  NEXT 3 (every request of the step brings one row): the row mixed with the
+// one before it in its sequence, next_out[r, c] = T(x[r, c] + (p - x[r, c]) * next_w[c]) with p = shift_state[
+// slot, c], which then takes x[r, c] (what shift_mix does in a launch of its own).
 template <typename T, int NEXT>
 __global__ __launch_bounds__(256) void rmsnorm_add_kernel(float* __restrict__ x, const float* __restrict__ y, int pieces,
                                                           size_t piece_stride, const float* __restrict__ w, float eps,
                                                           int width, const float* __restrict__ next_w, float next_eps,
-                                                          T* __restrict__ next_out) {
+                                                          T* __restrict__ next_out, float* __restrict__ shift_state,
+                                                          const int* __restrict__ req_rows) {
   __shared__ float red[17];
   const size_t row = (size_t)blockIdx.x * width;
+  float* before = NEXT == 3 ? shift_state + (size_t)req_rows[blockIdx.x] * width : nullptr;
   float keep[NORM_ADD_KEEP], xs[NORM_ADD_KEEP], ws[NORM_ADD_KEEP];
+  float ps[NEXT == 3 ? NORM_ADD_KEEP : 1], ms[NEXT == 3 ? NORM_ADD_KEEP : 1];
   float ss = 0.f;
   auto value = [&](int c) {
     float v = y[row + c];
@@ -438,6 +443,10 @@ __global__ __launch_bounds__(256) void rmsnorm_add_kernel(float* __restrict__ x,
     keep[n] = c < width ? value(c) : 0.f;
     xs[n] = c < width ? x[row + c] : 0.f;
     ws[n] = c < width ? w[c] : 0.f;
+    if (NEXT == 3) {
+      ps[n] = c < width ? before[c] : 0.f;
+      ms[n] = c < width ? next_w[c] : 0.f;
+    }
     ss = fmaf(keep[n], keep[n], ss);
   }
   for (int c = threadIdx.x + 256 * NORM_ADD_KEEP; c < width; c += 256) {
@@ -453,6 +462,10 @@ __global__ __launch_bounds__(256) void rmsnorm_add_kernel(float* __restrict__ x,
       keep[n] = xs[n] + keep[n] * inv * ws[n];
       x[row + c] = keep[n];
       if (NEXT == 2) next_out[row + c] = from_float<T>(keep[n]);
+      if (NEXT == 3) {
+        next_out[row + c] = from_float<T>(fmaf(ps[n] - keep[n], ms[n], keep[n]));
+        before[c] = keep[n];
+      }
       ss2 = fmaf(keep[n], keep[n], ss2);
     }
   }
@@ -460,6 +473,10 @@ __global__ __launch_bounds__(256) void rmsnorm_add_kernel(float* __restrict__ x,
     const float v = x[row + c] + value(c) * inv * w[c];
     x[row + c] = v;
     if (NEXT == 2) next_out[row + c] = from_float<T>(v);
+    if (NEXT == 3) {
+      next_out[row + c] = from_float<T>(fmaf(before[c] - v, next_w[c], v));
+      before[c] = v;
+    }
     ss2 = fmaf(v, v, ss2);
   }
   if (NEXT != 1) return;
@@ -475,15 +492,18 @@ __global__ __launch_bounds__(256) void rmsnorm_add_kernel(float* __restrict__ x,
 
 extern "C" int llmlab_rmsnorm_add(float* x, const float* y, int pieces, size_t piece_stride, const float* w, float eps,
                                   int rows, int width, const float* next_w, float next_eps, void* next_out,
-                                  int next_dtype, hipStream_t stream) {
+                                  int next_dtype, float* shift_state, const int* req_rows, hipStream_t stream) {
+  LLMLAB_REQUIRE(shift_state == nullptr || (next_w && next_out && req_rows), "rmsnorm_add: a shift needs its mix, slots and output");
   LLMLAB_REQUIRE(rows >= 0 && width > 0 && pieces >= 1 && x && y && w, "rmsnorm_add: bad arguments rows=%d width=%d pieces=%d",
                  rows, width, pieces);
   LLMLAB_REQUIRE(next_w == nullptr || next_out, "rmsnorm_add: the next norm needs an output");
   if (rows == 0) return 0;
 #define LLMLAB_NORM_ADD(T, NEXT)                                                                                           \
   hipLaunchKernelGGL((rmsnorm_add_kernel<T, NEXT>), dim3(rows), dim3(256), 0, stream, x, y, pieces, piece_stride, w, eps, \
-                     width, next_w, next_eps, (T*)next_out)
+                     width, next_w, next_eps, (T*)next_out, shift_state, req_rows)
   if (!next_out) LLMLAB_NORM_ADD(float, 0);
+  else if (shift_state && next_dtype == DT_BF16) LLMLAB_NORM_ADD(bf16_t, 3);
+  else if (shift_state) LLMLAB_NORM_ADD(float, 3);
   else if (next_w && next_dtype == DT_BF16) LLMLAB_NORM_ADD(bf16_t, 1);
   else if (next_w) LLMLAB_NORM_ADD(float, 1);
   else if (next_dtype == DT_BF16) LLMLAB_NORM_ADD(bf16_t, 2);
@@ -510,12 +530,17 @@ extern "C" int llmlab_scaled_sum(float* out, const float* y1, float a, const flo
   return 0;
 }
 
-// out[r] = a * norm(y1[r]) * w1 + b * norm(y2[r]) * w2, each row over its own root mean square (eps
-// inside the root).  One block a row, all float32.
+// s[r] = a * norm(y1[r]) * w1 + b * norm(y2[r]) * w2, each row over its own root mean square (eps
+// inside the root).  ADD false: out = s.  ADD true: the norm of s on its way into the stream, out[r] += s /
+// sqrt(mean(s^2) + add_eps) * add_w, and (copy not null) copy[r] = T(the new row).  One block a row, all
+// float32; a thread keeps up to NORM_ADD_KEEP of the row's numbers, wider rows are read again.
+template <typename T, bool ADD>
 __global__ __launch_bounds__(256) void normed_sum_kernel(float* __restrict__ out, const float* __restrict__ y1,
                                                          const float* __restrict__ w1, float a, const float* __restrict__ y2,
-                                                         const float* __restrict__ w2, float b, float eps, int width) {
-  __shared__ float red1[17], red2[17];
+                                                         const float* __restrict__ w2, float b, float eps, int width,
+                                                         const float* __restrict__ add_w, float add_eps,
+                                                         T* __restrict__ copy) {
+  __shared__ float red1[17], red2[17], red3[17];
   const size_t row = (size_t)blockIdx.x * width;
   float k1[NORM_ADD_KEEP], k2[NORM_ADD_KEEP];
   float s1 = 0.f, s2 = 0.f;
@@ -534,21 +559,51 @@ __global__ __launch_bounds__(256) void normed_sum_kernel(float* __restrict__ out
   }
   const float i1 = a / sqrtf(block_sum(s1, red1) / (float)width + eps);
   const float i2 = b / sqrtf(block_sum(s2, red2) / (float)width + eps);
+  float ss = 0.f;
 #pragma unroll
   for (int n = 0; n < NORM_ADD_KEEP; ++n) {
     const int c = threadIdx.x + 256 * n;
-    if (c < width) out[row + c] = k1[n] * i1 * w1[c] + k2[n] * i2 * w2[c];
+    if (c < width) {
+      k1[n] = k1[n] * i1 * w1[c] + k2[n] * i2 * w2[c];
+      if (!ADD) out[row + c] = k1[n];
+      ss = fmaf(k1[n], k1[n], ss);
+    }
+  }
+  for (int c = threadIdx.x + 256 * NORM_ADD_KEEP; c < width; c += 256) {
+    const float v = y1[row + c] * i1 * w1[c] + y2[row + c] * i2 * w2[c];
+    if (!ADD) out[row + c] = v;
+    ss = fmaf(v, v, ss);
+  }
+  if (!ADD) return;
+  const float inv = 1.0f / sqrtf(block_sum(ss, red3) / (float)width + add_eps);
+  auto add = [&](int c, float v) {
+    v = out[row + c] + v * inv * add_w[c];
+    out[row + c] = v;
+    if (copy) copy[row + c] = from_float<T>(v);
+  };
+#pragma unroll
+  for (int n = 0; n < NORM_ADD_KEEP; ++n) {
+    const int c = threadIdx.x + 256 * n;
+    if (c < width) add(c, k1[n]);
   }
   for (int c = threadIdx.x + 256 * NORM_ADD_KEEP; c < width; c += 256)
-    out[row + c] = y1[row + c] * i1 * w1[c] + y2[row + c] * i2 * w2[c];
+    add(c, y1[row + c] * i1 * w1[c] + y2[row + c] * i2 * w2[c]);
 }
 
 extern "C" int llmlab_normed_sum(float* out, const float* y1, const float* w1, float a, const float* y2, const float* w2,
-                                 float b, float eps, int rows, int width, hipStream_t stream) {
+                                 float b, float eps, int rows, int width, const float* add_w, float add_eps, void* copy,
+                                 int copy_dtype, hipStream_t stream) {
   LLMLAB_REQUIRE(rows >= 0 && width > 0 && out && y1 && y2 && w1 && w2, "normed_sum: bad arguments rows=%d width=%d", rows,
                  width);
+  LLMLAB_REQUIRE(copy == nullptr || add_w, "normed_sum: a copy is the stream's, so the sum goes into the stream");
   if (rows == 0) return 0;
-  hipLaunchKernelGGL(normed_sum_kernel, dim3(rows), dim3(256), 0, stream, out, y1, w1, a, y2, w2, b, eps, width);
+#define LLMLAB_NORMED_SUM(T, ADD)                                                                                          \
+  hipLaunchKernelGGL((normed_sum_kernel<T, ADD>), dim3(rows), dim3(256), 0, stream, out, y1, w1, a, y2, w2, b, eps, width, \
+                     add_w, add_eps, (T*)copy)
+  if (!add_w) LLMLAB_NORMED_SUM(float, false);
+  else if (copy && copy_dtype == DT_BF16) LLMLAB_NORMED_SUM(bf16_t, true);
+  else LLMLAB_NORMED_SUM(float, true);
+#undef LLMLAB_NORMED_SUM
   LLMLAB_LAUNCH_CHECK("normed_sum");
   return 0;
 }

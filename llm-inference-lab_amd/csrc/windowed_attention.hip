@@ -196,24 +196,28 @@ extern "C" int llmlab_project_rotate_write(const float* proj, int ld, int rows, 
 // a sequence's start).  Of every query and key head the first rot_dims channels turn by positions[r] *
 // freq[i]: channel i with i + rot_dims / 2, or (neighbours) channel 2i with 2i + 1.  unit: the head is
 // then divided by its root mean square over D.  Queries and keys are laid out DK >= D channels wide
-// (zeros behind), values E.  A wave a head; the head's numbers lie in LDS between the steps.
-// own_state: every request brings one row, and the row's block moves its slot on after it has read
-// it (a thread owns its channels); else conv_slots_kernel does.
+// (zeros behind), values E.  own_state: every request brings one row, and the row's block moves its
+// slot on after it has read it (a thread owns its channels); else conv_slots_kernel does.
+//
+// A block a row, `group` heads (queries, keys, values in this order) at a time: a thread a channel
+// first, PER channels a thread whose loads (projections of the row and of the rows before it, taps,
+// slot) are asked for together, results to LDS; then a wave a head.
 struct ConvArgs {
   const float* proj; int ld, n_heads, n_kv, D, DK, E; const float* bias; const float* w; int taps;
   float* state; const int* q_start; const int* req_rows; const float* freq; int rot_dims, neighbours, unit; float eps;
-  int page_size; const int* positions; const int* row_req; const int* table; int max_pages, own_state;
+  int page_size; const int* positions; const int* row_req; const int* table; int max_pages, own_state, group;
 };
 
-template <typename T>
-__global__ __launch_bounds__(256) void project_conv_write_kernel(ConvArgs a, T* __restrict__ q_out,
-                                                                 T* __restrict__ k_cache, T* __restrict__ v_cache) {
-  extern __shared__ float conv_lds[];           // cos [half], sin [half], then D numbers a wave
+constexpr int CONV_LDS_FLOATS = 12288;      // channels of a group of heads in LDS
+template <typename T, int TAPS, int PER>    // TAPS 0: any number, from the arguments
+__global__ __launch_bounds__(1024) void project_conv_write_kernel(ConvArgs a, T* __restrict__ q_out,
+                                                                  T* __restrict__ k_cache, T* __restrict__ v_cache) {
+  extern __shared__ float conv_lds[];           // cos [half], sin [half], then the group's channels
   const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
-  const int half = a.rot_dims >> 1, D = a.D, E = a.E, keep = a.taps - 1;
+  const int half = a.rot_dims >> 1, D = a.D, E = a.E, taps = TAPS > 0 ? TAPS : a.taps, keep = taps - 1;
   float* s_cos = conv_lds;
   float* s_sin = conv_lds + half;
-  float* s_head = conv_lds + 2 * half + wave * (D > E ? D : E);
+  float* s_row = conv_lds + 2 * half;
   const float* src = a.proj + (size_t)r * a.ld;
   const int pos = a.positions[r], b = a.row_req[r];
   const int inside = r - a.q_start[b];          // rows of this request before r in the step
@@ -225,65 +229,105 @@ __global__ __launch_bounds__(256) void project_conv_write_kernel(ConvArgs a, T* 
     s_cos[i] = cs;
     s_sin[i] = sn;
   }
-  __syncthreads();
   const int page = a.table[(size_t)b * a.max_pages + pos / a.page_size];
   const int slot = pos % a.page_size;
-  // channel c of the row after bias and convolution
-  auto channel = [&](int c) {
-    const float bias = a.bias ? a.bias[c] : 0.f;
-    const float own = src[c] + bias;
-    if (a.taps <= 0) return own;
-    const float* w = a.w + (size_t)c * a.taps;
-    float acc = 0.f;
-    for (int j = 0; j < keep; ++j) {
-      const int back = keep - j;
-      const float u = back <= inside ? src[c - (ptrdiff_t)back * a.ld] + bias
-                                     : st[(size_t)(keep - (back - inside)) * channels + c];
-      acc = fmaf(w[j], u, acc);
-    }
-    acc = fmaf(w[keep], own, acc);
-    if (a.own_state && keep > 0) {
-      for (int j = 0; j + 1 < keep; ++j) st[(size_t)j * channels + c] = st[(size_t)(j + 1) * channels + c];
-      st[(size_t)(keep - 1) * channels + c] = own;
-    }
-    return acc;
-  };
   const int heads = a.n_heads + 2 * a.n_kv;     // query heads, key heads, value heads
-  for (int h0 = 0; h0 < heads; h0 += waves) {   // (every wave takes part in the barriers)
-    const int h = h0 + wave;
-    const bool turns = h < a.n_heads + a.n_kv, live = h < heads;
-    const int width = turns ? D : E;
-    const int c0 = turns ? h * D : q_size + k_size + (h - a.n_heads - a.n_kv) * E;
-    if (live)
-      for (int d = lane; d < width; d += 64) s_head[d] = channel(c0 + d);
-    __syncthreads();
-    if (live && turns) {
-      float ss = 0.f;
-      auto turned = [&](int d) {
-        float x = s_head[d];
-        if (d < a.rot_dims) {
-          const int i = a.neighbours ? d >> 1 : (d < half ? d : d - half);
-          const bool first = a.neighbours ? (d & 1) == 0 : d < half;
-          const float other = s_head[a.neighbours ? d ^ 1 : (first ? d + half : d - half)];
-          x = first ? x * s_cos[i] - other * s_sin[i] : x * s_cos[i] + other * s_sin[i];
+  auto first_channel = [&](int h) {             // of head h (h == heads: the number of channels)
+    return h <= a.n_heads + a.n_kv ? h * D : q_size + k_size + (h - a.n_heads - a.n_kv) * E;
+  };
+  for (int h0 = 0; h0 < heads; h0 += a.group) {
+    const int h1 = h0 + a.group < heads ? h0 + a.group : heads;
+    const int c_lo = first_channel(h0), c_hi = first_channel(h1);
+    if (TAPS > 0) {
+      constexpr int K = TAPS > 1 ? TAPS - 1 : 1;
+      for (int c0 = c_lo + (int)threadIdx.x; c0 < c_hi; c0 += blockDim.x * PER) {
+        float own[PER], bias[PER], w[PER][TAPS], u[PER][K];
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {         // (past the end: the last channel again, dropped below)
+          const int c = min(c0 + i * (int)blockDim.x, c_hi - 1);
+          own[i] = src[c];
+          bias[i] = a.bias ? a.bias[c] : 0.f;
+#pragma unroll
+          for (int j = 0; j < TAPS; ++j) w[i][j] = a.w[(size_t)c * TAPS + j];
+#pragma unroll
+          for (int j = 0; j < TAPS - 1; ++j) {
+            const int back = TAPS - 1 - j;
+            const float* at = back <= inside ? src + c - (ptrdiff_t)back * a.ld
+                                             : st + (size_t)(TAPS - 1 - (back - inside)) * channels + c;
+            u[i][j] = *at;
+          }
         }
-        return x;
-      };
-      float inv = 1.f;
-      if (a.unit) {
-        for (int d = lane; d < D; d += 64) {
-          const float x = turned(d);
-          ss = fmaf(x, x, ss);
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+          const int c = c0 + i * (int)blockDim.x;
+          if (c >= c_hi) break;
+          own[i] += bias[i];
+          float acc = 0.f;
+#pragma unroll
+          for (int j = 0; j < TAPS - 1; ++j) {
+            if (TAPS - 1 - j <= inside) u[i][j] += bias[i];
+            acc = fmaf(w[i][j], u[i][j], acc);
+          }
+          s_row[c - c_lo] = fmaf(w[i][TAPS - 1], own[i], acc);
+          if (a.own_state && TAPS > 1) {
+#pragma unroll
+            for (int j = 0; j + 1 < TAPS - 1; ++j) st[(size_t)j * channels + c] = u[i][j + 1];
+            st[(size_t)(TAPS - 2) * channels + c] = own[i];
+          }
         }
-        inv = 1.0f / sqrtf(wave_sum(ss) / (float)D + a.eps);
       }
-      T* dst = h < a.n_heads ? q_out + ((size_t)r * a.n_heads + h) * a.DK
-                             : k_cache + (((size_t)page * a.n_kv + (h - a.n_heads)) * a.page_size + slot) * a.DK;
-      for (int d = lane; d < a.DK; d += 64) dst[d] = from_float<T>(d < D ? turned(d) * inv : 0.f);
-    } else if (live) {
-      const int g = h - a.n_heads - a.n_kv;
-      for (int e = lane; e < E; e += 64)
-        v_cache[((size_t)page * a.n_kv + g) * a.page_size * E + value_index(slot, e, E)] = from_float<T>(s_head[e]);
+    } else {
+      for (int c = c_lo + (int)threadIdx.x; c < c_hi; c += blockDim.x) {
+        const float bias = a.bias ? a.bias[c] : 0.f, own = src[c] + bias;
+        float acc = own;
+        if (taps > 0) {
+          const float* w = a.w + (size_t)c * taps;
+          acc = w[keep] * own;
+          for (int j = 0; j < keep; ++j) {
+            const int back = keep - j;
+            const float u = back <= inside ? src[c - (ptrdiff_t)back * a.ld] + bias
+                                           : st[(size_t)(keep - (back - inside)) * channels + c];
+            acc = fmaf(w[j], u, acc);
+          }
+          if (a.own_state && keep > 0) {
+            for (int j = 0; j + 1 < keep; ++j) st[(size_t)j * channels + c] = st[(size_t)(j + 1) * channels + c];
+            st[(size_t)(keep - 1) * channels + c] = own;
+          }
+        }
+        s_row[c - c_lo] = acc;
+      }
+    }
+    __syncthreads();
+    for (int h = h0 + wave; h < h1; h += waves) {
+      const float* s_head = s_row + (first_channel(h) - c_lo);
+      if (h < a.n_heads + a.n_kv) {
+        auto turned = [&](int d) {
+          float x = s_head[d];
+          if (d < a.rot_dims) {
+            const int i = a.neighbours ? d >> 1 : (d < half ? d : d - half);
+            const bool first = a.neighbours ? (d & 1) == 0 : d < half;
+            const float other = s_head[a.neighbours ? d ^ 1 : (first ? d + half : d - half)];
+            x = first ? x * s_cos[i] - other * s_sin[i] : x * s_cos[i] + other * s_sin[i];
+          }
+          return x;
+        };
+        float inv = 1.f;
+        if (a.unit) {
+          float ss = 0.f;
+          for (int d = lane; d < D; d += 64) {
+            const float x = turned(d);
+            ss = fmaf(x, x, ss);
+          }
+          inv = 1.0f / sqrtf(wave_sum(ss) / (float)D + a.eps);
+        }
+        T* dst = h < a.n_heads ? q_out + ((size_t)r * a.n_heads + h) * a.DK
+                               : k_cache + (((size_t)page * a.n_kv + (h - a.n_heads)) * a.page_size + slot) * a.DK;
+        for (int d = lane; d < a.DK; d += 64) dst[d] = from_float<T>(d < D ? turned(d) * inv : 0.f);
+      } else {
+        const int g = h - a.n_heads - a.n_kv;
+        for (int e = lane; e < E; e += 64)
+          v_cache[((size_t)page * a.n_kv + g) * a.page_size * E + value_index(slot, e, E)] = from_float<T>(s_head[e]);
+      }
     }
     __syncthreads();
   }
@@ -315,7 +359,7 @@ extern "C" int llmlab_project_conv_write(const float* proj, int ld, int rows, in
                                          const int* positions, const int* row_req, const int* table, int max_pages,
                                          int one_row_each, hipStream_t stream) {
   LLMLAB_REQUIRE(rows >= 0 && n_heads > 0 && n_kv > 0 && D > 0 && DK >= D && E > 0 && page_size > 0 && page_size % 4 == 0 &&
-                     D <= 2048 && E <= 2048,
+                     D <= 2048 && E <= 2048 && rot_dims <= 2048,
                  "project_conv_write: bad sizes rows=%d heads=%d kv=%d D=%d/%d E=%d page=%d", rows, n_heads, n_kv, D, DK, E,
                  page_size);
   LLMLAB_REQUIRE(ld >= (n_heads + n_kv) * D + n_kv * E, "project_conv_write: rows of %d numbers do not hold the projections",
@@ -327,43 +371,37 @@ extern "C" int llmlab_project_conv_write(const float* proj, int ld, int rows, in
   LLMLAB_REQUIRE(q_out && k_cache && v_cache && positions && row_req && table && q_start,
                  "project_conv_write: queries, pages and the step's description are needed");
   if (rows == 0) return 0;
+  const int widest = D > E ? D : E, heads = n_heads + 2 * n_kv;
+  int group = CONV_LDS_FLOATS / widest;
+  if (group > heads) group = heads;
   ConvArgs a{proj, ld, n_heads, n_kv, D, DK, E, bias, w, taps, state, q_start, req_rows, freq, rot_dims, neighbours, unit, eps,
-             page_size, positions, row_req, table, max_pages, one_row_each};
-  const size_t lds = (size_t)(rot_dims + 4 * (D > E ? D : E)) * sizeof(float);
-  if (dtype == DT_BF16)
-    hipLaunchKernelGGL(project_conv_write_kernel<bf16_t>, dim3(rows), dim3(256), lds, stream, a, (bf16_t*)q_out,
-                       (bf16_t*)k_cache, (bf16_t*)v_cache);
-  else
-    hipLaunchKernelGGL(project_conv_write_kernel<float>, dim3(rows), dim3(256), lds, stream, a, (float*)q_out,
-                       (float*)k_cache, (float*)v_cache);
+             page_size, positions, row_req, table, max_pages, one_row_each, group};
+  const size_t lds = (size_t)(rot_dims + group * widest) * sizeof(float);
+  // few rows (a step bound by latency): a thread a channel where a block holds them; many rows:
+  // blocks of which a compute unit holds several
+  const int channels = (n_heads + n_kv) * D + n_kv * E;
+  const bool few = rows <= 64;
+  const int threads = few ? (channels >= 1024 ? 1024 : (channels + 63) / 64 * 64) : 256;
+#define LLMLAB_CONV_WRITE(T, TAPS)                                                                                     \
+  do {                                                                                                                 \
+    if (few) hipLaunchKernelGGL((project_conv_write_kernel<T, TAPS, 2>), dim3(rows), dim3(threads), lds, stream, a,    \
+                                (T*)q_out, (T*)k_cache, (T*)v_cache);                                                  \
+    else hipLaunchKernelGGL((project_conv_write_kernel<T, TAPS, 5>), dim3(rows), dim3(threads), lds, stream, a,        \
+                            (T*)q_out, (T*)k_cache, (T*)v_cache);                                                      \
+  } while (0)
+#define LLMLAB_CONV_WRITE_TAPS(T)                     \
+  switch (taps) {                                     \
+    case 2: LLMLAB_CONV_WRITE(T, 2); break;           \
+    case 3: LLMLAB_CONV_WRITE(T, 3); break;           \
+    case 4: LLMLAB_CONV_WRITE(T, 4); break;           \
+    default: LLMLAB_CONV_WRITE(T, 0); break;          \
+  }
+  if (dtype == DT_BF16) LLMLAB_CONV_WRITE_TAPS(bf16_t)
+  else LLMLAB_CONV_WRITE_TAPS(float)
+#undef LLMLAB_CONV_WRITE_TAPS
+#undef LLMLAB_CONV_WRITE
   if (taps > 1 && !one_row_each) hipLaunchKernelGGL(conv_slots_kernel, dim3(rows), dim3(256), 0, stream, a);
   LLMLAB_LAUNCH_CHECK("project_conv_write");
-  return 0;
-}
-
-// out[r, c] = T(out[r, c] * sigmoid(gate[r, c])): a gate per channel of the heads' outputs, read
-// from the float32 projections (row stride ld).
-template <typename T>
-__global__ void gate_channels_kernel(T* __restrict__ out, const float* __restrict__ gate, int ld, int width, size_t n) {
-  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
-    const size_t r = i / width;
-    const float g = gate[r * ld + (i - r * width)];
-    out[i] = from_float<T>(to_float(out[i]) / (1.f + __expf(-g)));
-  }
-}
-
-extern "C" int llmlab_gate_channels(void* out, const float* gate, int ld, int rows, int width, int dtype,
-                                    hipStream_t stream) {
-  LLMLAB_REQUIRE(rows >= 0 && width > 0 && ld >= width && out && gate, "gate_channels: bad arguments rows=%d width=%d ld=%d",
-                 rows, width, ld);
-  const size_t n = (size_t)rows * width;
-  if (n == 0) return 0;
-  const int blocks = (int)((n + 255) / 256 < 65535 ? (n + 255) / 256 : 65535);
-  if (dtype == DT_BF16)
-    hipLaunchKernelGGL(gate_channels_kernel<bf16_t>, dim3(blocks), dim3(256), 0, stream, (bf16_t*)out, gate, ld, width, n);
-  else
-    hipLaunchKernelGGL(gate_channels_kernel<float>, dim3(blocks), dim3(256), 0, stream, (float*)out, gate, ld, width, n);
-  LLMLAB_LAUNCH_CHECK("gate_channels");
   return 0;
 }
 
@@ -394,6 +432,14 @@ struct Mask {
   __device__ __forceinline__ int low(int i) const {
     if (window > 0) return i - window + 1 > 0 ? i - window + 1 : 0;
     return chunk > 0 ? i - i % chunk : 0;
+  }
+};
+// A gate per channel of the heads' outputs, applied where an output is made final: column c of row r is
+// multiplied by sigmoid(p[r * ld + c]) (float32; p null: no gate).
+struct Gate {
+  const float* p; int ld;
+  __device__ __forceinline__ float at(int r, int c) const {
+    return p ? 1.0f / (1.0f + __expf(-p[(size_t)r * ld + c])) : 1.f;
   }
 };
 // (lo: the mask's low(i), taken once per query)
@@ -454,7 +500,7 @@ __global__ __launch_bounds__(64) void sink_window_attention_kernel(
     const T* __restrict__ v_cache, const int* __restrict__ table, int max_pages, int page_size,
     const int* __restrict__ positions, const int* __restrict__ row_req, Mask mask,
     const float* __restrict__ sink, float scale, T* __restrict__ out, const int* __restrict__ q_start, int long_from,
-    int mode) {
+    int mode, Gate gate) {
   if (long_from > 0) {      // (rows of requests that bring many rows are the other kernel's)
     const int b = row_req[blockIdx.x];
     if (q_start[b + 1] - q_start[b] >= long_from) return;
@@ -529,7 +575,7 @@ __global__ __launch_bounds__(64) void sink_window_attention_kernel(
 #pragma unroll
   for (int c = 0; c < MAX_E_PER_LANE; ++c) {
     const int e = lane + 64 * c;
-    if (e < E) out[((size_t)r * n_heads + h) * E + e] = from_float<T>(acc[c] * inv);
+    if (e < E) out[((size_t)r * n_heads + h) * E + e] = from_float<T>(acc[c] * inv * gate.at(r, h * E + e));
   }
 }
 
@@ -705,6 +751,7 @@ struct MfmaArgs {
   const int* positions; const int* row_req; Mask mask; const float* sink; float scale;
   bf16_t* out; const int* q_start; int long_from;
   int splits; float* part_o; float* part_ml;      // (decoding) [rows, heads, splits, E] and [rows, heads, splits, 2]
+  Gate gate;
   int mode;                                       // MODE_SOFTMAX, or MODE_SIGMOID (sink: the bias of the scores)
 };
 
@@ -759,7 +806,7 @@ __global__ __launch_bounds__(256) void sink_window_attention_mfma_kernel(MfmaArg
   for (int eb = 0; eb < EB; ++eb) {
     bf16x4 w;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) w[i] = (bf16_t)(run.o[eb][i] * inv);
+    for (int i = 0; i < 4; ++i) w[i] = (bf16_t)(run.o[eb][i] * inv * a.gate.at(r, h * E + 16 * eb + 4 * g4 + i));
     *(bf16x4*)(a.out + ((size_t)r * a.n_heads + h) * E + 16 * eb + 4 * g4) = w;
   }
 }
@@ -984,7 +1031,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
   for (int eb = 0; eb < EB; ++eb) {
     bf16x4 w;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) w[i] = (bf16_t)(run.o[eb][i] * inv);
+    for (int i = 0; i < 4; ++i) w[i] = (bf16_t)(run.o[eb][i] * inv * a.gate.at(r, h * E + 16 * eb + 4 * g4 + i));
     *(bf16x4*)(a.out + ((size_t)r * a.n_heads + h) * E + 16 * eb + 4 * g4) = w;
   }
 }
@@ -1035,7 +1082,7 @@ __global__ __launch_bounds__(64) void sink_window_attention_grouped_kernel(MfmaA
     for (int eb = 0; eb < EB; ++eb) {
       bf16x4 w;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) w[i] = (bf16_t)(run.o[eb][i] * inv);
+      for (int i = 0; i < 4; ++i) w[i] = (bf16_t)(run.o[eb][i] * inv * a.gate.at(r, h * E + 16 * eb + 4 * g4 + i));
       *(bf16x4*)(a.out + ((size_t)r * a.n_heads + h) * E + 16 * eb + 4 * g4) = w;
     }
     return;
@@ -1097,7 +1144,7 @@ __global__ __launch_bounds__(64) void sink_window_attention_merge_kernel(MfmaArg
       const float o = a.part_o[(first + z) * E + e];
       acc = fmaf(s_w[z], s_w[z] != 0.f ? o : 0.f, acc);
     }
-    a.out[((size_t)r * a.n_heads + h) * E + e] = (bf16_t)(acc * inv);
+    a.out[((size_t)r * a.n_heads + h) * E + e] = (bf16_t)(acc * inv * a.gate.at(r, h * E + e));
   }
 }
 
@@ -1160,7 +1207,10 @@ extern "C" int llmlab_sink_window_attention(const void* q, int dtype, int rows, 
                                             int keep_first, int chunk, const float* sink, float scale, void* out,
                                             const int* q_start, int long_from, int launches, int max_keys,
                                             float* workspace, size_t workspace_floats, int num_cus, int mode,
-                                            hipStream_t stream) {
+                                            const float* gate, int gate_ld, hipStream_t stream) {
+  LLMLAB_REQUIRE(gate == nullptr || gate_ld >= n_heads * E, "sink_window_attention: a gate per channel, rows of %d numbers",
+                 gate_ld);
+  const Gate gates{gate, gate_ld};
   LLMLAB_REQUIRE(mode == MODE_SOFTMAX || mode == MODE_SIGMOID, "sink_window_attention: unknown weighting %d", mode);
   LLMLAB_REQUIRE(rows >= 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0 && D > 0 && E > 0,
                  "sink_window_attention: bad sizes rows=%d heads=%d kv=%d D=%d E=%d", rows, n_heads, n_kv, D, E);
@@ -1179,7 +1229,7 @@ extern "C" int llmlab_sink_window_attention(const void* q, int dtype, int rows, 
   if (long_from > 0) {
     MfmaArgs a{(const bf16_t*)q, rows, n_heads, n_kv, (const bf16_t*)k_cache, (const bf16_t*)v_cache, table, max_pages,
                page_size, positions, row_req, mask, sink, scale, (bf16_t*)out, q_start, long_from, 1,
-               nullptr, nullptr, mode};
+               nullptr, nullptr, gates, mode};
     if (launches & 2) {
       // heads that read the same keys and values share the tiles a block stages in LDS
       const int group = n_heads / n_kv;
@@ -1220,11 +1270,11 @@ extern "C" int llmlab_sink_window_attention(const void* q, int dtype, int rows, 
   if (dtype == DT_BF16)
     hipLaunchKernelGGL(sink_window_attention_kernel<bf16_t>, grid, block, lds, stream, (const bf16_t*)q, n_heads, n_kv, D,
                        E, (const bf16_t*)k_cache, (const bf16_t*)v_cache, table, max_pages, page_size, positions,
-                       row_req, mask, sink, scale, (bf16_t*)out, q_start, long_from, mode);
+                       row_req, mask, sink, scale, (bf16_t*)out, q_start, long_from, mode, gates);
   else
     hipLaunchKernelGGL(sink_window_attention_kernel<float>, grid, block, lds, stream, (const float*)q, n_heads, n_kv, D,
                        E, (const float*)k_cache, (const float*)v_cache, table, max_pages, page_size, positions,
-                       row_req, mask, sink, scale, (float*)out, q_start, long_from, mode);
+                       row_req, mask, sink, scale, (float*)out, q_start, long_from, mode, gates);
   LLMLAB_LAUNCH_CHECK("sink_window_attention");
   return 0;
 }

@@ -33,6 +33,10 @@ class EntryView:
     writes_cache: bool = False
     cache: Dict[str, torch.Tensor] = dataclasses.field(default_factory=dict)   # name -> [pages, *page_shape]
     state: Dict[str, torch.Tensor] = dataclasses.field(default_factory=dict)
+    # a block whose last launch can begin the next run's work: that run's ``(block, view)``; and on
+    # the next run's side, that it may find this done
+    follower: Optional[tuple] = None
+    led: bool = False
 
     @property
     def k_cache(self) -> Optional[torch.Tensor]:
@@ -194,6 +198,12 @@ class CausalLM:
             if view.group is not None:
                 view.cache = {name: t[view.slot] for name, t in cache.storage[view.group].items()}
             view.state = cache.state.get(view.index, {})
+        for view, after in zip(self.entries, self.entries[1:]):
+            block, following = self.blocks[view.block], self.blocks[after.block]
+            # (a vector that the schedule adds to the stream in between keeps the two apart)
+            after.led = (hasattr(block, "leads") and self.spec.schedule[after.index].offset is None
+                         and block.leads(following))
+            view.follower = (following, after) if after.led else None
         if hasattr(self.embedding, "attach_state"):
             self.embedding.attach_state(cache.state.get(self.EMBEDDING_STATE, {}))
 

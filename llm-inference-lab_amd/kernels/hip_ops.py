@@ -72,6 +72,21 @@ class PackedWeight:
         return self.data.element_size()
 
 
+class SegmentedWeight:
+    """Matrices of one inner size kept as one (``HipOps.prepare_segments``): ``whole`` the packed stack of
+    all rows (bfloat16; None in float32), ``members`` each matrix by itself (runs of the stack),
+    ``offsets`` the stack's row where each begins, ``ends`` the strips where they end (host memory)."""
+
+    def __init__(self, whole, members, offsets, ends):
+        self.whole, self.members, self.offsets, self.ends = whole, members, offsets, ends
+
+    def numel(self) -> int:
+        return sum(m.shape[0] * m.shape[1] for m in self.members)
+
+    def element_size(self) -> int:
+        return self.members[0].element_size()
+
+
 class StackedWeight:
     """Several matrices of equal shape ``[n, k]`` kept as one operand (``HipOps.prepare_stacked``):
     ``data`` is the float32 tensor ``[members * n, k]`` or the packed bfloat16 matrix of ``members *
@@ -239,7 +254,7 @@ class HipOps:
             _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_float, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr,
             _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
             _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int,
-            _c_ptr, _c_int, _c_int, _c_size, _c_int, _c_size, _c_ptr]
+            _c_ptr, _c_int, _c_int, _c_size, _c_int, _c_size, _c_int, _c_ptr, _c_size, _c_ptr]
         c.llmlab_add_pending.argtypes = [_c_ptr, _c_ptr, _c_int, _c_size, _c_int, _c_int, _c_ptr]
         c.llmlab_add_pending.restype = _c_int
         c.llmlab_layernorm.argtypes = [_c_ptr, _c_ptr, _c_int, _c_float, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr]
@@ -575,7 +590,7 @@ class HipOps:
 
     def _skinny(self, x, norm, x_rows, norm_w, eps, w, bias, epilogue, out, m, n, k, ldo, n_out,
                 qkv=None, pending: Optional[PendingSums] = None, ksplit: int = 1,
-                part_stride: int = 0) -> None:
+                part_stride: int = 0, segments=None) -> None:
         if pending is not None:
             p = pending.parts
             if (p.dtype != torch.float32 or p.dim() != 3 or p.stride(2) != 1 or p.device != self.device
@@ -599,7 +614,44 @@ class HipOps:
             _dt(norm_w) if norm_w is not None else 0, float(eps), w.data_ptr(), self._ptr(bias),
             _dt(bias) if bias is not None else 0, epilogue, out.data_ptr(), m, n, k, ldo, n_out,
             *heads, self.num_cus, pend[0], pend[1], pend[2], pend[3], int(ksplit),
-            int(part_stride), self._stream())
+            int(part_stride), *(segments or (1, None, 0)), self._stream())
+
+    # --------------------------------------------- products whose columns read inputs of their own
+    def prepare_segments(self, weights) -> "SegmentedWeight":
+        """Matrices ``[n_s, k]`` of one inner size for ``segmented_products``."""
+        if not 1 <= len(weights) <= 8:
+            raise ValueError(f"1 to 8 segments, got {len(weights)}")
+        k = weights[0].shape[1]
+        if weights[0].dtype == torch.float32:
+            return SegmentedWeight(None, [self.prepare_weight(w.contiguous()) for w in weights], [], None)
+        rows, ends = [], []
+        for w in weights:                     # (every segment starts on a strip of 16 rows)
+            rows.append(torch.nn.functional.pad(w, (0, 0, 0, -w.shape[0] % 16)))
+            ends.append((ends[-1] if ends else 0) + rows[-1].shape[0] // 16)
+        whole = self.prepare_weight(torch.cat(rows).contiguous())
+        strip = whole.data.numel() // ends[-1]          # (a strip's rows lie together: a segment is a run of the whole)
+        members = [PackedWeight(whole.data[lo * strip:hi * strip], w.shape[0], k)
+                   for w, lo, hi in zip(weights, [0] + ends[:-1], ends)]
+        return SegmentedWeight(whole, members, [16 * e for e in [0] + ends[:-1]], (_c_int * len(ends))(*ends))
+
+    def segmented_products(self, x, w: "SegmentedWeight", out, offsets) -> None:
+        """``out[:, offsets[s]:] = x[s] w_s^T`` for every segment ``s``, float32 sums: ``x [segments, rows, k]``,
+        ``out [rows, columns]`` float32.  Few rows in bfloat16, with the segments' places in ``out`` as they
+        lie in the weight (``w.offsets``): one launch; else a product a segment."""
+        self._need(x, "inputs")
+        self._need(out, "sums", torch.float32)
+        segs, rows, k = x.shape
+        if segs != len(w.members) or out.shape[0] != rows:
+            raise ValueError(f"segmented_products: {segs} inputs for {len(w.members)} matrices, sums {tuple(out.shape)}")
+        if w.whole is not None and rows <= self.FEW_ROWS and list(offsets) == w.offsets and out.shape[1] == w.whole.shape[0]:
+            if x.dtype != torch.bfloat16 or w.whole.shape[1] != k:
+                raise ValueError(f"segmented_products: inputs {tuple(x.shape)} {x.dtype}, matrices {w.whole.shape}")
+            n = w.whole.shape[0]
+            self._skinny(x, False, None, None, 0.0, w.whole, None, EPI_PART, out, rows, n, k, out.stride(0), n, ksplit=1,
+                         part_stride=rows * out.stride(0), segments=(segs, w.ends, rows * k))
+            return
+        for s, (member, at) in enumerate(zip(w.members, offsets)):
+            self.linear_logits(x[s], member, out[:, at:at + member.shape[0]])
 
     # --------------------------------------------- sums left in pieces (deferred)
     MAX_SPLITS = 8
@@ -1062,15 +1114,13 @@ class HipOps:
                 lib.llmlab_sink_window_attention.argtypes = [
                     _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
                     _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_int, _c_int, _c_int,
-                    _c_ptr, _c_size, _c_int, _c_int, _c_ptr]
+                    _c_ptr, _c_size, _c_int, _c_int, _c_ptr, _c_int, _c_ptr]
                 lib.llmlab_sink_window_attention.restype = _c_int
                 lib.llmlab_project_conv_write.argtypes = [
                     _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr,
                     _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
                     _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr]
                 lib.llmlab_project_conv_write.restype = _c_int
-                lib.llmlab_gate_channels.argtypes = [_c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr]
-                lib.llmlab_gate_channels.restype = _c_int
                 lib.llmlab_project_rotate_write.argtypes = [
                     _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_float, _c_int,
                     _c_float, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
@@ -1106,12 +1156,12 @@ class HipOps:
                 lib.llmlab_softcap.argtypes = [_c_ptr, _c_float, _c_size, _c_ptr]
                 lib.llmlab_softcap.restype = _c_int
                 lib.llmlab_rmsnorm_add.argtypes = [_c_ptr, _c_ptr, _c_int, _c_size, _c_ptr, _c_float, _c_int, _c_int,
-                                                   _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr]
+                                                   _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr]
                 lib.llmlab_rmsnorm_add.restype = _c_int
                 lib.llmlab_scaled_sum.argtypes = [_c_ptr, _c_ptr, _c_float, _c_ptr, _c_float, _c_size, _c_ptr]
                 lib.llmlab_scaled_sum.restype = _c_int
                 lib.llmlab_normed_sum.argtypes = [_c_ptr, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_float,
-                                                  _c_int, _c_int, _c_ptr]
+                                                  _c_int, _c_int, _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr]
                 lib.llmlab_normed_sum.restype = _c_int
                 lib.llmlab_shift_mix.argtypes = [_c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
                                                  _c_int, _c_int, _c_int, _c_ptr]
@@ -1125,6 +1175,13 @@ class HipOps:
                                                     _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr]
                 lib.llmlab_memory_gates.restype = _c_int
                 lib.llmlab_gla_decay.restype = _c_int
+                lib.llmlab_recurrent_row_threads.argtypes = [_c_int, _c_int]
+                lib.llmlab_recurrent_row_threads.restype = _c_int
+                lib.llmlab_recurrent_row.argtypes = [
+                    _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
+                    _c_int, _c_ptr, _c_float, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int,
+                    _c_float, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr]
+                lib.llmlab_recurrent_row.restype = _c_int
                 lib.llmlab_gla_slices.argtypes = [_c_int]
                 lib.llmlab_gla_slices.restype = _c_int
                 lib.llmlab_gla_scan.argtypes = [_c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_float, _c_int, _c_int,
@@ -1423,14 +1480,16 @@ class HipOps:
     def sink_window_attention(self, q, num_heads, num_kv_heads, key_dim, value_dim, k_cache, v_cache, block_table,
                               page_size, positions, row_req, window, keep_first, sink, scale, out,
                               q_start=None, long_from=0, launches=3, max_keys=0, weights: str = "softmax",
-                              chunk=None) -> None:
+                              chunk=None, gate=None) -> None:
         """The query of row ``r`` at position ``i = positions[r]`` of request ``row_req[r]`` attends
         to the cached keys ``j <= i`` with ``i - j < window`` or ``j < keep_first`` (``window`` None:
         all); ``sink`` (float32 per head, or None) adds ``exp(sink)`` to the softmax's denominator.
         ``weights="sigmoid"``: no softmax; a visible key weighs ``sigmoid(score + sink[h])``
         (``sink``: then a bias per head on every score, None for none), not normalised over the keys.
         ``chunk`` (with ``window`` None): the keys of the query's own chunk of so many positions, ``j <=
-        i`` with ``j // chunk == i // chunk`` (or ``j < keep_first``).
+        i`` with ``j // chunk == i // chunk`` (or ``j < keep_first``).  ``gate = (proj, column)``: the output's
+        number ``c`` of row ``r`` is multiplied by ``sigmoid(proj[r, column + c])`` (float32 ``proj``) before it is
+        rounded.
         ``long_from > 0`` (``windowed_attention_long_rows``: sizes that the matrix cores take):
         requests that bring at least so many rows (by ``q_start``) are served in tiles of 16 rows
         of a head, the others a row and a group of heads at a time with the row's keys cut into
@@ -1459,6 +1518,14 @@ class HipOps:
             self._need(sink, "sink", torch.float32)
             if sink.numel() != num_heads:
                 raise ValueError("windowed attention: one sink per head")
+        gate_ptr, gate_ld = None, 0
+        if gate is not None:
+            gate_rows, column = gate
+            self._need(gate_rows, "gates", torch.float32)
+            if gate_rows.shape[0] != rows or column < 0 or column + num_heads * value_dim > gate_rows.shape[1]:
+                raise ValueError(f"windowed attention: gates at column {column} of {tuple(gate_rows.shape)} for outputs "
+                                 f"{tuple(out.shape)}")
+            gate_ptr, gate_ld = gate_rows.data_ptr() + 4 * int(column), gate_rows.stride(0)
         if value_dim > 1024:
             raise UnsupportedSizeError(f"windowed attention takes values up to 1024 wide, got {value_dim}")
         self._call(lib.llmlab_sink_window_attention, self._ptr(q), _dt(q), rows, num_heads, num_kv_heads, key_dim,
@@ -1467,7 +1534,7 @@ class HipOps:
                    int(keep_first or 0), int(chunk or 0), self._ptr(sink), float(scale), self._ptr(out),
                    self._ptr(q_start) if long_from else None, int(long_from), int(launches), int(max_keys),
                    self._ptr(self.workspace), self.workspace.numel(), self.num_cus, self.ATTENTION_WEIGHTS[weights],
-                   self._stream(), lib=lib)
+                   gate_ptr, gate_ld, self._stream(), lib=lib)
 
     ATTENTION_WEIGHTS = {"softmax": 0, "sigmoid": 1}
 
@@ -1580,18 +1647,6 @@ class HipOps:
                    self._ptr(q_out), self._ptr(k_cache), self._ptr(v_cache), _dt(q_out), page_size,
                    self._ptr(positions), self._ptr(row_req), self._ptr(block_table), block_table.stride(0),
                    1 if one_row_each else 0, self._stream(), lib=lib)
-
-    def gate_channels(self, out, proj, off_gate: int) -> None:
-        """``out[r, c] *= sigmoid(proj[r, off_gate + c])`` with the product in float32 (``out`` in a kernel
-        dtype, ``proj`` float32)."""
-        lib = self._mixer_lib("windowed_attention")
-        self._need(out, "heads' outputs")
-        self._need(proj, "projections", torch.float32)
-        rows, width = out.shape
-        if proj.shape[0] != rows or off_gate < 0 or off_gate + width > proj.shape[1]:
-            raise ValueError(f"gate_channels: gates at {off_gate} of {tuple(proj.shape)} for outputs {tuple(out.shape)}")
-        self._call(lib.llmlab_gate_channels, self._ptr(out), proj.data_ptr() + 4 * int(off_gate), proj.stride(0), rows, width,
-                   _dt(out), self._stream(), lib=lib)
 
     def gla_slices(self, key_dim: int) -> int:
         """Into how many pieces the scan leaves each output (one per slice of key channels)."""
@@ -1761,6 +1816,55 @@ class HipOps:
                    float(eps), self._ptr(proj), proj.stride(0), int(off_gate), self._ptr(out), _dt(out),
                    int(parts.shape[2]), per_head, self.OUTPUT_GATES[gate], int(norm_count or 0), self._ptr(norm_parts),
                    self._ptr(maxima), self._stream(), lib=lib)
+
+    RECURRENT_ROW_MAX_RANK = 512
+
+    def recurrent_row_takes(self, key_dim: int, value_dim: int, rank: int = 0) -> bool:
+        """Whether ``recurrent_row`` takes heads of these sizes."""
+        return (rank <= self.RECURRENT_ROW_MAX_RANK
+                and self._mixer_lib("linear_attention").llmlab_recurrent_row_threads(int(key_dim), int(value_dim)) > 0)
+
+    def recurrent_row(self, proj, off_q, off_k, off_v, off_gate, q_scale, num_heads, key_dim, value_dim, state, q_start,
+                      req_rows, n_reqs, weight, eps, gate: str, norm_count: int, out, decay=None, bonus=None,
+                      memory=None) -> None:
+        """A step in which every request brings ONE row: what ``gla_decay`` (or ``memory_gates``), ``gla_scan`` and
+        ``gla_output`` do, in one launch.  ``decay = (off_low, rank, w2, bias, kind, tau)``, with ``bonus`` for
+        the scan with a bonus; or ``memory = (off_i, off_f, bias_i, bias_f, cap, norm_state, max_state)``."""
+        lib = self._mixer_lib("linear_attention")
+        for t, name in ((proj, "projections"), (state, "recurrent state"), (weight, "output norm weight")):
+            self._need(t, name, torch.float32)
+        self._need(q_start, "request row starts", torch.int32)
+        self._need(req_rows, "state slots", torch.int32)
+        self._need(out, "mixer output")
+        rows, columns = proj.shape
+        if (rows != n_reqs or tuple(out.shape) != (rows, num_heads * value_dim) or q_start.numel() < n_reqs + 1
+                or req_rows.numel() < n_reqs or tuple(state.shape[1:]) != (num_heads, key_dim, value_dim)
+                or weight.numel() not in (value_dim, num_heads * value_dim) or (decay is None) == (memory is None)):
+            raise ValueError("recurrent_row: one row a request; the operands do not fit each other")
+        per_head = 1 if weight.numel() == num_heads * value_dim and num_heads > 1 else 0
+        kind = 2 if memory is not None else (1 if bonus is not None else 0)
+        off_low, rank, w2, bias, decay_kind, tau = decay if decay is not None else (0, 0, None, None, "sigmoid", 1.0)
+        off_i, off_f, bias_i, bias_f, cap, norm_state, max_state = memory if memory is not None else (0, 0, None, None, 1.0,
+                                                                                                      None, None)
+        for t, name, count in ((w2, "decay weight", num_heads * key_dim * rank), (bias, "decay bias", num_heads * key_dim),
+                               (bonus, "bonus", num_heads * key_dim), (bias_i, "gate bias", num_heads),
+                               (bias_f, "gate bias", num_heads)):
+            if t is not None:
+                self._need(t, name, torch.float32)
+                if t.numel() != count:
+                    raise ValueError(f"recurrent_row: {name} of {t.numel()} numbers, not {count}")
+        if memory is not None:
+            self._need(norm_state, "normaliser", torch.float32)
+            self._need(max_state, "maxima of the slots", torch.float32)
+            if (tuple(norm_state.shape) != (state.shape[0], num_heads, key_dim)
+                    or tuple(max_state.shape) != (state.shape[0], num_heads)):
+                raise ValueError("recurrent_row: the memory's slots do not fit the state's")
+        self._call(lib.llmlab_recurrent_row, self._ptr(proj), proj.stride(0), int(off_q), int(off_k), int(off_v), int(off_gate),
+                   float(q_scale), num_heads, key_dim, value_dim, self._ptr(state), self._ptr(q_start), self._ptr(req_rows),
+                   int(n_reqs), self._ptr(weight), float(eps), per_head, self.OUTPUT_GATES[gate], int(norm_count or 0), kind,
+                   int(off_low), int(rank), self._ptr(w2), self._ptr(bias), self.DECAY_KINDS[decay_kind], float(tau),
+                   self._ptr(bonus), int(off_i), int(off_f), self._ptr(bias_i), self._ptr(bias_f), float(cap),
+                   self._ptr(norm_state), self._ptr(max_state), self._ptr(out), _dt(out), self._stream(), lib=lib)
 
     def delta_gates(self, proj, off_low, rank, off_rate, off_k, w2, w0, rate_bias, decay_scale, key_eps, num_heads,
                     key_dim, decay, unit, removal) -> None:
@@ -1977,13 +2081,14 @@ class HipOps:
         self._call(lib.llmlab_gated_add, self._ptr(x), self._ptr(y), pieces, piece_stride, self._ptr(gate), cols,
                    self._ptr(bias), rows, width, self._stream(), lib=lib)
 
-    def rmsnorm_add(self, y, weight, eps: float, x, next_norm=None, copy=None) -> None:
+    def rmsnorm_add(self, y, weight, eps: float, x, next_norm=None, copy=None, shift=None) -> None:
         """``x += y / sqrt(mean(y^2) + eps) * weight`` row by row, all float32: the norm of a sublayer's
         result on its way into the stream.  ``y [rows, width]``, or a product left in pieces
         (``PendingSums``), which are summed on the way.  ``next_norm = (weight, eps, out)``: the RMS norm
         that reads the stream next, in the same launch: ``out = norm(x)`` of the new rows (float32
         weight, ``out`` in a kernel dtype).  ``copy``: a tensor of a kernel dtype that receives the new rows
-        rounded (instead of a next norm)."""
+        rounded (instead of a next norm).  ``shift = (mix, state, req_rows, out)`` (steps in which every request
+        brings ONE row): ``shift_mix`` of the new rows in the same launch, ``out [1, rows, width]``."""
         lib = self._mixer_lib("stream_ops")
         self._need(x, "stream", torch.float32)
         self._need(weight, "norm weight", torch.float32)
@@ -2008,6 +2113,16 @@ class HipOps:
             if next_norm is not None or tuple(copy.shape) != (rows, width):
                 raise ValueError("rmsnorm_add: a next norm or a copy of the stream's shape, not both")
             next_out = copy
+        shift_state = shift_rows = None
+        if shift is not None:
+            next_w, shift_state, shift_rows, next_out = shift
+            self._need(next_w, "mix", torch.float32)
+            self._need(shift_state, "rows before", torch.float32)
+            self._need(shift_rows, "request slots", torch.int32)
+            self._need(next_out, "mixed rows")
+            if (copy is not None or next_norm is not None or next_w.numel() != width or shift_rows.numel() < rows
+                    or tuple(shift_state.shape[1:]) != (width,) or next_out.numel() != rows * width):
+                raise ValueError("rmsnorm_add: the shift's mix, slots and output have the stream's width and rows")
         if next_norm is not None:
             next_w, next_eps, next_out = next_norm
             self._need(next_w, "next norm's weight", torch.float32)
@@ -2016,7 +2131,8 @@ class HipOps:
                 raise ValueError("rmsnorm_add: the next norm's weight and output have the stream's shape")
         self._call(lib.llmlab_rmsnorm_add, self._ptr(x), self._ptr(parts), int(pieces), int(stride), self._ptr(weight),
                    float(eps), rows, width, self._ptr(next_w), float(next_eps), self._ptr(next_out),
-                   _dt(next_out) if next_out is not None else 0, self._stream(), lib=lib)
+                   _dt(next_out) if next_out is not None else 0, self._ptr(shift_state), self._ptr(shift_rows),
+                   self._stream(), lib=lib)
 
     def scaled_sum(self, out, y1, a: float, y2, b: float) -> None:
         """``out = a * y1 + b * y2``, float32 tensors of one shape."""
@@ -2028,9 +2144,10 @@ class HipOps:
         self._call(lib.llmlab_scaled_sum, self._ptr(out), self._ptr(y1), float(a), self._ptr(y2), float(b), out.numel(),
                    self._stream(), lib=lib)
 
-    def normed_sum(self, out, y1, w1, a: float, y2, w2, b: float, eps: float) -> None:
-        """``out = a * rms(y1) * w1 + b * rms(y2) * w2`` row by row, ``rms(v) = v / sqrt(mean(v^2) + eps)``;
-        all float32."""
+    def normed_sum(self, out, y1, w1, a: float, y2, w2, b: float, eps: float, add=None, copy=None) -> None:
+        """``out = s`` with ``s = a * rms(y1) * w1 + b * rms(y2) * w2`` row by row, ``rms(v) = v / sqrt(mean(v^2) +
+        eps)``; all float32.  ``add = (weight, eps)``: ``out += rms(s) * weight`` instead (the norm of the sum
+        on its way into the stream), and ``copy`` (a kernel dtype, or None) receives the new rows."""
         lib = self._mixer_lib("stream_ops")
         for t, name in ((out, "sum"), (y1, "first term"), (y2, "second term"), (w1, "first weight"), (w2, "second weight")):
             self._need(t, name, torch.float32)
@@ -2039,8 +2156,18 @@ class HipOps:
             raise ValueError("normed_sum: three tensors of one shape")
         if w1.numel() != width or w2.numel() != width:
             raise ValueError("normed_sum: weights of the rows' width")
+        add_w, add_eps = add if add is not None else (None, 0.0)
+        if add is not None:
+            self._need(add_w, "norm weight", torch.float32)
+            if add_w.numel() != width:
+                raise ValueError("normed_sum: a weight of the stream's width")
+        if copy is not None:
+            self._need(copy, "stream copy")
+            if add is None or tuple(copy.shape) != (rows, width):
+                raise ValueError("normed_sum: a copy has the stream's shape and goes with the sum into it")
         self._call(lib.llmlab_normed_sum, self._ptr(out), self._ptr(y1), self._ptr(w1), float(a),
-                   self._ptr(y2), self._ptr(w2), float(b), float(eps), rows, width, self._stream(), lib=lib)
+                   self._ptr(y2), self._ptr(w2), float(b), float(eps), rows, width, self._ptr(add_w), float(add_eps),
+                   self._ptr(copy), _dt(copy) if copy is not None else 0, self._stream(), lib=lib)
 
     def shift_mix(self, h, mix, state, row_req, q_start, req_rows, out) -> None:
         """``out[m] = h + (p - h) * mix[m]`` for every row of ``mix [mixes, width]`` float32, ``p`` the row

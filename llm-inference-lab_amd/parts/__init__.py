@@ -1,5 +1,5 @@
 from .registry import register_part, unregister_part, part_class, build_part, FAMILIES
-from .base import (Part, Norm, NormedInput, PendingSums, PositionEncoding, Mixer, FeedForward, Block,
+from .base import (Part, Norm, NormedInput, NormedPair, PendingSums, PositionEncoding, Mixer, FeedForward, Block,
                    KVCacheSpec, CacheSpec, PageTensor)
 from .norms import RMSNorm, LayerNorm
 from .positions import RotaryEmbedding, PairRotary, NoPosition

@@ -569,6 +569,8 @@ class WindowedSinkAttention(Mixer):
         kind = dict(weights="sigmoid") if sigmoid else {}
         if self.chunk is not None:
             kind["chunk"] = self.chunk
+        if self.output_gate == "channels":
+            kind["gate"] = (proj, self.q_size + self.k_size + self.v_size)
         reach = self.window if self.window is not None else self.chunk
 
         def attend():
@@ -589,8 +591,6 @@ class WindowedSinkAttention(Mixer):
             attend()
         if gate is not None:
             ops.gate_heads(mixed, gate, self.num_heads, self.value_dim, self.output_gate)
-        if self.output_gate == "channels":
-            ops.gate_channels(mixed, proj, self.q_size + self.k_size + self.v_size)
         if self.b_o is not None:
             ops.linear_logits(mixed, self.w_o, out, self.b_o)
         else:

@@ -182,6 +182,16 @@ class PendingSums:
         self.parts, self.splits = parts, int(splits)
 
 
+class NormedPair:
+    """A result that is the weighted sum of two normed ones, ``a * rms(y1) * w1 + b * rms(y2) * w2`` (``rms`` with
+    ``eps`` inside the root), not summed yet: whoever takes it sums it on the way."""
+
+    __slots__ = ("y1", "w1", "a", "y2", "w2", "b", "eps")
+
+    def __init__(self, y1, w1, a, y2, w2, b, eps):
+        self.y1, self.w1, self.a, self.y2, self.w2, self.b, self.eps = y1, w1, float(a), y2, w2, float(b), float(eps)
+
+
 class NormedInput:
     """The input of a mixer, feed-forward or head whose norm has not run yet.
 

@@ -73,7 +73,9 @@ class SublayerNormBlock(Block):
     ``token_shift``: what the mixer reads is the stream's row mixed with the row before it in the
     sequence, ``h_t = x_t + (x_(t-1) - x_t) * shift`` element by element (``shift [width]``: tensor role
     ``shift``; zeros before the sequence's start), taken in float32 and rounded once.  The last row is
-    per-request state, so a sequence may be cut anywhere.  The feed-forward reads ``x`` itself."""
+    per-request state, so a sequence may be cut anywhere.  The feed-forward reads ``x`` itself.  Where
+    the next run of the schedule shifts its tokens too, and every request of the step brings one row,
+    the launch of this run's last sum does the next run's shift as well (``entry.follower``)."""
 
     def __init__(self, hidden_size: int, mixer: PartSpec, norm1: PartSpec, feed_forward: PartSpec = None,
                  norm2: PartSpec = None, tensors: Dict[str, str] = None, token_shift: bool = False):
@@ -144,9 +146,43 @@ class SublayerNormBlock(Block):
     def _shifted(self, residual, ctx, entry):
         """The mixer's input where tokens are shifted: every row of the stream mixed with the one before."""
         h = ctx.scratch("block.shifted", (1,) + tuple(residual.shape), self.dtype)
-        self.ops.shift_mix(residual, self.shift, entry.state["shifted_row"], ctx.row_req, ctx.all_q_start,
-                           ctx.all_req_rows, h)
+        led = getattr(entry, "led", False)
+
+        def launch():        # (whether every request brings one row is not a matter of the number of rows)
+            if led and ctx.n_rows == ctx.n_reqs:
+                return       # (the run before this one has done it)
+            self.ops.shift_mix(residual, self.shift, entry.state["shifted_row"], ctx.row_req, ctx.all_q_start,
+                               ctx.all_req_rows, h)
+        self._live(launch)
         return h[0]
+
+    def _live(self, launch):
+        live = getattr(self.ops, "live", None)
+        if live is not None:
+            live(launch)
+        else:
+            launch()
+
+    def leads(self, block) -> bool:
+        """Whether the launch of this block's last sum can do the token shift of ``block`` right after it."""
+        last = self.norm1 if self.feed_forward is None else self.norm2
+        return (isinstance(block, SublayerNormBlock) and block.token_shift and getattr(last, "adds_shift", False)
+                and not (self.feed_forward is None and hasattr(self.mixer, "forward_pending")))
+
+    def _last_sum(self, norm, y, residual, copy, ctx, entry):
+        follower = getattr(entry, "follower", None)
+        if follower is None:
+            norm.add_into(y, residual, copy)
+            return
+        block, view = follower
+        h = ctx.scratch("block.shifted", (1,) + tuple(residual.shape), self.dtype)
+
+        def launch():
+            if ctx.n_rows == ctx.n_reqs:
+                norm.add_into(y, residual, shift=(block.shift, view.state["shifted_row"], ctx.all_req_rows, h))
+            else:
+                norm.add_into(y, residual, copy)
+        self._live(launch)
 
     def _sublayer(self, part, norm, h, residual, ctx, *entry):
         y = ctx.scratch("block.sublayer_out", tuple(residual.shape), torch.float32)
@@ -173,10 +209,13 @@ class SublayerNormBlock(Block):
             mixed = h = self._input(residual, ctx, entry)
         copy = h if self.dtype != torch.float32 else None
         y = self._sublayer(self.mixer, self.norm1, mixed, residual, ctx, entry)
-        self.norm1.add_into(y, residual, copy if self.feed_forward is not None or not self.token_shift else None)
-        if self.feed_forward is not None:
+        last_copy = None if self.token_shift else copy
+        if self.feed_forward is None:
+            self._last_sum(self.norm1, y, residual, last_copy, ctx, entry)
+        else:
+            self.norm1.add_into(y, residual, copy)
             y = self._sublayer(self.feed_forward, self.norm2, h, residual, ctx)
-            self.norm2.add_into(y, residual, None if self.token_shift else copy)
+            self._last_sum(self.norm2, y, residual, last_copy, ctx, entry)
         memo = getattr(ctx, "memo", None)
         if memo is not None and copy is not None and not self.token_shift:
             memo[self.NOTE] = entry.index

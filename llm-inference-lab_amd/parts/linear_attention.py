@@ -84,20 +84,40 @@ class ScanMixer(Mixer):
                 kind["memory"] = tuple(memory) + (norm_parts, chunk_norm if chunk else None)
             ops.gla_scan(proj, off_q, off_k, off_v, decay, q_scale, heads, d, e, state, ctx.all_q_start, ctx.all_req_rows,
                          ctx.n_reqs, parts, chunk, chunk_state if chunk else None, chunk_decay if chunk else None, **kind)
-        live = getattr(ops, "live", None)
-        if live is not None:
-            live(scan)
-        else:
-            scan()
+        self._live(scan)
         return parts if memory is None else (parts, norm_parts)
 
-    def _output(self, parts, weight, eps, proj, off_gate, gate, ctx, **memory):
+    def _live(self, launch):
+        live = getattr(self.ops, "live", None)
+        if live is not None:
+            live(launch)
+        else:
+            launch()
+
+    def _recur(self, proj, ctx, entry, off, weight, eps, gate, q_scale, many_rows, rank=0, **kind):
+        """From the projections to the gated output ``[rows, heads * value_dim]`` (compute dtype).  Where every
+        request of the step brings one row and the sizes allow it: one launch; else ``many_rows()``.
+        ``off``: the columns of query, key, value and gate."""
+        ops = self.ops
         mixed = ctx.scratch("linear_attention.out", (proj.shape[0], self.v_size), self.dtype)
+        takes = getattr(ops, "recurrent_row_takes", None)
+        fits = takes is not None and takes(self.key_dim, self.value_dim, rank)
+        count = self.file_value_dim if self.file_value_dim != self.value_dim else 0
+
+        def launch():        # (whether every request brings one row is not a matter of the number of rows)
+            if fits and ctx.n_rows == ctx.n_reqs:
+                ops.recurrent_row(proj, *off, q_scale, self.num_heads, self.key_dim, self.value_dim, entry.state["s"],
+                                  ctx.all_q_start, ctx.all_req_rows, ctx.n_reqs, weight, eps, gate, count, mixed, **kind)
+            else:
+                many_rows(mixed)
+        self._live(launch)
+        return mixed
+
+    def _output(self, parts, weight, eps, proj, off_gate, gate, mixed, **memory):
         if self.file_value_dim != self.value_dim:      # (the heads' norm is over the file's channels)
             memory["norm_count"] = self.file_value_dim
         self.ops.gla_output(parts, self.num_heads, self.key_dim, self.value_dim, weight, eps, proj, off_gate, mixed, gate,
                             **memory)
-        return mixed
 
     def forward(self, h, residual, ctx, entry):
         if isinstance(h, NormedInput) and not self.takes_normed_input:
@@ -185,10 +205,16 @@ class GatedLinearAttention(ScanMixer):
         ops, rows, o = self.ops, h.shape[0], self.offsets
         proj = ctx.scratch("linear_attention.proj", (rows, self.in_size), torch.float32)
         ops.linear_logits(h, self.w_in, proj)
+        off = [o[role] for role in ("q_weight", "k_weight", "v_weight", "gate_weight")]
         decay = ctx.scratch("linear_attention.decay", (rows, self.qk_size), torch.float32)
-        ops.gla_decay(proj[:, o["decay_down"]:], self.decay_rank, self.w_decay, self.b_decay, self.tau, decay)
-        parts = self._scan(proj, o["q_weight"], o["k_weight"], o["v_weight"], decay, self.q_scale, entry.state["s"], ctx)
-        mixed = self._output(parts, self.norm_weight, self.norm_eps, proj, o["gate_weight"], "silu", ctx)
+
+        def many_rows(mixed):
+            ops.gla_decay(proj[:, o["decay_down"]:], self.decay_rank, self.w_decay, self.b_decay, self.tau, decay)
+            parts = self._scan(proj, *off[:3], decay, self.q_scale, entry.state["s"], ctx)
+            self._output(parts, self.norm_weight, self.norm_eps, proj, off[3], "silu", mixed)
+        mixed = self._recur(proj, ctx, entry, off, self.norm_weight, self.norm_eps, "silu", self.q_scale, many_rows,
+                            self.decay_rank,
+                            decay=(o["decay_down"], self.decay_rank, self.w_decay, self.b_decay, "sigmoid", self.tau))
         ops.linear_logits(mixed, self.w_o, out)
 
     def weight_bytes(self):
@@ -396,7 +422,7 @@ class TimeMixAttention(ScanMixer):
         self.gate = gate
         self.decay_rank = None
         self.mix = self.w_o = self.w_decay = self.b_decay = self.bonus = self.norm_weight = None
-        self.w_mixed, self.offsets, self.in_size = {}, {}, 0
+        self.w_mixed, self.offsets, self.in_size = None, {}, 0
 
     def tensor_specs(self):
         t, w = self.tensor_names, self.hidden_size
@@ -427,13 +453,13 @@ class TimeMixAttention(ScanMixer):
                              f"projection do not fit")
         self.decay_rank = rank
         self.mix = torch.stack([tensors[t[role]].float() for role, _ in self.MIXES]).contiguous()
-        at = 0
+        at, weights = 0, []
         for _, role in self.MIXES:
-            w = self._values(tensors[t[role]]) if role in ("v_weight", "gate_weight") else tensors[t[role]]
-            self.w_mixed[role] = ops.prepare_weight(w.contiguous())
+            weights.append(self._values(tensors[t[role]]) if role in ("v_weight", "gate_weight") else tensors[t[role]])
             self.offsets[role] = at
-            at += (w.shape[0] + 31) // 32 * 32       # (every product's columns start on a boundary of 128 bytes)
+            at += (weights[-1].shape[0] + 15) // 16 * 16       # (as the segments of the weight lie)
         self.in_size = at
+        self.w_mixed = ops.prepare_segments(weights)
         self.w_o = ops.prepare_weight(self._values(tensors[t["o_weight"]].t()).t().contiguous())
         # the second factor of the decays is applied in float32, inside the decay kernel
         self.w_decay = tensors[t["decay_up"]].float().contiguous()
@@ -449,21 +475,24 @@ class TimeMixAttention(ScanMixer):
         mixed = ctx.scratch("time_mix.mixed", (len(self.MIXES), rows, self.hidden_size), self.dtype)
         ops.shift_mix(h, self.mix, entry.state["previous_row"], ctx.row_req, ctx.all_q_start, ctx.all_req_rows, mixed)
         proj = ctx.scratch("time_mix.proj", (rows, self.in_size), torch.float32)
-        for i, (_, role) in enumerate(self.MIXES):
-            w = self.w_mixed[role]
-            ops.linear_logits(mixed[i], w, proj[:, o[role]:o[role] + w.shape[0]])
+        ops.segmented_products(mixed, self.w_mixed, proj, [o[role] for _, role in self.MIXES])
+        off = [o[role] for role in ("r_weight", "k_weight", "v_weight", "gate_weight")]
         decay = ctx.scratch("linear_attention.decay", (rows, self.qk_size), torch.float32)
-        ops.gla_decay(proj[:, o["decay_down"]:], self.decay_rank, self.w_decay, self.b_decay, 1.0, decay, "double_exp")
-        parts = self._scan(proj, o["r_weight"], o["k_weight"], o["v_weight"], decay, 1.0, entry.state["s"], ctx,
-                           bonus=self.bonus)
-        gated = self._output(parts, self.norm_weight, self.norm_eps, proj, o["gate_weight"], self.gate, ctx)
+
+        def many_rows(gated):
+            ops.gla_decay(proj[:, o["decay_down"]:], self.decay_rank, self.w_decay, self.b_decay, 1.0, decay, "double_exp")
+            parts = self._scan(proj, *off[:3], decay, 1.0, entry.state["s"], ctx, bonus=self.bonus)
+            self._output(parts, self.norm_weight, self.norm_eps, proj, off[3], self.gate, gated)
+        gated = self._recur(proj, ctx, entry, off, self.norm_weight, self.norm_eps, self.gate, 1.0, many_rows,
+                            self.decay_rank, bonus=self.bonus,
+                            decay=(o["decay_down"], self.decay_rank, self.w_decay, self.b_decay, "double_exp", 1.0))
         ops.linear_logits(gated, self.w_o, out)
 
     def kernel_libraries(self):
         return [("stream_ops", None), ("linear_attention", None)]
 
     def weight_bytes(self):
-        return sum(w.numel() * w.element_size() for w in (*self.w_mixed.values(), self.mix, self.w_o, self.w_decay,
+        return sum(w.numel() * w.element_size() for w in (self.w_mixed, self.mix, self.w_o, self.w_decay,
                                                           self.b_decay, self.bonus, self.norm_weight) if w is not None)
 
 
@@ -547,19 +576,18 @@ class MatrixMemoryAttention(ScanMixer):
         ops.linear_logits(h, self.w_in, proj)
         keep, take, maxima = (ctx.scratch("matrix_memory." + name, (rows, self.num_heads), torch.float32)
                               for name in ("keep", "take", "maxima"))
+        off = [o[role] for role in ("q_weight", "k_weight", "v_weight", "gate_weight")]
 
-        def gates():        # (how many requests the step has is read when the launch is made)
+        def many_rows(mixed):
             ops.memory_gates(proj, o["i_weight"], o["f_weight"], self.b_i, self.b_f, self.gate_cap, self.num_heads,
                              entry.state["m"], ctx.all_q_start, ctx.all_req_rows, ctx.n_reqs, keep, take, maxima)
-        live = getattr(ops, "live", None)
-        if live is not None:
-            live(gates)
-        else:
-            gates()
-        parts, norm_parts = self._scan(proj, o["q_weight"], o["k_weight"], o["v_weight"], None, self.q_scale,
-                                       entry.state["s"], ctx, memory=(keep, take, entry.state["n"]))
-        mixed = self._output(parts, self.norm_weight, self.norm_eps, proj, o["gate_weight"], self.gate, ctx,
-                             norm_parts=norm_parts, maxima=maxima)
+            parts, norm_parts = self._scan(proj, *off[:3], None, self.q_scale, entry.state["s"], ctx,
+                                           memory=(keep, take, entry.state["n"]))
+            self._output(parts, self.norm_weight, self.norm_eps, proj, off[3], self.gate, mixed, norm_parts=norm_parts,
+                         maxima=maxima)
+        mixed = self._recur(proj, ctx, entry, off, self.norm_weight, self.norm_eps, self.gate, self.q_scale, many_rows,
+                            memory=(o["i_weight"], o["f_weight"], self.b_i, self.b_f, self.gate_cap, entry.state["n"],
+                                    entry.state["m"]))
         ops.linear_logits(mixed, self.w_o, out)
 
     def weight_bytes(self):

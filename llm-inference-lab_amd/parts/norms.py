@@ -6,7 +6,7 @@ from typing import Dict, Optional
 import torch
 
 from ..weights.loader import TensorSpec, VECTOR, INIT_NORM, INIT_NORMAL
-from .base import Norm
+from .base import Norm, NormedPair
 from .registry import register_part
 
 
@@ -57,14 +57,20 @@ class RMSNorm(Norm):
     def rms_params(self):
         return self.weight, self.eps
 
-    adds_pieces = True      # ``add_into`` takes a result left in pieces as well
+    adds_pieces = True      # ``add_into`` takes a result left in pieces as well, or a ``NormedPair``,
+    adds_shift = True       # and may mix the new rows with the ones before (``HipOps.rmsnorm_add``'s ``shift``)
 
-    def add_into(self, y, stream, copy=None):
-        """``stream += norm(y)`` (``y`` float32, or ``PendingSums``); ``copy`` (compute dtype) receives the
-        stream's new rows.  (The kernel takes its weight in float32.)"""
+    def add_into(self, y, stream, copy=None, shift=None):
+        """``stream += norm(y)`` (``y`` float32, ``PendingSums`` or ``NormedPair``); ``copy`` (compute dtype)
+        receives the stream's new rows.  (The kernel takes its weight in float32.)"""
         if self.weight_f32 is None:
             self.weight_f32 = self.weight.float().contiguous()
-        self.ops.rmsnorm_add(y, self.weight_f32, self.eps, stream, copy=copy)
+        if isinstance(y, NormedPair):
+            self.ops.normed_sum(stream, y.y1, y.w1, y.a, y.y2, y.w2, y.b, y.eps, add=(self.weight_f32, self.eps), copy=copy)
+        elif shift is not None:
+            self.ops.rmsnorm_add(y, self.weight_f32, self.eps, stream, shift=shift)
+        else:
+            self.ops.rmsnorm_add(y, self.weight_f32, self.eps, stream, copy=copy)
 
     def weight_bytes(self):
         return self.weight.numel() * self.weight.element_size()

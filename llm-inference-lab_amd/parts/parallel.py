@@ -7,7 +7,7 @@ import torch
 
 from ..config.spec import PartSpec
 from ..weights.loader import TensorSpec, VECTOR, INIT_NORM
-from .base import Mixer, NormedInput, PendingSums
+from .base import Mixer, NormedInput, NormedPair, PendingSums
 from .registry import register_part, build_part
 
 
@@ -93,10 +93,21 @@ class ParallelMixers(Mixer):
                 ctx.pending = None
         return y
 
+    def forward_pending(self, h, out, ctx, entry):
+        """The two normed results as a ``NormedPair`` (where the results are normed), for a caller that sums
+        them on its own way; else their sum in ``out`` and None."""
+        if self.out_norms is None:
+            self.forward_into(h, out, ctx, entry)
+            return None
+        y1, y2 = self._results(h, tuple(out.shape), ctx, entry)
+        return NormedPair(y1, self.out_norms[0], self.left_scale, y2, self.out_norms[1], self.right_scale, self.norm_eps)
+
+    def _results(self, h, shape, ctx, entry):
+        return (self._result(self.left, "parallel.left", h, shape, ctx, entry),
+                self._result(self.right, "parallel.right", h, shape, ctx, entry))
+
     def forward_into(self, h, out, ctx, entry):
-        shape = tuple(out.shape)
-        y1 = self._result(self.left, "parallel.left", h, shape, ctx, entry)
-        y2 = self._result(self.right, "parallel.right", h, shape, ctx, entry)
+        y1, y2 = self._results(h, tuple(out.shape), ctx, entry)
         if self.out_norms is not None:
             self.ops.normed_sum(out, y1, self.out_norms[0], self.left_scale, y2, self.out_norms[1], self.right_scale,
                                 self.norm_eps)

@@ -10,6 +10,7 @@ All arithmetic is float32 whatever the storage dtype.
 from __future__ import annotations
 
 import math
+from types import SimpleNamespace
 
 import torch
 
@@ -55,7 +56,7 @@ class EmuRecord:
 class EmuOps:
     # the operations that do work on tensors: written down while a part is recorded, as the
     # product's kernel set writes down its calls into the kernel libraries
-    RECORDED = ("shift_mix", "poly_norm", "normed_sum", "project_conv_write", "gate_channels", "memory_gates",
+    RECORDED = ("shift_mix", "poly_norm", "normed_sum", "project_conv_write", "segmented_products", "memory_gates", "recurrent_row",
                 "embed", "gather_tokens", "rmsnorm", "linear", "linear_relu2", "linear_residual", "linear_partials",
                 "add_pending", "linear_logits", "linear_swiglu", "fused_norm_qkv", "qkv_rope_cache",
                 "fused_norm_swiglu", "fused_norm_logits", "rope_inplace", "rope_kv_write",
@@ -290,7 +291,7 @@ class EmuOps:
 
     def sink_window_attention(self, q, num_heads, num_kv_heads, key_dim, value_dim, k_cache, v_cache, block_table,
                               page_size, positions, row_req, window, keep_first, sink, scale, out,
-                              q_start=None, long_from=0, launches=3, max_keys=0, weights="softmax", chunk=None):
+                              q_start=None, long_from=0, launches=3, max_keys=0, weights="softmax", chunk=None, gate=None):
         """(``long_from``, ``launches``: how the kernels share the rows; the result is the same.)"""
         self._count("sink_window_attention")
         rows = q.shape[0]
@@ -315,7 +316,11 @@ class EmuOps:
                 if sink is not None:
                     s = torch.cat([s, sink[h].float().view(1)])
                 w = torch.softmax(s, 0)[:len(js)]
-                out[r, h * value_dim:(h + 1) * value_dim] = (w @ v[:, h // group]).to(out.dtype)
+                o = w @ v[:, h // group]
+                if gate is not None:
+                    at = gate[1] + h * value_dim
+                    o = o * torch.sigmoid(gate[0][r, at:at + value_dim].float())
+                out[r, h * value_dim:(h + 1) * value_dim] = o.to(out.dtype)
 
     def project_rotate_write(self, proj, num_heads, num_kv_heads, key_dim, value_dim, bias, freq, rot_dims, magnitude,
                              mix, mix_weight, v_first, gate_out, q_out, k_cache, v_cache, page_size, positions,
@@ -396,10 +401,16 @@ class EmuOps:
                 st.copy_(new)
                 o[t] = torch.einsum("hde,hd->he", st, r)
 
-    def normed_sum(self, out, y1, w1, a, y2, w2, b, eps):
+    def normed_sum(self, out, y1, w1, a, y2, w2, b, eps, add=None, copy=None):
         self._count("normed_sum")
-        rms = lambda y: y / torch.sqrt((y * y).mean(-1, keepdim=True) + eps)
-        out.copy_(a * rms(y1) * w1 + b * rms(y2) * w2)
+        rms = lambda y, e: y / torch.sqrt((y * y).mean(-1, keepdim=True) + e)
+        s = a * rms(y1, eps) * w1 + b * rms(y2, eps) * w2
+        if add is None:
+            out.copy_(s)
+            return
+        out += rms(s, add[1]) * add[0]
+        if copy is not None:
+            copy.copy_(out.to(copy.dtype))
 
     def shift_mix(self, h, mix, state, row_req, q_start, req_rows, out):
         self._count("shift_mix")
@@ -462,17 +473,53 @@ class EmuOps:
             k_cache[page, :, o] = k[r]
             cache_layout.value_quads(v_cache[page])[:, o >> 2, :, o & 3] = v[r]
 
-    def gate_channels(self, out, proj, off_gate):
-        self._count("gate_channels")
-        g = torch.sigmoid(proj[:, off_gate:off_gate + out.shape[1]].float())
-        out.copy_((out.float() * g).to(out.dtype))
+    def prepare_segments(self, weights):
+        return SimpleNamespace(members=[w.contiguous() for w in weights],
+                               numel=lambda: sum(w.numel() for w in weights), element_size=weights[0].element_size)
 
-    def rmsnorm_add(self, y, weight, eps, x, next_norm=None, copy=None):
+    def segmented_products(self, x, w, out, offsets):
+        self._count("segmented_products")
+        for s, (member, at) in enumerate(zip(w.members, offsets)):
+            out[:, at:at + member.shape[0]] = x[s].float() @ member.float().t()
+
+    def recurrent_row_takes(self, key_dim, value_dim, rank=0):
+        return key_dim * value_dim <= 1024 or key_dim % 3 == 0      # (both ways are exercised)
+
+    def recurrent_row(self, proj, off_q, off_k, off_v, off_gate, q_scale, num_heads, key_dim, value_dim, state, q_start,
+                      req_rows, n_reqs, weight, eps, gate, norm_count, out, decay=None, bonus=None, memory=None):
+        self._count("recurrent_row")
+        rows = proj.shape[0]
+        assert rows == n_reqs
+        parts = torch.zeros(rows, num_heads, self.gla_slices(key_dim), value_dim)
+        kind, a, norm = {}, None, {}
+        if decay is not None:
+            off_low, rank, w2, bias, decay_kind, tau = decay
+            a = torch.empty(rows, num_heads * key_dim)
+            self.gla_decay(proj[:, off_low:], rank, w2, bias, tau, a, decay_kind)
+            kind = dict(bonus=bonus) if bonus is not None else {}
+        else:
+            off_i, off_f, bias_i, bias_f, cap, norm_state, max_state = memory
+            keep, take, maxima = (torch.empty(rows, num_heads) for _ in range(3))
+            self.memory_gates(proj, off_i, off_f, bias_i, bias_f, cap, num_heads, max_state, q_start, req_rows, n_reqs, keep,
+                              take, maxima)
+            norm = dict(norm_parts=torch.zeros(rows, num_heads, parts.shape[2]), maxima=maxima)
+            kind = dict(memory=(keep, take, norm_state, norm["norm_parts"], None))
+        self.gla_scan(proj, off_q, off_k, off_v, a, q_scale, num_heads, key_dim, value_dim, state, q_start, req_rows, n_reqs,
+                      parts, **kind)
+        self.gla_output(parts, num_heads, key_dim, value_dim, weight, eps, proj, off_gate, out, gate, norm_count, **norm)
+
+    def rmsnorm_add(self, y, weight, eps, x, next_norm=None, copy=None, shift=None):
         self._count("rmsnorm_add")
         v = self._owed(y) if isinstance(y, PendingSums) else y.float()
         x.add_(v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * weight.float())
         if copy is not None:
             copy.copy_(x.to(copy.dtype))
+        if shift is not None:
+            mix, state, req_rows, out = shift
+            for r in range(x.shape[0]):
+                before = state[int(req_rows[r])]
+                out[0, r] = (x[r] + (before - x[r]) * mix[0]).to(out.dtype)
+                before.copy_(x[r])
         if next_norm is not None:
             w, e, out = next_norm
             out.copy_((x / torch.sqrt((x * x).mean(-1, keepdim=True) + e) * w.float()).to(out.dtype))
