@@ -21,16 +21,20 @@ constexpr int SLICE = 16;      // key channels of the state that one thread keep
 // key channels, j over the rank of the projection).  sigmoid(z)^(1/tau) = exp(-softplus(-z) / tau),
 // with softplus(u) = max(u, 0) + log1p(exp(-|u|)), so that neither end overflows.
 // kind 1 (DECAY_DOUBLE_EXP): a[r, c] = exp(-exp(z)), z = bias[c] + sum_j w2[c, j] * tanh(low[r, j]).
+// as_log: the decay's logarithm to the base 2 instead, at least LOG_FLOOR (what the chunked scan on the
+// matrix cores takes; a decay of 2^-60 leaves nothing of a state in 32 bits).
 constexpr int DECAY_SIGMOID = 0, DECAY_DOUBLE_EXP = 1;
-__device__ __forceinline__ float decay_of(float z, int kind, float inv_tau) {
-  if (kind == DECAY_DOUBLE_EXP) return expf(-expf(z));
+constexpr float LOG2_E = 1.4426950408889634f, LOG_FLOOR = -60.f;
+__device__ __forceinline__ float log_decay_of(float z, int kind, float inv_tau) {
+  if (kind == DECAY_DOUBLE_EXP) return -expf(z);
   const float u = -z;
-  const float sp = fmaxf(u, 0.f) + log1pf(expf(-fabsf(u)));
-  return expf(-sp * inv_tau);
+  return -(fmaxf(u, 0.f) + log1pf(expf(-fabsf(u)))) * inv_tau;
 }
+__device__ __forceinline__ float decay_of(float z, int kind, float inv_tau) { return expf(log_decay_of(z, kind, inv_tau)); }
 __global__ __launch_bounds__(256) void gla_decay_kernel(const float* __restrict__ low, int ld, int rank,
                                                         const float* __restrict__ w2, const float* __restrict__ bias,
-                                                        int kind, float inv_tau, float* __restrict__ decay, int channels) {
+                                                        int kind, float inv_tau, float* __restrict__ decay, int channels,
+                                                        int as_log) {
   extern __shared__ float s_low[];
   const int r = blockIdx.x;
   const float* t = low + (size_t)r * ld;
@@ -50,19 +54,20 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(const float* __restrict_
     } else {
       for (int j = 0; j < rank; ++j) z = fmaf(w[j], s_low[j], z);
     }
-    decay[(size_t)r * channels + c] = decay_of(z, kind, inv_tau);
+    const float lg = log_decay_of(z, kind, inv_tau);
+    decay[(size_t)r * channels + c] = as_log ? fmaxf(lg * LOG2_E, LOG_FLOOR) : expf(lg);
   }
 }
 
 extern "C" int llmlab_gla_decay(const float* low, int ld, int rows, int rank, const float* w2, const float* bias,
-                                int kind, float tau, float* decay, int channels, hipStream_t stream) {
+                                int kind, float tau, float* decay, int channels, int as_log, hipStream_t stream) {
   LLMLAB_REQUIRE(rows >= 0 && rank > 0 && rank <= 8192 && channels > 0 && ld >= rank && tau > 0.f &&
                      (kind == DECAY_SIGMOID || kind == DECAY_DOUBLE_EXP),
                  "gla_decay: bad sizes rows=%d rank=%d channels=%d ld=%d kind=%d tau=%g", rows, rank, channels, ld, kind,
                  (double)tau);
   if (rows == 0) return 0;
   hipLaunchKernelGGL(gla_decay_kernel, dim3(rows), dim3(256), rank * sizeof(float), stream, low, ld, rank, w2, bias, kind,
-                     1.0f / tau, decay, channels);
+                     1.0f / tau, decay, channels, as_log);
   LLMLAB_LAUNCH_CHECK("gla_decay");
   return 0;
 }
@@ -79,7 +84,8 @@ constexpr int MEMORY_TILE = 256;
 __global__ __launch_bounds__(MEMORY_TILE) void memory_gates_kernel(
     const float* __restrict__ proj, int ld, int off_i, int off_f, const float* __restrict__ bias_i,
     const float* __restrict__ bias_f, float cap, int n_heads, float* __restrict__ max_state, const int* __restrict__ q_start,
-    const int* __restrict__ req_rows, float* __restrict__ keep, float* __restrict__ take, float* __restrict__ maxima) {
+    const int* __restrict__ req_rows, float* __restrict__ keep, float* __restrict__ take, float* __restrict__ maxima,
+    int as_log) {
   __shared__ float s_f[MEMORY_TILE / 64], s_m[MEMORY_TILE / 64], s_max[MEMORY_TILE + 1];
   const int b = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int first = q_start[b], last = q_start[b + 1];
@@ -119,7 +125,8 @@ __global__ __launch_bounds__(MEMORY_TILE) void memory_gates_kernel(
     __syncthreads();
     if (in) {
       const size_t at = (size_t)t * n_heads + h;
-      keep[at] = expf(f + s_max[threadIdx.x] - m);
+      const float lg = f + s_max[threadIdx.x] - m;
+      keep[at] = as_log ? fmaxf(lg * LOG2_E, LOG_FLOOR) : expf(lg);      // (as for the decays)
       take[at] = expf(i - m);
       maxima[at] = m;
     }
@@ -131,14 +138,14 @@ __global__ __launch_bounds__(MEMORY_TILE) void memory_gates_kernel(
 
 extern "C" int llmlab_memory_gates(const float* proj, int ld, int off_i, int off_f, const float* bias_i, const float* bias_f,
                                    float cap, int n_heads, float* max_state, const int* q_start, const int* req_rows,
-                                   int n_reqs, float* keep, float* take, float* maxima, hipStream_t stream) {
+                                   int n_reqs, float* keep, float* take, float* maxima, int as_log, hipStream_t stream) {
   LLMLAB_REQUIRE(n_reqs >= 0 && n_heads > 0 && n_heads <= 65535 && cap > 0.f && off_i >= 0 && off_f >= 0 &&
                      ld >= off_i + n_heads && ld >= off_f + n_heads,
                  "memory_gates: bad sizes requests=%d heads=%d cap=%g ld=%d", n_reqs, n_heads, (double)cap, ld);
   LLMLAB_REQUIRE(proj && max_state && q_start && req_rows && keep && take && maxima, "memory_gates: an operand is missing");
   if (n_reqs == 0) return 0;
   hipLaunchKernelGGL(memory_gates_kernel, dim3(n_reqs, n_heads), dim3(MEMORY_TILE), 0, stream, proj, ld, off_i, off_f, bias_i,
-                     bias_f, cap, n_heads, max_state, q_start, req_rows, keep, take, maxima);
+                     bias_f, cap, n_heads, max_state, q_start, req_rows, keep, take, maxima, as_log);
   LLMLAB_LAUNCH_CHECK("memory_gates");
   return 0;
 }
@@ -517,6 +524,360 @@ extern "C" int llmlab_gla_output(const float* parts, int rows, int n_heads, int 
   return 0;
 }
 
+
+// ------------------------------------------------------------------ chunks on the matrix cores
+// Long portions, all three kinds, as products of 64-row chunks (float32 matrix instructions,
+// v_mfma_f32_16x16x4_f32: 32-bit products and sums), in the same three passes as above:
+//   LOCAL   per chunk and head: L = sum_s diag(decays behind s) k_s v_s^T as one product [D x 64] [64 x E];
+//   carry   (gla_carry_kernel);
+//   FINISH  per chunk and head, a wave 16 rows t: o_t = (decayed q_t)^T S_start + sum_(s <= t) p_ts v_s with the
+//           pair weights p_ts = sum_d q_t[d] k_s[d] (product of the decays a_u[d], s < u <= t), then the head's
+//           norm, its gate and the rounding (the output kernel's work) while the outputs are in registers.
+// Products of decays are taken as 2^(difference of sums of logarithms).  A sum covers at most the 16
+// rows of a sub-block; across sub-blocks the sub-blocks' totals are added, so that the terms of a
+// difference stay small and every exponent is at most 0: nothing overflows, and the ratio of two
+// neighbours is exact to a few units of a sum over 16 rows.  Pairs in different sub-blocks: their
+// decays split at the later sub-block's start into a factor of k_s and a factor of q_t, and the weights
+// are a matrix product.  Pairs in one sub-block: a lane takes the row t = lane % 16 and four rows s and
+// walks the key channels.  MEMORY has one decay per head: all its weights are products q_t . k_s times a
+// number per pair, and the normaliser's n_t . q_t is their sum.
+// The weights are taken transposed (rows s, columns t): an accumulator then is the next product's operand,
+// lane (t, g) holding s = 4 g + r in register r.
+struct ChunkArgs {
+  const float* proj; int ld, off_q, off_k, off_v, off_g; float q_scale; int n_heads, D, E;
+  const float* logs;                              // log2 of the decays: [rows, heads, D], or (MEMORY) [rows, heads]
+  const float* take; const float* bonus;          // MEMORY: [rows, heads]; BONUS: [heads, D]
+  const int* q_start; int n_reqs;
+  float* chunk_state; float* chunk_decay; float* chunk_norm;
+  const float* w; float eps; int w_per_head, gate_kind, count; const float* maxima;
+};
+constexpr int CK = 64, SUB = 16;
+__device__ __forceinline__ float exp2_(float x) { return __builtin_amdgcn_exp2f(x); }
+
+__device__ __forceinline__ bool chunk_rows(const int* __restrict__ q_start, int n_reqs, int index, int& first, int& n) {
+  int before = 0;
+  for (int b = 0; b < n_reqs; ++b) {
+    const int lo = q_start[b], hi = q_start[b + 1], chunks = (hi - lo + CK - 1) / CK;
+    if (index < before + chunks) {
+      first = lo + (index - before) * CK;
+      n = hi - first < CK ? hi - first : CK;
+      return true;
+    }
+    before += chunks;
+  }
+  return false;
+}
+
+// The sums of the logs within each sub-block (inclusive) to s_lb[row * stride + d], the sub-blocks' totals to
+// s_tot[sub * width + d]; channels d < width (width 1: MEMORY's one number a row, log_ld numbers apart).
+// Rows past the chunk's end do not decay; channels from D to width are zeros.
+__device__ __forceinline__ void chunk_log_sums(const float* __restrict__ logs, size_t log_ld, int D, int width, int n,
+                                               float* s_lb, int stride, float* s_tot) {
+  for (int c = threadIdx.x; c < (CK / SUB) * width; c += blockDim.x) {
+    const int sub = c / width, d = c - sub * width;
+    float lg[SUB], sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < SUB; ++i) {
+      const int row = sub * SUB + i;
+      lg[i] = (row < n && d < D) ? logs[(size_t)row * log_ld + d] : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < SUB; ++i) {
+      sum += lg[i];
+      s_lb[(sub * SUB + i) * stride + d] = sum;
+    }
+    s_tot[sub * width + d] = sum;
+  }
+}
+
+template <int KIND, int ET>
+__global__ __launch_bounds__(256) void chunk_local_kernel(ChunkArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float chunk_lds[];
+  int first, n;
+  if (!chunk_rows(a.q_start, a.n_reqs, blockIdx.x, first, n)) return;
+  const int h = blockIdx.y, D = a.D, E = a.E, DK = (D + 15) & ~15;
+  const int width = KIND == KIND_MEMORY ? 1 : DK, stride = KIND == KIND_MEMORY ? 1 : DK + 4;
+  float* s_lb = chunk_lds;
+  float* s_tot = s_lb + CK * stride;
+  if (KIND == KIND_MEMORY) chunk_log_sums(a.logs + (size_t)first * a.n_heads + h, a.n_heads, 1, 1, n, s_lb, 1, s_tot);
+  else chunk_log_sums(a.logs + ((size_t)first * a.n_heads + h) * D, (size_t)a.n_heads * D, D, DK, n, s_lb, stride, s_tot);
+  __syncthreads();
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
+  const size_t at = (size_t)blockIdx.x * a.n_heads + h;
+  for (int dt = wave; dt * 16 < D; dt += 4) {
+    const int d = dt * 16 + c, dl = KIND == KIND_MEMORY ? 0 : d;
+    float after[4];                              // the totals behind each sub-block
+    after[3] = 0.f;
+#pragma unroll
+    for (int j = 2; j >= 0; --j) after[j] = after[j + 1] + s_tot[(j + 1) * width + dl];
+    floatx4 acc[ET];
+#pragma unroll
+    for (int et = 0; et < ET; ++et) acc[et] = floatx4{0.f, 0.f, 0.f, 0.f};
+    float n_sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (j * SUB >= n) break;
+      const float tail = s_tot[j * width + dl] + after[j];
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const int s = j * SUB + 4 * q + g;
+        const bool in = s < n && d < D;
+        const float* row = a.proj + (size_t)(first + (s < n ? s : n - 1)) * a.ld;      // (past the end: the last row, dropped)
+        float k = in ? row[a.off_k + h * D + d] : 0.f;
+        k *= exp2_(tail - s_lb[s * stride + dl]);
+        if (KIND == KIND_MEMORY) k *= s < n ? a.take[(size_t)(first + s) * a.n_heads + h] : 0.f;
+        n_sum += k;
+        const float* v = row + a.off_v + h * E;
+#pragma unroll
+        for (int et = 0; et < ET; ++et) {
+          const int e = 16 * et + c;
+          acc[et] = __builtin_amdgcn_mfma_f32_16x16x4f32(k, v[e < E ? e : E - 1], acc[et], 0, 0, 0);
+        }
+      }
+    }
+    float* out = a.chunk_state + at * D * E;
+#pragma unroll
+    for (int et = 0; et < ET; ++et)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = dt * 16 + 4 * g + r, e = 16 * et + c;
+        if (row < D && e < E) out[(size_t)row * E + e] = acc[et][r];
+      }
+    if (KIND == KIND_MEMORY) {
+      n_sum += __shfl_xor(n_sum, 16, WAVE);
+      n_sum += __shfl_xor(n_sum, 32, WAVE);
+      if (g == 0 && d < D) a.chunk_norm[at * D + d] = n_sum;
+    }
+    if (g == 0 && d < D) a.chunk_decay[at * D + d] = exp2_(s_tot[dl] + after[0]);
+  }
+}
+
+template <int KIND, int ET, typename T>
+__global__ __launch_bounds__(256) void chunk_finish_kernel(ChunkArgs a, T* __restrict__ out) {
+  extern __shared__ __attribute__((aligned(16))) float chunk_lds[];
+  int first, n;
+  if (!chunk_rows(a.q_start, a.n_reqs, blockIdx.x, first, n)) return;
+  const int h = blockIdx.y, D = a.D, E = a.E, DK = (D + 15) & ~15, DS = DK + 4;
+  const int width = KIND == KIND_MEMORY ? 1 : DK, stride = KIND == KIND_MEMORY ? 1 : DS;
+  float* s_q = chunk_lds;
+  float* s_k = s_q + CK * DS;
+  float* s_lb = s_k + CK * DS;
+  float* s_tot = s_lb + CK * stride;
+  for (int i = threadIdx.x; i < CK * DK; i += 256) {
+    const int row = i / DK, d = i - row * DK;
+    const bool in = row < n && d < D;
+    const float* p = a.proj + (size_t)(first + (row < n ? row : 0)) * a.ld + h * D + d;
+    s_q[row * DS + d] = in ? p[a.off_q] * a.q_scale : 0.f;
+    s_k[row * DS + d] = in ? p[a.off_k] : 0.f;
+  }
+  if (KIND == KIND_MEMORY) chunk_log_sums(a.logs + (size_t)first * a.n_heads + h, a.n_heads, 1, 1, n, s_lb, 1, s_tot);
+  else chunk_log_sums(a.logs + ((size_t)first * a.n_heads + h) * D, (size_t)a.n_heads * D, D, DK, n, s_lb, stride, s_tot);
+  __syncthreads();
+  const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
+  const int i0 = __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));      // this wave's sub-block
+  if (i0 * SUB >= n) return;                     // (no barrier behind this point)
+  const int t = i0 * SUB + c;                    // this lane's row (as a row of an operand)
+  const size_t at = (size_t)blockIdx.x * a.n_heads + h;
+  const float* q_t = s_q + t * DS;
+  // the sum of the logs from the sub-block's start that row t's outputs see (BONUS: up to the row before)
+  auto seen = [&](int d) {
+    if (KIND == KIND_BONUS) return c == 0 ? 0.f : s_lb[(t - 1) * stride + d];
+    return s_lb[t * stride + (KIND == KIND_MEMORY ? 0 : d)];
+  };
+  floatx4 acc[ET];
+#pragma unroll
+  for (int et = 0; et < ET; ++et) acc[et] = floatx4{0.f, 0.f, 0.f, 0.f};
+  float nq = 0.f;
+  // ---- what the state before the chunk gives
+  const float* S0 = a.chunk_state + at * D * E;
+  for (int kk = 0; kk < DK / 4; ++kk) {
+    const int d = 4 * kk + g, dl = KIND == KIND_MEMORY ? 0 : d;
+    float lg = seen(d);
+    for (int j = 0; j < i0; ++j) lg += s_tot[j * width + dl];
+    const float q = q_t[d] * exp2_(lg);
+    const float* srow = S0 + (size_t)(d < D ? d : D - 1) * E;      // (past the end: q is zero)
+    if (KIND == KIND_MEMORY) nq = fmaf(q, a.chunk_norm[at * D + (d < D ? d : D - 1)], nq);
+#pragma unroll
+    for (int et = 0; et < ET; ++et) {
+      const int e = 16 * et + c;
+      acc[et] = __builtin_amdgcn_mfma_f32_16x16x4f32(q, srow[e < E ? e : E - 1], acc[et], 0, 0, 0);
+    }
+  }
+  // ---- what the rows of the chunk up to each row give
+  for (int j = 0; j <= i0; ++j) {
+    floatx4 p = floatx4{0.f, 0.f, 0.f, 0.f};     // the weights of row t and the rows s = 16 j + 4 g + r
+    if (KIND == KIND_MEMORY) {
+      for (int kk = 0; kk < DK / 4; ++kk)
+        p = __builtin_amdgcn_mfma_f32_16x16x4f32(s_k[(j * SUB + c) * DS + 4 * kk + g], q_t[4 * kk + g], p, 0, 0, 0);
+      float between = 0.f;                       // from the end of s's sub-block on (or, in one sub-block, nothing)
+      for (int b = j + 1; b < i0; ++b) between += s_tot[b];
+      const float base = seen(0) + between + (j < i0 ? s_tot[j] : 0.f);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int s = j * SUB + 4 * g + r;
+        const float take = s < n ? a.take[(size_t)(first + s) * a.n_heads + h] : 0.f;
+        p[r] = s <= t ? p[r] * exp2_(fminf(base - s_lb[s], 0.f)) * take : 0.f;
+        nq += p[r];
+      }
+    } else if (j < i0) {
+      for (int kk = 0; kk < DK / 4; ++kk) {
+        const int d = 4 * kk + g;
+        float lg = s_tot[j * width + d] - s_lb[(j * SUB + c) * stride + d];
+        for (int b = j + 1; b < i0; ++b) lg += s_tot[b * width + d];
+        p = __builtin_amdgcn_mfma_f32_16x16x4f32(s_k[(j * SUB + c) * DS + d] * exp2_(lg), q_t[d] * exp2_(seen(d)), p, 0, 0, 0);
+      }
+    } else {
+      const int s0 = j * SUB + 4 * g;
+      for (int d = 0; d < DK; d += 4) {
+        const floatx4 q4 = *(const floatx4*)(q_t + d);
+        floatx4 see4;
+        if (KIND == KIND_BONUS && c == 0) see4 = floatx4{0.f, 0.f, 0.f, 0.f};
+        else see4 = *(const floatx4*)(s_lb + (KIND == KIND_BONUS ? t - 1 : t) * stride + d);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const floatx4 k4 = *(const floatx4*)(s_k + (s0 + r) * DS + d);
+          const floatx4 lb4 = *(const floatx4*)(s_lb + (s0 + r) * stride + d);
+#pragma unroll
+          for (int x = 0; x < 4; ++x) {
+            float f = exp2_(fminf(see4[x] - lb4[x], 0.f));
+            if (KIND == KIND_BONUS && s0 + r == t) f = d + x < D ? a.bonus[h * D + d + x] : 0.f;
+            p[r] = fmaf(q4[x] * k4[x], f, p[r]);
+          }
+        }
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (s0 + r > t) p[r] = 0.f;
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int s = j * SUB + 4 * g + r;
+      const float* v = a.proj + (size_t)(first + (s < n ? s : n - 1)) * a.ld + a.off_v + h * E;      // (past the end: the weight is zero)
+#pragma unroll
+      for (int et = 0; et < ET; ++et) {
+        const int e = 16 * et + c;
+        acc[et] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[r], v[e < E ? e : E - 1], acc[et], 0, 0, 0);
+      }
+    }
+  }
+  // ---- norm, gate, rounding: this lane now holds the columns 16 et + c of the rows 4 g + r
+  if (KIND == KIND_MEMORY) {
+    nq += __shfl_xor(nq, 16, WAVE);
+    nq += __shfl_xor(nq, 32, WAVE);
+  }
+  float inv[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int row = i0 * SUB + 4 * g + r;
+    if (KIND == KIND_MEMORY) {
+      const float size = memory_size(__shfl(nq, 4 * g + r, WAVE), a.maxima[(size_t)(first + (row < n ? row : n - 1)) * a.n_heads + h]);
+#pragma unroll
+      for (int et = 0; et < ET; ++et) acc[et][r] /= size;
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int et = 0; et < ET; ++et) ss = fmaf(acc[et][r], 16 * et + c < E ? acc[et][r] : 0.f, ss);
+#pragma unroll
+    for (int off = 8; off > 0; off >>= 1) ss += __shfl_xor(ss, off, WAVE);
+    inv[r] = 1.0f / sqrtf(ss / (float)a.count + a.eps);
+  }
+#pragma unroll
+  for (int et = 0; et < ET; ++et) {
+    const int e = 16 * et + c;
+    if (e >= E) break;
+    const float w = a.w[a.w_per_head ? h * E + e : e];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = i0 * SUB + 4 * g + r;
+      if (row >= n) break;
+      const float gate = a.proj[(size_t)(first + row) * a.ld + a.off_g + h * E + e];
+      const float sg = 1.0f / (1.0f + expf(-gate));
+      out[((size_t)(first + row) * a.n_heads + h) * E + e] =
+          from_float<T>(acc[et][r] * inv[r] * w * (a.gate_kind == 1 ? sg : gate * sg));
+    }
+  }
+}
+
+constexpr int CHUNK_MAX_D = 128, CHUNK_MAX_E = 256;
+extern "C" int llmlab_chunk_scan_takes(int D, int E) { return D > 0 && E > 0 && D <= CHUNK_MAX_D && E <= CHUNK_MAX_E; }
+extern "C" int llmlab_chunk_scan_rows() { return CK; }
+
+// From the projections and the logarithms of the decays to the gated outputs (as gla_scan and gla_output).
+// chunk_state [max_chunks, heads, D, E], chunk_decay and (memory) chunk_norm [max_chunks, heads, D], with
+// max_chunks >= rows / CK + n_reqs.
+extern "C" int llmlab_chunk_scan(const float* proj, int ld, int off_q, int off_k, int off_v, int off_g, float q_scale,
+                                 int n_heads, int D, int E, const float* logs, float* state, const int* q_start,
+                                 const int* req_rows, int n_reqs, int rows, int kind, const float* bonus, const float* take,
+                                 float* norm_state, const float* maxima, float* chunk_state, float* chunk_decay,
+                                 float* chunk_norm, int max_chunks, const float* w, float eps, int w_per_head, int gate_kind,
+                                 int norm_count, void* out, int dtype, hipStream_t stream) {
+  LLMLAB_REQUIRE(llmlab_chunk_scan_takes(D, E) && n_heads > 0 && n_heads <= 65535 && n_reqs >= 0 && n_reqs <= 65535 && rows >= 0,
+                 "chunk_scan: sizes D=%d E=%d heads=%d are not taken", D, E, n_heads);
+  LLMLAB_REQUIRE(ld >= off_q + n_heads * D && ld >= off_k + n_heads * D && ld >= off_v + n_heads * E &&
+                     ld >= off_g + n_heads * E && off_q >= 0 && off_k >= 0 && off_v >= 0 && off_g >= 0,
+                 "chunk_scan: rows of %d numbers do not hold the projections", ld);
+  LLMLAB_REQUIRE(proj && logs && state && q_start && req_rows && chunk_state && chunk_decay && w && out &&
+                     norm_count >= 0 && norm_count <= E && (gate_kind == 0 || gate_kind == 1) &&
+                     kind >= KIND_DECAY && kind <= KIND_MEMORY && (kind != KIND_BONUS || bonus) &&
+                     (kind != KIND_MEMORY || (take && norm_state && maxima && chunk_norm)),
+                 "chunk_scan: an operand of kind %d is missing", kind);
+  if (rows == 0 || n_reqs == 0) return 0;
+  const int chunks = rows / CK + n_reqs;
+  LLMLAB_REQUIRE(max_chunks >= chunks, "chunk_scan: %d rows of %d requests need room for %d chunks, got %d", rows, n_reqs,
+                 chunks, max_chunks);
+  const ChunkArgs a{proj, ld, off_q, off_k, off_v, off_g, q_scale, n_heads, D, E, logs, take, bonus, q_start, n_reqs,
+                    chunk_state, chunk_decay, chunk_norm, w, eps, w_per_head, gate_kind, norm_count > 0 ? norm_count : E,
+                    maxima};
+  const int DK = (D + 15) & ~15, et = (E + 15) / 16;
+  const size_t sums = kind == KIND_MEMORY ? CK + 4 : (size_t)CK * (DK + 4) + 4 * DK;
+  const size_t lds_local = sums * sizeof(float), lds_finish = (sums + 2 * (size_t)CK * (DK + 4)) * sizeof(float);
+  const dim3 grid(chunks, n_heads), block(256);
+  // (LDS beyond 64 KB is asked for once per kernel)
+#define LLMLAB_CHUNK_FINISH(KIND, ETV, T)                                                                                 \
+  do {                                                                                                                    \
+    static bool raised = false;                                                                                           \
+    if (lds_finish > 64 * 1024 && !raised) {                                                                              \
+      LLMLAB_REQUIRE(hipFuncSetAttribute((const void*)chunk_finish_kernel<KIND, ETV, T>,                                  \
+                                         hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024) == hipSuccess,          \
+                     "chunk_scan: no %zu bytes of LDS", lds_finish);                                                     \
+      raised = true;                                                                                                      \
+    }                                                                                                                     \
+    hipLaunchKernelGGL((chunk_finish_kernel<KIND, ETV, T>), grid, block, lds_finish, stream, a, (T*)out);                 \
+  } while (0)
+#define LLMLAB_CHUNK(KIND, ETV, PASS)                                                                            \
+  do {                                                                                                           \
+    if (PASS == 0) hipLaunchKernelGGL((chunk_local_kernel<KIND, ETV>), grid, block, lds_local, stream, a);        \
+    else if (dtype == DT_BF16) LLMLAB_CHUNK_FINISH(KIND, ETV, bf16_t);                                           \
+    else LLMLAB_CHUNK_FINISH(KIND, ETV, float);                                                                  \
+  } while (0)
+#define LLMLAB_CHUNK_ET(KIND, PASS)                 \
+  do {                                              \
+    if (et <= 2) LLMLAB_CHUNK(KIND, 2, PASS);       \
+    else if (et <= 4) LLMLAB_CHUNK(KIND, 4, PASS);  \
+    else if (et <= 8) LLMLAB_CHUNK(KIND, 8, PASS);  \
+    else LLMLAB_CHUNK(KIND, 16, PASS);              \
+  } while (0)
+#define LLMLAB_CHUNK_PASS(PASS)                                       \
+  do {                                                                \
+    if (kind == KIND_DECAY) LLMLAB_CHUNK_ET(KIND_DECAY, PASS);        \
+    else if (kind == KIND_BONUS) LLMLAB_CHUNK_ET(KIND_BONUS, PASS);   \
+    else LLMLAB_CHUNK_ET(KIND_MEMORY, PASS);                          \
+  } while (0)
+  LLMLAB_CHUNK_PASS(0);
+  ScanArgs carry{};
+  carry.n_heads = n_heads; carry.D = D; carry.E = E; carry.state = state; carry.q_start = q_start; carry.req_rows = req_rows;
+  carry.n_reqs = n_reqs; carry.chunk = CK; carry.chunk_state = chunk_state; carry.chunk_decay = chunk_decay;
+  carry.norm_state = kind == KIND_MEMORY ? norm_state : nullptr; carry.chunk_norm = chunk_norm;
+  const size_t per = (size_t)n_heads * D * E + (kind == KIND_MEMORY ? (size_t)n_heads * D : 0);
+  hipLaunchKernelGGL(gla_carry_kernel, dim3((unsigned)((per + 255) / 256), n_reqs), dim3(256), 0, stream, carry);
+  LLMLAB_CHUNK_PASS(1);
+#undef LLMLAB_CHUNK_PASS
+#undef LLMLAB_CHUNK_ET
+#undef LLMLAB_CHUNK
+#undef LLMLAB_CHUNK_FINISH
+  LLMLAB_LAUNCH_CHECK("chunk_scan");
+  return 0;
+}
 
 // ------------------------------------------------------------------ one row, whole
 // Decoding: every request brings ONE row.  A block takes a request's row for one head and does what

@@ -68,6 +68,9 @@ class DispatchRules:
     # most ``scan_max_chunk`` rows, shorter while that leaves fewer than ``scan_blocks_per_cu``
     # blocks to a compute unit.  2,048 rows, 7 heads of 64 x 128: 1.53 ms in one run, 0.17 ms in
     # chunks of 16 (the pass that joins 128 chunks takes 40 us of it), 0.13 ms in chunks of 64.
+    # From this many rows of a step's longest request on, heads of up to 128 key and 256 value channels
+    # go through the chunked scan on the matrix cores instead (0: never).
+    chunk_scan_min_rows: int = 32
     scan_min_chunk: int = 16
     scan_max_chunk: int = 64
     scan_blocks_per_cu: int = 1

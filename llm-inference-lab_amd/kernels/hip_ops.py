@@ -1170,9 +1170,19 @@ class HipOps:
                 lib.llmlab_poly_norm.restype = _c_int
             elif kind == "linear_attention":
                 lib.llmlab_gla_decay.argtypes = [_c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_float, _c_ptr,
-                                                 _c_int, _c_ptr]
+                                                 _c_int, _c_int, _c_ptr]
                 lib.llmlab_memory_gates.argtypes = [_c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_float, _c_int,
-                                                    _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr]
+                                                    _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int,
+                                                    _c_ptr]
+                lib.llmlab_chunk_scan_takes.argtypes = [_c_int, _c_int]
+                lib.llmlab_chunk_scan_takes.restype = _c_int
+                lib.llmlab_chunk_scan_rows.argtypes = []
+                lib.llmlab_chunk_scan_rows.restype = _c_int
+                lib.llmlab_chunk_scan.argtypes = [
+                    _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
+                    _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr,
+                    _c_float, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_ptr]
+                lib.llmlab_chunk_scan.restype = _c_int
                 lib.llmlab_memory_gates.restype = _c_int
                 lib.llmlab_gla_decay.restype = _c_int
                 lib.llmlab_recurrent_row_threads.argtypes = [_c_int, _c_int]
@@ -1654,9 +1664,10 @@ class HipOps:
 
     DECAY_KINDS = {"sigmoid": 0, "double_exp": 1}
 
-    def gla_decay(self, low, rank, w2, bias, tau, decay, kind: str = "sigmoid") -> None:
+    def gla_decay(self, low, rank, w2, bias, tau, decay, kind: str = "sigmoid", as_log: bool = False) -> None:
         """``decay[r, c] = sigmoid(bias[c] + w2[c] . low[r, :rank]) ** (1 / tau)``, all float32;
-        ``kind="double_exp"``: ``exp(-exp(bias[c] + w2[c] . tanh(low[r, :rank])))`` (no ``tau``)."""
+        ``kind="double_exp"``: ``exp(-exp(bias[c] + w2[c] . tanh(low[r, :rank])))`` (no ``tau``).  ``as_log``: the
+        decays' logarithms to the base 2 (at least -60), what ``chunk_scan`` takes."""
         lib = self._mixer_lib("linear_attention")
         for t, name in ((low, "low-rank projection"), (w2, "decay weight"), (decay, "decays")):
             self._need(t, name, torch.float32, contiguous=name != "low-rank projection")
@@ -1669,16 +1680,16 @@ class HipOps:
             if bias.numel() != channels:
                 raise ValueError("gla_decay: one bias per channel")
         self._call(lib.llmlab_gla_decay, self._ptr(low), low.stride(0), rows, int(rank), self._ptr(w2),
-                   self._ptr(bias), self.DECAY_KINDS[kind], float(tau), self._ptr(decay), channels, self._stream(),
-                   lib=lib)
+                   self._ptr(bias), self.DECAY_KINDS[kind], float(tau), self._ptr(decay), channels,
+                   1 if as_log else 0, self._stream(), lib=lib)
 
     def memory_gates(self, proj, off_i, off_f, bias_i, bias_f, cap: float, num_heads: int, max_state, q_start, req_rows,
-                     n_reqs, keep, take, maxima) -> None:
+                     n_reqs, keep, take, maxima, as_log: bool = False) -> None:
         """The gates of a matrix memory for the rows of every request: log gates ``i = cap * tanh((proj[:,
         off_i + h] + bias_i) / cap)`` and ``f = logsigmoid(cap * tanh((proj[:, off_f + h] + bias_f) / cap))``,
         the running maximum ``m_t = max(f_t + m_(t-1), i_t)`` from ``max_state [slots, heads]`` (left at the
         last row's), ``keep = exp(f_t + m_(t-1) - m_t)``, ``take = exp(i_t - m_t)`` and ``maxima = m_t``, each
-        ``[rows, heads]``; all float32."""
+        ``[rows, heads]``; all float32.  ``as_log``: ``keep``'s logarithm to the base 2 (at least -60) instead."""
         lib = self._mixer_lib("linear_attention")
         for t, name in ((proj, "projections"), (max_state, "maxima of the slots"), (keep, "keep"), (take, "take"),
                         (maxima, "maxima")):
@@ -1699,7 +1710,8 @@ class HipOps:
             raise ValueError("memory_gates: the operands do not fit each other")
         self._call(lib.llmlab_memory_gates, self._ptr(proj), proj.stride(0), int(off_i), int(off_f), self._ptr(bias_i),
                    self._ptr(bias_f), float(cap), num_heads, self._ptr(max_state), self._ptr(q_start), self._ptr(req_rows),
-                   int(n_reqs), self._ptr(keep), self._ptr(take), self._ptr(maxima), self._stream(), lib=lib)
+                   int(n_reqs), self._ptr(keep), self._ptr(take), self._ptr(maxima), 1 if as_log else 0, self._stream(),
+                   lib=lib)
 
     def gla_scan_chunk(self, rows: int, longest: int, num_heads: int, value_dim: int) -> int:
         """Into chunks of how many rows the scan cuts a step whose longest request brings
@@ -1816,6 +1828,60 @@ class HipOps:
                    float(eps), self._ptr(proj), proj.stride(0), int(off_gate), self._ptr(out), _dt(out),
                    int(parts.shape[2]), per_head, self.OUTPUT_GATES[gate], int(norm_count or 0), self._ptr(norm_parts),
                    self._ptr(maxima), self._stream(), lib=lib)
+
+    def chunk_scan_takes(self, longest: int, key_dim: int, value_dim: int) -> bool:
+        """Whether a step whose longest request brings ``longest`` rows goes through ``chunk_scan``."""
+        return bool(self.rules.chunk_scan_min_rows and longest >= self.rules.chunk_scan_min_rows
+                    and self._mixer_lib("linear_attention").llmlab_chunk_scan_takes(int(key_dim), int(value_dim)))
+
+    CHUNK_SCAN_ROWS = 64
+
+    def chunk_scan(self, proj, off_q, off_k, off_v, off_gate, q_scale, num_heads, key_dim, value_dim, logs, state, q_start,
+                   req_rows, n_reqs, chunk_state, chunk_decay, weight, eps, gate: str, norm_count: int, out, bonus=None,
+                   memory=None) -> None:
+        """What ``gla_scan`` and ``gla_output`` do, for long portions: every request's rows in chunks of 64 side
+        by side, as products on the matrix cores (float32).  ``logs``: the decays' logarithms to the base 2
+        (``as_log``), ``[rows, heads * key_dim]``, or, with ``memory = (take, norm_state, maxima, chunk_norm)``,
+        ``[rows, heads]``.  ``chunk_state [chunks, heads, key_dim, value_dim]``, ``chunk_decay`` and ``chunk_norm
+        [chunks, heads, key_dim]``: float32 scratch, ``chunks >= rows // 64 + n_reqs``."""
+        lib = self._mixer_lib("linear_attention")
+        for t, name in ((proj, "projections"), (logs, "log decays"), (state, "recurrent state"),
+                        (weight, "output norm weight"), (chunk_state, "chunk states"), (chunk_decay, "chunk decays")):
+            self._need(t, name, torch.float32)
+        self._need(q_start, "request row starts", torch.int32)
+        self._need(req_rows, "state slots", torch.int32)
+        self._need(out, "mixer output")
+        rows = proj.shape[0]
+        if (tuple(logs.shape) != (rows, num_heads * (key_dim if memory is None else 1))
+                or tuple(out.shape) != (rows, num_heads * value_dim)
+                or tuple(state.shape[1:]) != (num_heads, key_dim, value_dim)
+                or q_start.numel() < n_reqs + 1 or req_rows.numel() < n_reqs
+                or weight.numel() not in (value_dim, num_heads * value_dim)
+                or tuple(chunk_state.shape[1:]) != (num_heads, key_dim, value_dim)
+                or tuple(chunk_decay.shape) != (chunk_state.shape[0], num_heads, key_dim)
+                or chunk_state.shape[0] < rows // self.CHUNK_SCAN_ROWS + n_reqs):
+            raise ValueError("chunk_scan: the operands do not fit each other")
+        per_head = 1 if weight.numel() == num_heads * value_dim and num_heads > 1 else 0
+        kind = 2 if memory is not None else (1 if bonus is not None else 0)
+        take = norm_state = maxima = chunk_norm = None
+        if memory is not None:
+            take, norm_state, maxima, chunk_norm = memory
+            for t, name, shape in ((take, "take", (rows, num_heads)), (maxima, "maxima", (rows, num_heads)),
+                                   (norm_state, "normaliser", (state.shape[0], num_heads, key_dim)),
+                                   (chunk_norm, "chunk normalisers", tuple(chunk_decay.shape))):
+                self._need(t, name, torch.float32)
+                if tuple(t.shape) != shape:
+                    raise ValueError(f"chunk_scan: {name} is {tuple(t.shape)}, not {shape}")
+        if bonus is not None:
+            self._need(bonus, "bonus", torch.float32)
+            if bonus.numel() != num_heads * key_dim:
+                raise ValueError("chunk_scan: one bonus per head and key channel")
+        self._call(lib.llmlab_chunk_scan, self._ptr(proj), proj.stride(0), int(off_q), int(off_k), int(off_v), int(off_gate),
+                   float(q_scale), num_heads, key_dim, value_dim, self._ptr(logs), self._ptr(state), self._ptr(q_start),
+                   self._ptr(req_rows), int(n_reqs), rows, kind, self._ptr(bonus), self._ptr(take), self._ptr(norm_state),
+                   self._ptr(maxima), self._ptr(chunk_state), self._ptr(chunk_decay), self._ptr(chunk_norm),
+                   chunk_state.shape[0], self._ptr(weight), float(eps), per_head, self.OUTPUT_GATES[gate],
+                   int(norm_count or 0), self._ptr(out), _dt(out), self._stream(), lib=lib)
 
     RECURRENT_ROW_MAX_RANK = 512
 

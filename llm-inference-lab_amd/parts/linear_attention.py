@@ -94,9 +94,10 @@ class ScanMixer(Mixer):
         else:
             launch()
 
-    def _recur(self, proj, ctx, entry, off, weight, eps, gate, q_scale, many_rows, rank=0, **kind):
+    def _recur(self, proj, ctx, entry, off, weight, eps, gate, q_scale, many_rows, in_chunks, rank=0, **kind):
         """From the projections to the gated output ``[rows, heads * value_dim]`` (compute dtype).  Where every
-        request of the step brings one row and the sizes allow it: one launch; else ``many_rows()``.
+        request of the step brings one row and the sizes allow it: one launch; where some bring many:
+        ``in_chunks(out)``; else ``many_rows(out)``.
         ``off``: the columns of query, key, value and gate."""
         ops = self.ops
         mixed = ctx.scratch("linear_attention.out", (proj.shape[0], self.v_size), self.dtype)
@@ -104,14 +105,35 @@ class ScanMixer(Mixer):
         fits = takes is not None and takes(self.key_dim, self.value_dim, rank)
         count = self.file_value_dim if self.file_value_dim != self.value_dim else 0
 
-        def launch():        # (whether every request brings one row is not a matter of the number of rows)
+        def launch():        # (how many rows the requests bring is not a matter of the number of rows)
             if fits and ctx.n_rows == ctx.n_reqs:
                 ops.recurrent_row(proj, *off, q_scale, self.num_heads, self.key_dim, self.value_dim, entry.state["s"],
                                   ctx.all_q_start, ctx.all_req_rows, ctx.n_reqs, weight, eps, gate, count, mixed, **kind)
+                return
+            chunked = getattr(ops, "chunk_scan_takes", None)
+            if chunked is not None and chunked(ctx.max_q_len, self.key_dim, self.value_dim):
+                in_chunks(mixed)
             else:
                 many_rows(mixed)
         self._live(launch)
         return mixed
+
+    def _in_chunks(self, proj, ctx, entry, off, logs, weight, eps, gate, q_scale, mixed, bonus=None, memory=None):
+        """Long portions: chunks of rows side by side on the matrix cores, from the logarithms of the decays
+        to the gated output.  ``memory``: ``(take, maxima)``."""
+        heads, d, e = self.num_heads, self.key_dim, self.value_dim
+        most = proj.shape[0] // self.ops.CHUNK_SCAN_ROWS + ctx.max_reqs
+        chunk_state = ctx.scratch("linear_attention.chunk_state", (most, heads, d, e), torch.float32)
+        chunk_decay = ctx.scratch("linear_attention.chunk_decay", (most, heads, d), torch.float32)
+        kind = {}
+        if bonus is not None:
+            kind["bonus"] = bonus
+        if memory is not None:
+            chunk_norm = ctx.scratch("linear_attention.chunk_norm", (most, heads, d), torch.float32)
+            kind["memory"] = (memory[0], entry.state["n"], memory[1], chunk_norm)
+        self.ops.chunk_scan(proj, *off, q_scale, heads, d, e, logs, entry.state["s"], ctx.all_q_start, ctx.all_req_rows,
+                            ctx.n_reqs, chunk_state, chunk_decay, weight, eps, gate,
+                            self.file_value_dim if self.file_value_dim != self.value_dim else 0, mixed, **kind)
 
     def _output(self, parts, weight, eps, proj, off_gate, gate, mixed, **memory):
         if self.file_value_dim != self.value_dim:      # (the heads' norm is over the file's channels)
@@ -212,8 +234,12 @@ class GatedLinearAttention(ScanMixer):
             ops.gla_decay(proj[:, o["decay_down"]:], self.decay_rank, self.w_decay, self.b_decay, self.tau, decay)
             parts = self._scan(proj, *off[:3], decay, self.q_scale, entry.state["s"], ctx)
             self._output(parts, self.norm_weight, self.norm_eps, proj, off[3], "silu", mixed)
+
+        def in_chunks(mixed):
+            ops.gla_decay(proj[:, o["decay_down"]:], self.decay_rank, self.w_decay, self.b_decay, self.tau, decay, as_log=True)
+            self._in_chunks(proj, ctx, entry, off, decay, self.norm_weight, self.norm_eps, "silu", self.q_scale, mixed)
         mixed = self._recur(proj, ctx, entry, off, self.norm_weight, self.norm_eps, "silu", self.q_scale, many_rows,
-                            self.decay_rank,
+                            in_chunks, self.decay_rank,
                             decay=(o["decay_down"], self.decay_rank, self.w_decay, self.b_decay, "sigmoid", self.tau))
         ops.linear_logits(mixed, self.w_o, out)
 
@@ -483,7 +509,13 @@ class TimeMixAttention(ScanMixer):
             ops.gla_decay(proj[:, o["decay_down"]:], self.decay_rank, self.w_decay, self.b_decay, 1.0, decay, "double_exp")
             parts = self._scan(proj, *off[:3], decay, 1.0, entry.state["s"], ctx, bonus=self.bonus)
             self._output(parts, self.norm_weight, self.norm_eps, proj, off[3], self.gate, gated)
-        gated = self._recur(proj, ctx, entry, off, self.norm_weight, self.norm_eps, self.gate, 1.0, many_rows,
+
+        def in_chunks(gated):
+            ops.gla_decay(proj[:, o["decay_down"]:], self.decay_rank, self.w_decay, self.b_decay, 1.0, decay, "double_exp",
+                          as_log=True)
+            self._in_chunks(proj, ctx, entry, off, decay, self.norm_weight, self.norm_eps, self.gate, 1.0, gated,
+                            bonus=self.bonus)
+        gated = self._recur(proj, ctx, entry, off, self.norm_weight, self.norm_eps, self.gate, 1.0, many_rows, in_chunks,
                             self.decay_rank, bonus=self.bonus,
                             decay=(o["decay_down"], self.decay_rank, self.w_decay, self.b_decay, "double_exp", 1.0))
         ops.linear_logits(gated, self.w_o, out)
@@ -578,15 +610,23 @@ class MatrixMemoryAttention(ScanMixer):
                               for name in ("keep", "take", "maxima"))
         off = [o[role] for role in ("q_weight", "k_weight", "v_weight", "gate_weight")]
 
-        def many_rows(mixed):
+        def gates(**how):
             ops.memory_gates(proj, o["i_weight"], o["f_weight"], self.b_i, self.b_f, self.gate_cap, self.num_heads,
-                             entry.state["m"], ctx.all_q_start, ctx.all_req_rows, ctx.n_reqs, keep, take, maxima)
+                             entry.state["m"], ctx.all_q_start, ctx.all_req_rows, ctx.n_reqs, keep, take, maxima, **how)
+
+        def in_chunks(mixed):
+            gates(as_log=True)
+            self._in_chunks(proj, ctx, entry, off, keep, self.norm_weight, self.norm_eps, self.gate, self.q_scale, mixed,
+                            memory=(take, maxima))
+
+        def many_rows(mixed):
+            gates()
             parts, norm_parts = self._scan(proj, *off[:3], None, self.q_scale, entry.state["s"], ctx,
                                            memory=(keep, take, entry.state["n"]))
             self._output(parts, self.norm_weight, self.norm_eps, proj, off[3], self.gate, mixed, norm_parts=norm_parts,
                          maxima=maxima)
         mixed = self._recur(proj, ctx, entry, off, self.norm_weight, self.norm_eps, self.gate, self.q_scale, many_rows,
-                            memory=(o["i_weight"], o["f_weight"], self.b_i, self.b_f, self.gate_cap, entry.state["n"],
+                            in_chunks, memory=(o["i_weight"], o["f_weight"], self.b_i, self.b_f, self.gate_cap, entry.state["n"],
                                     entry.state["m"]))
         ops.linear_logits(mixed, self.w_o, out)
 
