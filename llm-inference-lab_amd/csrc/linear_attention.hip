@@ -10,6 +10,8 @@
 // Three kernels: the decays from their low-rank projection; the scan over the tokens of every
 // request of the step (prompts' portions and single decoded tokens alike); the output
 // (norm over each head's values, gate, rounding to the compute dtype).
+#include <type_traits>
+
 #include "common.h"
 
 extern "C" const char* llmlab_last_error() { return g_llmlab_error; }
@@ -80,7 +82,7 @@ extern "C" int llmlab_gla_decay(const float* low, int ld, int rows, int rank, co
 // row; the maxima of a tile by a scan over (sum of f, maximum so far) pairs, (F1, M1) then (F2, M2) =
 // (F1 + F2, max(M1 + F2, M2)).  Whatever rounding the scan adds to an m, keep and take of all rows
 // are taken from the same m's, so the state stays exact in them.
-constexpr int MEMORY_TILE = 256;
+constexpr int MEMORY_TILE = 1024;
 __global__ __launch_bounds__(MEMORY_TILE) void memory_gates_kernel(
     const float* __restrict__ proj, int ld, int off_i, int off_f, const float* __restrict__ bias_i,
     const float* __restrict__ bias_f, float cap, int n_heads, float* __restrict__ max_state, const int* __restrict__ q_start,
@@ -355,7 +357,9 @@ __global__ __launch_bounds__(THREADS) void gla_scan_kernel(ScanArgs a) {
 }
 
 // One thread per element (h, d, e) of a request's state, chunk after chunk:
-// chunk_state[c] <- the state before chunk c; the slot <- the state after the last chunk.
+// chunk_state[c] <- the state before chunk c; the slot <- the state after the last chunk.  The numbers of
+// CARRY_AHEAD chunks are asked for together.
+constexpr int CARRY_AHEAD = 8;
 __global__ __launch_bounds__(256) void gla_carry_kernel(ScanArgs a) {
   const int b = blockIdx.y;
   const size_t per = (size_t)a.n_heads * a.D * a.E;
@@ -369,11 +373,20 @@ __global__ __launch_bounds__(256) void gla_carry_kernel(ScanArgs a) {
     const int last = c + (a.q_start[b + 1] - a.q_start[b] + a.chunk - 1) / a.chunk;
     float* slot = a.norm_state + (size_t)a.req_rows[b] * hd_all + i;
     float N = *slot;
-    for (; c < last; ++c) {
-      float* l = a.chunk_norm + (size_t)c * hd_all + i;
-      const float built = *l;
-      *l = N;
-      N = fmaf(a.chunk_decay[(size_t)c * hd_all + i], N, built);
+    for (; c < last; c += CARRY_AHEAD) {
+      float built[CARRY_AHEAD], decay[CARRY_AHEAD];
+#pragma unroll
+      for (int x = 0; x < CARRY_AHEAD; ++x) {
+        const size_t at = (size_t)(c + x < last ? c + x : last - 1) * hd_all + i;
+        built[x] = a.chunk_norm[at];
+        decay[x] = a.chunk_decay[at];
+      }
+#pragma unroll
+      for (int x = 0; x < CARRY_AHEAD; ++x)
+        if (c + x < last) {
+          a.chunk_norm[(size_t)(c + x) * hd_all + i] = N;
+          N = fmaf(decay[x], N, built[x]);
+        }
     }
     *slot = N;
     return;
@@ -384,11 +397,20 @@ __global__ __launch_bounds__(256) void gla_carry_kernel(ScanArgs a) {
   float* slot = a.state + (size_t)a.req_rows[b] * per + i;
   float S = *slot;
   const size_t hd = i / a.E;
-  for (int c = before; c < before + n; ++c) {
-    float* l = a.chunk_state + (size_t)c * per + i;
-    const float built = *l;
-    *l = S;
-    S = fmaf(a.chunk_decay[(size_t)c * a.n_heads * a.D + hd], S, built);
+  for (int c = before; c < before + n; c += CARRY_AHEAD) {
+    float built[CARRY_AHEAD], decay[CARRY_AHEAD];
+#pragma unroll
+    for (int x = 0; x < CARRY_AHEAD; ++x) {      // (past the last: the last again, dropped)
+      const size_t at = (size_t)(c + x < before + n ? c + x : before + n - 1);
+      built[x] = a.chunk_state[at * per + i];
+      decay[x] = a.chunk_decay[at * a.n_heads * a.D + hd];
+    }
+#pragma unroll
+    for (int x = 0; x < CARRY_AHEAD; ++x)
+      if (c + x < before + n) {
+        a.chunk_state[(size_t)(c + x) * per + i] = S;
+        S = fmaf(decay[x], S, built[x]);
+      }
   }
   *slot = S;
 }
@@ -577,79 +599,139 @@ __device__ __forceinline__ void chunk_log_sums(const float* __restrict__ logs, s
     const int sub = c / width, d = c - sub * width;
     float lg[SUB], sum = 0.f;
 #pragma unroll
-    for (int i = 0; i < SUB; ++i) {
+    for (int i = 0; i < SUB; ++i) {              // (past the end: the last ones, set aside below; no load under a branch)
       const int row = sub * SUB + i;
-      lg[i] = (row < n && d < D) ? logs[(size_t)row * log_ld + d] : 0.f;
+      lg[i] = logs[(size_t)(row < n ? row : n - 1) * log_ld + (d < D ? d : D - 1)];
     }
 #pragma unroll
     for (int i = 0; i < SUB; ++i) {
-      sum += lg[i];
+      sum += (sub * SUB + i < n && d < D) ? lg[i] : 0.f;
       s_lb[(sub * SUB + i) * stride + d] = sum;
     }
     s_tot[sub * width + d] = sum;
   }
 }
 
-template <int KIND, int ET>
+// Operands of the products lie in LDS in rows of a multiple of 64 floats plus 16: the lanes (c, g) of a read
+// then are 16 consecutive numbers of four rows in all 64 banks.  Values and states pass through one buffer
+// SLAB columns at a time; a slab's numbers are asked for into registers while the products before it run.
+constexpr int SLAB = 64, SLAB_STRIDE = SLAB + 16;
+__host__ __device__ inline int product_stride(int columns) { return (columns + 63) / 64 * 64 + 16; }
+// the slab e0 .. of the chunk's values (this thread's 16 numbers: one row of 64 columns a wave at a time)
+__device__ __forceinline__ void fetch_values(const ChunkArgs& a, int first, int n, int h, int e0, float (&reg)[16]) {
+  const int e = e0 + (int)(threadIdx.x & 63), ec = e < a.E ? e : a.E - 1;
+#pragma unroll
+  for (int i = 0; i < 16; ++i) {
+    const int s = 4 * i + (int)(threadIdx.x >> 6);      // (past the end: the last row, which weighs nothing)
+    reg[i] = a.proj[(size_t)(first + (s < n ? s : n - 1)) * a.ld + a.off_v + h * a.E + ec];
+  }
+}
+__device__ __forceinline__ void stash_slab(float* buf, const float (&reg)[16], int row0) {
+#pragma unroll
+  for (int i = 0; i < 16; ++i) buf[(row0 + 4 * i + (int)(threadIdx.x >> 6)) * SLAB_STRIDE + (int)(threadIdx.x & 63)] = reg[i];
+}
+
+template <int KIND>
 __global__ __launch_bounds__(256) void chunk_local_kernel(ChunkArgs a) {
   extern __shared__ __attribute__((aligned(16))) float chunk_lds[];
   int first, n;
   if (!chunk_rows(a.q_start, a.n_reqs, blockIdx.x, first, n)) return;
-  const int h = blockIdx.y, D = a.D, E = a.E, DK = (D + 15) & ~15;
-  const int width = KIND == KIND_MEMORY ? 1 : DK, stride = KIND == KIND_MEMORY ? 1 : DK + 4;
-  float* s_lb = chunk_lds;
-  float* s_tot = s_lb + CK * stride;
-  if (KIND == KIND_MEMORY) chunk_log_sums(a.logs + (size_t)first * a.n_heads + h, a.n_heads, 1, 1, n, s_lb, 1, s_tot);
-  else chunk_log_sums(a.logs + ((size_t)first * a.n_heads + h) * D, (size_t)a.n_heads * D, D, DK, n, s_lb, stride, s_tot);
+  const int h = blockIdx.y, D = a.D, E = a.E, DK = (D + 15) & ~15, KS = product_stride(DK);
+  const int width = KIND == KIND_MEMORY ? 1 : DK;
+  float* s_k = chunk_lds;                        // the decayed keys [64][KS]
+  float* s_v = s_k + CK * KS;                    // a slab of the values [64][SLAB_STRIDE]
+  float* s_tot = s_v + CK * SLAB_STRIDE;         // totals of the sub-blocks' logs [4][width]
+  float* s_lb = s_tot + 4 * width;               // MEMORY: the sums of the logs and takes [64] [64]
+  float vreg[16];
+  fetch_values(a, first, n, h, 0, vreg);
+  constexpr int ITEMS = 2;                       // (sub-block, key channel) pairs a thread takes: D <= 128
+  float lb[KIND == KIND_MEMORY ? 1 : ITEMS][SUB], kk[ITEMS][SUB];
+#pragma unroll
+  for (int it = 0; it < ITEMS; ++it) {
+    const int item = threadIdx.x + 256 * it, sub = item / DK, d = item - sub * DK;
+    if (sub < 4) {
+      const int dc = d < D ? d : D - 1;
+#pragma unroll
+      for (int i = 0; i < SUB; ++i) {            // (rows past the end: the last one, set aside below)
+        const int row = sub * SUB + i, rc = first + (row < n ? row : n - 1);
+        kk[it][i] = a.proj[(size_t)rc * a.ld + a.off_k + h * D + dc];
+        if (KIND != KIND_MEMORY) lb[it][i] = a.logs[((size_t)rc * a.n_heads + h) * D + dc];
+      }
+      if (KIND != KIND_MEMORY) {
+        float sum = 0.f;
+#pragma unroll
+        for (int i = 0; i < SUB; ++i) {
+          sum += (sub * SUB + i < n && d < D) ? lb[it][i] : 0.f;
+          lb[it][i] = sum;
+        }
+        s_tot[sub * width + d] = sum;
+      }
+    }
+  }
+  if (KIND == KIND_MEMORY) {
+    chunk_log_sums(a.logs + (size_t)first * a.n_heads + h, a.n_heads, 1, 1, n, s_lb, 1, s_tot);
+    if (threadIdx.x < CK) s_lb[CK + threadIdx.x] = (int)threadIdx.x < n ? a.take[(size_t)(first + threadIdx.x) * a.n_heads + h] : 0.f;
+  }
+  __syncthreads();
+  const size_t at = (size_t)blockIdx.x * a.n_heads + h;
+#pragma unroll
+  for (int it = 0; it < ITEMS; ++it) {
+    const int item = threadIdx.x + 256 * it, sub = item / DK, d = item - sub * DK;
+    if (sub < 4) {
+      const int dl = KIND == KIND_MEMORY ? 0 : d;
+      float tail = s_tot[sub * width + dl];      // from the sub-block's start to the chunk's end
+      for (int b = sub + 1; b < 4; ++b) tail += s_tot[b * width + dl];
+#pragma unroll
+      for (int i = 0; i < SUB; ++i) {
+        const int row = sub * SUB + i;
+        float k = (row < n && d < D) ? kk[it][i] : 0.f;
+        if (KIND == KIND_MEMORY) k *= exp2_(tail - s_lb[row]) * s_lb[CK + row];
+        else k *= exp2_(tail - lb[it][i]);
+        s_k[row * KS + d] = k;
+      }
+      if (sub == 0 && d < D) a.chunk_decay[at * D + d] = exp2_(tail);
+    }
+  }
+  stash_slab(s_v, vreg, 0);
   __syncthreads();
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
-  const size_t at = (size_t)blockIdx.x * a.n_heads + h;
-  for (int dt = wave; dt * 16 < D; dt += 4) {
-    const int d = dt * 16 + c, dl = KIND == KIND_MEMORY ? 0 : d;
-    float after[4];                              // the totals behind each sub-block
-    after[3] = 0.f;
+  const int tiles = DK / 16, steps = (n + 15) >> 4 << 2;      // (four rows a step, steps in fours)
+  float* out = a.chunk_state + at * D * E;
+  for (int e0 = 0; e0 < E; e0 += SLAB) {
+    const bool more = e0 + SLAB < E;
+    if (more) fetch_values(a, first, n, h, e0 + SLAB, vreg);
+    for (int item = wave; item < 2 * tiles; item += 4) {      // a tile of 16 key channels x half the slab
+      const int dt = item >> 1, half = (item & 1) * 32;
+      if (e0 + half >= E) continue;
+      floatx4 acc[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
+      for (int q0 = 0; q0 < steps; q0 += 4)
 #pragma unroll
-    for (int j = 2; j >= 0; --j) after[j] = after[j + 1] + s_tot[(j + 1) * width + dl];
-    floatx4 acc[ET];
+      for (int u = 0; u < 4; ++u) {
+        const int q = q0 + u;
+        const float k = s_k[(4 * q + g) * KS + dt * 16 + c];
+        const float* v = s_v + (4 * q + g) * SLAB_STRIDE + half + c;
+        acc[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(k, v[0], acc[0], 0, 0, 0);
+        acc[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(k, v[16], acc[1], 0, 0, 0);
+      }
 #pragma unroll
-    for (int et = 0; et < ET; ++et) acc[et] = floatx4{0.f, 0.f, 0.f, 0.f};
-    float n_sum = 0.f;
+      for (int x = 0; x < 2; ++x)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      if (j * SUB >= n) break;
-      const float tail = s_tot[j * width + dl] + after[j];
-#pragma unroll
-      for (int q = 0; q < 4; ++q) {
-        const int s = j * SUB + 4 * q + g;
-        const bool in = s < n && d < D;
-        const float* row = a.proj + (size_t)(first + (s < n ? s : n - 1)) * a.ld;      // (past the end: the last row, dropped)
-        float k = in ? row[a.off_k + h * D + d] : 0.f;
-        k *= exp2_(tail - s_lb[s * stride + dl]);
-        if (KIND == KIND_MEMORY) k *= s < n ? a.take[(size_t)(first + s) * a.n_heads + h] : 0.f;
-        n_sum += k;
-        const float* v = row + a.off_v + h * E;
-#pragma unroll
-        for (int et = 0; et < ET; ++et) {
-          const int e = 16 * et + c;
-          acc[et] = __builtin_amdgcn_mfma_f32_16x16x4f32(k, v[e < E ? e : E - 1], acc[et], 0, 0, 0);
+        for (int r = 0; r < 4; ++r) {
+          const int row = dt * 16 + 4 * g + r, e = e0 + half + 16 * x + c;
+          if (row < D && e < E) out[(size_t)row * E + e] = acc[x][r];
         }
-      }
     }
-    float* out = a.chunk_state + at * D * E;
-#pragma unroll
-    for (int et = 0; et < ET; ++et)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int row = dt * 16 + 4 * g + r, e = 16 * et + c;
-        if (row < D && e < E) out[(size_t)row * E + e] = acc[et][r];
-      }
-    if (KIND == KIND_MEMORY) {
-      n_sum += __shfl_xor(n_sum, 16, WAVE);
-      n_sum += __shfl_xor(n_sum, 32, WAVE);
-      if (g == 0 && d < D) a.chunk_norm[at * D + d] = n_sum;
-    }
-    if (g == 0 && d < D) a.chunk_decay[at * D + d] = exp2_(s_tot[dl] + after[0]);
+    __syncthreads();
+    if (!more) break;
+    stash_slab(s_v, vreg, 0);
+    __syncthreads();
   }
+  if (KIND == KIND_MEMORY)
+    for (int d = threadIdx.x; d < D; d += 256) {
+      float sum = 0.f;
+      for (int s = 0; s < n; ++s) sum += s_k[s * KS + d];
+      a.chunk_norm[at * D + d] = sum;
+    }
 }
 
 template <int KIND, int ET, typename T>
@@ -663,68 +745,92 @@ __global__ __launch_bounds__(256) void chunk_finish_kernel(ChunkArgs a, T* __res
   float* s_k = s_q + CK * DS;
   float* s_lb = s_k + CK * DS;
   float* s_tot = s_lb + CK * stride;
-  for (int i = threadIdx.x; i < CK * DK; i += 256) {
+  float* s_one = s_tot + 4 * (width > 4 ? width : 4);      // BONUS: the bonus [DK]; MEMORY: the normaliser [DK], takes [64]
+  float* s_buf = s_one + DK + CK;                            // a slab of the state [DK] or of the values [64]
+  const size_t at = (size_t)blockIdx.x * a.n_heads + h;
+  const float* S0 = a.chunk_state + at * D * E;
+  // a slab of the state: 64 rows d a time, as many times as it takes
+  auto fetch_state = [&](int d0, int e0, float (&reg)[16]) {
+    const int e = e0 + (int)(threadIdx.x & 63), ec = e < E ? e : E - 1;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const int d = d0 + 4 * i + (int)(threadIdx.x >> 6);      // (past the end: the last row, which meets zeros)
+      reg[i] = S0[(size_t)(d < D ? d : D - 1) * E + ec];
+    }
+  };
+  float sreg[2][16], vreg[16];
+  fetch_state(0, 0, sreg[0]);
+  if (DK > 64) fetch_state(64, 0, sreg[1]);
+  for (int i0 = 0; i0 < CK * DK; i0 += 1024)
+#pragma unroll
+  for (int u = 0; u < 4; ++u) {                  // (CK * DK is a multiple of 1,024)
+    const int i = i0 + 256 * u + (int)threadIdx.x;
     const int row = i / DK, d = i - row * DK;
     const bool in = row < n && d < D;
-    const float* p = a.proj + (size_t)(first + (row < n ? row : 0)) * a.ld + h * D + d;
-    s_q[row * DS + d] = in ? p[a.off_q] * a.q_scale : 0.f;
-    s_k[row * DS + d] = in ? p[a.off_k] : 0.f;
+    const float* p = a.proj + (size_t)(first + (row < n ? row : n - 1)) * a.ld + h * D + (d < D ? d : D - 1);
+    const float q = p[a.off_q], k = p[a.off_k];
+    s_q[row * DS + d] = in ? q * a.q_scale : 0.f;
+    s_k[row * DS + d] = in ? k : 0.f;
   }
   if (KIND == KIND_MEMORY) chunk_log_sums(a.logs + (size_t)first * a.n_heads + h, a.n_heads, 1, 1, n, s_lb, 1, s_tot);
   else chunk_log_sums(a.logs + ((size_t)first * a.n_heads + h) * D, (size_t)a.n_heads * D, D, DK, n, s_lb, stride, s_tot);
+  if (KIND != KIND_DECAY)
+    for (int d = threadIdx.x; d < DK; d += 256) {
+      const int dc = d < D ? d : D - 1;
+      s_one[d] = d < D ? (KIND == KIND_BONUS ? a.bonus[h * D + dc] : a.chunk_norm[at * D + dc]) : 0.f;
+    }
+  if (KIND == KIND_MEMORY && threadIdx.x < CK) {
+    const int row = (int)threadIdx.x;
+    s_one[DK + row] = row < n ? a.take[(size_t)(first + row) * a.n_heads + h] : 0.f;
+  }
+  auto stash_state = [&]() {
+    stash_slab(s_buf, sreg[0], 0);
+    if (DK > 64) stash_slab(s_buf, sreg[1], 64);
+  };
+  stash_state();
   __syncthreads();
+  fetch_values(a, first, n, h, 0, vreg);
   const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
   const int i0 = __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));      // this wave's sub-block
-  if (i0 * SUB >= n) return;                     // (no barrier behind this point)
+  const bool busy = i0 * SUB < n;                // (a wave without rows takes part in the barriers only)
   const int t = i0 * SUB + c;                    // this lane's row (as a row of an operand)
-  const size_t at = (size_t)blockIdx.x * a.n_heads + h;
   const float* q_t = s_q + t * DS;
   // the sum of the logs from the sub-block's start that row t's outputs see (BONUS: up to the row before)
   auto seen = [&](int d) {
     if (KIND == KIND_BONUS) return c == 0 ? 0.f : s_lb[(t - 1) * stride + d];
     return s_lb[t * stride + (KIND == KIND_MEMORY ? 0 : d)];
   };
-  floatx4 acc[ET];
-#pragma unroll
-  for (int et = 0; et < ET; ++et) acc[et] = floatx4{0.f, 0.f, 0.f, 0.f};
+  // ---- the weights of row t and the rows s = 16 j + 4 g + r of the chunk
+  floatx4 p[4];
   float nq = 0.f;
-  // ---- what the state before the chunk gives
-  const float* S0 = a.chunk_state + at * D * E;
-  for (int kk = 0; kk < DK / 4; ++kk) {
-    const int d = 4 * kk + g, dl = KIND == KIND_MEMORY ? 0 : d;
-    float lg = seen(d);
-    for (int j = 0; j < i0; ++j) lg += s_tot[j * width + dl];
-    const float q = q_t[d] * exp2_(lg);
-    const float* srow = S0 + (size_t)(d < D ? d : D - 1) * E;      // (past the end: q is zero)
-    if (KIND == KIND_MEMORY) nq = fmaf(q, a.chunk_norm[at * D + (d < D ? d : D - 1)], nq);
 #pragma unroll
-    for (int et = 0; et < ET; ++et) {
-      const int e = 16 * et + c;
-      acc[et] = __builtin_amdgcn_mfma_f32_16x16x4f32(q, srow[e < E ? e : E - 1], acc[et], 0, 0, 0);
-    }
-  }
-  // ---- what the rows of the chunk up to each row give
-  for (int j = 0; j <= i0; ++j) {
-    floatx4 p = floatx4{0.f, 0.f, 0.f, 0.f};     // the weights of row t and the rows s = 16 j + 4 g + r
+  for (int j = 0; j < 4; ++j) {
+    p[j] = floatx4{0.f, 0.f, 0.f, 0.f};
+    if (!busy || j > i0) continue;
     if (KIND == KIND_MEMORY) {
-      for (int kk = 0; kk < DK / 4; ++kk)
-        p = __builtin_amdgcn_mfma_f32_16x16x4f32(s_k[(j * SUB + c) * DS + 4 * kk + g], q_t[4 * kk + g], p, 0, 0, 0);
+      for (int k0 = 0; k0 < DK; k0 += 16)
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          const int d = k0 + 4 * u + g;
+          p[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(s_k[(j * SUB + c) * DS + d], q_t[d], p[j], 0, 0, 0);
+        }
       float between = 0.f;                       // from the end of s's sub-block on (or, in one sub-block, nothing)
       for (int b = j + 1; b < i0; ++b) between += s_tot[b];
       const float base = seen(0) + between + (j < i0 ? s_tot[j] : 0.f);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int s = j * SUB + 4 * g + r;
-        const float take = s < n ? a.take[(size_t)(first + s) * a.n_heads + h] : 0.f;
-        p[r] = s <= t ? p[r] * exp2_(fminf(base - s_lb[s], 0.f)) * take : 0.f;
-        nq += p[r];
+        p[j][r] = s <= t ? p[j][r] * exp2_(fminf(base - s_lb[s], 0.f)) * s_one[DK + s] : 0.f;
+        nq += p[j][r];
       }
     } else if (j < i0) {
-      for (int kk = 0; kk < DK / 4; ++kk) {
-        const int d = 4 * kk + g;
+      for (int k0 = 0; k0 < DK; k0 += 16)
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int d = k0 + 4 * u + g;
         float lg = s_tot[j * width + d] - s_lb[(j * SUB + c) * stride + d];
         for (int b = j + 1; b < i0; ++b) lg += s_tot[b * width + d];
-        p = __builtin_amdgcn_mfma_f32_16x16x4f32(s_k[(j * SUB + c) * DS + d] * exp2_(lg), q_t[d] * exp2_(seen(d)), p, 0, 0, 0);
+        p[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(s_k[(j * SUB + c) * DS + d] * exp2_(lg), q_t[d] * exp2_(seen(d)), p[j], 0, 0, 0);
       }
     } else {
       const int s0 = j * SUB + 4 * g;
@@ -738,29 +844,90 @@ __global__ __launch_bounds__(256) void chunk_finish_kernel(ChunkArgs a, T* __res
           const floatx4 k4 = *(const floatx4*)(s_k + (s0 + r) * DS + d);
           const floatx4 lb4 = *(const floatx4*)(s_lb + (s0 + r) * stride + d);
 #pragma unroll
-          for (int x = 0; x < 4; ++x) {
-            float f = exp2_(fminf(see4[x] - lb4[x], 0.f));
-            if (KIND == KIND_BONUS && s0 + r == t) f = d + x < D ? a.bonus[h * D + d + x] : 0.f;
-            p[r] = fmaf(q4[x] * k4[x], f, p[r]);
-          }
+          for (int x = 0; x < 4; ++x) p[j][r] = fmaf(q4[x] * k4[x], exp2_(fminf(see4[x] - lb4[x], 0.f)), p[j][r]);
         }
       }
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        if (s0 + r > t) p[r] = 0.f;
-    }
+        if (s0 + r > t || (KIND == KIND_BONUS && s0 + r == t)) p[j][r] = 0.f;
+      if (KIND == KIND_BONUS) {                  // the row itself, through the bonus: a quarter of the channels a lane
+        float own = 0.f;
+        for (int d = g; d < DK; d += 4) own = fmaf(q_t[d] * s_k[t * DS + d], s_one[d], own);
+        own += __shfl_xor(own, 16, WAVE);
+        own += __shfl_xor(own, 32, WAVE);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int s = j * SUB + 4 * g + r;
-      const float* v = a.proj + (size_t)(first + (s < n ? s : n - 1)) * a.ld + a.off_v + h * E;      // (past the end: the weight is zero)
-#pragma unroll
-      for (int et = 0; et < ET; ++et) {
-        const int e = 16 * et + c;
-        acc[et] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[r], v[e < E ? e : E - 1], acc[et], 0, 0, 0);
+        for (int r = 0; r < 4; ++r)
+          if (s0 + r == t) p[j][r] = own;
       }
     }
   }
+  // ---- slab by slab: what the state before the chunk gives, and what the chunk's rows give
+  floatx4 acc[ET];
+#pragma unroll
+  for (int et = 0; et < ET; ++et) acc[et] = floatx4{0.f, 0.f, 0.f, 0.f};
+  auto slab = [&](auto number) {                 // (returns whether there is another one behind it)
+    constexpr int TILES = ET < 4 ? ET : 4, X0 = 4 * decltype(number)::value, e0 = 16 * X0;
+    const bool more = X0 + 4 < ET && e0 + SLAB < E;
+    if (busy) {
+      for (int k0 = 0; k0 < DK; k0 += 16)
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int d = k0 + 4 * u + g, dl = KIND == KIND_MEMORY ? 0 : d;
+        float lg = seen(d);
+        for (int j = 0; j < i0; ++j) lg += s_tot[j * width + dl];
+        const float q = q_t[d] * exp2_(lg);
+        if (KIND == KIND_MEMORY && e0 == 0) nq = fmaf(q, s_one[d], nq);
+        const float* srow = s_buf + d * SLAB_STRIDE + c;
+#pragma unroll
+        for (int x = 0; x < TILES; ++x)
+          acc[X0 + x] = __builtin_amdgcn_mfma_f32_16x16x4f32(q, srow[16 * x], acc[X0 + x], 0, 0, 0);
+      }
+    }
+    __syncthreads();
+    stash_slab(s_buf, vreg, 0);
+    __syncthreads();
+    if (more) {
+      fetch_state(0, e0 + SLAB, sreg[0]);
+      if (DK > 64) fetch_state(64, e0 + SLAB, sreg[1]);
+    }
+    if (busy) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        if (j > i0) continue;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float* v = s_buf + (j * SUB + 4 * g + r) * SLAB_STRIDE + c;
+#pragma unroll
+          for (int x = 0; x < TILES; ++x)
+            acc[X0 + x] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[j][r], v[16 * x], acc[X0 + x], 0, 0, 0);
+        }
+      }
+    }
+    if (!more) return false;
+    __syncthreads();
+    stash_state();
+    __syncthreads();
+    fetch_values(a, first, n, h, e0 + SLAB, vreg);
+    return true;
+  };
+  bool again = slab(std::integral_constant<int, 0>{});
+  if constexpr (ET > 4) again = again && slab(std::integral_constant<int, 1>{});
+  if constexpr (ET > 8) again = again && slab(std::integral_constant<int, 2>{});
+  if constexpr (ET > 12) again = again && slab(std::integral_constant<int, 3>{});
+  if (!busy) return;
   // ---- norm, gate, rounding: this lane now holds the columns 16 et + c of the rows 4 g + r
+  // (all gates and weights are asked for together; past the end the last ones, dropped)
+  float gates[ET][4], ws[ET];
+#pragma unroll
+  for (int et = 0; et < ET; ++et) {
+    const int e = 16 * et + c < E ? 16 * et + c : E - 1;
+    ws[et] = a.w[a.w_per_head ? h * E + e : e];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = i0 * SUB + 4 * g + r;
+      gates[et][r] = a.proj[(size_t)(first + (row < n ? row : n - 1)) * a.ld + a.off_g + h * E + e];
+    }
+  }
   if (KIND == KIND_MEMORY) {
     nq += __shfl_xor(nq, 16, WAVE);
     nq += __shfl_xor(nq, 32, WAVE);
@@ -784,21 +951,18 @@ __global__ __launch_bounds__(256) void chunk_finish_kernel(ChunkArgs a, T* __res
 #pragma unroll
   for (int et = 0; et < ET; ++et) {
     const int e = 16 * et + c;
-    if (e >= E) break;
-    const float w = a.w[a.w_per_head ? h * E + e : e];
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int row = i0 * SUB + 4 * g + r;
-      if (row >= n) break;
-      const float gate = a.proj[(size_t)(first + row) * a.ld + a.off_g + h * E + e];
+      const float gate = gates[et][r];
       const float sg = 1.0f / (1.0f + expf(-gate));
-      out[((size_t)(first + row) * a.n_heads + h) * E + e] =
-          from_float<T>(acc[et][r] * inv[r] * w * (a.gate_kind == 1 ? sg : gate * sg));
+      const T y = from_float<T>(acc[et][r] * inv[r] * ws[et] * (a.gate_kind == 1 ? sg : gate * sg));
+      if (row < n && e < E) out[((size_t)(first + row) * a.n_heads + h) * E + e] = y;
     }
   }
 }
 
-constexpr int CHUNK_MAX_D = 128, CHUNK_MAX_E = 256;
+constexpr int CHUNK_MAX_D = 128, CHUNK_MAX_E = 256, CHUNK_MAX_LDS = 152 * 1024;
 extern "C" int llmlab_chunk_scan_takes(int D, int E) { return D > 0 && E > 0 && D <= CHUNK_MAX_D && E <= CHUNK_MAX_E; }
 extern "C" int llmlab_chunk_scan_rows() { return CK; }
 
@@ -829,52 +993,61 @@ extern "C" int llmlab_chunk_scan(const float* proj, int ld, int off_q, int off_k
                     chunk_state, chunk_decay, chunk_norm, w, eps, w_per_head, gate_kind, norm_count > 0 ? norm_count : E,
                     maxima};
   const int DK = (D + 15) & ~15, et = (E + 15) / 16;
-  const size_t sums = kind == KIND_MEMORY ? CK + 4 : (size_t)CK * (DK + 4) + 4 * DK;
-  const size_t lds_local = sums * sizeof(float), lds_finish = (sums + 2 * (size_t)CK * (DK + 4)) * sizeof(float);
+  const size_t lds_local = ((size_t)CK * product_stride(DK) + (size_t)CK * SLAB_STRIDE + 4 * DK + 2 * CK) * sizeof(float);
+  const size_t lds_finish = ((size_t)(kind == KIND_MEMORY ? 2 : 3) * CK * (DK + 4) + CK + 4 * DK + 16 +
+                             DK + (DK > CK ? 2 * CK : CK) * SLAB_STRIDE) * sizeof(float);
   const dim3 grid(chunks, n_heads), block(256);
   // (LDS beyond 64 KB is asked for once per kernel)
-#define LLMLAB_CHUNK_FINISH(KIND, ETV, T)                                                                                 \
+#define LLMLAB_CHUNK_LDS(KERNEL, BYTES)                                                                                   \
   do {                                                                                                                    \
     static bool raised = false;                                                                                           \
-    if (lds_finish > 64 * 1024 && !raised) {                                                                              \
-      LLMLAB_REQUIRE(hipFuncSetAttribute((const void*)chunk_finish_kernel<KIND, ETV, T>,                                  \
-                                         hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024) == hipSuccess,          \
-                     "chunk_scan: no %zu bytes of LDS", lds_finish);                                                     \
+    if ((BYTES) > 64 * 1024 && !raised) {                                                                                 \
+      LLMLAB_REQUIRE(hipFuncSetAttribute((const void*)KERNEL, hipFuncAttributeMaxDynamicSharedMemorySize,                 \
+                                         CHUNK_MAX_LDS) == hipSuccess, "chunk_scan: no %zu bytes of LDS", (size_t)(BYTES)); \
       raised = true;                                                                                                      \
     }                                                                                                                     \
-    hipLaunchKernelGGL((chunk_finish_kernel<KIND, ETV, T>), grid, block, lds_finish, stream, a, (T*)out);                 \
   } while (0)
-#define LLMLAB_CHUNK(KIND, ETV, PASS)                                                                            \
+#define LLMLAB_CHUNK_FINISH(KIND, ETV, T)                                                                                 \
+  do {                                                                                                                    \
+    auto kernel = chunk_finish_kernel<KIND, ETV, T>;                                                                      \
+    LLMLAB_CHUNK_LDS(kernel, lds_finish);                                                                                 \
+    hipLaunchKernelGGL(kernel, grid, block, lds_finish, stream, a, (T*)out);                                              \
+  } while (0)
+#define LLMLAB_CHUNK_LOCAL(KIND)                                              \
+  do {                                                                        \
+    auto kernel = chunk_local_kernel<KIND>;                                   \
+    LLMLAB_CHUNK_LDS(kernel, lds_local);                                      \
+    hipLaunchKernelGGL(kernel, grid, block, lds_local, stream, a);            \
+  } while (0)
+#define LLMLAB_CHUNK(KIND, ETV)                                                                                  \
   do {                                                                                                           \
-    if (PASS == 0) hipLaunchKernelGGL((chunk_local_kernel<KIND, ETV>), grid, block, lds_local, stream, a);        \
-    else if (dtype == DT_BF16) LLMLAB_CHUNK_FINISH(KIND, ETV, bf16_t);                                           \
+    if (dtype == DT_BF16) LLMLAB_CHUNK_FINISH(KIND, ETV, bf16_t);                                           \
     else LLMLAB_CHUNK_FINISH(KIND, ETV, float);                                                                  \
   } while (0)
-#define LLMLAB_CHUNK_ET(KIND, PASS)                 \
-  do {                                              \
-    if (et <= 2) LLMLAB_CHUNK(KIND, 2, PASS);       \
-    else if (et <= 4) LLMLAB_CHUNK(KIND, 4, PASS);  \
-    else if (et <= 8) LLMLAB_CHUNK(KIND, 8, PASS);  \
-    else LLMLAB_CHUNK(KIND, 16, PASS);              \
+#define LLMLAB_CHUNK_ET(KIND)                 \
+  do {                                        \
+    if (et <= 2) LLMLAB_CHUNK(KIND, 2);       \
+    else if (et <= 4) LLMLAB_CHUNK(KIND, 4);  \
+    else if (et <= 8) LLMLAB_CHUNK(KIND, 8);  \
+    else LLMLAB_CHUNK(KIND, 16);              \
   } while (0)
-#define LLMLAB_CHUNK_PASS(PASS)                                       \
-  do {                                                                \
-    if (kind == KIND_DECAY) LLMLAB_CHUNK_ET(KIND_DECAY, PASS);        \
-    else if (kind == KIND_BONUS) LLMLAB_CHUNK_ET(KIND_BONUS, PASS);   \
-    else LLMLAB_CHUNK_ET(KIND_MEMORY, PASS);                          \
-  } while (0)
-  LLMLAB_CHUNK_PASS(0);
+  if (kind == KIND_DECAY) LLMLAB_CHUNK_LOCAL(KIND_DECAY);
+  else if (kind == KIND_BONUS) LLMLAB_CHUNK_LOCAL(KIND_BONUS);
+  else LLMLAB_CHUNK_LOCAL(KIND_MEMORY);
   ScanArgs carry{};
   carry.n_heads = n_heads; carry.D = D; carry.E = E; carry.state = state; carry.q_start = q_start; carry.req_rows = req_rows;
   carry.n_reqs = n_reqs; carry.chunk = CK; carry.chunk_state = chunk_state; carry.chunk_decay = chunk_decay;
   carry.norm_state = kind == KIND_MEMORY ? norm_state : nullptr; carry.chunk_norm = chunk_norm;
   const size_t per = (size_t)n_heads * D * E + (kind == KIND_MEMORY ? (size_t)n_heads * D : 0);
   hipLaunchKernelGGL(gla_carry_kernel, dim3((unsigned)((per + 255) / 256), n_reqs), dim3(256), 0, stream, carry);
-  LLMLAB_CHUNK_PASS(1);
-#undef LLMLAB_CHUNK_PASS
+  if (kind == KIND_DECAY) LLMLAB_CHUNK_ET(KIND_DECAY);
+  else if (kind == KIND_BONUS) LLMLAB_CHUNK_ET(KIND_BONUS);
+  else LLMLAB_CHUNK_ET(KIND_MEMORY);
 #undef LLMLAB_CHUNK_ET
 #undef LLMLAB_CHUNK
+#undef LLMLAB_CHUNK_LOCAL
 #undef LLMLAB_CHUNK_FINISH
+#undef LLMLAB_CHUNK_LDS
   LLMLAB_LAUNCH_CHECK("chunk_scan");
   return 0;
 }
