@@ -56,7 +56,7 @@ class EmuRecord:
 class EmuOps:
     # the operations that do work on tensors: written down while a part is recorded, as the
     # product's kernel set writes down its calls into the kernel libraries
-    RECORDED = ("shift_mix", "poly_norm", "normed_sum", "project_conv_write", "segmented_products", "memory_gates", "recurrent_row",
+    RECORDED = ("shift_mix", "poly_norm", "normed_sum", "project_conv_write", "segmented_products", "memory_gates", "recurrent_row", "chunk_scan",
                 "embed", "gather_tokens", "rmsnorm", "linear", "linear_relu2", "linear_residual", "linear_partials",
                 "add_pending", "linear_logits", "linear_swiglu", "fused_norm_qkv", "qkv_rope_cache",
                 "fused_norm_swiglu", "fused_norm_logits", "rope_inplace", "rope_kv_write",
@@ -482,6 +482,29 @@ class EmuOps:
         for s, (member, at) in enumerate(zip(w.members, offsets)):
             out[:, at:at + member.shape[0]] = x[s].float() @ member.float().t()
 
+    CHUNK_SCAN_ROWS = 64
+
+    def chunk_scan_takes(self, longest, key_dim, value_dim):
+        return longest >= 32 and key_dim != 24      # (both ways are exercised)
+
+    def chunk_scan(self, proj, off_q, off_k, off_v, off_gate, q_scale, num_heads, key_dim, value_dim, logs, state, q_start,
+                   req_rows, n_reqs, chunk_state, chunk_decay, weight, eps, gate, norm_count, out, bonus=None, memory=None):
+        """(The recurrence row by row; the chunks are how the kernel spreads the work.)"""
+        self._count("chunk_scan")
+        rows = proj.shape[0]
+        assert chunk_state.shape[0] >= rows // self.CHUNK_SCAN_ROWS + n_reqs and chunk_decay.shape[0] == chunk_state.shape[0]
+        parts = torch.zeros(rows, num_heads, self.gla_slices(key_dim), value_dim)
+        decay, kind, norm = torch.exp2(logs), {}, {}
+        if memory is not None:
+            take, norm_state, maxima, _ = memory
+            norm = dict(norm_parts=torch.zeros(rows, num_heads, parts.shape[2]), maxima=maxima)
+            kind, decay = dict(memory=(decay, take, norm_state, norm["norm_parts"], None)), None
+        elif bonus is not None:
+            kind = dict(bonus=bonus)
+        self.gla_scan(proj, off_q, off_k, off_v, decay, q_scale, num_heads, key_dim, value_dim, state, q_start, req_rows, n_reqs,
+                      parts, **kind)
+        self.gla_output(parts, num_heads, key_dim, value_dim, weight, eps, proj, off_gate, out, gate, norm_count, **norm)
+
     def recurrent_row_takes(self, key_dim, value_dim, rank=0):
         return key_dim * value_dim <= 1024 or key_dim % 3 == 0      # (both ways are exercised)
 
@@ -533,17 +556,17 @@ class EmuOps:
     def gla_slices(self, key_dim):
         return (key_dim + self.SCAN_SLICE - 1) // self.SCAN_SLICE
 
-    def gla_decay(self, low, rank, w2, bias, tau, decay, kind="sigmoid"):
+    def gla_decay(self, low, rank, w2, bias, tau, decay, kind="sigmoid", as_log=False):
         self._count("gla_decay")
         x = low[:, :rank].float()
         z = (torch.tanh(x) if kind == "double_exp" else x) @ w2.float().t()
         if bias is not None:
             z = z + bias.float()
-        decay.copy_(torch.exp(-torch.exp(z)) if kind == "double_exp"
-                    else torch.exp(torch.nn.functional.logsigmoid(z) / tau))
+        log = -torch.exp(z) if kind == "double_exp" else torch.nn.functional.logsigmoid(z) / tau
+        decay.copy_(torch.clamp(log / math.log(2.0), min=-60.0) if as_log else torch.exp(log))
 
     def memory_gates(self, proj, off_i, off_f, bias_i, bias_f, cap, num_heads, max_state, q_start, req_rows, n_reqs, keep,
-                     take, maxima):
+                     take, maxima, as_log=False):
         self._count("memory_gates")
         z = lambda at, b: cap * torch.tanh((proj[:, at:at + num_heads] + (0.0 if b is None else b)) / cap)
         i, f = z(off_i, bias_i), torch.nn.functional.logsigmoid(z(off_f, bias_f))
@@ -551,7 +574,9 @@ class EmuOps:
             m = max_state[int(req_rows[b])]
             for t in range(int(q_start[b]), int(q_start[b + 1])):
                 new = torch.maximum(f[t] + m, i[t])
-                keep[t], take[t], maxima[t] = torch.exp(f[t] + m - new), torch.exp(i[t] - new), new
+                log = f[t] + m - new
+                keep[t] = torch.clamp(log / math.log(2.0), min=-60.0) if as_log else torch.exp(log)
+                take[t], maxima[t] = torch.exp(i[t] - new), new
                 m.copy_(new)
 
     def gla_scan_chunk(self, rows, longest, num_heads, value_dim):
