@@ -114,6 +114,53 @@ def test_page_need_bounds_what_a_request_ever_holds():
                     assert need == pages_for_tokens(500, page)
 
 
+def chunked(chunk, pages=64, page_size=16, keep_first=0, max_seq_len=1024):
+    spec = CacheSpec((("k", PageTensor((1, 16), 1)),), chunk=chunk, keep_first=keep_first)
+    return CacheManager([GroupLayout(spec, [0], pages)], page_size, 2, max_seq_len, {}, torch.float32, "cpu")
+
+
+@pytest.mark.parametrize("chunk", [1, 5, 16, 24, 40, 64, 100])
+def test_chunks_give_back_the_pages_they_have_passed(chunk):
+    """A group whose layers read the current chunk of positions only: after every step it holds the pages
+    from the next position's chunk on, and never more than the admission arithmetic says."""
+    for page in (16, 64):
+        for step in (1, 7, 48):
+            m = chunked(chunk, page_size=page)
+            a = m.admit("a")
+            need, worst = m.page_need(500, step)[0], 0
+            while a.computed_len < 500:
+                m.reserve(a, min(step, 500 - a.computed_len))
+                worst = max(worst, sum(p >= 0 for p in a.pages[0]))
+                m.commit(a)
+                held = [lp for lp, p in enumerate(a.pages[0]) if p >= 0]
+                first = min(a.computed_len // chunk * chunk // page, len(a.pages[0]))
+                assert held == list(range(first, len(a.pages[0]))), (a.computed_len, held)
+                m.check()
+            assert worst <= need, (page, step, worst, need)
+            m.release(a)
+            assert m.free_pages(0) == 64
+
+
+def test_a_chunk_stands_in_place_of_a_window():
+    tensors = (("k", PageTensor((1, 16), 1)),)
+    with pytest.raises(ValueError):
+        CacheSpec(tensors, window=8, chunk=8)
+    with pytest.raises(ValueError):
+        CacheSpec(tensors, chunk=0)
+    a = CacheSpec(tensors, chunk=8)
+    assert a.bounded and a.reach == 8 and [a.lowest_read(p) for p in (0, 7, 8, 20)] == [0, 0, 8, 16]
+    # a reader with chunks of another size, or with a window: everything is kept
+    assert a.widened_by(CacheSpec(tensors, chunk=8)).chunk == 8
+    for other in (CacheSpec(tensors, chunk=6), CacheSpec(tensors, window=4), CacheSpec(tensors)):
+        assert not a.widened_by(other).bounded
+    m = chunked(24, keep_first=20)
+    r = m.admit("a")
+    for _ in range(10):
+        m.reserve(r, 16)
+        m.commit(r)
+    assert [lp for lp, p in enumerate(r.pages[0]) if p >= 0][:2] == [0, 1]        # the kept first positions' pages
+
+
 @pytest.mark.parametrize("seed", range(8))
 def test_random_orders_keep_every_invariant(seed):
     rng = random.Random(seed)
