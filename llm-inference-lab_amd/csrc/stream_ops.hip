@@ -535,24 +535,25 @@ extern "C" int llmlab_scaled_sum(float* out, const float* y1, float a, const flo
 // sqrt(mean(s^2) + add_eps) * add_w, and (copy not null) copy[r] = T(the new row).  One block a row, all
 // float32; a thread keeps up to NORM_ADD_KEEP of the row's numbers, wider rows are read again.
 template <typename T, bool ADD>
-__global__ __launch_bounds__(256) void normed_sum_kernel(float* __restrict__ out, const float* __restrict__ y1,
+__global__ __launch_bounds__(1024) void normed_sum_kernel(float* __restrict__ out, const float* __restrict__ y1,
                                                          const float* __restrict__ w1, float a, const float* __restrict__ y2,
                                                          const float* __restrict__ w2, float b, float eps, int width,
                                                          const float* __restrict__ add_w, float add_eps,
                                                          T* __restrict__ copy) {
   __shared__ float red1[17], red2[17], red3[17];
+  const int threads = blockDim.x;
   const size_t row = (size_t)blockIdx.x * width;
   float k1[NORM_ADD_KEEP], k2[NORM_ADD_KEEP];
   float s1 = 0.f, s2 = 0.f;
 #pragma unroll
   for (int n = 0; n < NORM_ADD_KEEP; ++n) {
-    const int c = threadIdx.x + 256 * n;
+    const int c = threadIdx.x + threads * n;
     k1[n] = c < width ? y1[row + c] : 0.f;
     k2[n] = c < width ? y2[row + c] : 0.f;
     s1 = fmaf(k1[n], k1[n], s1);
     s2 = fmaf(k2[n], k2[n], s2);
   }
-  for (int c = threadIdx.x + 256 * NORM_ADD_KEEP; c < width; c += 256) {
+  for (int c = threadIdx.x + threads * NORM_ADD_KEEP; c < width; c += threads) {
     const float v1 = y1[row + c], v2 = y2[row + c];
     s1 = fmaf(v1, v1, s1);
     s2 = fmaf(v2, v2, s2);
@@ -562,14 +563,14 @@ __global__ __launch_bounds__(256) void normed_sum_kernel(float* __restrict__ out
   float ss = 0.f;
 #pragma unroll
   for (int n = 0; n < NORM_ADD_KEEP; ++n) {
-    const int c = threadIdx.x + 256 * n;
+    const int c = threadIdx.x + threads * n;
     if (c < width) {
       k1[n] = k1[n] * i1 * w1[c] + k2[n] * i2 * w2[c];
       if (!ADD) out[row + c] = k1[n];
       ss = fmaf(k1[n], k1[n], ss);
     }
   }
-  for (int c = threadIdx.x + 256 * NORM_ADD_KEEP; c < width; c += 256) {
+  for (int c = threadIdx.x + threads * NORM_ADD_KEEP; c < width; c += threads) {
     const float v = y1[row + c] * i1 * w1[c] + y2[row + c] * i2 * w2[c];
     if (!ADD) out[row + c] = v;
     ss = fmaf(v, v, ss);
@@ -583,10 +584,10 @@ __global__ __launch_bounds__(256) void normed_sum_kernel(float* __restrict__ out
   };
 #pragma unroll
   for (int n = 0; n < NORM_ADD_KEEP; ++n) {
-    const int c = threadIdx.x + 256 * n;
+    const int c = threadIdx.x + threads * n;
     if (c < width) add(c, k1[n]);
   }
-  for (int c = threadIdx.x + 256 * NORM_ADD_KEEP; c < width; c += 256)
+  for (int c = threadIdx.x + threads * NORM_ADD_KEEP; c < width; c += threads)
     add(c, y1[row + c] * i1 * w1[c] + y2[row + c] * i2 * w2[c]);
 }
 
@@ -597,8 +598,10 @@ extern "C" int llmlab_normed_sum(float* out, const float* y1, const float* w1, f
                  width);
   LLMLAB_REQUIRE(copy == nullptr || add_w, "normed_sum: a copy is the stream's, so the sum goes into the stream");
   if (rows == 0) return 0;
+  // few wide rows: more threads, so that a row is one trip to memory
+  const int threads = rows <= 64 && width > 1024 ? 1024 : 256;
 #define LLMLAB_NORMED_SUM(T, ADD)                                                                                          \
-  hipLaunchKernelGGL((normed_sum_kernel<T, ADD>), dim3(rows), dim3(256), 0, stream, out, y1, w1, a, y2, w2, b, eps, width, \
+  hipLaunchKernelGGL((normed_sum_kernel<T, ADD>), dim3(rows), dim3(threads), 0, stream, out, y1, w1, a, y2, w2, b, eps, width, \
                      add_w, add_eps, (T*)copy)
   if (!add_w) LLMLAB_NORMED_SUM(float, false);
   else if (copy && copy_dtype == DT_BF16) LLMLAB_NORMED_SUM(bf16_t, true);
@@ -624,8 +627,8 @@ __device__ __forceinline__ void store4(bf16_t* p, floatx4 v) {
   *(bf16x4*)p = bf16x4{(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
 }
 
-template <typename TI, typename TO, bool VEC>
-__global__ __launch_bounds__(256) void shift_mix_kernel(const TI* __restrict__ h, const float* __restrict__ mix, int n_mix,
+template <typename TI, typename TO, bool VEC, int MIXES>      // MIXES 0: any number, from the arguments
+__global__ __launch_bounds__(1024) void shift_mix_kernel(const TI* __restrict__ h, const float* __restrict__ mix, int n_mix,
                                                         TI* __restrict__ state, const int* __restrict__ row_req,
                                                         const int* __restrict__ q_start, const int* __restrict__ req_rows,
                                                         TO* __restrict__ out, size_t out_stride, int width) {
@@ -638,8 +641,16 @@ __global__ __launch_bounds__(256) void shift_mix_kernel(const TI* __restrict__ h
   if (VEC) {
     for (int c = threadIdx.x * 4; c < width; c += blockDim.x * 4) {
       const floatx4 own = load4(own_row + c), d = load4(before + c) - own;
-      for (int m = 0; m < n_mix; ++m)
-        store4(out + m * out_stride + (size_t)r * width + c, own + d * load4(mix + (size_t)m * width + c));
+      if (MIXES > 0) {
+        floatx4 w[MIXES > 0 ? MIXES : 1];
+#pragma unroll
+        for (int m = 0; m < MIXES; ++m) w[m] = load4(mix + (size_t)m * width + c);
+#pragma unroll
+        for (int m = 0; m < MIXES; ++m) store4(out + m * out_stride + (size_t)r * width + c, own + d * w[m]);
+      } else {
+        for (int m = 0; m < n_mix; ++m)
+          store4(out + m * out_stride + (size_t)r * width + c, own + d * load4(mix + (size_t)m * width + c));
+      }
       if (lead) store4(st + c, load4(latest + c));
     }
   } else {
@@ -660,13 +671,18 @@ extern "C" int llmlab_shift_mix(const void* h, int h_dtype, const float* mix, in
   if (rows == 0) return 0;
   const bool vec = width % 4 == 0 && (((uintptr_t)h | (uintptr_t)mix | (uintptr_t)state | (uintptr_t)out) & 15) == 0;
   const size_t stride = (size_t)rows * width;
-#define LLMLAB_SHIFT(TI, TO, VEC)                                                                                          \
-  hipLaunchKernelGGL((shift_mix_kernel<TI, TO, VEC>), dim3(rows), dim3(256), 0, stream, (const TI*)h, mix, n_mix,         \
-                     (TI*)state, row_req, q_start, req_rows, (TO*)out, stride, width)
-#define LLMLAB_SHIFT_ANY(TI, TO)        \
-  do {                                  \
-    if (vec) LLMLAB_SHIFT(TI, TO, true); \
-    else LLMLAB_SHIFT(TI, TO, false);   \
+  // few rows: a thread four channels up to a block's 1,024 threads; many rows: blocks of 256
+  int threads = 256;
+  if (rows <= 64 && width > 1024) threads = width >= 4096 ? 1024 : (width / 4 + 63) / 64 * 64;
+#define LLMLAB_SHIFT(TI, TO, VEC, MIXES)                                                                                  \
+  hipLaunchKernelGGL((shift_mix_kernel<TI, TO, VEC, MIXES>), dim3(rows), dim3(threads), 0, stream, (const TI*)h, mix,     \
+                     n_mix, (TI*)state, row_req, q_start, req_rows, (TO*)out, stride, width)
+#define LLMLAB_SHIFT_ANY(TI, TO)                            \
+  do {                                                      \
+    if (vec && n_mix == 1) LLMLAB_SHIFT(TI, TO, true, 1);   \
+    else if (vec && n_mix == 5) LLMLAB_SHIFT(TI, TO, true, 5); \
+    else if (vec) LLMLAB_SHIFT(TI, TO, true, 0);            \
+    else LLMLAB_SHIFT(TI, TO, false, 0);                    \
   } while (0)
   if (h_dtype == DT_F32 && out_dtype == DT_F32) LLMLAB_SHIFT_ANY(float, float);
   else if (h_dtype == DT_F32) LLMLAB_SHIFT_ANY(float, bf16_t);

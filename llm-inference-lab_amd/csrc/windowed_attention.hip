@@ -191,7 +191,7 @@ extern "C" int llmlab_project_rotate_write(const float* proj, int ld, int rows, 
 // The same for layers whose projections pass a short causal convolution, turn, and are brought to
 // unit root mean square head by head.  proj[r, :] = q | k | v (float32 sums; heads of D, D and E
 // channels).  Channel by channel: `bias` is added (null: none); with taps > 0 the convolution over
-// the positions of the row's request, y_t = sum_j w[c, j] u_(t - taps + 1 + j), u the biased
+// the positions of the row's request, y_t = sum_j w[j, c] u_(t - taps + 1 + j), u the biased
 // projection, inputs from before the step from state [slots, taps - 1, channels] float32 (zeros before
 // a sequence's start).  Of every query and key head the first rot_dims channels turn by positions[r] *
 // freq[i]: channel i with i + rot_dims / 2, or (neighbours) channel 2i with 2i + 1.  unit: the head is
@@ -209,19 +209,80 @@ struct ConvArgs {
 };
 
 constexpr int CONV_LDS_FLOATS = 12288;      // channels of a group of heads in LDS
+constexpr int CONV_BLOCK_CHANNELS = 512;    // channels of a block of several rows (its other heads: other blocks)
+
+// first channel of head h in [queries | keys | values] (h one past the last: the number of channels)
+__device__ __forceinline__ int conv_first_channel(const ConvArgs& a, int h) {
+  const int turned = a.n_heads + a.n_kv;
+  return h <= turned ? h * a.D : turned * a.D + (h - turned) * a.E;
+}
+
+// A wave's work on head h of row r, its channels ready in LDS: rotation, unit norm, the query's row
+// or the page's.
+template <typename T>
+__device__ __forceinline__ void conv_head(const ConvArgs& a, int h, int r, int page, int slot, const float* s_head,
+                                          const float* s_cos, const float* s_sin, int lane, T* __restrict__ q_out,
+                                          T* __restrict__ k_cache, T* __restrict__ v_cache) {
+  const int D = a.D, E = a.E, half = a.rot_dims >> 1;
+  if (h < a.n_heads + a.n_kv) {
+    auto turned = [&](int d) {
+      float x = s_head[d];
+      if (d < a.rot_dims) {
+        const int i = a.neighbours ? d >> 1 : (d < half ? d : d - half);
+        const bool first = a.neighbours ? (d & 1) == 0 : d < half;
+        const float other = s_head[a.neighbours ? d ^ 1 : (first ? d + half : d - half)];
+        x = first ? x * s_cos[i] - other * s_sin[i] : x * s_cos[i] + other * s_sin[i];
+      }
+      return x;
+    };
+    T* dst = h < a.n_heads ? q_out + ((size_t)r * a.n_heads + h) * a.DK
+                           : k_cache + (((size_t)page * a.n_kv + (h - a.n_heads)) * a.page_size + slot) * a.DK;
+    constexpr int HELD = 2;                     // heads of this many times 64 channels stay in registers
+    if (a.DK <= 64 * HELD) {
+      float x[HELD], ss = 0.f;
+#pragma unroll
+      for (int n = 0; n < HELD; ++n) {
+        const int d = lane + 64 * n;
+        x[n] = d < D ? turned(d) : 0.f;
+        ss = fmaf(x[n], x[n], ss);
+      }
+      const float inv = a.unit ? 1.0f / sqrtf(wave_sum(ss) / (float)D + a.eps) : 1.f;
+#pragma unroll
+      for (int n = 0; n < HELD; ++n)
+        if (lane + 64 * n < a.DK) dst[lane + 64 * n] = from_float<T>(x[n] * inv);
+      return;
+    }
+    float inv = 1.f;
+    if (a.unit) {
+      float ss = 0.f;
+      for (int d = lane; d < D; d += 64) {
+        const float x = turned(d);
+        ss = fmaf(x, x, ss);
+      }
+      inv = 1.0f / sqrtf(wave_sum(ss) / (float)D + a.eps);
+    }
+    for (int d = lane; d < a.DK; d += 64) dst[d] = from_float<T>(d < D ? turned(d) * inv : 0.f);
+  } else {
+    const int g = h - a.n_heads - a.n_kv;
+    for (int e = lane; e < E; e += 64)
+      v_cache[((size_t)page * a.n_kv + g) * a.page_size * E + value_index(slot, e, E)] = from_float<T>(s_head[e]);
+  }
+}
+
 template <typename T, int TAPS, int PER>    // TAPS 0: any number, from the arguments
 __global__ __launch_bounds__(1024) void project_conv_write_kernel(ConvArgs a, T* __restrict__ q_out,
                                                                   T* __restrict__ k_cache, T* __restrict__ v_cache) {
   extern __shared__ float conv_lds[];           // cos [half], sin [half], then the group's channels
-  const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
-  const int half = a.rot_dims >> 1, D = a.D, E = a.E, taps = TAPS > 0 ? TAPS : a.taps, keep = taps - 1;
+  const int r = blockIdx.x, lane = threadIdx.x & 63, waves = blockDim.x >> 6;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int half = a.rot_dims >> 1, taps = TAPS > 0 ? TAPS : a.taps, keep = taps - 1;
   float* s_cos = conv_lds;
   float* s_sin = conv_lds + half;
   float* s_row = conv_lds + 2 * half;
   const float* src = a.proj + (size_t)r * a.ld;
   const int pos = a.positions[r], b = a.row_req[r];
   const int inside = r - a.q_start[b];          // rows of this request before r in the step
-  const int q_size = a.n_heads * D, k_size = a.n_kv * D, channels = q_size + k_size + a.n_kv * E;
+  const int channels = (a.n_heads + a.n_kv) * a.D + a.n_kv * a.E;
   float* st = keep > 0 ? a.state + (size_t)a.req_rows[b] * keep * channels : nullptr;
   for (int i = threadIdx.x; i < half; i += blockDim.x) {
     float sn, cs;
@@ -232,12 +293,9 @@ __global__ __launch_bounds__(1024) void project_conv_write_kernel(ConvArgs a, T*
   const int page = a.table[(size_t)b * a.max_pages + pos / a.page_size];
   const int slot = pos % a.page_size;
   const int heads = a.n_heads + 2 * a.n_kv;     // query heads, key heads, value heads
-  auto first_channel = [&](int h) {             // of head h (h == heads: the number of channels)
-    return h <= a.n_heads + a.n_kv ? h * D : q_size + k_size + (h - a.n_heads - a.n_kv) * E;
-  };
   for (int h0 = 0; h0 < heads; h0 += a.group) {
     const int h1 = h0 + a.group < heads ? h0 + a.group : heads;
-    const int c_lo = first_channel(h0), c_hi = first_channel(h1);
+    const int c_lo = conv_first_channel(a, h0), c_hi = conv_first_channel(a, h1);
     if (TAPS > 0) {
       constexpr int K = TAPS > 1 ? TAPS - 1 : 1;
       for (int c0 = c_lo + (int)threadIdx.x; c0 < c_hi; c0 += blockDim.x * PER) {
@@ -248,7 +306,7 @@ __global__ __launch_bounds__(1024) void project_conv_write_kernel(ConvArgs a, T*
           own[i] = src[c];
           bias[i] = a.bias ? a.bias[c] : 0.f;
 #pragma unroll
-          for (int j = 0; j < TAPS; ++j) w[i][j] = a.w[(size_t)c * TAPS + j];
+          for (int j = 0; j < TAPS; ++j) w[i][j] = a.w[(size_t)j * channels + c];
 #pragma unroll
           for (int j = 0; j < TAPS - 1; ++j) {
             const int back = TAPS - 1 - j;
@@ -281,13 +339,13 @@ __global__ __launch_bounds__(1024) void project_conv_write_kernel(ConvArgs a, T*
         const float bias = a.bias ? a.bias[c] : 0.f, own = src[c] + bias;
         float acc = own;
         if (taps > 0) {
-          const float* w = a.w + (size_t)c * taps;
-          acc = w[keep] * own;
+          const float* w = a.w + c;               // (tap j: channels numbers further on each)
+          acc = w[(size_t)keep * channels] * own;
           for (int j = 0; j < keep; ++j) {
             const int back = keep - j;
             const float u = back <= inside ? src[c - (ptrdiff_t)back * a.ld] + bias
                                            : st[(size_t)(keep - (back - inside)) * channels + c];
-            acc = fmaf(w[j], u, acc);
+            acc = fmaf(w[(size_t)j * channels], u, acc);
           }
           if (a.own_state && keep > 0) {
             for (int j = 0; j + 1 < keep; ++j) st[(size_t)j * channels + c] = st[(size_t)(j + 1) * channels + c];
@@ -298,51 +356,89 @@ __global__ __launch_bounds__(1024) void project_conv_write_kernel(ConvArgs a, T*
       }
     }
     __syncthreads();
-    for (int h = h0 + wave; h < h1; h += waves) {
-      const float* s_head = s_row + (first_channel(h) - c_lo);
-      if (h < a.n_heads + a.n_kv) {
-        auto turned = [&](int d) {
-          float x = s_head[d];
-          if (d < a.rot_dims) {
-            const int i = a.neighbours ? d >> 1 : (d < half ? d : d - half);
-            const bool first = a.neighbours ? (d & 1) == 0 : d < half;
-            const float other = s_head[a.neighbours ? d ^ 1 : (first ? d + half : d - half)];
-            x = first ? x * s_cos[i] - other * s_sin[i] : x * s_cos[i] + other * s_sin[i];
-          }
-          return x;
-        };
-        float inv = 1.f;
-        if (a.unit) {
-          float ss = 0.f;
-          for (int d = lane; d < D; d += 64) {
-            const float x = turned(d);
-            ss = fmaf(x, x, ss);
-          }
-          inv = 1.0f / sqrtf(wave_sum(ss) / (float)D + a.eps);
-        }
-        T* dst = h < a.n_heads ? q_out + ((size_t)r * a.n_heads + h) * a.DK
-                               : k_cache + (((size_t)page * a.n_kv + (h - a.n_heads)) * a.page_size + slot) * a.DK;
-        for (int d = lane; d < a.DK; d += 64) dst[d] = from_float<T>(d < D ? turned(d) * inv : 0.f);
-      } else {
-        const int g = h - a.n_heads - a.n_kv;
-        for (int e = lane; e < E; e += 64)
-          v_cache[((size_t)page * a.n_kv + g) * a.page_size * E + value_index(slot, e, E)] = from_float<T>(s_head[e]);
-      }
-    }
+    for (int h = h0 + wave; h < h1; h += waves)
+      conv_head(a, h, r, page, slot, s_row + (conv_first_channel(a, h) - c_lo), s_cos, s_sin, lane, q_out, k_cache, v_cache);
     __syncthreads();
   }
 }
 
+// Long portions: a block takes a group of heads of ROWS rows that follow each other and a thread a
+// channel of all of them, so that taps, bias and the rows before are read once for ROWS rows.
+// Rows near the start of a request (of which the block may hold several) take their earlier inputs
+// from its slot.
+template <typename T, int TAPS, int ROWS>
+__global__ __launch_bounds__(256) void project_conv_rows_kernel(ConvArgs a, int rows, T* __restrict__ q_out,
+                                                                T* __restrict__ k_cache, T* __restrict__ v_cache) {
+  extern __shared__ float conv_lds[];           // per row: cos [half], sin [half]; then the group's channels
+  constexpr int K = TAPS - 1;
+  const int r0 = blockIdx.x * ROWS, lane = threadIdx.x & 63, waves = blockDim.x >> 6;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int half = a.rot_dims >> 1;
+  float* s_row = conv_lds + ROWS * 2 * half;
+  const int own = wave % ROWS;                  // a wave works on the heads of one row
+  const float* s_cos = conv_lds + own * 2 * half;
+  const int own_row = min(r0 + own, rows - 1), pos = a.positions[own_row];
+  const int page = a.table[(size_t)a.row_req[own_row] * a.max_pages + pos / a.page_size], slot = pos % a.page_size;
+  const int channels = (a.n_heads + a.n_kv) * a.D + a.n_kv * a.E;
+  int inside[ROWS];                             // (rows past the end: the last row again, not written)
+  bool whole = true;                            // every earlier input is a row of the step
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    const int r = min(r0 + i, rows - 1);
+    inside[i] = r - a.q_start[a.row_req[r]];
+    whole = whole && inside[i] >= K;
+  }
+  for (int n = threadIdx.x; n < ROWS * half; n += blockDim.x) {
+    const int i = n / half, f = n - i * half;
+    float sn, cs;
+    sincosf((float)a.positions[min(r0 + i, rows - 1)] * a.freq[f], &sn, &cs);
+    conv_lds[i * 2 * half + f] = cs;
+    conv_lds[i * 2 * half + half + f] = sn;
+  }
+  const int heads = a.n_heads + 2 * a.n_kv, h0 = blockIdx.y * a.group, h1 = min(h0 + a.group, heads);
+  const int c_lo = conv_first_channel(a, h0), c_hi = conv_first_channel(a, h1), wide = c_hi - c_lo;
+  for (int c = c_lo + (int)threadIdx.x; c < c_hi; c += blockDim.x) {
+    const float bias = a.bias ? a.bias[c] : 0.f;
+    float w[TAPS], u[K + ROWS];                 // u[K + i]: row i; u[0 .. K): the rows before the block
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[j] = a.w[(size_t)j * channels + c];
+#pragma unroll
+    for (int i = 0; i < K + ROWS; ++i) u[i] = a.proj[(size_t)min(max(r0 + i - K, 0), rows - 1) * a.ld + c];
+#pragma unroll
+    for (int i = 0; i < K + ROWS; ++i) u[i] += bias;
+#pragma unroll
+    for (int i = 0; i < ROWS; ++i) {
+      float acc = 0.f;
+#pragma unroll
+      for (int j = 0; j < K; ++j) {
+        float x = u[i + j];
+        if (!whole && K - j > inside[i]) {
+          const int b = a.row_req[min(r0 + i, rows - 1)];
+          x = a.state[((size_t)a.req_rows[b] * K + (K - (K - j - inside[i]))) * channels + c];
+        }
+        acc = fmaf(w[j], x, acc);
+      }
+      s_row[i * wide + c - c_lo] = fmaf(w[K], u[K + i], acc);
+    }
+  }
+  __syncthreads();
+  if (r0 + own < rows)
+    for (int h = h0 + wave / ROWS; h < h1; h += waves / ROWS)
+      conv_head(a, h, r0 + own, page, slot, s_row + own * wide + conv_first_channel(a, h) - c_lo, s_cos, s_cos + half, lane,
+                q_out, k_cache, v_cache);
+}
+
 // The slots after the step: the last taps - 1 inputs (biased projections) of every request.  The
-// block of a request's first row does it for the request; a thread reads place n + s before it
-// writes place s, in rising order, so nothing is read after it changed.
-__global__ __launch_bounds__(256) void conv_slots_kernel(ConvArgs a) {
-  const int r = blockIdx.x, b = a.row_req[r], first = a.q_start[b];
-  if (r != first) return;
+// step's description holds room for more requests than a step has: a place whose first row does not name
+// it back is none.  A thread reads place n + s before it writes place s, in rising order, so nothing
+// is read after it changed.
+__global__ __launch_bounds__(256) void conv_slots_kernel(ConvArgs a, int rows) {
+  const int b = blockIdx.x, first = a.q_start[b];
+  if (first < 0 || first >= rows || a.row_req[first] != b) return;
   const int n = a.q_start[b + 1] - first, keep = a.taps - 1;
   const int channels = (a.n_heads + a.n_kv) * a.D + a.n_kv * a.E;
   float* st = a.state + (size_t)a.req_rows[b] * keep * channels;
-  for (int c = threadIdx.x; c < channels; c += blockDim.x) {
+  for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < channels; c += gridDim.y * blockDim.x) {
     const float bias = a.bias ? a.bias[c] : 0.f;
     for (int s = 0; s < keep; ++s) {
       const int at = n + s;                    // place in [what the slot held | the step's rows]
@@ -357,7 +453,7 @@ extern "C" int llmlab_project_conv_write(const float* proj, int ld, int rows, in
                                          const int* req_rows, const float* freq, int rot_dims, int neighbours, int unit,
                                          float eps, void* q_out, void* k_cache, void* v_cache, int dtype, int page_size,
                                          const int* positions, const int* row_req, const int* table, int max_pages,
-                                         int one_row_each, hipStream_t stream) {
+                                         int max_reqs, int one_row_each, hipStream_t stream) {
   LLMLAB_REQUIRE(rows >= 0 && n_heads > 0 && n_kv > 0 && D > 0 && DK >= D && E > 0 && page_size > 0 && page_size % 4 == 0 &&
                      D <= 2048 && E <= 2048 && rot_dims <= 2048,
                  "project_conv_write: bad sizes rows=%d heads=%d kv=%d D=%d/%d E=%d page=%d", rows, n_heads, n_kv, D, DK, E,
@@ -370,6 +466,7 @@ extern "C" int llmlab_project_conv_write(const float* proj, int ld, int rows, in
                  "project_conv_write: %d of %d channels cannot turn in pairs", rot_dims, D);
   LLMLAB_REQUIRE(q_out && k_cache && v_cache && positions && row_req && table && q_start,
                  "project_conv_write: queries, pages and the step's description are needed");
+  LLMLAB_REQUIRE(rows == 0 || max_reqs > 0, "project_conv_write: room for %d requests", max_reqs);
   if (rows == 0) return 0;
   const int widest = D > E ? D : E, heads = n_heads + 2 * n_kv;
   int group = CONV_LDS_FLOATS / widest;
@@ -382,12 +479,24 @@ extern "C" int llmlab_project_conv_write(const float* proj, int ld, int rows, in
   const int channels = (n_heads + n_kv) * D + n_kv * E;
   const bool few = rows <= 64;
   const int threads = few ? (channels >= 1024 ? 1024 : (channels + 63) / 64 * 64) : 256;
+  constexpr int ROWS = 4;
+  ConvArgs wide = a;
+  wide.group = CONV_BLOCK_CHANNELS / widest > 0 ? CONV_BLOCK_CHANNELS / widest : 1;
+  const int groups = (heads + wide.group - 1) / wide.group;
+  const size_t wide_lds = (size_t)ROWS * (rot_dims + wide.group * widest) * sizeof(float);
+  const bool several = !few && !one_row_each && wide_lds <= 64 * 1024;
 #define LLMLAB_CONV_WRITE(T, TAPS)                                                                                     \
   do {                                                                                                                 \
-    if (few) hipLaunchKernelGGL((project_conv_write_kernel<T, TAPS, 2>), dim3(rows), dim3(threads), lds, stream, a,    \
-                                (T*)q_out, (T*)k_cache, (T*)v_cache);                                                  \
-    else hipLaunchKernelGGL((project_conv_write_kernel<T, TAPS, 5>), dim3(rows), dim3(threads), lds, stream, a,        \
-                            (T*)q_out, (T*)k_cache, (T*)v_cache);                                                      \
+    if (several && TAPS > 1)                                                                                           \
+      hipLaunchKernelGGL((project_conv_rows_kernel<T, (TAPS > 1 ? TAPS : 2), ROWS>),                                   \
+                         dim3((rows + ROWS - 1) / ROWS, groups), dim3(256), wide_lds, stream, wide, rows, (T*)q_out,   \
+                         (T*)k_cache, (T*)v_cache);                                                                    \
+    else if (few)                                                                                                      \
+      hipLaunchKernelGGL((project_conv_write_kernel<T, TAPS, 2>), dim3(rows), dim3(threads), lds, stream, a,           \
+                         (T*)q_out, (T*)k_cache, (T*)v_cache);                                                         \
+    else                                                                                                               \
+      hipLaunchKernelGGL((project_conv_write_kernel<T, TAPS, 5>), dim3(rows), dim3(threads), lds, stream, a,           \
+                         (T*)q_out, (T*)k_cache, (T*)v_cache);                                                         \
   } while (0)
 #define LLMLAB_CONV_WRITE_TAPS(T)                     \
   switch (taps) {                                     \
@@ -400,7 +509,10 @@ extern "C" int llmlab_project_conv_write(const float* proj, int ld, int rows, in
   else LLMLAB_CONV_WRITE_TAPS(float)
 #undef LLMLAB_CONV_WRITE_TAPS
 #undef LLMLAB_CONV_WRITE
-  if (taps > 1 && !one_row_each) hipLaunchKernelGGL(conv_slots_kernel, dim3(rows), dim3(256), 0, stream, a);
+  if (taps > 1 && !one_row_each) {
+    const int places = max_reqs < rows ? max_reqs : rows;
+    hipLaunchKernelGGL(conv_slots_kernel, dim3(places, (channels + 255) / 256), dim3(256), 0, stream, a, rows);
+  }
   LLMLAB_LAUNCH_CHECK("project_conv_write");
   return 0;
 }

@@ -62,15 +62,14 @@ class DispatchRules:
     # q/k/v of this many rows up to 64 goes through pieces when the matrix is a large one
     # (64 rows of 7168 x 5120: 26 us against 52 with a head per block; slower below 24 rows).
     qkv_pieces_min_rows: int = 24
-    # The scan of a recurrent mixer (gated linear attention) walks a request's rows one after
-    # the other; from twice ``scan_min_chunk`` rows on a request's rows are cut into chunks that
-    # run side by side and are joined afterwards (the rows are walked twice then), chunks of at
-    # most ``scan_max_chunk`` rows, shorter while that leaves fewer than ``scan_blocks_per_cu``
+    # From this many rows of a step's longest request on, the recurrences of heads of up to 128 key
+    # and 256 value channels go through the chunked scan on the matrix cores (0: never).
+    chunk_scan_min_rows: int = 32
+    # The scan below that walks a request's rows one after the other; from twice ``scan_min_chunk``
+    # rows on a request's rows are cut into chunks that run side by side and are joined afterwards
+    # (the rows are walked twice then), chunks of at most ``scan_max_chunk`` rows, shorter while that leaves fewer than ``scan_blocks_per_cu``
     # blocks to a compute unit.  2,048 rows, 7 heads of 64 x 128: 1.53 ms in one run, 0.17 ms in
     # chunks of 16 (the pass that joins 128 chunks takes 40 us of it), 0.13 ms in chunks of 64.
-    # From this many rows of a step's longest request on, heads of up to 128 key and 256 value channels
-    # go through the chunked scan on the matrix cores instead (0: never).
-    chunk_scan_min_rows: int = 32
     scan_min_chunk: int = 16
     scan_max_chunk: int = 64
     scan_blocks_per_cu: int = 1

@@ -1119,7 +1119,7 @@ class HipOps:
                 lib.llmlab_project_conv_write.argtypes = [
                     _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr,
                     _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
-                    _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr]
+                    _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr]
                 lib.llmlab_project_conv_write.restype = _c_int
                 lib.llmlab_project_rotate_write.argtypes = [
                     _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_float, _c_int,
@@ -1603,9 +1603,9 @@ class HipOps:
                            freq, rot_dims, pairing: str, unit_eps, q_out, k_cache, v_cache, page_size, positions, row_req,
                            block_table, one_row_each: bool) -> None:
         """From the float32 projections ``proj [rows, q | k | v (| ...)]`` (heads of ``key_dim``, ``key_dim``
-        and ``value_dim`` channels): ``bias`` (float32, the same order, or None) is added; ``conv [q + k +
-        v, taps]`` float32 (or None): a causal convolution channel by channel over the positions of each
-        request, ``y_t = sum_j conv[:, j] u_(t - taps + 1 + j)`` of the biased projections ``u``, whose last
+        and ``value_dim`` channels): ``bias`` (float32, the same order, or None) is added; ``conv [taps, q
+        + k + v]`` float32 (or None): a causal convolution channel by channel over the positions of each
+        request, ``y_t = sum_j conv[j] u_(t - taps + 1 + j)`` of the biased projections ``u``, whose last
         ``taps - 1`` rows live in ``state [slots, taps - 1, q + k + v]`` float32; the first ``rot_dims``
         channels of every query and key head turn by ``positions[r] * freq[i]``, channel ``i`` with ``i +
         rot_dims / 2`` (``pairing="halves"``) or ``2i`` with ``2i + 1`` (``"neighbours"``); ``unit_eps`` (None:
@@ -1630,8 +1630,8 @@ class HipOps:
         taps = 0
         if conv is not None:
             self._need(conv, "convolution taps", torch.float32)
-            taps = conv.shape[1]
-            if conv.shape[0] != sizes:
+            taps = conv.shape[0]
+            if conv.shape[1] != sizes:
                 raise ValueError(f"project_conv_write: taps {tuple(conv.shape)} for {sizes} channels")
         if taps > 1:
             self._need(state, "convolution state", torch.float32)
@@ -1656,7 +1656,7 @@ class HipOps:
                    {"halves": 0, "neighbours": 1}[pairing], 0 if unit_eps is None else 1, float(unit_eps or 0.0),
                    self._ptr(q_out), self._ptr(k_cache), self._ptr(v_cache), _dt(q_out), page_size,
                    self._ptr(positions), self._ptr(row_req), self._ptr(block_table), block_table.stride(0),
-                   1 if one_row_each else 0, self._stream(), lib=lib)
+                   min(q_start.numel() - 1, req_rows.numel()), 1 if one_row_each else 0, self._stream(), lib=lib)
 
     def gla_slices(self, key_dim: int) -> int:
         """Into how many pieces the scan leaves each output (one per slice of key channels)."""

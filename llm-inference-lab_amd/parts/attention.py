@@ -486,7 +486,7 @@ class WindowedSinkAttention(Mixer):
             self.b_in = torch.cat(bias).contiguous()
         if self.conv_taps:
             self.conv = torch.cat([tensors[t["q_conv"]].float(), tensors[t["k_conv"]].float(),
-                                   value_heads(tensors[t["v_conv"]].float(), self.num_kv_heads)]).contiguous()
+                                   value_heads(tensors[t["v_conv"]].float(), self.num_kv_heads)]).t().contiguous()
         if self.out_bias:
             self.b_o = tensors[t["o_bias"]].contiguous()
         if self.has_score_bias:

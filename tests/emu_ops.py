@@ -441,12 +441,12 @@ class EmuOps:
         assert not one_row_each or rows == len(reqs)
         y = u
         if conv is not None:
-            taps, y = conv.shape[1], torch.zeros_like(u)
+            taps, y = conv.shape[0], torch.zeros_like(u)
             for b in reqs:
                 lo, hi, slot = int(q_start[b]), int(q_start[b + 1]), int(req_rows[b])
                 joined = torch.cat([state[slot], u[lo:hi]], dim=0) if taps > 1 else u[lo:hi]
                 for j in range(taps):
-                    y[lo:hi] += conv[:, j] * joined[j:j + hi - lo]
+                    y[lo:hi] += conv[j] * joined[j:j + hi - lo]
                 if taps > 1:
                     state[slot] = joined[-(taps - 1):]
 

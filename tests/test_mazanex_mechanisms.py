@@ -172,8 +172,11 @@ def shaped(u, w, positions, heads, D, rot, eps):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("H_,G,D,E,taps,dims", [(3, 1, 16, 24, 4, 16), (4, 2, 24, 8, 3, 6), (6, 3, 9, 16, 2, 4), (2, 2, 32, 40, 1, 0),
                                                 (5, 1, 14, 12, 7, 14), (70, 2, 192, 96, 4, 128)])
-def test_bias_convolution_rotation_unit_norm_and_the_cache_write(backend, dtype, H_, G, D, E, taps, dims):
-    """Two requests in portions (down to one row) and then single rows, against whole sequences: biases
+@pytest.mark.parametrize("plan", ["short", "long"])
+def test_bias_convolution_rotation_unit_norm_and_the_cache_write(backend, dtype, H_, G, D, E, taps, dims, plan):
+    """Requests in portions (down to one row) and then single rows, against whole sequences, with few
+    rows in a step and with many (short ones between long ones, and a description with room for more
+    requests than the step has, which says something stale there): biases
     enter the convolution's inputs (but not what stands before a sequence), the last inputs are
     carried in slots, the first ``dims`` channels of a head turn in halves, the norm comes last."""
     if backend == "emu" and H_ > 10:
@@ -181,7 +184,11 @@ def test_bias_convolution_rotation_unit_norm_and_the_cache_write(backend, dtype,
     ops = ops_of(backend)
     dev = ops.device
     laid = (D + 31) // 32 * 32
-    lengths = [41, 23]
+    portions = {"short": ([17, 1], [2, 3], [5, 16], [1, 1], [1, 1], [15, 1]),
+                "long": ([66, 1, 2], [2, 67, 1], [1, 2, 70], [1, 1, 1], [64, 1, 3])}[plan]
+    lengths = [sum(spans[b] for spans in portions) for b in range(len(portions[0]))]
+    stale = [-1, 5, 10 ** 6, 0] if plan == "long" else []
+    slots = ints([3, 1, 4][:len(lengths)] + [2] * len(stale), dev)
     rot = dict(dims=dims, base=60.0) if dims else None
     sizes = (H_ * D, G * D, G * E)
     total = sum(sizes)
@@ -201,15 +208,16 @@ def test_bias_convolution_rotation_unit_norm_and_the_cache_write(backend, dtype,
         want_q.append(shaped(u[:, :cut[1]], w[:cut[1]], range(n), H_, D, rot, 1e-4))
         want_k.append(shaped(u[:, cut[1]:cut[2]], w[cut[1]:cut[2]], range(n), G, D, rot, 1e-4))
         want_v.append(P.short_conv(u[:, cut[2]:], w[cut[2]:]).view(n, G, E))
-    done = [0, 0]
-    for spans in ([17, 1], [2, 3], [5, 16], [1, 1], [1, 1], [15, 1]):
+    done = [0] * len(lengths)
+    for spans in portions:
         rows = torch.cat([proj[b][done[b]:done[b] + n] for b, n in enumerate(spans)]).to(dev)
         positions = [done[b] + i for b, n in enumerate(spans) for i in range(n)]
         q_start, row_req = batch(spans, dev)
         q = torch.full((rows.shape[0], H_ * laid), float("nan"), dtype=dtype, device=dev)
-        ops.project_conv_write(rows, H_, G, D, E, bias.to(dev), conv.to(dev), state, q_start, ints([3, 1], dev), freq, dims,
-                               "halves", 1e-4, q, cache.k_cache, cache.v_cache, cache.page, ints(positions, dev), row_req,
-                               cache.table, all(n == 1 for n in spans))
+        ops.project_conv_write(rows, H_, G, D, E, bias.to(dev), conv.t().contiguous().to(dev), state,
+                               torch.cat([q_start, ints(stale, dev)]), slots, freq, dims, "halves", 1e-4, q, cache.k_cache,
+                               cache.v_cache, cache.page, ints(positions, dev), row_req, cache.table,
+                               all(n == 1 for n in spans))
         got = q.view(rows.shape[0], H_, laid)
         want = torch.cat([want_q[b][done[b]:done[b] + n] for b, n in enumerate(spans)])
         close(got[..., :D], want, dtype, f"queries of {spans}", f32=2e-5)
