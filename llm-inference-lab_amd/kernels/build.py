@@ -147,11 +147,13 @@ MIXER_SOURCES = {"windowed_attention": "windowed_attention.hip", "linear_attenti
 
 
 def mixer_library(kind: str, force: bool = False) -> str:
-    """``windowed_attention``: sliding window with a kept prefix and a sink term;
-    ``linear_attention``: the gated recurrence with a matrix state per head; ``routed_experts``: a
+    """``windowed_attention``: sliding window with a kept prefix, or chunks, and a sink term, with what
+    stands between the projections and the cache; ``linear_attention``: recurrences with a matrix state
+    per head; ``routed_experts``: a
     feed-forward of many experts of which a row uses a few (choice, sorting, grouped products);
     ``stream_ops``: what lies around the sublayers of a layer (an embedding with hashed token pairs, a
-    short causal convolution with per-request state, a gated sum into the stream, a soft cap)."""
+    short causal convolution with per-request state, a token shift, norms of results summed into the
+    stream, a cubic of normed powers, a gated sum into the stream, a soft cap)."""
     return _compile(kind, (MIXER_SOURCES[kind],), (), force)
 
 
