@@ -5,3 +5,4 @@ from . import ruvalorn  # noqa: F401
 from . import minodra  # noqa: F401
 from . import ninisun  # noqa: F401
 from . import mazanex  # noqa: F401
+from . import molotar  # noqa: F401

@@ -89,7 +89,8 @@ struct SkinnyArgs {
   // (no residual, bias in group 0) in out[s][M][ldo], part_stride numbers apart.
   int ksplit;
   size_t part_stride;
-  int act;         // SK_STORE: 1 = max(z, 0)^2 before the rounding; SK_SWIGLU: 2 = gelu (tanh form) gate
+  int act;         // SK_STORE: 1 = max(z, 0)^2 before the rounding; SK_SWIGLU: 2 = gelu (tanh form) gate, 3 = the clamped pair
+  float limit, slope, shift;      // the clamped pair's constants
   // SK_PART: segments of the columns may read inputs of their own: the strips from seg_end[s - 1] to
   // seg_end[s] - 1 multiply the rows x + s * seg_stride (segs <= 1: all strips read x).
   int segs;
@@ -104,6 +105,14 @@ __device__ __forceinline__ float sk_silu(float z) { return z / (1.f + __expf(-z)
 __device__ __forceinline__ float sk_gelu_tanh(float z) {
   const float t = 0.7978845608028654f * (z + 0.044715f * z * z * z);
   return z / (1.f + __expf(-2.f * t));
+}
+
+// act(gate) * up; the clamped pair: g = min(gate, limit), u = up held within -limit .. limit,
+// g * sigmoid(slope * g) * (u + shift)
+__device__ __forceinline__ float sk_pair(float g, float u, const SkinnyArgs& a) {
+  if (a.act != 3) return (a.act == 2 ? sk_gelu_tanh(g) : sk_silu(g)) * u;
+  g = fminf(g, a.limit);
+  return g / (1.f + __expf(-a.slope * g)) * (fminf(fmaxf(u, -a.limit), a.limit) + a.shift);
 }
 
 // Loads of W (and of x where it is not staged) run R steps ahead of the MFMAs in a
@@ -505,7 +514,7 @@ __global__ __launch_bounds__(MB >= 4 ? 512 : 1024) void skinny_block_kernel(Skin
       const int pr = j >> 4, cc = j & 15;
       const float gv = tile[m * cols + pr * 32 + cc], uv = tile[m * cols + pr * 32 + 16 + cc];
       const int o = ((n0 >> 5) + pr) * 16 + cc;
-      if (o < a.n_out) ((bf16_t*)a.out)[(size_t)m * a.ldo + o] = (bf16_t)((a.act == 2 ? sk_gelu_tanh(gv) : sk_silu(gv)) * uv);
+      if (o < a.n_out) ((bf16_t*)a.out)[(size_t)m * a.ldo + o] = (bf16_t)sk_pair(gv, uv, a);
     }
   }
   if constexpr (EPI == SK_QKV) {
@@ -742,15 +751,17 @@ extern "C" int llmlab_skinny_linear(const void* x, int norm, const int* x_rows, 
                                     int page_size, void* kcache, void* vcache, int nq, int nkv, int d,
                                     int num_cus, const float* pend, int pend_splits, int pend_ld,
                                     size_t pend_stride, int ksplit, size_t part_stride, int segs,
-                                    const int* seg_ends, size_t seg_stride, hipStream_t stream) {
+                                    const int* seg_ends, size_t seg_stride, float limit, float slope,
+                                    float shift, hipStream_t stream) {
   LLMLAB_REQUIRE(segs <= 1 || (segs <= 8 && seg_ends && epilogue == SK_PART && seg_stride % 8 == 0),
                  "skinny_linear: up to 8 segments with inputs of their own, in pieces, got %d", segs);
   LLMLAB_REQUIRE(M >= 0 && M <= SK_MAX_ROWS, "skinny_linear: takes at most %d rows, got %d", SK_MAX_ROWS, M);
   LLMLAB_REQUIRE(N > 0 && K > 0 && K % 8 == 0, "skinny_linear: bad sizes N=%d K=%d (K must be a multiple of 8)", N, K);
-  // (6 at this interface: STORE through the squared relu; 7: the paired product with a gelu gate)
-  const int act = epilogue == 6 ? 1 : epilogue == 7 ? 2 : 0;
+  // (6 at this interface: STORE through the squared relu; 7: the paired product with a gelu gate;
+  // 8: the clamped pair)
+  const int act = epilogue == 6 ? 1 : epilogue == 7 ? 2 : epilogue == 8 ? 3 : 0;
   if (act == 1) epilogue = SK_STORE;
-  if (act == 2) epilogue = SK_SWIGLU;
+  if (act > 1) epilogue = SK_SWIGLU;
   LLMLAB_REQUIRE(epilogue >= 0 && epilogue <= 5, "skinny_linear: unknown epilogue %d", epilogue);
   LLMLAB_REQUIRE(pend_splits >= 0 && (pend_splits == 0 || (pend != nullptr && (norm || epilogue == SK_RESID))),
                  "skinny_linear: pending sums go with a norm or into the residual");
@@ -809,6 +820,7 @@ extern "C" int llmlab_skinny_linear(const void* x, int norm, const int* x_rows, 
   a.ksplit = ksplit; a.part_stride = part_stride; a.tiles = tiles; a.col_blocks = blocks;
   a.qsplit = shape.qsplit;
   a.act = act;
+  a.limit = limit; a.slope = slope; a.shift = shift;
   a.x = x; a.x_rows = x_rows; a.norm_w = norm_w; a.W = (const bf16_t*)w; a.bias = bias; a.out = out;
   a.inv_freq = inv_freq; a.positions = positions; a.row_req = row_req; a.table = table;
   a.kcache = (bf16_t*)kcache; a.vcache = (bf16_t*)vcache;

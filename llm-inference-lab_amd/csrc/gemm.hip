@@ -71,7 +71,7 @@ struct EpiArgs {
   bf16_t* vcache;
   int table_stride, page_size, nq, nkv, d;
   // STORE: 1 = the sum goes through max(z, 0)^2 (in float32) before it is rounded;
-  // SWIGLU: 2 = the gate goes through gelu (tanh form) instead of silu
+  // SWIGLU: 2 = the gate goes through gelu (tanh form) instead of silu; 3 = the clamped pair (below)
   int act;
   // Grouped products (several matrices of equal shape, one below the other in W; every tile of
   // rows belongs to one of them): g_tile[tile of rows] is the tile's matrix (-1: the tile is
@@ -80,6 +80,7 @@ struct EpiArgs {
   const int* g_tile;
   const int* g_rows;
   size_t g_w_stride;
+  float limit, slope, shift;      // constants of the clamped pair
 };
 
 __device__ __forceinline__ float relu2_f(float z) {
@@ -102,6 +103,19 @@ __device__ __forceinline__ float gelu_tanh_exact_f(float z) {
 __device__ __forceinline__ float gate_act_f(float z, int act) { return act == 2 ? gelu_tanh_f(z) : silu_f(z); }
 __device__ __forceinline__ float gate_act_exact_f(float z, int act) {
   return act == 2 ? gelu_tanh_exact_f(z) : z / (1.f + expf(-z));
+}
+
+// A gated pair: act(gate) * up; act 3, the clamped pair: with g = min(gate, limit) and u = up held within
+// -limit .. limit, g * sigmoid(slope * g) * (u + shift).
+__device__ __forceinline__ float pair_f(float g, float u, const EpiArgs& e) {
+  if (e.act != 3) return gate_act_f(g, e.act) * u;
+  g = fminf(g, e.limit);
+  return g / (1.f + __expf(-e.slope * g)) * (fminf(fmaxf(u, -e.limit), e.limit) + e.shift);
+}
+__device__ __forceinline__ float pair_exact_f(float g, float u, const EpiArgs& e) {
+  if (e.act != 3) return gate_act_exact_f(g, e.act) * u;
+  g = fminf(g, e.limit);
+  return g / (1.f + expf(-e.slope * g)) * (fminf(fmaxf(u, -e.limit), e.limit) + e.shift);
 }
 
 // One output element (non-SWIGLU).
@@ -257,8 +271,8 @@ __device__ __forceinline__ void tile_epilogue(const float* Cs, const EpiArgs& e,
       bf16x8 v;
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
-        v[q] = (bf16_t)(gate_act_f(g0[q], e.act) * u0[q]);
-        v[4 + q] = (bf16_t)(gate_act_f(g1[q], e.act) * u1[q]);
+        v[q] = (bf16_t)pair_f(g0[q], u0[q], e);
+        v[4 + q] = (bf16_t)pair_f(g1[q], u1[q], e);
       }
       bf16_t* dst = out + (size_t)m * e.ldo + o0 + oc;
       if (vec && o0 + oc + 8 <= e.n_out) *(bf16x8*)dst = v;
@@ -796,10 +810,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const float* __restrict__
         if (j & 1) continue;
         const int nb = n0 + 16 * j;
         const int o = (nb >> 5) * 16 + tx;
-        if (o < e.n_out) {
-          const float z = acc[i][j];
-          ((float*)e.out)[(size_t)m * e.ldo + o] = gate_act_exact_f(z, e.act) * acc[i][j + 1];
-        }
+        if (o < e.n_out) ((float*)e.out)[(size_t)m * e.ldo + o] = pair_exact_f(acc[i][j], acc[i][j + 1], e);
       } else {
         const int n = n0 + tx + 16 * j;
         if (n < N) epi_store<float, EPI>(e, m, n, acc[i][j]);
@@ -905,10 +916,7 @@ __global__ __launch_bounds__(256) void gemm_f32_mfma_kernel(const float* __restr
 #pragma unroll
         for (int x = 0; x < 8; ++x) {
           const int o = (nb >> 5) * 16 + 8 * (x >> 2) + 4 * kk + (x & 3);
-          if (o < e.n_out) {
-            const float z = acc[j][i][x];
-            ((float*)e.out)[(size_t)m * e.ldo + o] = gate_act_exact_f(z, e.act) * acc[j][i][x + 8];
-          }
+          if (o < e.n_out) ((float*)e.out)[(size_t)m * e.ldo + o] = pair_exact_f(acc[j][i][x], acc[j][i][x + 8], e);
         }
       } else {
 #pragma unroll
@@ -1060,10 +1068,7 @@ __global__ __launch_bounds__(64 * KW) void gemm_f32_rows_kernel(const float* __r
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         const int o = (rows_w[j] >> 5) * 16 + (rows_w[j] & 15);
-        if (o < e.n_out) {
-          const float z = acc[i][j];
-          ((float*)e.out)[(size_t)m * e.ldo + o] = gate_act_exact_f(z, e.act) * acc[i][j + 2];
-        }
+        if (o < e.n_out) ((float*)e.out)[(size_t)m * e.ldo + o] = pair_exact_f(acc[i][j], acc[i][j + 2], e);
       }
     } else {
 #pragma unroll
@@ -1287,17 +1292,18 @@ static void launch_tile(int kind, const bf16_t* A, const bf16_t* W, const EpiArg
 // W (every member whole strips of 16 rows: N % 16 == 0); tile t of bm rows of the product belongs
 // to member tile_member[t] (-1: empty, its block leaves at once); row m reads row rows_index[m]
 // of x (null: row m).  out has M rows (a multiple of bm).  Epilogues: SWIGLU, F32, and STORE
-// (compute dtype; epilogue 6: through max(z, 0)^2 first).
+// (compute dtype; epilogue 6: through max(z, 0)^2 first; epilogue 8: SWIGLU as the clamped pair).
 extern "C" int llmlab_linear_grouped(const void* x, const void* w, int epilogue, void* out, int M, int N, int K,
                                      int ldo, int n_out, const int* tile_member, const int* rows_index, int bm,
-                                     int wide, hipStream_t stream) {
+                                     int wide, float limit, float slope, float shift, hipStream_t stream) {
   LLMLAB_REQUIRE(M >= 0 && N > 0 && K > 0 && K % 8 == 0 && N % 16 == 0, "linear_grouped: bad sizes M=%d N=%d K=%d", M,
                  N, K);
   LLMLAB_REQUIRE((bm == 64 || bm == 128) && M % bm == 0, "linear_grouped: %d rows in tiles of %d", M, bm);
   if (g_force_tile == 129) wide = 0;
   if (g_force_tile == 131) wide = 1;
-  const int act = epilogue == 6 ? 1 : 0;
-  if (act) epilogue = EPI_STORE;
+  const int act = epilogue == 6 ? 1 : epilogue == 8 ? 3 : 0;
+  if (act == 1) epilogue = EPI_STORE;
+  if (act == 3) epilogue = EPI_SWIGLU;
   LLMLAB_REQUIRE(epilogue == EPI_SWIGLU || epilogue == EPI_F32 || epilogue == EPI_STORE, "linear_grouped: epilogue %d",
                  epilogue);
   if (epilogue == EPI_SWIGLU)
@@ -1308,7 +1314,7 @@ extern "C" int llmlab_linear_grouped(const void* x, const void* w, int epilogue,
   LLMLAB_REQUIRE(ldo >= n_out && tile_member != nullptr, "linear_grouped: output stride or tile table");
   if (M == 0) return 0;
   EpiArgs e{out, nullptr, 0, ldo, n_out, 0, 0, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0, 0, 0, 0, act,
-            tile_member, rows_index, (size_t)(N / 16) * (size_t)((K + 31) / 32) * 512};
+            tile_member, rows_index, (size_t)(N / 16) * (size_t)((K + 31) / 32) * 512, limit, slope, shift};
   const bf16_t* A = (const bf16_t*)x;
   const bf16_t* W = (const bf16_t*)w;
   // (the columns past n_out of an F32 product are the zero rows that pad a member to whole strips)
@@ -1466,13 +1472,13 @@ extern "C" int llmlab_linear_partials(const void* x, const void* w, float* parts
 // is the number of interleaved weight rows (2 * ceil16(n_out)).
 extern "C" int llmlab_linear(const void* x, const void* w, int dtype, int epilogue, void* out,
                              const void* bias, int bias_dtype, int M, int N, int K, int ldo, int n_out,
-                             int num_cus, hipStream_t stream) {
+                             int num_cus, float limit, float slope, float shift, hipStream_t stream) {
   LLMLAB_REQUIRE(M >= 0 && N > 0 && K > 0, "linear: bad sizes M=%d N=%d K=%d", M, N, K);
   // 6 at this interface: STORE with the squared-relu activation on the way; 7: the paired
-  // product whose gate goes through gelu (tanh form)
-  const int act = epilogue == 6 ? 1 : epilogue == 7 ? 2 : 0;
+  // product whose gate goes through gelu (tanh form); 8: the clamped pair with its three constants
+  const int act = epilogue == 6 ? 1 : epilogue == 7 ? 2 : epilogue == 8 ? 3 : 0;
   if (act == 1) epilogue = EPI_STORE;
-  if (act == 2) epilogue = EPI_SWIGLU;
+  if (act > 1) epilogue = EPI_SWIGLU;
   LLMLAB_REQUIRE(epilogue >= 0 && epilogue <= 3, "linear: unknown epilogue %d", epilogue);
   if (epilogue == EPI_SWIGLU) {
     LLMLAB_REQUIRE(N % 32 == 0 && n_out > 0 && 2 * ((n_out + 15) / 16 * 16) == N,
@@ -1484,7 +1490,7 @@ extern "C" int llmlab_linear(const void* x, const void* w, int dtype, int epilog
   LLMLAB_REQUIRE(ldo >= n_out, "linear: output row stride %d < %d columns", ldo, n_out);
   if (M == 0) return 0;
   EpiArgs e{out, bias, bias_dtype == DT_BF16, ldo, n_out, 0, 0,
-            nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0, 0, 0, 0, act};
+            nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0, 0, 0, 0, act, nullptr, nullptr, 0, limit, slope, shift};
   if (num_cus <= 0) num_cus = 256;
   if (dtype == DT_BF16) {
     LLMLAB_REQUIRE(K % 8 == 0, "linear(bfloat16): inner size %d must be a multiple of 8", K);

@@ -3,6 +3,7 @@
 //
 //   select      per row: softmax over the router's outputs, choice value = score + correction,
 //               the best groups of neighbours, the top outputs among them; weight = score * scale
+//               (or the score's share of the chosen scores' sum, times scale)
 //   add_chosen  resid[r] += (sum of the weights of row r's choices within [first, last)) * src[r]
 #include "common.h"
 
@@ -10,11 +11,28 @@ extern "C" const char* llmlab_last_error() { return g_llmlab_error; }
 
 constexpr int SELECT_MAX_OUTPUTS = 1024;     // router outputs a row's wave keeps in LDS
 
+// How a row's outputs are scored, grouped and weighed.  sigmoid: every output by itself, else a softmax.
+// pairs: a group counts as the sum of its two largest choice values, else as its largest.  share_eps >= 0:
+// the chosen scores are divided by their sum + share_eps before they are scaled.
+struct Choice {
+  int outputs, groups, keep, top; float scale; int sigmoid, pairs; float share_eps;
+};
+
+// the value of a group of `per` neighbours
+__device__ __forceinline__ float group_value(const float* choice, int per, int pairs) {
+  float best = -INFINITY, next = -INFINITY;
+  for (int i = 0; i < per; ++i) {
+    const float v = choice[i];
+    next = fmaxf(next, fminf(best, v));
+    best = fmaxf(best, v);
+  }
+  return pairs && per > 1 ? best + next : best;
+}
+
 // One wave a row.  Everything in float32; ties go to the smaller index, as a scan in order does.
 __global__ __launch_bounds__(64) void moe_select_kernel(const float* __restrict__ logits, const float* __restrict__ correction,
-                                                        int outputs, int groups, int keep, int top, float scale,
-                                                        int* __restrict__ chosen, float* __restrict__ weights,
-                                                        int sigmoid) {
+                                                        Choice how, int* __restrict__ chosen, float* __restrict__ weights) {
+  const int outputs = how.outputs, groups = how.groups, keep = how.keep, top = how.top, sigmoid = how.sigmoid;
   __shared__ float s_score[SELECT_MAX_OUTPUTS], s_choice[SELECT_MAX_OUTPUTS];
   __shared__ float s_group[SELECT_MAX_OUTPUTS];
   const int row = blockIdx.x, lane = threadIdx.x;
@@ -39,9 +57,7 @@ __global__ __launch_bounds__(64) void moe_select_kernel(const float* __restrict_
   const int per = outputs / groups;
   if (keep < groups) {
     for (int g = lane; g < groups; g += WAVE) {
-      float best = -INFINITY;
-      for (int i = 0; i < per; ++i) best = fmaxf(best, s_choice[g * per + i]);
-      s_group[g] = best;
+      s_group[g] = group_value(s_choice + g * per, per, how.pairs);
     }
     __syncthreads();
     // a group is kept if fewer than `keep` groups come before it in the order (value down, index up)
@@ -57,6 +73,7 @@ __global__ __launch_bounds__(64) void moe_select_kernel(const float* __restrict_
     }
     __syncthreads();
   }
+  float sum_chosen = 0.f;
   for (int k = 0; k < top; ++k) {
     float best = -INFINITY;
     int at = outputs;             // (when every value left is minus infinity: the smallest index left)
@@ -76,13 +93,16 @@ __global__ __launch_bounds__(64) void moe_select_kernel(const float* __restrict_
       }
     }
     at = min(at, outputs - 1);
+    sum_chosen += s_score[at];
     if (lane == 0) {
       chosen[(size_t)row * top + k] = at;
-      weights[(size_t)row * top + k] = s_score[at] * scale;
+      weights[(size_t)row * top + k] = s_score[at] * how.scale;
       s_choice[at] = -INFINITY;          // taken
     }
     __syncthreads();
   }
+  if (how.share_eps >= 0.f && lane == 0)       // (the numbers this lane has just written)
+    for (int k = 0; k < top; ++k) weights[(size_t)row * top + k] /= sum_chosen + how.share_eps;
 }
 
 // The same for a router of up to 64 outputs: a lane an output, a wave a row, no block barrier.
@@ -98,9 +118,9 @@ __device__ __forceinline__ void wave_sync() {
 }
 
 __device__ __forceinline__ void select_row_by_wave(const float* __restrict__ logits, const float* __restrict__ correction,
-                                                   int outputs, int groups, int keep, int top, float scale,
-                                                   int* __restrict__ chosen, float* __restrict__ weights, int row,
-                                                   int lane, float* s_wave, int sigmoid) {
+                                                   const Choice& how, int* __restrict__ chosen,
+                                                   float* __restrict__ weights, int row, int lane, float* s_wave) {
+  const int outputs = how.outputs, groups = how.groups, keep = how.keep, top = how.top, sigmoid = how.sigmoid;
   const bool mine = lane < outputs;
   const float z = mine ? logits[(size_t)row * outputs + lane] : -INFINITY;
   wave_sync();                                 // (the row before is read out)
@@ -120,9 +140,7 @@ __device__ __forceinline__ void select_row_by_wave(const float* __restrict__ log
   wave_sync();
   if (keep < groups) {
     const int per = outputs / groups, g = mine ? lane / per : groups;
-    float best = -INFINITY;                    // of this lane's group
-    if (mine)
-      for (int i = 0; i < per; ++i) best = fmaxf(best, s_wave[g * per + i]);
+    const float best = mine ? group_value(s_wave + g * per, per, how.pairs) : -INFINITY;      // of this lane's group
     wave_sync();
     s_wave[WAVE + lane] = best;
     wave_sync();
@@ -141,25 +159,25 @@ __device__ __forceinline__ void select_row_by_wave(const float* __restrict__ log
     const float c = s_wave[j];
     place += (c > choice) || (c == choice && j < lane);
   }
-  if (mine && place < top) {
+  const bool taken = mine && place < top;
+  const float weight = how.share_eps >= 0.f ? score / (wave_sum(taken ? score : 0.f) + how.share_eps) : score;
+  if (taken) {
     chosen[(size_t)row * top + place] = lane;
-    weights[(size_t)row * top + place] = score * scale;
+    weights[(size_t)row * top + place] = weight * how.scale;
   }
 }
 
 __global__ __launch_bounds__(64) void moe_select_wave_kernel(const float* __restrict__ logits,
-                                                             const float* __restrict__ correction, int outputs, int groups,
-                                                             int keep, int top, float scale, int* __restrict__ chosen,
-                                                             float* __restrict__ weights, int sigmoid) {
+                                                             const float* __restrict__ correction, Choice how,
+                                                             int* __restrict__ chosen, float* __restrict__ weights) {
   __shared__ float s_wave[2 * WAVE];
-  select_row_by_wave(logits, correction, outputs, groups, keep, top, scale, chosen, weights, blockIdx.x, threadIdx.x,
-                     s_wave, sigmoid);
+  select_row_by_wave(logits, correction, how, chosen, weights, blockIdx.x, threadIdx.x, s_wave);
 }
 
-// scoring: 0 softmax over the outputs, 1 the sigmoid of each output by itself
+// scoring: 0 softmax over the outputs, 1 the sigmoid of each output by itself; pairs, share_eps: see Choice
 extern "C" int llmlab_moe_select(const float* logits, const float* correction, int rows, int outputs, int groups,
-                                 int keep, int top, float scale, int* chosen, float* weights, int scoring,
-                                 hipStream_t stream) {
+                                 int keep, int top, float scale, int* chosen, float* weights, int scoring, int pairs,
+                                 float share_eps, hipStream_t stream) {
   LLMLAB_REQUIRE(scoring == 0 || scoring == 1, "moe_select: scoring %d", scoring);
   LLMLAB_REQUIRE(rows >= 0 && outputs > 0 && outputs <= SELECT_MAX_OUTPUTS,
                  "moe_select: a router of 1 to %d outputs, got %d", SELECT_MAX_OUTPUTS, outputs);
@@ -167,12 +185,11 @@ extern "C" int llmlab_moe_select(const float* logits, const float* correction, i
                      top <= keep * (outputs / groups),
                  "moe_select: %d outputs in %d groups of which %d are kept, top %d", outputs, groups, keep, top);
   if (rows == 0) return 0;
+  const Choice how{outputs, groups, keep, top, scale, scoring, pairs, share_eps};
   if (outputs <= WAVE)
-    hipLaunchKernelGGL(moe_select_wave_kernel, dim3(rows), dim3(64), 0, stream, logits, correction, outputs, groups,
-                       keep, top, scale, chosen, weights, scoring);
+    hipLaunchKernelGGL(moe_select_wave_kernel, dim3(rows), dim3(64), 0, stream, logits, correction, how, chosen, weights);
   else
-    hipLaunchKernelGGL(moe_select_kernel, dim3(rows), dim3(64), 0, stream, logits, correction, outputs, groups, keep,
-                       top, scale, chosen, weights, scoring);
+    hipLaunchKernelGGL(moe_select_kernel, dim3(rows), dim3(64), 0, stream, logits, correction, how, chosen, weights);
   LLMLAB_LAUNCH_CHECK("moe_select");
   return 0;
 }
@@ -298,27 +315,24 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
 // in turn, then the block sorts what they chose (their writes are the block's own: a barrier
 // makes them seen).
 __global__ __launch_bounds__(1024) void moe_select_plan_kernel(const float* __restrict__ logits,
-                                                               const float* __restrict__ correction, int rows, int outputs,
-                                                               int groups, int keep, int top, float scale,
+                                                               const float* __restrict__ correction, int rows, Choice how,
                                                                int* __restrict__ chosen, float* __restrict__ weights,
                                                                int experts, int bm, int capacity, int* __restrict__ place_of,
-                                                               int* __restrict__ place_row, int* __restrict__ tile_member,
-                                                               int sigmoid) {
+                                                               int* __restrict__ place_row, int* __restrict__ tile_member) {
   __shared__ int s_count[PLAN_MAX_EXPERTS], s_start[PLAN_MAX_EXPERTS];
   __shared__ float s_waves[16][2 * WAVE];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, waves = blockDim.x >> 6;
   for (int row = wave; row < rows; row += waves)
-    select_row_by_wave(logits, correction, outputs, groups, keep, top, scale, chosen, weights, row, lane, s_waves[wave],
-                       sigmoid);
+    select_row_by_wave(logits, correction, how, chosen, weights, row, lane, s_waves[wave]);
   __threadfence_block();
   __syncthreads();
-  plan_by_block(chosen, rows * top, experts, bm, capacity, place_of, place_row, tile_member, top, s_count, s_start);
+  plan_by_block(chosen, rows * how.top, experts, bm, capacity, place_of, place_row, tile_member, how.top, s_count, s_start);
 }
 
 extern "C" int llmlab_moe_select_plan(const float* logits, const float* correction, int rows, int outputs, int groups,
                                       int keep, int top, float scale, int* chosen, float* weights, int experts, int bm,
-                                      int capacity, int* place_of, int* place_row, int* tile_member, int scoring,
-                                      hipStream_t stream) {
+                                      int capacity, int* place_of, int* place_row, int* tile_member, int scoring, int pairs,
+                                      float share_eps, hipStream_t stream) {
   LLMLAB_REQUIRE(rows >= 0 && outputs > 0 && outputs <= WAVE, "moe_select_plan: a router of 1 to 64 outputs, got %d",
                  outputs);
   LLMLAB_REQUIRE(scoring == 0 || scoring == 1, "moe_select_plan: scoring %d", scoring);
@@ -330,8 +344,9 @@ extern "C" int llmlab_moe_select_plan(const float* logits, const float* correcti
   LLMLAB_REQUIRE(capacity % bm == 0 && capacity >= need, "moe_select_plan: %d places for %d pairs of %d experts", capacity,
                  rows * top, experts);
   if (rows == 0) return 0;
-  hipLaunchKernelGGL(moe_select_plan_kernel, dim3(1), dim3(1024), 0, stream, logits, correction, rows, outputs, groups,
-                     keep, top, scale, chosen, weights, experts, bm, capacity, place_of, place_row, tile_member, scoring);
+  const Choice how{outputs, groups, keep, top, scale, scoring, pairs, share_eps};
+  hipLaunchKernelGGL(moe_select_plan_kernel, dim3(1), dim3(1024), 0, stream, logits, correction, rows, how, chosen, weights,
+                     experts, bm, capacity, place_of, place_row, tile_member);
   LLMLAB_LAUNCH_CHECK("moe_select_plan");
   return 0;
 }

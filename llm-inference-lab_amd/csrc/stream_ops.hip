@@ -6,6 +6,7 @@
 //   softcap         x = cap * tanh(x / cap)
 //   rmsnorm_add     x += y / sqrt(mean(y^2) + eps) * w   (a norm on a sublayer's result, before the sum;
 //                   the norm that reads the stream next, or a rounded copy, may come out of the same launch)
+//   post_norm       x = (alpha * x + y) / sqrt(mean((alpha * x + y)^2) + eps) * w   (a norm BEHIND the sum)
 //   scaled_sum      out = a * y1 + b * y2
 //   normed_sum      out = a * norm1(y1) + b * norm2(y2)
 //   shift_mix       out_m = h + (previous row's h - h) * mix_m, for one or several mixes
@@ -693,6 +694,144 @@ extern "C" int llmlab_shift_mix(const void* h, int h_dtype, const float* mix, in
 #undef LLMLAB_SHIFT_ANY
 #undef LLMLAB_SHIFT
   LLMLAB_LAUNCH_CHECK("shift_mix");
+  return 0;
+}
+
+// ------------------------------------------------------------------ a norm behind the sum
+// v = alpha * x[r] + y, x[r, c] = v[c] / sqrt(mean(v^2) + eps) * w[c], and (copy not null) copy[r] = T(the new row).
+// All float32.  y is a row of a result, or the sum of its pieces in the pieces' order, or (top > 0) the
+// weighted sum of the rows of y at the places place_of[r, k], the choices in their order (a place below zero:
+// none).  One block a row, V numbers a load; a thread keeps up to POST_KEEP loads of the row in registers
+// between the sum and the result, wider rows are read again.
+constexpr int POST_KEEP = 4, POST_CHOICES = 4;
+struct PostNorm {
+  float* x; float alpha; const float* y; int pieces; size_t piece_stride;
+  const int* place_of; const float* weights; int top;
+  const float* w; float eps; int width;
+};
+
+template <int V>
+struct Numbers { float f[V]; };
+template <int V>
+__device__ __forceinline__ Numbers<V> load_numbers(const float* p) {
+  Numbers<V> n;
+  if (V == 4) {
+    const floatx4 t = *(const floatx4*)p;
+#pragma unroll
+    for (int q = 0; q < V; ++q) n.f[q] = t[q & 3];
+  } else {
+    n.f[0] = p[0];
+  }
+  return n;
+}
+
+template <typename T, int V>
+__global__ __launch_bounds__(1024) void post_norm_kernel(PostNorm a, T* __restrict__ copy) {
+  __shared__ float red[17];
+  const int threads = blockDim.x, units = a.width / V;
+  const size_t row = (size_t)blockIdx.x * a.width;
+  const int* places = a.place_of + (size_t)blockIdx.x * a.top;
+  const float* shares = a.weights + (size_t)blockIdx.x * a.top;
+  auto summed = [&](int i) {
+    const size_t c = (size_t)i * V;
+    Numbers<V> v = load_numbers<V>(a.x + row + c);
+    if (a.top > 0) {
+      Numbers<V> s;
+#pragma unroll
+      for (int q = 0; q < V; ++q) s.f[q] = 0.f;
+      for (int k0 = 0; k0 < a.top; k0 += POST_CHOICES) {      // (a few choices' loads travel together)
+        Numbers<V> p[POST_CHOICES];
+        float share[POST_CHOICES];
+#pragma unroll
+        for (int k = 0; k < POST_CHOICES; ++k) {
+          const int at = min(k0 + k, a.top - 1), place = places[at];
+          share[k] = k0 + k < a.top && place >= 0 ? shares[at] : 0.f;
+          p[k] = load_numbers<V>(a.y + (size_t)max(place, 0) * a.width + c);
+        }
+#pragma unroll
+        for (int k = 0; k < POST_CHOICES; ++k)
+          if (share[k] != 0.f)
+#pragma unroll
+            for (int q = 0; q < V; ++q) s.f[q] = fmaf(share[k], p[k].f[q], s.f[q]);
+      }
+#pragma unroll
+      for (int q = 0; q < V; ++q) v.f[q] = fmaf(a.alpha, v.f[q], s.f[q]);
+      return v;
+    }
+    Numbers<V> s = load_numbers<V>(a.y + row + c);
+    for (int k = 1; k < a.pieces; ++k) {
+      const Numbers<V> p = load_numbers<V>(a.y + k * a.piece_stride + row + c);
+#pragma unroll
+      for (int q = 0; q < V; ++q) s.f[q] += p.f[q];
+    }
+#pragma unroll
+    for (int q = 0; q < V; ++q) v.f[q] = fmaf(a.alpha, v.f[q], s.f[q]);
+    return v;
+  };
+  Numbers<V> keep[POST_KEEP], ws[POST_KEEP];
+  float ss = 0.f;
+#pragma unroll
+  for (int n = 0; n < POST_KEEP; ++n) {
+    const int i = threadIdx.x + threads * n;
+    if (i < units) {
+      keep[n] = summed(i);
+      ws[n] = load_numbers<V>(a.w + (size_t)i * V);
+#pragma unroll
+      for (int q = 0; q < V; ++q) ss = fmaf(keep[n].f[q], keep[n].f[q], ss);
+    }
+  }
+  for (int i = threadIdx.x + threads * POST_KEEP; i < units; i += threads) {
+    const Numbers<V> v = summed(i);
+#pragma unroll
+    for (int q = 0; q < V; ++q) ss = fmaf(v.f[q], v.f[q], ss);
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)a.width + a.eps);
+  auto result = [&](int i, const Numbers<V>& v, const Numbers<V>& w) {
+    const size_t c = row + (size_t)i * V;
+    if (V == 4) {
+      floatx4 o;
+#pragma unroll
+      for (int q = 0; q < 4; ++q) o[q] = v.f[q % V] * inv * w.f[q % V];
+      store4(a.x + c, o);
+      if (copy) store4(copy + c, o);
+    } else {
+      const float o = v.f[0] * inv * w.f[0];
+      a.x[c] = o;
+      if (copy) copy[c] = from_float<T>(o);
+    }
+  };
+#pragma unroll
+  for (int n = 0; n < POST_KEEP; ++n) {
+    const int i = threadIdx.x + threads * n;
+    if (i < units) result(i, keep[n], ws[n]);
+  }
+  for (int i = threadIdx.x + threads * POST_KEEP; i < units; i += threads)      // (a thread's own numbers, not yet replaced)
+    result(i, summed(i), load_numbers<V>(a.w + (size_t)i * V));
+}
+
+extern "C" int llmlab_post_norm(float* x, float alpha, const float* y, int pieces, size_t piece_stride, const int* place_of,
+                                const float* weights, int top, const float* w, float eps, int rows, int width, void* copy,
+                                int copy_dtype, hipStream_t stream) {
+  LLMLAB_REQUIRE(rows >= 0 && width > 0 && x && y && w && pieces >= 1 && top >= 0,
+                 "post_norm: bad arguments rows=%d width=%d pieces=%d choices=%d", rows, width, pieces, top);
+  LLMLAB_REQUIRE(top == 0 || (place_of && weights && pieces == 1), "post_norm: choices need their places and weights");
+  if (rows == 0) return 0;
+  const PostNorm a{x, alpha, y, pieces, piece_stride, place_of, weights, top, w, eps, width};
+  const bool vec = width % 4 == 0 && piece_stride % 4 == 0 &&
+                   (((uintptr_t)x | (uintptr_t)y | (uintptr_t)w | (uintptr_t)copy) & 15) == 0;
+  // few rows: a thread a load, up to a block's 1,024 threads; many rows: blocks of which several share a unit
+  const int units = vec ? width / 4 : width, most = rows <= 64 ? 1024 : 256;
+  int threads = (units + 63) / 64 * 64;
+  if (threads > most) threads = most;
+#define LLMLAB_POST_NORM(T, V) \
+  hipLaunchKernelGGL((post_norm_kernel<T, V>), dim3(rows), dim3(threads), 0, stream, a, (T*)copy)
+  if (copy && copy_dtype == DT_BF16) {
+    if (vec) LLMLAB_POST_NORM(bf16_t, 4); else LLMLAB_POST_NORM(bf16_t, 1);
+  } else {
+    if (vec) LLMLAB_POST_NORM(float, 4); else LLMLAB_POST_NORM(float, 1);
+  }
+#undef LLMLAB_POST_NORM
+  LLMLAB_LAUNCH_CHECK("post_norm");
   return 0;
 }
 

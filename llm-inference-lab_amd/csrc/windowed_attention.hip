@@ -21,54 +21,96 @@ __host__ __device__ inline size_t value_index(int o, int e, int E) { return ((si
 // q at column 0 (q_size = heads * D wide), then (if the layer has keys and values of its
 // own) k (kv heads * D) and v (kv heads * E).  NORM: q and k are each divided by the root
 // mean square over their WHOLE width (all heads together) and multiplied by a weight of
-// that width, in float32.  q goes to q_out (compute dtype), k and v to the row's place
-// in the pages.
+// that width, in float32.  Then the first rot_dims channels of every query and key head turn by
+// positions[r] * freq[i], channel i with i + rot_dims / 2, or (neighbours) 2i with 2i + 1.  q goes to
+// q_out (compute dtype), k and v to the row's place in the pages; query and key heads are laid out
+// DK >= D channels wide there (zeros behind).  A wave a head.
+struct NormWrite {
+  const float* proj; int ld, n_heads, n_kv, D, DK, E, own, norm; float eps; const float* q_w; const float* k_w;
+  const float* freq; int rot_dims, neighbours, page_size; const int* positions; const int* row_req; const int* table;
+  int max_pages;
+};
 template <typename T>
-__global__ __launch_bounds__(256) void project_norm_write_kernel(
-    const float* __restrict__ proj, int ld, int q_size, int k_size, int v_size, int norm, float eps,
-    const float* __restrict__ q_w, const float* __restrict__ k_w, T* __restrict__ q_out,
-    T* __restrict__ k_cache, T* __restrict__ v_cache, int n_kv, int D, int E, int page_size,
-    const int* __restrict__ positions, const int* __restrict__ row_req, const int* __restrict__ table,
-    int max_pages) {
-  __shared__ float red[17];
-  const int r = blockIdx.x;
-  const float* src = proj + (size_t)r * ld;
+__global__ __launch_bounds__(1024) void project_norm_write_kernel(NormWrite a, T* __restrict__ q_out, T* __restrict__ k_cache,
+                                                                  T* __restrict__ v_cache) {
+  extern __shared__ float norm_lds[];            // cos [half], sin [half]
+  __shared__ float red_q[16], red_k[16];
+  const int r = blockIdx.x, lane = threadIdx.x & 63, waves = blockDim.x >> 6;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const float* src = a.proj + (size_t)r * a.ld;
+  const int q_size = a.n_heads * a.D, k_size = a.own ? a.n_kv * a.D : 0, half = a.rot_dims >> 1;
+  float* s_cos = norm_lds;
+  float* s_sin = norm_lds + half;
+  const int pos = a.positions ? a.positions[r] : 0;
+  for (int i = threadIdx.x; i < half; i += blockDim.x) {
+    float sn, cs;
+    sincosf((float)pos * a.freq[i], &sn, &cs);
+    s_cos[i] = cs;
+    s_sin[i] = sn;
+  }
   float inv_q = 1.f, inv_k = 1.f;
-  if (norm) {
-    float s = 0.f;
-    for (int c = threadIdx.x; c < q_size; c += blockDim.x) s += src[c] * src[c];
-    inv_q = 1.0f / sqrtf(block_sum(s, red) / (float)q_size + eps);
-    if (k_size > 0) {
-      s = 0.f;
-      for (int c = threadIdx.x; c < k_size; c += blockDim.x) s += src[q_size + c] * src[q_size + c];
-      inv_k = 1.0f / sqrtf(block_sum(s, red) / (float)k_size + eps);
+  if (a.norm) {                                  // (both sums in one pass)
+    float sq = 0.f, sk = 0.f;
+    for (int c = threadIdx.x; c < q_size; c += blockDim.x) sq = fmaf(src[c], src[c], sq);
+    for (int c = threadIdx.x; c < k_size; c += blockDim.x) sk = fmaf(src[q_size + c], src[q_size + c], sk);
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if (lane == 0) {
+      red_q[wave] = sq;
+      red_k[wave] = sk;
     }
   }
-  for (int c = threadIdx.x; c < q_size; c += blockDim.x)
-    q_out[(size_t)r * q_size + c] = from_float<T>(norm ? src[c] * inv_q * q_w[c] : src[c]);
-  if (k_size <= 0) return;
-  const int pos = positions[r];
-  const int page = table[(size_t)row_req[r] * max_pages + pos / page_size];
-  const int slot = pos % page_size;
-  for (int c = threadIdx.x; c < k_size; c += blockDim.x) {
-    const int g = c / D, d = c - g * D;
-    const float v = norm ? src[q_size + c] * inv_k * k_w[c] : src[q_size + c];
-    k_cache[(((size_t)page * n_kv + g) * page_size + slot) * D + d] = from_float<T>(v);
+  __syncthreads();
+  if (a.norm) {
+    float sq = 0.f, sk = 0.f;
+    for (int n = 0; n < waves; ++n) {
+      sq += red_q[n];
+      sk += red_k[n];
+    }
+    inv_q = 1.0f / sqrtf(sq / (float)q_size + a.eps);
+    if (k_size > 0) inv_k = 1.0f / sqrtf(sk / (float)k_size + a.eps);
   }
-  for (int c = threadIdx.x; c < v_size; c += blockDim.x) {
-    const int g = c / E, e = c - g * E;
-    v_cache[((size_t)page * n_kv + g) * page_size * E + value_index(slot, e, E)] = from_float<T>(src[q_size + k_size + c]);
+  const int page = a.own ? a.table[(size_t)a.row_req[r] * a.max_pages + pos / a.page_size] : 0;
+  const int slot = pos % a.page_size;
+  for (int h = wave; h < a.n_heads + (a.own ? a.n_kv : 0); h += waves) {
+    const bool query = h < a.n_heads;
+    const float* x = src + (size_t)h * a.D;      // (the key heads follow the query heads)
+    const float* w = !a.norm ? nullptr : query ? a.q_w + (size_t)h * a.D : a.k_w + (size_t)(h - a.n_heads) * a.D;
+    const float inv = query ? inv_q : inv_k;
+    T* dst = query ? q_out + ((size_t)r * a.n_heads + h) * a.DK
+                   : k_cache + (((size_t)page * a.n_kv + (h - a.n_heads)) * a.page_size + slot) * a.DK;
+    for (int d = lane; d < a.DK; d += 64) {
+      float v = 0.f;
+      if (d < a.D) {
+        v = w ? x[d] * inv * w[d] : x[d];
+        if (d < a.rot_dims) {
+          const int i = a.neighbours ? d >> 1 : (d < half ? d : d - half);
+          const bool first = a.neighbours ? (d & 1) == 0 : d < half;
+          const int o = a.neighbours ? d ^ 1 : (first ? d + half : d - half);
+          const float other = w ? x[o] * inv * w[o] : x[o];
+          v = first ? v * s_cos[i] - other * s_sin[i] : v * s_cos[i] + other * s_sin[i];
+        }
+      }
+      dst[d] = from_float<T>(v);
+    }
   }
+  if (!a.own) return;
+  for (int g = wave; g < a.n_kv; g += waves)
+    for (int e = lane; e < a.E; e += 64)
+      v_cache[((size_t)page * a.n_kv + g) * a.page_size * a.E + value_index(slot, e, a.E)] =
+          from_float<T>(src[q_size + k_size + (size_t)g * a.E + e]);
 }
 
-extern "C" int llmlab_project_norm_write(const float* proj, int ld, int rows, int n_heads, int n_kv, int D, int E,
+extern "C" int llmlab_project_norm_write(const float* proj, int ld, int rows, int n_heads, int n_kv, int D, int DK, int E,
                                          int own_kv, int norm, float eps, const float* q_w, const float* k_w,
-                                         void* q_out, void* k_cache, void* v_cache, int dtype, int page_size,
-                                         const int* positions, const int* row_req, const int* table,
-                                         int max_pages, hipStream_t stream) {
-  LLMLAB_REQUIRE(rows >= 0 && n_heads > 0 && n_kv > 0 && D > 0 && E > 0 && page_size > 0,
-                 "project_norm_write: bad sizes rows=%d heads=%d kv=%d D=%d E=%d page=%d", rows, n_heads, n_kv, D, E,
-                 page_size);
+                                         const float* freq, int rot_dims, int neighbours, void* q_out, void* k_cache,
+                                         void* v_cache, int dtype, int page_size, const int* positions,
+                                         const int* row_req, const int* table, int max_pages, hipStream_t stream) {
+  LLMLAB_REQUIRE(rows >= 0 && n_heads > 0 && n_kv > 0 && D > 0 && DK >= D && E > 0 && page_size > 0,
+                 "project_norm_write: bad sizes rows=%d heads=%d kv=%d D=%d (%d) E=%d page=%d", rows, n_heads, n_kv, D, DK,
+                 E, page_size);
+  LLMLAB_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= D && (rot_dims == 0 || (freq && positions)),
+                 "project_norm_write: %d of %d channels cannot turn in pairs", rot_dims, D);
   const int q_size = n_heads * D, k_size = own_kv ? n_kv * D : 0, v_size = own_kv ? n_kv * E : 0;
   LLMLAB_REQUIRE(ld >= q_size + k_size + v_size, "project_norm_write: rows of %d numbers do not hold %d", ld,
                  q_size + k_size + v_size);
@@ -76,14 +118,17 @@ extern "C" int llmlab_project_norm_write(const float* proj, int ld, int rows, in
   LLMLAB_REQUIRE(!own_kv || (k_cache && v_cache && positions && row_req && table),
                  "project_norm_write: keys and values need pages to go to");
   if (rows == 0) return 0;
+  const NormWrite a{proj, ld, n_heads, n_kv, D, DK, E, own_kv, norm, eps, q_w, k_w, freq, rot_dims, neighbours, page_size,
+                    positions, row_req, table, max_pages};
+  // few rows: more waves, a head a wave
+  const int threads = rows <= 64 && n_heads > 4 ? 1024 : 256;
+  const size_t lds = (size_t)rot_dims * sizeof(float);
   if (dtype == DT_BF16)
-    hipLaunchKernelGGL(project_norm_write_kernel<bf16_t>, dim3(rows), dim3(256), 0, stream, proj, ld, q_size, k_size,
-                       v_size, norm, eps, q_w, k_w, (bf16_t*)q_out, (bf16_t*)k_cache, (bf16_t*)v_cache, n_kv, D, E,
-                       page_size, positions, row_req, table, max_pages);
+    hipLaunchKernelGGL(project_norm_write_kernel<bf16_t>, dim3(rows), dim3(threads), lds, stream, a, (bf16_t*)q_out,
+                       (bf16_t*)k_cache, (bf16_t*)v_cache);
   else
-    hipLaunchKernelGGL(project_norm_write_kernel<float>, dim3(rows), dim3(256), 0, stream, proj, ld, q_size, k_size,
-                       v_size, norm, eps, q_w, k_w, (float*)q_out, (float*)k_cache, (float*)v_cache, n_kv, D, E,
-                       page_size, positions, row_req, table, max_pages);
+    hipLaunchKernelGGL(project_norm_write_kernel<float>, dim3(rows), dim3(threads), lds, stream, a, (float*)q_out,
+                       (float*)k_cache, (float*)v_cache);
   LLMLAB_LAUNCH_CHECK("project_norm_write");
   return 0;
 }
@@ -546,12 +591,15 @@ struct Mask {
     return chunk > 0 ? i - i % chunk : 0;
   }
 };
-// A gate per channel of the heads' outputs, applied where an output is made final: column c of row r is
-// multiplied by sigmoid(p[r * ld + c]) (float32; p null: no gate).
+// A gate on the heads' outputs, applied where an output is made final: column c of row r is multiplied by
+// sigmoid(p[r * ld + c]), or (per_head) all of head h by sigmoid(p[r * ld + h]) (float32; p null: no gate).
 struct Gate {
-  const float* p; int ld;
+  const float* p; int ld, per_head;
   __device__ __forceinline__ float at(int r, int c) const {
-    return p ? 1.0f / (1.0f + __expf(-p[(size_t)r * ld + c])) : 1.f;
+    return p && !per_head ? 1.0f / (1.0f + __expf(-p[(size_t)r * ld + c])) : 1.f;
+  }
+  __device__ __forceinline__ float head(int r, int h) const {
+    return p && per_head ? 1.0f / (1.0f + __expf(-p[(size_t)r * ld + h])) : 1.f;
   }
 };
 // (lo: the mask's low(i), taken once per query)
@@ -683,7 +731,7 @@ __global__ __launch_bounds__(64) void sink_window_attention_kernel(
       __syncthreads();
     }
   }
-  const float inv = 1.0f / l;
+  const float inv = gate.head(r, h) / l;
 #pragma unroll
   for (int c = 0; c < MAX_E_PER_LANE; ++c) {
     const int e = lane + 64 * c;
@@ -913,7 +961,7 @@ __global__ __launch_bounds__(256) void sink_window_attention_mfma_kernel(MfmaArg
   }
   if (!row_ok) return;
   if (a.long_from > 0 && a.q_start[req + 1] - a.q_start[req] < a.long_from) return;
-  const float inv = 1.0f / run.l;
+  const float inv = a.gate.head(r, h) / run.l;
 #pragma unroll
   for (int eb = 0; eb < EB; ++eb) {
     bf16x4 w;
@@ -1138,7 +1186,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
   }
   if (!row_ok || !head_ok) return;
   if (a.long_from > 0 && a.q_start[req + 1] - a.q_start[req] < a.long_from) return;
-  const float inv = 1.0f / run.l;
+  const float inv = a.gate.head(r, h) / run.l;
 #pragma unroll
   for (int eb = 0; eb < EB; ++eb) {
     bf16x4 w;
@@ -1189,7 +1237,7 @@ __global__ __launch_bounds__(64) void sink_window_attention_grouped_kernel(MfmaA
                        a.k_cache, a.v_cache, a.mask, a.scale, run, a.mode, bias);
   if (!head_ok) return;
   if (a.splits == 1) {
-    const float inv = 1.0f / run.l;
+    const float inv = a.gate.head(r, h) / run.l;
 #pragma unroll
     for (int eb = 0; eb < EB; ++eb) {
       bf16x4 w;
@@ -1241,7 +1289,7 @@ __global__ __launch_bounds__(64) void sink_window_attention_merge_kernel(MfmaArg
   }
   den = wave_sum(den);
   __syncthreads();
-  const float inv = 1.0f / den;
+  const float inv = a.gate.head(r, h) / den;
   for (int e = threadIdx.x; e < E; e += 64) {
     float acc = 0.f;
     int z = 0;
@@ -1319,10 +1367,10 @@ extern "C" int llmlab_sink_window_attention(const void* q, int dtype, int rows, 
                                             int keep_first, int chunk, const float* sink, float scale, void* out,
                                             const int* q_start, int long_from, int launches, int max_keys,
                                             float* workspace, size_t workspace_floats, int num_cus, int mode,
-                                            const float* gate, int gate_ld, hipStream_t stream) {
-  LLMLAB_REQUIRE(gate == nullptr || gate_ld >= n_heads * E, "sink_window_attention: a gate per channel, rows of %d numbers",
-                 gate_ld);
-  const Gate gates{gate, gate_ld};
+                                            const float* gate, int gate_ld, int gate_per_head, hipStream_t stream) {
+  LLMLAB_REQUIRE(gate == nullptr || gate_ld >= (gate_per_head ? n_heads : n_heads * E),
+                 "sink_window_attention: a gate per channel or head, rows of %d numbers", gate_ld);
+  const Gate gates{gate, gate_ld, gate_per_head};
   LLMLAB_REQUIRE(mode == MODE_SOFTMAX || mode == MODE_SIGMOID, "sink_window_attention: unknown weighting %d", mode);
   LLMLAB_REQUIRE(rows >= 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0 && D > 0 && E > 0,
                  "sink_window_attention: bad sizes rows=%d heads=%d kv=%d D=%d E=%d", rows, n_heads, n_kv, D, E);

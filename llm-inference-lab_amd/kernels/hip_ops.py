@@ -16,7 +16,7 @@ from typing import Dict, Optional
 import torch
 
 from ..config.errors import UnsupportedSizeError
-from ..parts.base import PendingSums
+from ..parts.base import ChosenSums, PendingSums
 from . import build
 from .debug import DispatchRules, KernelDebug
 
@@ -24,7 +24,9 @@ DT_F32, DT_BF16 = 0, 1
 EPI_STORE, EPI_RESID, EPI_F32, EPI_SWIGLU, EPI_QKV, EPI_PART = 0, 1, 2, 3, 4, 5
 EPI_RELU2 = 6        # STORE through max(z, 0)^2, taken on the float32 sum
 EPI_GEGLU = 7        # the paired product with gelu (tanh form) on the gate instead of silu
-GATE_EPILOGUES = {"silu": EPI_SWIGLU, "gelu_tanh": EPI_GEGLU}
+EPI_CLAMPED = 8      # the paired product as the clamped pair (limit, slope, shift)
+GATE_EPILOGUES = {"silu": EPI_SWIGLU, "gelu_tanh": EPI_GEGLU, "clamped": EPI_CLAMPED}
+NO_CONSTANTS = (0.0, 0.0, 0.0)
 
 _c_int, _c_long, _c_float, _c_size, _c_ptr = (ctypes.c_int, ctypes.c_long, ctypes.c_float,
                                               ctypes.c_size_t, ctypes.c_void_p)
@@ -187,7 +189,7 @@ class HipOps:
             self.device = torch.device("cuda", torch.cuda.current_device())
         self._core = self._load(build.core_library())
         self._declare_core()
-        if self._core.llmlab_abi_version() != 8:
+        if self._core.llmlab_abi_version() != 9:
             raise RuntimeError("kernel library and Python bindings disagree on the interface")
         self._attn: Dict[int, ctypes.CDLL] = {}
         self._mixer_libs: Dict[str, ctypes.CDLL] = {}
@@ -226,7 +228,7 @@ class HipOps:
         c.llmlab_rope_inplace.argtypes = [_c_ptr, _c_int, _c_int, _c_int, _c_int, _c_long, _c_long,
                                           _c_ptr, _c_ptr, _c_ptr]
         c.llmlab_linear.argtypes = [_c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_int,
-                                    _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr]
+                                    _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_ptr]
         c.llmlab_sample.argtypes = [_c_ptr, _c_long, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr]
         c.llmlab_gather_tokens.argtypes = [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr]
         c.llmlab_gather_tokens.restype = _c_int
@@ -254,7 +256,7 @@ class HipOps:
             _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_float, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr,
             _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
             _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int,
-            _c_ptr, _c_int, _c_int, _c_size, _c_int, _c_size, _c_int, _c_ptr, _c_size, _c_ptr]
+            _c_ptr, _c_int, _c_int, _c_size, _c_int, _c_size, _c_int, _c_ptr, _c_size, _c_float, _c_float, _c_float, _c_ptr]
         c.llmlab_add_pending.argtypes = [_c_ptr, _c_ptr, _c_int, _c_size, _c_int, _c_int, _c_ptr]
         c.llmlab_add_pending.restype = _c_int
         c.llmlab_layernorm.argtypes = [_c_ptr, _c_ptr, _c_int, _c_float, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr]
@@ -269,7 +271,7 @@ class HipOps:
         c.llmlab_add_row_vector.argtypes = [_c_ptr, _c_ptr, _c_int, _c_int, _c_ptr]
         c.llmlab_add_row_vector.restype = _c_int
         c.llmlab_linear_grouped.argtypes = [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int,
-                                            _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr]
+                                            _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_float, _c_float, _c_ptr]
         c.llmlab_linear_grouped.restype = _c_int
         for fn in (c.llmlab_embed, c.llmlab_rmsnorm, c.llmlab_rope_kv_write, c.llmlab_rope_inplace,
                    c.llmlab_linear, c.llmlab_sample, c.llmlab_skinny_linear,
@@ -499,7 +501,8 @@ class HipOps:
                                               pend[0], pend[1], pend[2], self._stream())
 
     # ----------------------------------------------------------------- linear
-    def _linear(self, x, w, out, bias, epilogue, n_out, pending: Optional[PendingSums] = None) -> None:
+    def _linear(self, x, w, out, bias, epilogue, n_out, pending: Optional[PendingSums] = None,
+                constants=NO_CONSTANTS) -> None:
         self._need(x, "linear input")
         w = self._weight(w, "linear weight")
         if x.dtype != w.dtype:
@@ -514,7 +517,7 @@ class HipOps:
         if x.dtype == torch.bfloat16 and k % 8 != 0:
             raise UnsupportedSizeError(
                 f"bfloat16 matrix products need an inner size that is a multiple of 8, got {k}")
-        want_out = x.dtype if epilogue in (EPI_STORE, EPI_SWIGLU, EPI_RELU2, EPI_GEGLU) else torch.float32
+        want_out = x.dtype if epilogue in (EPI_STORE, EPI_SWIGLU, EPI_RELU2, EPI_GEGLU, EPI_CLAMPED) else torch.float32
         if out.dtype != want_out:
             raise TypeError(f"linear: output must be {want_out}, got {out.dtype}")
         if bias is not None:
@@ -526,13 +529,13 @@ class HipOps:
         # for narrow outputs (the tiled kernel has too few tiles there), measured
         if x.dtype == torch.bfloat16 and (m <= 16 or (n < 8192 and self.few_rows_take(m, n, k))):
             self._skinny(x, False, None, None, 0.0, w, bias, epilogue, out, m, n, k, ldo, n_out,
-                         pending=pending)
+                         pending=pending, constants=constants)
             return
         if pending is not None:
             self.add_pending(out, pending)
         self._call(self._core.llmlab_linear,
             self._ptr(x), self._ptr(w), _dt(x), epilogue, self._ptr(out), self._ptr(bias),
-            _dt(bias) if bias is not None else 0, m, n, k, ldo, n_out, self.num_cus, self._stream())
+            _dt(bias) if bias is not None else 0, m, n, k, ldo, n_out, self.num_cus, *constants, self._stream())
 
     def linear(self, x, w, out, bias=None) -> None:
         self._linear(x, w, out, bias, EPI_STORE, w.shape[0])
@@ -549,16 +552,25 @@ class HipOps:
     def linear_logits(self, x, w, out, bias=None) -> None:
         self._linear(x, w, out, bias, EPI_F32, w.shape[0])
 
-    def linear_swiglu(self, x, w_gate_up, out, activation: str = "silu") -> None:
+    @staticmethod
+    def _pair_constants(activation: str, constants):
+        if (activation == "clamped") != (constants is not None):
+            raise ValueError("the clamped pair has three constants (limit, slope, shift), the other activations none")
+        return NO_CONSTANTS if constants is None else tuple(float(c) for c in constants)
+
+    def linear_swiglu(self, x, w_gate_up, out, activation: str = "silu", constants=None) -> None:
         """``out = act(x Wg^T) * (x Wu^T)`` with the rows of gate and up interleaved in runs of 16;
-        ``activation``: ``silu`` or ``gelu_tanh``, taken on the float32 sums."""
+        ``activation``: ``silu`` or ``gelu_tanh``, taken on the float32 sums; or ``clamped`` with ``constants =
+        (limit, slope, shift)``: ``g * sigmoid(slope * g) * (u + shift)``, ``g`` the gate's number held to at most
+        ``limit`` and ``u`` the other held within ``-limit .. limit``."""
         inter = out.shape[1]
         if w_gate_up.shape[0] != 2 * ((inter + 15) // 16 * 16):
             raise ValueError(f"linear_swiglu: {w_gate_up.shape[0]} interleaved rows do not belong "
                              f"to {inter} outputs")
         if activation not in GATE_EPILOGUES:
             raise ValueError(f"linear_swiglu: the gate's activation is one of {sorted(GATE_EPILOGUES)}, got {activation!r}")
-        self._linear(x, w_gate_up, out, None, GATE_EPILOGUES[activation], inter)
+        self._linear(x, w_gate_up, out, None, GATE_EPILOGUES[activation], inter,
+                     constants=self._pair_constants(activation, constants))
 
     # ----------------------------------------------- few rows: fused kernels
     FUSED_MAX_ROWS = 1024         # most rows the few-row kernels take at all
@@ -590,7 +602,7 @@ class HipOps:
 
     def _skinny(self, x, norm, x_rows, norm_w, eps, w, bias, epilogue, out, m, n, k, ldo, n_out,
                 qkv=None, pending: Optional[PendingSums] = None, ksplit: int = 1,
-                part_stride: int = 0, segments=None) -> None:
+                part_stride: int = 0, segments=None, constants=NO_CONSTANTS) -> None:
         if pending is not None:
             p = pending.parts
             if (p.dtype != torch.float32 or p.dim() != 3 or p.stride(2) != 1 or p.device != self.device
@@ -614,7 +626,7 @@ class HipOps:
             _dt(norm_w) if norm_w is not None else 0, float(eps), w.data_ptr(), self._ptr(bias),
             _dt(bias) if bias is not None else 0, epilogue, out.data_ptr(), m, n, k, ldo, n_out,
             *heads, self.num_cus, pend[0], pend[1], pend[2], pend[3], int(ksplit),
-            int(part_stride), *(segments or (1, None, 0)), self._stream())
+            int(part_stride), *(segments or (1, None, 0)), *constants, self._stream())
 
     # --------------------------------------------- products whose columns read inputs of their own
     def prepare_segments(self, weights) -> "SegmentedWeight":
@@ -1108,13 +1120,14 @@ class HipOps:
             lib.llmlab_last_error.restype = ctypes.c_char_p
             if kind == "windowed_attention":
                 lib.llmlab_project_norm_write.argtypes = [
-                    _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_ptr,
-                    _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr]
+                    _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_ptr,
+                    _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int,
+                    _c_ptr]
                 lib.llmlab_project_norm_write.restype = _c_int
                 lib.llmlab_sink_window_attention.argtypes = [
                     _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
                     _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_int, _c_int, _c_int,
-                    _c_ptr, _c_size, _c_int, _c_int, _c_ptr, _c_int, _c_ptr]
+                    _c_ptr, _c_size, _c_int, _c_int, _c_ptr, _c_int, _c_int, _c_ptr]
                 lib.llmlab_sink_window_attention.restype = _c_int
                 lib.llmlab_project_conv_write.argtypes = [
                     _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr,
@@ -1158,6 +1171,9 @@ class HipOps:
                 lib.llmlab_rmsnorm_add.argtypes = [_c_ptr, _c_ptr, _c_int, _c_size, _c_ptr, _c_float, _c_int, _c_int,
                                                    _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr]
                 lib.llmlab_rmsnorm_add.restype = _c_int
+                lib.llmlab_post_norm.argtypes = [_c_ptr, _c_float, _c_ptr, _c_int, _c_size, _c_ptr, _c_ptr, _c_int, _c_ptr,
+                                                 _c_float, _c_int, _c_int, _c_ptr, _c_int, _c_ptr]
+                lib.llmlab_post_norm.restype = _c_int
                 lib.llmlab_scaled_sum.argtypes = [_c_ptr, _c_ptr, _c_float, _c_ptr, _c_float, _c_size, _c_ptr]
                 lib.llmlab_scaled_sum.restype = _c_int
                 lib.llmlab_normed_sum.argtypes = [_c_ptr, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_float,
@@ -1211,9 +1227,14 @@ class HipOps:
                                                   _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int,
                                                   _c_ptr, _c_ptr, _c_int, _c_ptr]
                 lib.llmlab_delta_scan.restype = _c_int
+            elif kind == "gated_recurrence":
+                lib.llmlab_gated_recurrence.argtypes = [
+                    _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
+                    _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr]
+                lib.llmlab_gated_recurrence.restype = _c_int
             elif kind == "routed_experts":
                 lib.llmlab_moe_select.argtypes = [_c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
-                                                  _c_ptr, _c_ptr, _c_int, _c_ptr]
+                                                  _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_ptr]
                 lib.llmlab_moe_select.restype = _c_int
                 lib.llmlab_moe_add_chosen.argtypes = [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_int,
                                                       _c_int, _c_int, _c_ptr]
@@ -1223,7 +1244,7 @@ class HipOps:
                 lib.llmlab_moe_plan.restype = _c_int
                 lib.llmlab_moe_select_plan.argtypes = [_c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
                                                        _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
-                                                       _c_int, _c_ptr]
+                                                       _c_int, _c_int, _c_float, _c_ptr]
                 lib.llmlab_moe_select_plan.restype = _c_int
                 lib.llmlab_moe_combine.argtypes = [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
                                                    _c_int, _c_int, _c_ptr]
@@ -1278,9 +1299,16 @@ class HipOps:
         return 0 < rows <= self.rules.select_plan_max_rows and outputs <= 64
 
     SCORINGS = {"softmax": 0, "sigmoid": 1}
+    GROUP_SCORES = {"max": 0, "top2": 1}
+
+    def _choice(self, group_score: str, share_eps):
+        if share_eps is not None and share_eps < 0:
+            raise ValueError(f"what is added to the sum of the chosen scores is not negative, got {share_eps}")
+        return self.GROUP_SCORES[group_score], -1.0 if share_eps is None else float(share_eps)
 
     def moe_select_plan(self, logits, correction, groups: int, groups_keep: int, scale: float, chosen, weights,
-                        num_experts: int, scratch, scoring: str = "softmax") -> "MoePlan":
+                        num_experts: int, scratch, scoring: str = "softmax", group_score: str = "max",
+                        share_eps=None) -> "MoePlan":
         """``moe_select`` and ``moe_plan`` in one launch of one block, for steps of few rows."""
         lib = self._mixer_lib("routed_experts")
         for t, name, dt in ((logits, "router logits", torch.float32), (correction, "router correction", torch.float32),
@@ -1295,7 +1323,7 @@ class HipOps:
         self._call(lib.llmlab_moe_select_plan, self._ptr(logits), self._ptr(correction), rows, outputs, int(groups),
                    int(groups_keep), top, float(scale), self._ptr(chosen), self._ptr(weights), int(num_experts), plan.bm,
                    plan.capacity, self._ptr(plan.place_of), self._ptr(plan.place_row), self._ptr(plan.tile_member),
-                   self.SCORINGS[scoring], self._stream(), lib=lib)
+                   self.SCORINGS[scoring], *self._choice(group_score, share_eps), self._stream(), lib=lib)
         return plan
 
     def moe_plan(self, chosen, num_experts: int, scratch) -> "MoePlan":
@@ -1312,7 +1340,8 @@ class HipOps:
                    lib=lib)
         return plan
 
-    def _grouped(self, x, stacked: "StackedWeight", plan: "MoePlan", out, epilogue, n_out, rows_index) -> None:
+    def _grouped(self, x, stacked: "StackedWeight", plan: "MoePlan", out, epilogue, n_out, rows_index,
+                 constants=NO_CONSTANTS) -> None:
         w = stacked.data
         if not isinstance(w, PackedWeight) or x.dtype != torch.bfloat16:
             raise TypeError("grouped products are bfloat16 products over a packed stack of matrices")
@@ -1327,14 +1356,19 @@ class HipOps:
                    plan.capacity, stacked.padded, stacked.k, out.stride(0), int(n_out), self._ptr(plan.tile_member),
                    self._ptr(rows_index), plan.bm,
                    1 if plan.bm == 128 and stacked.padded >= self.rules.grouped_wide_min_columns else 0,
-                   self._stream())
+                   *constants, self._stream())
 
-    def moe_gate_up(self, h, w_gate_up: "StackedWeight", plan: "MoePlan", act) -> None:
+    def moe_gate_up(self, h, w_gate_up: "StackedWeight", plan: "MoePlan", act, activation: str = "silu",
+                    constants=None) -> None:
         """``act[place] = silu(h[row] Wg_e^T) * (h[row] Wu_e^T)`` for every place of the plan, ``e`` the
-        expert of the place's tile and ``row`` the row of ``h`` at the place."""
+        expert of the place's tile and ``row`` the row of ``h`` at the place; ``activation="clamped"`` with its
+        ``constants`` as in ``linear_swiglu``."""
+        if activation not in ("silu", "clamped"):
+            raise ValueError(f"moe_gate_up: 'silu' or 'clamped', got {activation!r}")
         if act.dtype != torch.bfloat16 or 2 * ((act.shape[1] + 15) // 16 * 16) != w_gate_up.n:
             raise ValueError("moe_gate_up: the experts' gate and up rows do not interleave the outputs")
-        self._grouped(h, w_gate_up, plan, act, EPI_SWIGLU, act.shape[1], plan.place_row)
+        self._grouped(h, w_gate_up, plan, act, GATE_EPILOGUES[activation], act.shape[1], plan.place_row,
+                      self._pair_constants(activation, constants))
 
     def moe_up_relu2(self, h, w_up: "StackedWeight", plan: "MoePlan", act) -> None:
         """``act[place] = max(h[row] Wu_e^T, 0) ** 2`` for every place of the plan (experts without a
@@ -1365,13 +1399,15 @@ class HipOps:
                    int(num_experts), hidden, self._stream(), lib=lib)
 
     def moe_select(self, logits, correction, groups: int, groups_keep: int, scale: float, chosen, weights,
-                   scoring: str = "softmax") -> None:
+                   scoring: str = "softmax", group_score: str = "max", share_eps=None) -> None:
         """Per row of the router's float32 ``logits [rows, outputs]``: scores ``softmax(logits)``
         (``scoring="sigmoid"``: the sigmoid of every logit by itself); choice
         values ``score + correction``; the outputs form ``groups`` equal groups of neighbours of which
         the ``groups_keep`` with the largest best choice value stay; ``chosen [rows, top]`` (int32) are
         the outputs with the largest choice values among those (ties: the smaller index), ``weights
-        [rows, top]`` their scores times ``scale``."""
+        [rows, top]`` their scores times ``scale``.  ``group_score="top2"``: a group counts as the sum of its two
+        largest choice values.  ``share_eps`` (None: as they are): the chosen scores are divided by their sum
+        plus so much before they are scaled."""
         lib = self._mixer_lib("routed_experts")
         self._need(logits, "router logits", torch.float32)
         self._need(correction, "router correction", torch.float32)
@@ -1383,7 +1419,7 @@ class HipOps:
             raise ValueError("moe_select: shapes do not fit")
         self._call(lib.llmlab_moe_select, self._ptr(logits), self._ptr(correction), rows, outputs, int(groups),
                    int(groups_keep), top, float(scale), self._ptr(chosen), self._ptr(weights), self.SCORINGS[scoring],
-                   self._stream(), lib=lib)
+                   *self._choice(group_score, share_eps), self._stream(), lib=lib)
 
     def moe_add_chosen(self, resid, src, chosen, weights, first: int, last: int) -> None:
         """``resid[r] += w_r * src[r]`` with ``w_r`` the sum of ``weights[r, k]`` over the ``k`` whose
@@ -1430,18 +1466,24 @@ class HipOps:
             raise TypeError("windowed attention: queries and cache share one dtype")
 
     def project_norm_write(self, proj, num_heads, num_kv_heads, key_dim, value_dim, own_kv, q_norm, k_norm, eps,
-                           q_out, k_cache, v_cache, page_size, positions, row_req, block_table) -> None:
+                           q_out, k_cache, v_cache, page_size, positions, row_req, block_table, freq=None,
+                           rot_dims: int = 0, pairing: str = "halves") -> None:
         """From the float32 projections ``proj [rows, >= q (+ k + v)]``: the queries (divided by
         the root mean square over their whole width and multiplied by ``q_norm`` if that is
         given) into ``q_out``, and, if the layer has keys and values of its own, the keys
-        (normed alike with ``k_norm``) and values into the rows' places in the pages."""
+        (normed alike with ``k_norm``) and values into the rows' places in the pages.  ``rot_dims``: after
+        the norm so many first channels of every query and key head turn by ``positions[r] * freq[i]``,
+        channel ``i`` with ``i + rot_dims / 2`` (``pairing="neighbours"``: ``2i`` with ``2i + 1``).  Heads may be laid
+        out wider than ``key_dim`` in ``q_out [rows, heads * DK]`` and the key pages (zeros behind)."""
         lib = self._mixer_lib("windowed_attention")
         self._need(proj, "projections", torch.float32)
         self._need(q_out, "queries")
         rows = q_out.shape[0]
         q_size = num_heads * key_dim
         need = q_size + (num_kv_heads * (key_dim + value_dim) if own_kv else 0)
-        if proj.shape[0] != rows or proj.shape[1] < need or tuple(q_out.shape) != (rows, q_size):
+        laid = q_out.shape[1] // num_heads
+        if (proj.shape[0] != rows or proj.shape[1] < need or tuple(q_out.shape) != (rows, num_heads * laid)
+                or laid < key_dim):
             raise ValueError(f"project_norm_write: projections {tuple(proj.shape)}, queries {tuple(q_out.shape)} "
                              f"do not fit {need} numbers a row")
         norm = q_norm is not None
@@ -1449,8 +1491,14 @@ class HipOps:
             self._need(q_norm, "query norm weight", torch.float32)
             if q_norm.numel() != q_size:
                 raise ValueError("project_norm_write: the query norm's weight spans all heads")
+        rot_dims = int(rot_dims or 0)
+        if rot_dims:
+            self._need(freq, "rotation frequencies", torch.float32)
+            self._need(positions, "positions", torch.int32)
+            if rot_dims % 2 or rot_dims > key_dim or freq.numel() != rot_dims // 2 or positions.numel() < rows:
+                raise ValueError(f"project_norm_write: {rot_dims} of {key_dim} channels with {freq.numel()} frequencies")
         if own_kv:
-            self._paged(k_cache, v_cache, num_kv_heads, page_size, key_dim, value_dim, q_out.dtype)
+            self._paged(k_cache, v_cache, num_kv_heads, page_size, laid, value_dim, q_out.dtype)
             if norm:
                 self._need(k_norm, "key norm weight", torch.float32)
                 if k_norm.numel() != num_kv_heads * key_dim:
@@ -1460,10 +1508,12 @@ class HipOps:
             if positions.numel() < rows or row_req.numel() < rows or block_table.stride(1) != 1:
                 raise ValueError("project_norm_write: one position and one request index per row")
         self._call(lib.llmlab_project_norm_write, self._ptr(proj), proj.stride(0), rows, num_heads, num_kv_heads,
-                   key_dim, value_dim, 1 if own_kv else 0, 1 if norm else 0, float(eps), self._ptr(q_norm),
-                   self._ptr(k_norm) if own_kv and norm else None, self._ptr(q_out),
+                   key_dim, laid, value_dim, 1 if own_kv else 0, 1 if norm else 0, float(eps), self._ptr(q_norm),
+                   self._ptr(k_norm) if own_kv and norm else None, self._ptr(freq) if rot_dims else None, rot_dims,
+                   {"halves": 0, "neighbours": 1}[pairing], self._ptr(q_out),
                    self._ptr(k_cache) if own_kv else None, self._ptr(v_cache) if own_kv else None, _dt(q_out),
-                   page_size, self._ptr(positions) if own_kv else None, self._ptr(row_req) if own_kv else None,
+                   page_size, self._ptr(positions) if own_kv or rot_dims else None,
+                   self._ptr(row_req) if own_kv else None,
                    self._ptr(block_table) if own_kv else None, block_table.stride(0) if own_kv else 0,
                    self._stream(), lib=lib)
 
@@ -1490,7 +1540,7 @@ class HipOps:
     def sink_window_attention(self, q, num_heads, num_kv_heads, key_dim, value_dim, k_cache, v_cache, block_table,
                               page_size, positions, row_req, window, keep_first, sink, scale, out,
                               q_start=None, long_from=0, launches=3, max_keys=0, weights: str = "softmax",
-                              chunk=None, gate=None) -> None:
+                              chunk=None, gate=None, head_gate=None) -> None:
         """The query of row ``r`` at position ``i = positions[r]`` of request ``row_req[r]`` attends
         to the cached keys ``j <= i`` with ``i - j < window`` or ``j < keep_first`` (``window`` None:
         all); ``sink`` (float32 per head, or None) adds ``exp(sink)`` to the softmax's denominator.
@@ -1499,7 +1549,7 @@ class HipOps:
         ``chunk`` (with ``window`` None): the keys of the query's own chunk of so many positions, ``j <=
         i`` with ``j // chunk == i // chunk`` (or ``j < keep_first``).  ``gate = (proj, column)``: the output's
         number ``c`` of row ``r`` is multiplied by ``sigmoid(proj[r, column + c])`` (float32 ``proj``) before it is
-        rounded.
+        rounded; ``head_gate = (proj, column)``: all of head ``h`` by ``sigmoid(proj[r, column + h])``.
         ``long_from > 0`` (``windowed_attention_long_rows``: sizes that the matrix cores take):
         requests that bring at least so many rows (by ``q_start``) are served in tiles of 16 rows
         of a head, the others a row and a group of heads at a time with the row's keys cut into
@@ -1529,10 +1579,13 @@ class HipOps:
             if sink.numel() != num_heads:
                 raise ValueError("windowed attention: one sink per head")
         gate_ptr, gate_ld = None, 0
-        if gate is not None:
-            gate_rows, column = gate
+        if gate is not None and head_gate is not None:
+            raise ValueError("windowed attention: a gate per channel or one per head")
+        if gate is not None or head_gate is not None:
+            gate_rows, column = gate if gate is not None else head_gate
+            gates = num_heads * (value_dim if gate is not None else 1)
             self._need(gate_rows, "gates", torch.float32)
-            if gate_rows.shape[0] != rows or column < 0 or column + num_heads * value_dim > gate_rows.shape[1]:
+            if gate_rows.shape[0] != rows or column < 0 or column + gates > gate_rows.shape[1]:
                 raise ValueError(f"windowed attention: gates at column {column} of {tuple(gate_rows.shape)} for outputs "
                                  f"{tuple(out.shape)}")
             gate_ptr, gate_ld = gate_rows.data_ptr() + 4 * int(column), gate_rows.stride(0)
@@ -1544,7 +1597,7 @@ class HipOps:
                    int(keep_first or 0), int(chunk or 0), self._ptr(sink), float(scale), self._ptr(out),
                    self._ptr(q_start) if long_from else None, int(long_from), int(launches), int(max_keys),
                    self._ptr(self.workspace), self.workspace.numel(), self.num_cus, self.ATTENTION_WEIGHTS[weights],
-                   gate_ptr, gate_ld, self._stream(), lib=lib)
+                   gate_ptr, gate_ld, 1 if head_gate is not None else 0, self._stream(), lib=lib)
 
     ATTENTION_WEIGHTS = {"softmax": 0, "sigmoid": 1}
 
@@ -2199,6 +2252,107 @@ class HipOps:
                    float(eps), rows, width, self._ptr(next_w), float(next_eps), self._ptr(next_out),
                    _dt(next_out) if next_out is not None else 0, self._ptr(shift_state), self._ptr(shift_rows),
                    self._stream(), lib=lib)
+
+    def post_norm(self, x, alpha: float, y, weight, eps: float, copy=None) -> None:
+        """``x = v / sqrt(mean(v^2) + eps) * weight`` with ``v = alpha * x + y`` row by row, all float32: a norm behind
+        the sum of a sublayer's result and the stream.  ``y [rows, width]``, a product left in pieces
+        (``PendingSums``), or experts' results not summed yet (``ChosenSums``), summed on the way.  ``copy``
+        (a kernel dtype, or None) receives the new rows."""
+        lib = self._mixer_lib("stream_ops")
+        self._need(x, "stream", torch.float32)
+        self._need(weight, "norm weight", torch.float32)
+        rows, width = x.shape
+        places = shares = None
+        pieces, stride, top = 1, 0, 0
+        if isinstance(y, ChosenSums):
+            places, shares, y = y.place_of, y.weights, y.rows
+            self._need(places, "places of the choices", torch.int32)
+            self._need(shares, "weights of the choices", torch.float32)
+            self._need(y, "experts' results", torch.float32)
+            top = places.shape[1]
+            if places.shape[0] != rows or tuple(shares.shape) != tuple(places.shape) or y.shape[1] != width:
+                raise ValueError(f"post_norm: choices {tuple(places.shape)} of results {tuple(y.shape)} onto {tuple(x.shape)}")
+        elif isinstance(y, PendingSums):
+            parts, pieces = y.parts, y.splits
+            if (parts.dtype != torch.float32 or parts.dim() != 3 or tuple(parts.shape[1:]) != (rows, width)
+                    or not parts.is_contiguous() or not 1 <= pieces <= parts.shape[0]):
+                raise ValueError("post_norm: pieces are float32 [pieces, rows, width]")
+            stride, y = parts.stride(0), parts
+        else:
+            self._need(y, "sublayer result", torch.float32)
+            if tuple(y.shape) != (rows, width):
+                raise ValueError(f"post_norm: result {tuple(y.shape)} onto a stream {tuple(x.shape)}")
+        if weight.numel() != width:
+            raise ValueError("post_norm: one weight per column")
+        if copy is not None:
+            self._need(copy, "stream copy")
+            if tuple(copy.shape) != (rows, width):
+                raise ValueError("post_norm: a copy has the stream's shape")
+        self._call(lib.llmlab_post_norm, self._ptr(x), float(alpha), self._ptr(y), int(pieces), int(stride),
+                   self._ptr(places), self._ptr(shares), int(top), self._ptr(weight), float(eps), rows, width,
+                   self._ptr(copy), _dt(copy) if copy is not None else 0, self._stream(), lib=lib)
+
+    # ------------------------------------- recurrences of single numbers with block-diagonal gates
+    def prepare_block_gates(self, w_r: torch.Tensor, w_i: torch.Tensor) -> torch.Tensor:
+        """Two stacks of square matrices ``[parts, size, size]`` (``[out, in]``, ``size`` a multiple of 32) in the
+        order the recurrence's kernels read them: per part, strip of 16 outputs and 32 inputs the operand of
+        either matrix, a lane eight numbers."""
+        parts, size, inner = w_r.shape
+        if tuple(w_i.shape) != tuple(w_r.shape) or inner != size or size % 32 or w_r.dtype != w_i.dtype:
+            raise ValueError(f"prepare_block_gates: {tuple(w_r.shape)} and {tuple(w_i.shape)}")
+        both = torch.stack([w_r, w_i])                                   # [2, parts, out, in]
+        both = both.view(2, parts, size // 16, 16, size // 32, 4, 8)     # [2, part, strip, c, step, g, 8]
+        return self._need(both.permute(1, 2, 4, 0, 5, 3, 6).contiguous(), "gates")
+
+    def gated_recurrence(self, proj, off_x: int, off_y: int, size: int, conv, conv_bias, ring, gates, r_bias, i_bias,
+                         decay, state, positions, q_start, req_rows, n_reqs: int, decays, states, out,
+                         one_row_each: bool) -> None:
+        """Per channel of ``out [rows, channels]``: ``u = conv_bias + sum_j conv[j] x_(t - taps + 1 + j)`` over the
+        positions of each request (``x``: the float32 columns ``off_x ..`` of ``proj``); part by part of ``size``
+        channels ``r = sigmoid(R u + r_bias)`` and ``i = sigmoid(I u + i_bias)`` (``gates``:
+        ``prepare_block_gates``); ``a = exp(decay * r)``, ``S = a S + sqrt(1 - a^2) i u``, ``out = S * gelu(y)`` (tanh
+        form; ``y``: the columns ``off_y ..``).  ``state [slots, channels]`` float32 is carried on, and so is ``ring
+        [slots, taps, channels]`` float32, the input of position ``p`` at place ``p mod taps`` (None: one tap).
+        ``one_row_each``: every request of the step brings one row; else ``decays`` and ``states`` (float32
+        ``[rows, channels]``) are room for the tiles of rows."""
+        lib = self._mixer_lib("gated_recurrence")
+        self._need(proj, "projections", torch.float32)
+        self._need(out, "output")
+        rows, channels = out.shape
+        taps = conv.shape[0]
+        if proj.shape[0] != rows or size <= 0 or channels % size:
+            raise ValueError(f"gated_recurrence: projections {tuple(proj.shape)}, output {tuple(out.shape)} in parts of {size}")
+        for t, name, count in ((conv, "convolution taps", taps * channels), (conv_bias, "convolution bias", channels),
+                               (r_bias, "gate bias", channels), (i_bias, "gate bias", channels),
+                               (decay, "decay", channels), (state, "state", None)):
+            self._need(t, name, torch.float32)
+            if count is not None and t.numel() != count:
+                raise ValueError(f"gated_recurrence: {name} of {t.numel()} numbers, not {count}")
+        self._need(gates, "gates", out.dtype)
+        if gates.numel() != 2 * channels * size or tuple(state.shape[1:]) != (channels,):
+            raise ValueError(f"gated_recurrence: gates of {gates.numel()} numbers, state {tuple(state.shape)}")
+        if taps > 1:
+            self._need(ring, "convolution inputs", torch.float32)
+            if tuple(ring.shape[1:]) != (taps, channels) or ring.shape[0] != state.shape[0]:
+                raise ValueError(f"gated_recurrence: inputs {tuple(ring.shape)} of {taps} taps")
+        for t, name, least in ((positions, "positions", rows), (q_start, "request row starts", n_reqs + 1),
+                               (req_rows, "request slots", n_reqs)):
+            self._need(t, name, torch.int32)
+            if t.numel() < least:
+                raise ValueError(f"gated_recurrence: {name} is too short")
+        if one_row_each != (rows == n_reqs):
+            raise ValueError(f"gated_recurrence: {rows} rows of {n_reqs} requests, one_row_each {one_row_each}")
+        if not one_row_each:
+            for t in (decays, states):
+                self._need(t, "room for the tiles", torch.float32)
+                if tuple(t.shape) != (rows, channels):
+                    raise ValueError(f"gated_recurrence: room {tuple(t.shape)} for {tuple(out.shape)}")
+        self._call(lib.llmlab_gated_recurrence, self._ptr(proj), proj.stride(0), int(off_x), int(off_y), channels, int(size),
+                   self._ptr(conv), self._ptr(conv_bias), taps, self._ptr(ring) if taps > 1 else None, self._ptr(gates),
+                   self._ptr(r_bias), self._ptr(i_bias), self._ptr(decay), self._ptr(state), self._ptr(positions),
+                   self._ptr(q_start), self._ptr(req_rows), int(n_reqs), rows,
+                   None if one_row_each else self._ptr(decays), None if one_row_each else self._ptr(states),
+                   self._ptr(out), _dt(out), 1 if one_row_each else 0, self._stream(), lib=lib)
 
     def scaled_sum(self, out, y1, a: float, y2, b: float) -> None:
         """``out = a * y1 + b * y2``, float32 tensors of one shape."""

@@ -335,6 +335,12 @@ class WindowedSinkAttention(Mixer):
     heads are laid out in multiples of 32 channels and their value heads of 16 (zeros behind), the
     sizes of the matrix cores.
 
+    ``qk_norm="whole"`` goes with a position encoding (a ``half_table()`` or a ``pair_table()`` without a
+    magnitude; queries and keys turn after the norm) and with ``output_gate="sigmoid"`` too, with keys and
+    values of the layer's own or another run's; heads are then laid out as above, and the gates are read
+    where an output is made final.  ``plus_one``: the denominator holds one more term of 1 (a sink whose
+    score is 0, with no number of its own).
+
     Pages: keys ``[kv_heads, P, key_dim]``, values ``[kv_heads, P, value_dim]``.  The products'
     inner sizes are multiples of 8: a value head of another width is laid out with zeros behind
     its channels (zero rows of the value projection, zero columns of the output projection), which
@@ -352,7 +358,7 @@ class WindowedSinkAttention(Mixer):
                  own_kv: bool = True, position: Optional[PartSpec] = None, qkv_bias: bool = False,
                  weights: str = "softmax", score_bias: bool = False, output_gate: Optional[str] = None,
                  value_mix: Optional[str] = None, chunk: Optional[int] = None, conv_taps: int = 0,
-                 out_bias: bool = False):
+                 out_bias: bool = False, plus_one: bool = False):
         super().__init__(tensors)
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads are not a multiple of {num_kv_heads} kv heads")
@@ -370,20 +376,27 @@ class WindowedSinkAttention(Mixer):
         self.position = build_part("position", position) if position is not None else None
         # the projections that turn, carry biases, mix values or gate heads go through one kernel
         # of their own, which knows no norm over the whole projection and writes keys and values
+        self.whole = qk_norm == "whole"
         self.shaped = bool(self.conv_taps or qk_norm == "head" or output_gate == "channels"
-                           or (self.position is not None and not hasattr(self.position, "pair_table")))
-        self.rotates = not self.shaped and bool(self.position is not None or qkv_bias or value_mix or output_gate)
+                           or (self.position is not None and not self.whole and not hasattr(self.position, "pair_table")))
+        self.rotates = not self.shaped and not self.whole and bool(self.position is not None or qkv_bias or value_mix
+                                                                   or output_gate)
+        if self.whole and (qkv_bias or value_mix):
+            raise ValueError("a norm over the whole projection goes without biases and mixed values")
         if self.shaped and (qk_norm == "whole" or not own_kv or value_mix or output_gate == "sigmoid"):
             raise ValueError("convolutions, norms head by head, halves that turn and gates per channel go with keys and "
                              "values of the layer's own, without a norm over the whole projection, mixed values or a "
                              "gate per head")
-        if self.rotates and (qk_norm or not own_kv):
-            raise ValueError("a position encoding, biases, mixed values or an output gate go with keys and values "
-                             "of the layer's own and without a norm over the whole projection")
+        if self.rotates and not own_kv:
+            raise ValueError("without a norm over the whole projection, a position encoding, biases, mixed values or an "
+                             "output gate go with keys and values of the layer's own")
         if self.position is not None and not (hasattr(self.position, "pair_table") or hasattr(self.position, "half_table")):
             raise ValueError(f"{type(self.position).__name__} has neither a pair_table() nor a half_table()")
-        if weights == "sigmoid" and sink:
+        if weights == "sigmoid" and (sink or plus_one):
             raise ValueError("a sink belongs to a softmax's denominator; sigmoid weights have none")
+        if sink and plus_one:
+            raise ValueError("one extra term in the denominator: a learned sink or a one")
+        self.plus_one = bool(plus_one)
         if score_bias and weights != "sigmoid":
             raise ValueError("score_bias goes with sigmoid weights")
         self.w_gate_rows = 0
@@ -392,9 +405,10 @@ class WindowedSinkAttention(Mixer):
         self.hidden_size, self.num_heads, self.num_kv_heads = int(hidden_size), int(num_heads), int(num_kv_heads)
         self.key_dim = int(key_dim)
         self.file_value_dim = int(value_dim)                       # a value head as the model file has it
-        unit = 16 if self.shaped else 8
+        tiled = self.shaped or (self.whole and bool(self.position is not None or output_gate))
+        unit = 16 if tiled else 8
         self.value_dim = (self.file_value_dim + unit - 1) // unit * unit      # and as the kernels and the pages see it
-        self.laid_dim = (self.key_dim + 31) // 32 * 32 if self.shaped else self.key_dim      # a key head in the pages
+        self.laid_dim = (self.key_dim + 31) // 32 * 32 if tiled else self.key_dim      # a key head in the pages
         self.scale = float(scale)
         self.window = None if window is None else int(window)
         self.keep_first = int(keep_first or 0)
@@ -501,6 +515,8 @@ class WindowedSinkAttention(Mixer):
             self.k_norm = tensors[t["k_norm"]].float().contiguous() if self.own_kv else None
         if self.has_sink:
             self.sink = tensors[t["sink"]].float().contiguous()
+        elif self.plus_one:
+            self.sink = torch.zeros(self.num_heads, dtype=torch.float32, device=tensors[t["q_weight"]].device)
 
     def cache_spec(self):
         return CacheSpec((("k", PageTensor((self.num_kv_heads, self.laid_dim), 1)),
@@ -512,17 +528,21 @@ class WindowedSinkAttention(Mixer):
             return {}
         return {"conv": ((self.conv_taps - 1, self.q_size + self.k_size + self.v_size), torch.float32)}
 
+    def _turn(self):
+        """The position encoding as the kernels take it: frequencies, how many channels turn, which with which."""
+        if self.position is None:
+            return None, 0, "halves"
+        if hasattr(self.position, "half_table"):
+            return (*self.position.half_table(), "halves")
+        freq, rot_dims, magnitude = self.position.pair_table()
+        if magnitude != 1.0:
+            raise ValueError("this mixer's kernel turns channels without a magnitude")
+        return freq, rot_dims, "neighbours"
+
     def _shape_and_write(self, proj, q, ctx, entry, group):
         """Convolution, rotation and norms of the projections; queries out, keys and values to the pages."""
         ops = self.ops
-        freq, rot_dims, pairing = None, 0, "halves"
-        if self.position is not None and hasattr(self.position, "half_table"):
-            freq, rot_dims = self.position.half_table()
-        elif self.position is not None:
-            freq, rot_dims, magnitude = self.position.pair_table()
-            pairing = "neighbours"
-            if magnitude != 1.0:
-                raise ValueError("this mixer's kernel turns channels without a magnitude")
+        freq, rot_dims, pairing = self._turn()
 
         def launch():
             # (whether every request brings one row is not a matter of the number of rows)
@@ -537,7 +557,8 @@ class WindowedSinkAttention(Mixer):
         else:
             launch()
 
-    def forward_into(self, h, out, ctx, entry):
+    def _mixed(self, h, ctx, entry):
+        """The heads' outputs of this step's rows, side by side, in the compute dtype."""
         ops, rows = self.ops, h.shape[0]
         if self.own_kv != bool(entry.writes_cache):
             raise ValueError("an attention layer without keys and values of its own reads another run's cache, "
@@ -563,7 +584,7 @@ class WindowedSinkAttention(Mixer):
         else:
             ops.project_norm_write(proj, self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim, self.own_kv,
                                    self.q_norm, self.k_norm, self.norm_eps, q, entry.k_cache, entry.v_cache,
-                                   group.page_size, ctx.positions, ctx.row_req, group.block_table)
+                                   group.page_size, ctx.positions, ctx.row_req, group.block_table, **self._turned())
         mixed = ctx.scratch("windowed_attention.out", (rows, self.num_heads * self.value_dim), self.dtype)
         sigmoid = self.weights == "sigmoid"
         kind = dict(weights="sigmoid") if sigmoid else {}
@@ -571,6 +592,8 @@ class WindowedSinkAttention(Mixer):
             kind["chunk"] = self.chunk
         if self.output_gate == "channels":
             kind["gate"] = (proj, self.q_size + self.k_size + self.v_size)
+        elif self.whole and self.output_gate:
+            kind["head_gate"] = (proj, self.in_size - self.gate_size)
         reach = self.window if self.window is not None else self.chunk
 
         def attend():
@@ -591,6 +614,23 @@ class WindowedSinkAttention(Mixer):
             attend()
         if gate is not None:
             ops.gate_heads(mixed, gate, self.num_heads, self.value_dim, self.output_gate)
+        return mixed
+
+    def _turned(self):
+        if not self.whole or self.position is None:
+            return {}
+        freq, rot_dims, pairing = self._turn()
+        return dict(freq=freq, rot_dims=rot_dims, pairing=pairing)
+
+    def forward_split(self, h, out, ctx, entry):
+        if self.b_o is not None:
+            self.forward_into(h, out, ctx, entry)
+            return None
+        return self._product_split(self._mixed(h, ctx, entry), self.w_o, out, ctx)
+
+    def forward_into(self, h, out, ctx, entry):
+        ops = self.ops
+        mixed = self._mixed(h, ctx, entry)
         if self.b_o is not None:
             ops.linear_logits(mixed, self.w_o, out, self.b_o)
         else:

@@ -182,6 +182,17 @@ class PendingSums:
         self.parts, self.splits = parts, int(splits)
 
 
+class ChosenSums:
+    """A result that is a weighted sum of experts' results, not summed yet: row ``r`` is ``sum_k weights[r, k] *
+    rows[place_of[r, k], :]``, the choices in their order (a place below zero: none).  Whoever takes it sums it
+    on the way."""
+
+    __slots__ = ("rows", "place_of", "weights")
+
+    def __init__(self, rows, place_of, weights):
+        self.rows, self.place_of, self.weights = rows, place_of, weights
+
+
 class NormedPair:
     """A result that is the weighted sum of two normed ones, ``a * rms(y1) * w1 + b * rms(y2) * w2`` (``rms`` with
     ``eps`` inside the root), not summed yet: whoever takes it sums it on the way."""
@@ -282,8 +293,21 @@ class Mixer(Part):
     # True: the part also has ``forward_into(h, out, ctx, ...)``, which WRITES its result into
     # the float32 ``out`` instead of adding it into the stream (for blocks that put a norm
     # between the sublayer and the sum).  Without it such a block hands ``forward`` a zeroed
-    # buffer in place of the stream.
+    # buffer in place of the stream.  A mixer with ``forward_split(h, out, ctx, entry)`` may hand its last
+    # product over in pieces instead (``_product_split``).
     writes_output = False
+
+    def _product_split(self, x, w, out, ctx):
+        """A mixer's last product ``x W^T`` for a caller that does something else with the result than add it to
+        the stream: into ``out`` (None comes back), or, where it spreads over the chip better cut along its
+        inner size, the pieces themselves (``PendingSums``; ``out`` is not written)."""
+        rows, width = out.shape
+        splits = self.ops.split_count(rows, self.dtype, width, x.shape[1])
+        if splits > 1:
+            parts = ctx.scratch("mixer.pieces", (splits, rows, width), torch.float32)
+            return self.ops.linear_partials(x, w, parts, splits)
+        self.ops.linear_logits(x, w, out)
+        return None
 
     def cache_spec(self) -> Optional[CacheSpec]:
         """Per-token cache need (``KVCacheSpec(...)`` for keys and values, or any

@@ -224,6 +224,48 @@ class SublayerNormBlock(Block):
         return sum(p.weight_bytes() for p in self.parts())
 
 
+class PostNormBlock(SublayerNormBlock):
+    """A norm BEHIND each sum: ``x = norm1(alpha * x + mixer(x)); x = norm2(alpha * x + feed_forward(x))``, the
+    sublayers reading the stream itself.  A block without a feed-forward has the first half only.  The
+    stream, both sums and both norms are float32; the sublayers' products read the stream rounded to the
+    compute dtype, and the launch of a sum leaves that copy for the next reader.
+
+    A part with ``forward_split`` may hand its result over in pieces, or as experts' results not summed yet;
+    the launch of the norm sums them on the way."""
+
+    def __init__(self, hidden_size: int, mixer: PartSpec, norm1: PartSpec, feed_forward: PartSpec = None,
+                 norm2: PartSpec = None, tensors: Dict[str, str] = None, alpha: float = 1.0):
+        super().__init__(hidden_size, mixer, norm1, feed_forward, norm2, tensors)
+        self.alpha = float(alpha)
+        for n in (self.norm1, self.norm2):
+            if n is not None and not hasattr(n, "post_into"):
+                raise ValueError(f"{type(n).__name__} cannot norm the sum of the stream and a result (no post_into)")
+
+    def leads(self, block) -> bool:
+        return False
+
+    def _result(self, part, h, residual, ctx, *entry):
+        y = ctx.scratch("block.sublayer_out", tuple(residual.shape), torch.float32)
+        if hasattr(part, "forward_split"):
+            split = part.forward_split(h, y, ctx, *entry)
+            return y if split is None else split
+        if hasattr(part, "forward_pending"):
+            pieces = part.forward_pending(h, y, ctx, *entry)
+            return y if pieces is None else pieces
+        return self._sublayer(part, None, h, residual, ctx, *entry)
+
+    def forward(self, residual, ctx, entry):
+        self._fold(residual, ctx)
+        h = self._input(residual, ctx, entry)
+        copy = h if self.dtype != torch.float32 else None
+        self.norm1.post_into(self._result(self.mixer, h, residual, ctx, entry), self.alpha, residual, copy)
+        if self.feed_forward is not None:
+            self.norm2.post_into(self._result(self.feed_forward, h, residual, ctx), self.alpha, residual, copy)
+        memo = getattr(ctx, "memo", None)
+        if memo is not None and copy is not None:
+            memo[self.NOTE] = entry.index
+
+
 class SandwichNormBlock(Block):
     """A norm before AND behind each sublayer::
 
@@ -617,6 +659,7 @@ register_part("block", "prenorm", PreNormBlock)
 register_part("block", "gated_conv", GatedConvBlock)
 register_part("embedding", "pair_hash_embedding", PairHashEmbedding)
 register_part("block", "sublayer_norm", SublayerNormBlock)
+register_part("block", "post_norm", PostNormBlock)
 register_part("block", "sandwich_norm", SandwichNormBlock)
 register_part("embedding", "token_embedding", TokenEmbedding)
 register_part("head", "linear_head", LinearHead)

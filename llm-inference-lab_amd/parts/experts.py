@@ -7,7 +7,7 @@ import torch
 
 from ..config.spec import PartSpec
 from ..weights.loader import TensorSpec, MATRIX, VECTOR, INIT_ZEROS
-from .base import FeedForward, NormedInput
+from .base import ChosenSums, FeedForward, NormedInput
 from .feed_forward import interleave_gate_up, pad_columns, pad_rows
 from .registry import register_part, build_part
 
@@ -29,8 +29,12 @@ class RoutedExperts(FeedForward):
 
     ``scoring="sigmoid"``: the scores are ``sigmoid(z)``, each output by itself, instead of the
     softmax.  ``expert_form="relu2"``: the experts are ``W_down relu(W_up h)^2`` without a gate
-    matrix.  ``shared_gate=True``: the shared part's result is multiplied by ``sigmoid(w_sg . h)``,
-    one number per token (``shared_gate [1, hidden]``), before it is added.
+    matrix; ``expert_form="clamped"``: ``W_down (g sigmoid(slope g) (u + shift))`` with ``g = min(W_gate h, limit)`` and
+    ``u = W_up h`` held within ``-limit .. limit`` (``expert_constants = (limit, slope, shift)``).
+    ``group_score="top2"``: a group counts as the sum of its two largest ``c``.  ``share_eps`` (None: as they are):
+    the chosen outputs' scores are divided by their sum plus so much before ``scale``.
+    ``shared_gate=True``: the shared part's result is multiplied by ``sigmoid(w_sg . h)``, one number per
+    token (``shared_gate [1, hidden]``), before it is added.
 
     Tensor roles: ``router [outputs, hidden]``, ``correction [outputs]`` (absent: none), and the
     experts' ``expert_gate``, ``expert_up``, ``expert_down``, each a name with ``{}`` in the place of
@@ -44,12 +48,25 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, expert_size: int, num_experts: int, top: int, tensors: Dict[str, str],
                  identity: int = 0, scale: float = 1.0, groups: int = 1, groups_keep: int = 1,
                  correction: bool = True, shared: Optional[PartSpec] = None, scoring: str = "softmax",
-                 expert_form: str = "swiglu", shared_gate: bool = False):
+                 expert_form: str = "swiglu", shared_gate: bool = False, expert_constants=None,
+                 group_score: str = "max", share_eps: Optional[float] = None):
         super().__init__(tensors)
         if scoring not in ("softmax", "sigmoid"):
             raise ValueError(f"a router scores by 'softmax' or 'sigmoid', got {scoring!r}")
-        if expert_form not in ("swiglu", "relu2"):
-            raise ValueError(f"experts are 'swiglu' or 'relu2' feed-forwards, got {expert_form!r}")
+        if expert_form not in ("swiglu", "relu2", "clamped"):
+            raise ValueError(f"experts are 'swiglu', 'relu2' or 'clamped' feed-forwards, got {expert_form!r}")
+        if (expert_form == "clamped") != (expert_constants is not None):
+            raise ValueError("clamped experts have three constants (limit, slope, shift), the other forms none")
+        if group_score not in ("max", "top2"):
+            raise ValueError(f"a group counts as its 'max' or its 'top2', got {group_score!r}")
+        # (what the kernels are told; silu, a group's largest and plain scores are what they do when told nothing)
+        self._pair = {} if expert_constants is None else dict(activation="clamped",
+                                                              constants=tuple(float(c) for c in expert_constants))
+        self._how = {} if scoring == "softmax" else dict(scoring=scoring)
+        if group_score != "max":
+            self._how["group_score"] = group_score
+        if share_eps is not None:
+            self._how["share_eps"] = float(share_eps)
         if shared_gate and shared is None:
             raise ValueError("a gate on the shared part needs a shared part")
         self.scoring, self.expert_form, self.has_shared_gate = scoring, expert_form, bool(shared_gate)
@@ -73,7 +90,7 @@ class RoutedExperts(FeedForward):
 
     def _expert_names(self, e: int):
         t = self.tensor_names
-        gate = t["expert_gate"].format(e) if self.expert_form == "swiglu" else None
+        gate = t["expert_gate"].format(e) if self.expert_form != "relu2" else None
         return gate, t["expert_up"].format(e), t["expert_down"].format(e)
 
     def tensor_specs(self):
@@ -123,24 +140,50 @@ class RoutedExperts(FeedForward):
 
     takes_normed_input = True
 
-    def forward(self, h, residual, ctx):
+    @property
+    def grouped(self) -> bool:
         ops = self.ops
-        if isinstance(h, NormedInput):
-            h = h.tensor()
-        rows, top = h.shape[0], self.top
+        return bool(self.num_experts and getattr(ops, "moe_grouped", None) is not None and ops.moe_grouped(self.dtype))
+
+    def _route(self, h, ctx):
+        """Chosen outputs and their weights, and the plan of the grouped products if choice and sorting were one
+        launch."""
+        ops, rows, top = self.ops, h.shape[0], self.top
         logits = ctx.scratch("experts.logits", (rows, self.outputs), torch.float32)
         ops.linear_logits(h, self.w_router, logits)
         chosen = ctx.scratch("experts.chosen", (rows, top), torch.int32)
         weights = ctx.scratch("experts.weights", (rows, top), torch.float32)
-        grouped = self.num_experts and getattr(ops, "moe_grouped", None) is not None and ops.moe_grouped(self.dtype)
         plan = None
-        how = {} if self.scoring == "softmax" else dict(scoring=self.scoring)
-        if grouped and ops.moe_select_plan_takes(rows, self.outputs):       # few rows: choice and sorting in one launch
+        if self.grouped and ops.moe_select_plan_takes(rows, self.outputs):       # few rows: choice and sorting in one launch
             plan = ops.moe_select_plan(logits, self.correction, self.groups, self.groups_keep, self.scale, chosen,
-                                       weights, self.num_experts, ctx.scratch, **how)
+                                       weights, self.num_experts, ctx.scratch, **self._how)
         else:
-            ops.moe_select(logits, self.correction, self.groups, self.groups_keep, self.scale, chosen, weights, **how)
-        if grouped:
+            ops.moe_select(logits, self.correction, self.groups, self.groups_keep, self.scale, chosen, weights, **self._how)
+        return chosen, weights, plan
+
+    def forward_split(self, h, out, ctx):
+        """For a caller that does something else with the result than add it to the stream: the experts'
+        results not summed yet (``ChosenSums``), or the result in ``out`` (None comes back)."""
+        if isinstance(h, NormedInput):
+            h = h.tensor()
+        if not self.grouped or self.identity or self.shared is not None:
+            self.ops.activation(out, out, "zero")
+            self.forward(h, out, ctx)
+            if getattr(ctx, "pending", None) is not None:       # (pieces the shared part left belong to the result)
+                self.ops.add_pending(out, ctx.pending)
+                ctx.pending = None
+            return None
+        chosen, weights, plan = self._route(h, ctx)
+        y, plan = self._products(h, ctx, chosen, plan)
+        return ChosenSums(y, plan.place_of, weights)
+
+    def forward(self, h, residual, ctx):
+        ops = self.ops
+        if isinstance(h, NormedInput):
+            h = h.tensor()
+        rows = h.shape[0]
+        chosen, weights, plan = self._route(h, ctx)
+        if self.grouped:
             self._grouped(h, residual, ctx, chosen, weights, plan)
         elif self.num_experts:
             relu2 = self.expert_form == "relu2"
@@ -150,7 +193,7 @@ class RoutedExperts(FeedForward):
                 if relu2:
                     ops.linear_relu2(h, ops.stacked_member(self.w_gate_up, e), act)
                 else:
-                    ops.linear_swiglu(h, ops.stacked_member(self.w_gate_up, e), act)
+                    ops.linear_swiglu(h, ops.stacked_member(self.w_gate_up, e), act, **self._pair)
                 ops.linear_logits(act, ops.stacked_member(self.w_down, e), y)
                 ops.moe_add_chosen(residual, y, chosen, weights, e, e + 1)
             if self.identity:
@@ -174,6 +217,11 @@ class RoutedExperts(FeedForward):
             ops.gated_add(residual, y, g, None)
 
     def _grouped(self, h, residual, ctx, chosen, weights, plan=None):
+        y, plan = self._products(h, ctx, chosen, plan)
+        self.ops.moe_combine(residual, y, plan, chosen, weights, self.num_experts, h)     # (identity outputs too)
+
+    def _products(self, h, ctx, chosen, plan):
+        """The experts' results at the places of the plan."""
         ops = self.ops
         if plan is None:
             plan = ops.moe_plan(chosen, self.num_experts, ctx.scratch)
@@ -182,10 +230,10 @@ class RoutedExperts(FeedForward):
             ops.moe_up_relu2(h, self.w_gate_up, plan, act)
         else:
             act = ctx.scratch("experts.act", (plan.capacity, self.kernel_size), self.dtype)
-            ops.moe_gate_up(h, self.w_gate_up, plan, act)
+            ops.moe_gate_up(h, self.w_gate_up, plan, act, **self._pair)
         y = ctx.scratch("experts.out", (plan.capacity, self.hidden_size), torch.float32)
         ops.moe_down(act, self.w_down, plan, y)
-        ops.moe_combine(residual, y, plan, chosen, weights, self.num_experts, h)     # (identity outputs too)
+        return y, plan
 
     @property
     def graph_safe(self):

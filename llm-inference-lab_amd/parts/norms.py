@@ -72,6 +72,13 @@ class RMSNorm(Norm):
         else:
             self.ops.rmsnorm_add(y, self.weight_f32, self.eps, stream, copy=copy)
 
+    def post_into(self, y, alpha: float, stream, copy=None):
+        """``stream = norm(alpha * stream + y)`` (``y`` float32, ``PendingSums`` or ``ChosenSums``); ``copy`` (compute
+        dtype) receives the stream's new rows."""
+        if self.weight_f32 is None:
+            self.weight_f32 = self.weight.float().contiguous()
+        self.ops.post_norm(stream, alpha, y, self.weight_f32, self.eps, copy)
+
     def weight_bytes(self):
         return self.weight.numel() * self.weight.element_size()
 

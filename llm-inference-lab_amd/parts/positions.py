@@ -1,6 +1,7 @@
 """Position encodings."""
 from __future__ import annotations
 
+import math
 from typing import Dict, Optional
 
 import torch
@@ -24,11 +25,22 @@ class RotaryEmbedding(PositionEncoding):
     query and key heads (``channel_order()``: scores do not depend on a common order of both)
     and gives the channels that do not turn the frequency 0: an angle of exactly 0, whose cosine
     is 1 and whose sine is 0.  ``padded_dim``: the mixer's kernels work on heads of that many
-    channels (the head's own, then zeros); the table and the order are made for those."""
+    channels (the head's own, then zeros); the table and the order are made for those.
+
+    ``scaling`` (``factor, low, high, original``) stretches the slow waves for sequences longer than the
+    ``original`` length: a pair whose wave (``2 pi / f`` positions) is shorter than ``original / high`` keeps
+    its frequency, one longer than ``original / low`` turns ``factor`` times slower, and between the two, with
+    ``s = (original / wave - low) / (high - low)``, the frequency is ``(1 - s) f / factor + s f``."""
 
     def __init__(self, dim: int, theta: float, tensors: Optional[Dict[str, str]] = None,
-                 rotary_dim: Optional[int] = None, padded_dim: Optional[int] = None):
+                 rotary_dim: Optional[int] = None, padded_dim: Optional[int] = None,
+                 scaling: Optional[Dict[str, float]] = None):
         super().__init__(tensors)
+        self.scaling = dict(scaling) if scaling else None
+        if self.scaling is not None:
+            missing = [k for k in ("factor", "low", "high", "original") if k not in self.scaling]
+            if missing:
+                raise ValueError(f"frequency scaling needs {missing}")
         self.dim = int(dim)
         self.rotary_dim = self.dim if rotary_dim is None else int(rotary_dim)
         self.padded_dim = self.dim if padded_dim is None else int(padded_dim)
@@ -45,11 +57,22 @@ class RotaryEmbedding(PositionEncoding):
         rotary_dim / 2`` in the file's own order."""
         return self.half_freq, self.rotary_dim
 
+    def frequencies(self) -> torch.Tensor:
+        """``f [rotary_dim / 2]`` in double precision."""
+        exponent = torch.arange(0, self.rotary_dim, 2, dtype=torch.float64) / max(self.rotary_dim, 1)
+        f = 1.0 / (torch.tensor(self.theta, dtype=torch.float64) ** exponent)
+        if self.scaling is None:
+            return f
+        factor, low, high, original = (float(self.scaling[k]) for k in ("factor", "low", "high", "original"))
+        wave = 2.0 * math.pi / f
+        s = (original / wave - low) / (high - low) if high != low else torch.zeros_like(f)
+        between = (1.0 - s) * f / factor + s * f
+        return torch.where(wave < original / high, f, torch.where(wave > original / low, f / factor, between))
+
     def bind(self, tensors, ops, dtype):
         super().bind(tensors, ops, dtype)
-        exponent = torch.arange(0, self.rotary_dim, 2, dtype=torch.float64) / max(self.rotary_dim, 1)
         freq = torch.zeros(self.padded_dim // 2, dtype=torch.float64)
-        freq[:self.rotary_dim // 2] = 1.0 / (torch.tensor(self.theta, dtype=torch.float64) ** exponent)
+        freq[:self.rotary_dim // 2] = self.frequencies()
         self.inv_freq = freq.to(torch.float32).to(ops.device)
         self.half_freq = self.inv_freq[:self.rotary_dim // 2].contiguous()
 
@@ -114,7 +137,6 @@ class PairRotary(PositionEncoding):
 
     def frequencies(self):
         """``(f [rotary_dim / 2] as Python floats, magnitude)``, worked out in double precision."""
-        import math
         n = self.rotary_dim
         f = [self.theta ** (-2.0 * i / n) for i in range(n // 2)]
         sc = self.scaling

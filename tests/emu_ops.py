@@ -15,7 +15,7 @@ from types import SimpleNamespace
 import torch
 
 from llm_inference_lab_amd.cache import layout as cache_layout
-from llm_inference_lab_amd.parts import PendingSums
+from llm_inference_lab_amd.parts import ChosenSums, PendingSums
 
 
 class EmuRecord:
@@ -64,7 +64,7 @@ class EmuOps:
                 "project_norm_write", "sink_window_attention", "gla_decay", "gla_scan", "gla_output",
                 "gate_heads", "add_row_vector", "moe_select", "moe_add_chosen", "embed_pairs", "causal_conv", "norm_conv",
                 "gated_add", "latent_norm_write", "head_products", "softcap", "project_rotate_write", "delta_gates",
-                "delta_scan", "rmsnorm_add", "scaled_sum")
+                "delta_scan", "rmsnorm_add", "scaled_sum", "post_norm", "gated_recurrence")
 
     def __init__(self, device="cpu", fuse=True):
         self.device = torch.device(device)
@@ -222,7 +222,7 @@ class EmuOps:
         self._count("linear_logits")
         out.copy_(x.float() @ w.float().t() + (0.0 if bias is None else bias.float()))
 
-    def linear_swiglu(self, x, w_gu, out, activation="silu"):
+    def linear_swiglu(self, x, w_gu, out, activation="silu", constants=None):
         """w_gu rows alternate in runs of 16: gate rows of 16 outputs, then the
         up rows of the same outputs."""
         self._count("linear_swiglu")
@@ -231,7 +231,11 @@ class EmuOps:
         y = y.view(x.shape[0], -1, 2, 16)
         gate = y[:, :, 0, :].reshape(x.shape[0], -1)[:, :inter]
         up = y[:, :, 1, :].reshape(x.shape[0], -1)[:, :inter]
-        if activation == "gelu_tanh":
+        if activation == "clamped":
+            limit, slope, shift = constants
+            gate, up = gate.clamp(max=limit), up.clamp(-limit, limit) + shift
+            act = gate * torch.sigmoid(slope * gate)
+        elif activation == "gelu_tanh":
             act = 0.5 * gate * (1.0 + torch.tanh(0.7978845608028654 * (gate + 0.044715 * gate ** 3)))
         else:
             act = gate / (1.0 + torch.exp(-gate))
@@ -269,18 +273,31 @@ class EmuOps:
         pass
 
     def project_norm_write(self, proj, num_heads, num_kv_heads, key_dim, value_dim, own_kv, q_norm, k_norm, eps,
-                           q_out, k_cache, v_cache, page_size, positions, row_req, block_table):
+                           q_out, k_cache, v_cache, page_size, positions, row_req, block_table, freq=None, rot_dims=0,
+                           pairing="halves"):
         self._count("project_norm_write")
-        rows = q_out.shape[0]
+        rows, laid = q_out.shape[0], q_out.shape[1] // num_heads
         qs, ks, vs = num_heads * key_dim, num_kv_heads * key_dim, num_kv_heads * value_dim
 
         def whole(v, w):
             return v if w is None else v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * w.float()
         p = proj.float()
-        q_out.copy_(whole(p[:, :qs], q_norm).to(q_out.dtype))
+
+        def heads(v, n):
+            v = v.reshape(rows, n, key_dim).clone()
+            if rot_dims:
+                angle = positions[:rows].float()[:, None] * freq
+                c, s = torch.cos(angle)[:, None], torch.sin(angle)[:, None]
+                half = rot_dims // 2
+                first = slice(0, half) if pairing == "halves" else slice(0, rot_dims, 2)
+                second = slice(half, rot_dims) if pairing == "halves" else slice(1, rot_dims, 2)
+                a, b = v[..., first].clone(), v[..., second].clone()
+                v[..., first], v[..., second] = a * c - b * s, b * c + a * s
+            return torch.nn.functional.pad(v, (0, laid - key_dim))
+        q_out.copy_(heads(whole(p[:, :qs], q_norm), num_heads).reshape(rows, -1).to(q_out.dtype))
         if not own_kv:
             return
-        k = whole(p[:, qs:qs + ks], k_norm).to(k_cache.dtype).view(rows, num_kv_heads, key_dim)
+        k = heads(whole(p[:, qs:qs + ks], k_norm), num_kv_heads).to(k_cache.dtype)
         v = p[:, qs + ks:qs + ks + vs].to(v_cache.dtype).view(rows, num_kv_heads, value_dim)
         for r in range(rows):
             pos = int(positions[r])
@@ -291,7 +308,8 @@ class EmuOps:
 
     def sink_window_attention(self, q, num_heads, num_kv_heads, key_dim, value_dim, k_cache, v_cache, block_table,
                               page_size, positions, row_req, window, keep_first, sink, scale, out,
-                              q_start=None, long_from=0, launches=3, max_keys=0, weights="softmax", chunk=None, gate=None):
+                              q_start=None, long_from=0, launches=3, max_keys=0, weights="softmax", chunk=None, gate=None,
+                              head_gate=None):
         """(``long_from``, ``launches``: how the kernels share the rows; the result is the same.)"""
         self._count("sink_window_attention")
         rows = q.shape[0]
@@ -320,6 +338,8 @@ class EmuOps:
                 if gate is not None:
                     at = gate[1] + h * value_dim
                     o = o * torch.sigmoid(gate[0][r, at:at + value_dim].float())
+                if head_gate is not None:
+                    o = o * torch.sigmoid(head_gate[0][r, head_gate[1] + h].float())
                 out[r, h * value_dim:(h + 1) * value_dim] = o.to(out.dtype)
 
     def project_rotate_write(self, proj, num_heads, num_kv_heads, key_dim, value_dim, bias, freq, rot_dims, magnitude,
@@ -547,6 +567,47 @@ class EmuOps:
             w, e, out = next_norm
             out.copy_((x / torch.sqrt((x * x).mean(-1, keepdim=True) + e) * w.float()).to(out.dtype))
 
+    def post_norm(self, x, alpha, y, weight, eps, copy=None):
+        self._count("post_norm")
+        if isinstance(y, ChosenSums):
+            w = torch.where(y.place_of >= 0, y.weights, torch.zeros_like(y.weights)).float()
+            y = (w[..., None] * y.rows[y.place_of.clamp(min=0).long()].float()).sum(1)
+        v = alpha * x + (self._owed(y) if isinstance(y, PendingSums) else y.float())
+        x.copy_(v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * weight.float())
+        if copy is not None:
+            copy.copy_(x.to(copy.dtype))
+
+    def prepare_block_gates(self, w_r, w_i):
+        return torch.stack([w_r, w_i])
+
+    def gated_recurrence(self, proj, off_x, off_y, size, conv, conv_bias, ring, gates, r_bias, i_bias, decay, state,
+                         positions, q_start, req_rows, n_reqs, decays, states, out, one_row_each):
+        """(``decays``, ``states``: the kernels' room for tiles of rows; untouched here.)"""
+        self._count("gated_recurrence")
+        channels, taps = out.shape[1], conv.shape[0]
+        x, y = proj[:, off_x:off_x + channels].float(), proj[:, off_y:off_y + channels].float()
+        gelu = 0.5 * y * (1.0 + torch.tanh(0.7978845608028654 * (y + 0.044715 * y ** 3)))
+        for b in range(n_reqs):
+            first, n, slot = int(q_start[b]), int(q_start[b + 1]) - int(q_start[b]), int(req_rows[b])
+            assert not one_row_each or n == 1
+            p0 = int(positions[first])
+            s = state[slot].clone()
+            for k in range(n):
+                u = conv_bias.clone()
+                for j in range(taps):
+                    back = taps - 1 - j
+                    v = x[first + k - back] if back <= k else ring[slot, (p0 + k - back) % taps]
+                    u += conv[j] * v
+                parts = u.to(gates.dtype).float().view(-1, size)
+                z = torch.einsum("mpoi,pi->mpo", gates.float(), parts).reshape(2, channels)
+                a_log = decay * torch.sigmoid(z[0] + r_bias)
+                s = torch.exp(a_log) * s + torch.sqrt(-torch.expm1(2 * a_log)) * torch.sigmoid(z[1] + i_bias) * u
+                out[first + k] = (s * gelu[first + k]).to(out.dtype)
+            for k in range(max(0, n - taps), n):
+                if taps > 1:
+                    ring[slot, (p0 + k) % taps] = x[first + k]
+            state[slot] = s
+
     def scaled_sum(self, out, y1, a, y2, b):
         self._count("scaled_sum")
         out.copy_(a * y1 + b * y2)
@@ -665,7 +726,8 @@ class EmuOps:
     def moe_grouped(self, dtype):
         return False
 
-    def moe_select(self, logits, correction, groups, groups_keep, scale, chosen, weights, scoring="softmax"):
+    def moe_select(self, logits, correction, groups, groups_keep, scale, chosen, weights, scoring="softmax",
+                   group_score="max", share_eps=None):
         """Per row: softmax (or, ``scoring="sigmoid"``, the sigmoid) of the logits, the choice value
         (score + correction), the kept groups by their best choice value, the ``top`` best of their
         members; ties to the smaller index."""
@@ -677,7 +739,7 @@ class EmuOps:
         s = e / e.sum(-1, keepdim=True) if scoring == "softmax" else torch.sigmoid(z)
         c = s + correction.float()
         per = outputs // groups
-        best = c.view(rows, groups, per).max(-1).values
+        best = c.view(rows, groups, per).sort(-1, descending=True).values[..., :2 if group_score == "top2" else 1].sum(-1)
         allowed = torch.zeros(rows, groups, dtype=torch.bool)
         left = best.clone()
         for _ in range(groups_keep):
@@ -689,8 +751,11 @@ class EmuOps:
         for k in range(top):
             e_k = torch.argmax(c, dim=-1)
             chosen[:, k] = e_k.to(torch.int32)
-            weights[:, k] = s[torch.arange(rows), e_k] * scale
+            weights[:, k] = s[torch.arange(rows), e_k]
             c[torch.arange(rows), e_k] = -float("inf")
+        if share_eps is not None:
+            weights /= weights.sum(-1, keepdim=True) + share_eps
+        weights *= scale
 
     # ------------------------------- hashed pairs, short convolution, gates, latent attention
     def embed_pairs(self, table, pairs, ids, positions, row_req, q_start, req_rows, previous, scale, buckets,
