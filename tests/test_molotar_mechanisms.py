@@ -1,0 +1,457 @@
+"""Each mechanism of Molotar alone, against the plain implementation's function for it: the kernel set's
+operation on the engine's own layouts (pages, block tables, state slots), once as the PyTorch reference
+on the CPU and once as the HIP kernel on the GPU.  Where random numbers would hide a fault (a key at a
+window's edge or far back, the one in the denominator, an early input after hundreds of tokens), the
+inputs are made so that it shows."""
+import math
+
+import pytest
+import torch
+
+import helpers as H          # noqa: F401
+import plain_molotar as P
+from test_vivevik_mechanisms import BACKENDS, DTYPES, F64, Paged, close, ops_of, randn
+from test_mazanex_mechanisms import batch, ints
+from llm_inference_lab_amd.cache.layout import value_quads
+from llm_inference_lab_amd.parts import ChosenSums, GatedLinearRecurrence, PendingSums, RotaryEmbedding, RoutedExperts
+
+
+class Scratch:
+    """The least a part needs of a step: named scratch buffers and no sums owed."""
+
+    def __init__(self, device):
+        self.device, self.pending, self.memo = device, None, {}
+
+    def scratch(self, name, shape, dtype):
+        return torch.zeros(shape, dtype=dtype, device=self.device)
+
+
+# ------------------------------------------------------------------ the stream
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("hidden,rows", [(7, 3), (8, 5), (72, 5), (1000, 70), (2600, 5), (4100, 3), (20000, 2)])
+def test_norm_behind_the_sum(backend, hidden, rows):
+    """The norm of alpha times the stream plus a result: whole, left in pieces, or experts' results with
+    their places and weights (none for some choices), with a rounded copy; a row in a thread's registers
+    up to rows that are read twice."""
+    ops = ops_of(backend)
+    dev = ops.device
+    w = (1.0 + randn(hidden, seed=2, scale=0.3)).to(dev)
+    pieces = randn(3, rows, hidden, seed=4).to(dev)
+    top = 6
+    place_of = torch.randint(0, 9, (rows, top), generator=torch.Generator().manual_seed(5)).to(torch.int32)
+    place_of[0, 1] = -1
+    shares = torch.rand(rows, top, generator=torch.Generator().manual_seed(6))
+    y = randn(9, hidden, seed=7).to(dev)
+    kept = torch.where(place_of >= 0, shares, torch.zeros(())).to(F64)
+    chosen = (kept[..., None] * y.cpu().to(F64)[place_of.clamp(min=0).long()]).sum(1)
+    results = [(pieces[0].clone(), pieces[0].cpu().to(F64)), (PendingSums(pieces, 3), pieces.cpu().to(F64).sum(0)),
+               (ChosenSums(y, place_of.to(dev), shares.to(dev)), chosen)]
+    for result, y64 in results:
+        for alpha in (1.0, 2.75, 0.0):
+            for dtype in (None,) + tuple(DTYPES):
+                x = randn(rows, hidden, seed=3).to(dev)
+                want = P.post_norm(x.cpu().to(F64), y64, w.cpu(), alpha, 1e-4)
+                copy = None if dtype is None else torch.full((rows, hidden), float("nan"), dtype=dtype, device=dev)
+                ops.post_norm(x, alpha, result, w, 1e-4, copy)
+                close(x, want, torch.float32, "norm(alpha x + y)", f32=5e-6)
+                if copy is not None:
+                    close(copy, want, dtype, "its copy", f32=5e-6, bf16=8e-3)
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+def test_pairs_without_a_norm(backend):
+    """The scaled token vector plus the pair's row, no norm behind; the token before a step's first one
+    comes out of the slot; a sequence's first token takes the row behind the buckets."""
+    ops = ops_of(backend)
+    dev = ops.device
+    vocab, width, buckets, mul_prev, mul_cur = 40, 24, 11, 29, 7
+    table, pairs = randn(vocab, width, seed=1), randn(buckets + 1, width, seed=2)
+    cfg = dict(embedding=dict(scale=4.5, bigram=dict(buckets=buckets, mul_prev=mul_prev, mul_cur=mul_cur)))
+    ids = torch.randint(0, vocab, (12,), generator=torch.Generator().manual_seed(3)).tolist()
+    want = P.embed(ids, cfg, {"embed": table, "bigram": pairs})
+    slots = torch.full((3, 1), 5, dtype=torch.int32, device=dev)
+    at = 0
+    for n in (1, 2, 6, 1, 2):
+        q_start, row_req = batch([n], dev)
+        out = torch.full((n, width), float("nan"), device=dev)
+        ops.embed_pairs(table.to(dev), pairs.to(dev), ints(ids[at:at + n], dev), ints(range(at, at + n), dev), row_req, q_start,
+                        ints([2], dev), slots, 4.5, buckets, mul_prev, mul_cur, None, 0.0, out)
+        close(out, want[at:at + n], torch.float32, f"rows {at} ..", f32=1e-6)
+        at += n
+        assert int(slots[2]) == ids[at - 1] and int(slots[0]) == 5
+
+
+# ------------------------------------------------------------------ rotation
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("dim,dims,base,scaling", [
+    (32, 32, 1e4, None), (20, 8, 50.0, None), (64, 48, 5e5, (8.0, 1.0, 4.0, 256)), (16, 16, 100.0, (2.0, 0.5, 32.0, 40)),
+    (24, 10, 3e3, (16.0, 2.0, 2.0, 100)), (12, 4, 7.0, (1.0, 1.0, 4.0, 20))])
+def test_stretched_frequencies(backend, dim, dims, base, scaling):
+    """Short waves keep their frequency, long ones are stretched by the factor, those between are mixed."""
+    sc = None if scaling is None else dict(zip(("factor", "low", "high", "original"), scaling))
+    part = RotaryEmbedding(dim, base, rotary_dim=dims, scaling=sc)
+    part.bind({}, ops_of(backend), torch.float32)
+    freq, turning = part.half_table()
+    want = torch.tensor(P.frequencies(dict(dims=dims, base=base, scaling=sc)), dtype=F64)
+    assert turning == dims and float(((freq.cpu().double() - want) / want).abs().max()) < 1e-6
+    if scaling == (8.0, 1.0, 4.0, 256):          # (all three kinds of waves)
+        ratio = want * torch.tensor([base ** (2.0 * i / dims) for i in range(dims // 2)], dtype=F64)
+        assert float(ratio[0]) == 1.0 and abs(float(ratio[-1]) - 0.125) < 1e-12
+        assert ((ratio > 0.13) & (ratio < 0.99)).any()
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H_,G,D,E,dims,rows", [(4, 2, 16, 16, 8, 37), (3, 1, 10, 24, 10, 5), (8, 2, 32, 16, 32, 70),
+                                                (20, 5, 72, 32, 40, 9), (6, 6, 128, 128, 64, 80)])
+def test_whole_norm_rotation_and_the_cache_write(backend, dtype, H_, G, D, E, dims, rows):
+    """Queries and keys normed over ALL their heads at once, then turned, laid out in multiples of 32
+    channels; values as projected; a layer without keys of its own turns its queries alike."""
+    ops = ops_of(backend)
+    dev = ops.device
+    laid = (D + 31) // 32 * 32
+    cache = Paged(ops, dtype, [rows + 3, 20], G, laid, E)
+    qs, ks = H_ * D, G * D
+    proj = randn(rows, qs + ks + G * E + H_, seed=5, scale=2.0)
+    proj[:, :D] *= 5.0           # one head much larger than the others: a norm per head would differ
+    qw, kw = (1.0 + randn(qs, seed=6, scale=0.3)).to(dev), (1.0 + randn(ks, seed=7, scale=0.3)).to(dev)
+    rot = dict(dims=dims, base=40.0, scaling=dict(factor=3.0, low=1.0, high=4.0, original=60))
+    freq = torch.tensor(P.frequencies(rot), dtype=F64).float().to(dev)
+    first = 3                    # (the rows' first position)
+    pos = ints(range(first, first + rows), dev)
+    row_req = ints([0] * rows, dev)
+    p64 = torch.cat([torch.zeros(first, proj.shape[1], dtype=F64), proj.to(F64)])      # (rotate() counts from position 0)
+    want_q = P.rotate(P.whole_norm(p64[:, :qs], qw.cpu(), 1e-5).view(-1, H_, D), rot)[first:]
+    want_k = P.rotate(P.whole_norm(p64[:, qs:qs + ks], kw.cpu(), 1e-5).view(-1, G, D), rot)[first:]
+    want_v = p64[first:, qs + ks:qs + ks + G * E].reshape(rows, G, E)
+    q = torch.full((rows, H_ * laid), float("nan"), dtype=dtype, device=dev)
+    ops.project_norm_write(proj.to(dev), H_, G, D, E, True, qw, kw, 1e-5, q, cache.k_cache, cache.v_cache, 16, pos, row_req,
+                           cache.table, freq=freq, rot_dims=dims)
+    got = q.view(rows, H_, laid)
+    close(got[..., :D], want_q, dtype, "queries", f32=3e-5)
+    assert float(got[..., D:].float().abs().sum()) == 0.0
+    for i in range(rows):
+        page, o = int(cache.table[0, (first + i) // 16]), (first + i) % 16
+        close(cache.k_cache[page, :, o, :D], want_k[i], dtype, f"key {i}", f32=3e-5)
+        assert float(cache.k_cache[page, :, o, D:].float().abs().sum()) == 0.0
+        close(value_quads(cache.v_cache[page])[:, o >> 2, :, o & 3], want_v[i], dtype, f"value {i}")
+    before = cache.k_cache.clone(), cache.v_cache.clone()
+    again = torch.full_like(q, float("nan"))
+    alone = torch.cat([proj[:, :qs], proj[:, -H_:]], 1).contiguous().to(dev)
+    ops.project_norm_write(alone, H_, G, D, E, False, qw, None, 1e-5, again, None, None, 16, pos, row_req, cache.table,
+                           freq=freq, rot_dims=dims)
+    assert torch.equal(again, q) and torch.equal(before[0], cache.k_cache) and torch.equal(before[1], cache.v_cache)
+
+
+# ------------------------------------------------------------------ attention
+SHAPES = [(4, 2, 32, 16), (8, 2, 64, 64), (4, 1, 96, 48), (3, 3, 128, 128), (6, 2, 32, 192)]
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H_,G,D,E", SHAPES)
+@pytest.mark.parametrize("window", [1, 2, 16, 21, 64, 1000, None])
+def test_windows_the_one_in_the_denominator_and_gates_per_head(backend, dtype, H_, G, D, E, window):
+    """A long portion, a short one and decoded rows in one step: every head's queries point at one key just
+    inside the window, just outside it, far back, at a page's border, or at none (then the one in the
+    denominator takes most of the weight); a gate per head where the outputs are made final."""
+    if backend == "emu" and (D > 64 or window in (64, 1000)):
+        pytest.skip("the references on the CPU take the small shapes; the kernels all of them")
+    ops = ops_of(backend)
+    dev = ops.device
+    lengths, spans, scale = [90, 45, 70, 33], [(0, 90), (40, 45), (69, 70), (0, 33)], 0.6
+    cache = Paged(ops, dtype, lengths, G, D, E, seed=3)
+    rounded = lambda t: t.to(dtype).to(F64)
+    ks, vs, qs = [], [], []
+    for b, n in enumerate(lengths):
+        k, v = randn(n, G, D, seed=10 + b) / D ** 0.5, randn(n, G, E, seed=20 + b)
+        q = randn(n, H_, D, seed=30 + b, scale=0.5)
+        size = n + 5 if window is None else window
+        for i in range(n):
+            target = [i, i - size + 1, i - size, i // 16 * 16, i // 16 * 16 - 1, 0, None][(3 * i + b) % 7]
+            if target is not None and 0 <= target <= i:
+                for h in range(H_):
+                    kk = k[target, h // (H_ // G)]
+                    q[i, h] = kk / kk.norm() ** 2 * 6.0 / scale
+        cache.write(torch.cat([torch.zeros(n, H_ * D), k.reshape(n, -1), v.reshape(n, -1)], 1), H_, list(range(n)), [b] * n)
+        ks.append(rounded(k)), vs.append(rounded(v)), qs.append(rounded(q))
+    positions = [p for lo, hi in spans for p in range(lo, hi)]
+    row_req = [b for b, (lo, hi) in enumerate(spans) for _ in range(lo, hi)]
+    rows = len(positions)
+    gates = randn(rows, 5 + H_, seed=40, scale=1.5)
+    want = torch.cat([P.gate_heads(P.attend(qs[b], ks[b], vs[b], scale, window)[lo:hi],
+                                   gates[[r for r in range(rows) if row_req[r] == b], 5:].to(F64)) for b, (lo, hi) in enumerate(spans)])
+    q = torch.cat([qs[b][lo:hi] for b, (lo, hi) in enumerate(spans)]).reshape(rows, -1).to(dtype).to(dev)
+    out = torch.full((rows, H_ * E), float("nan"), dtype=dtype, device=dev)
+    pick = getattr(ops, "windowed_attention_long_rows", None)
+    long_from = pick(dtype, D, E, 16) if pick is not None else 0
+    q_start, _ = batch([hi - lo for lo, hi in spans], dev)
+    ops.sink_window_attention(q, H_, G, D, E, cache.k_cache, cache.v_cache, cache.table, 16, ints(positions, dev),
+                              ints(row_req, dev), window, 0, torch.zeros(H_, device=dev), scale, out, q_start, long_from,
+                              3 if long_from else 1, 90 if window is None else min(window, 90), head_gate=(gates.to(dev), 5))
+    close(out, want.reshape(rows, -1), dtype, "gated heads", f32=2e-5, bf16=1.5e-2)
+
+
+def test_the_oracle_s_window_and_one():
+    """A window one token off, or no one in the denominator, would show in the case above."""
+    n, D = 30, 8
+    k, v = randn(n, 1, D, seed=1).to(F64), randn(n, 1, D, seed=2).to(F64)
+    q = torch.zeros(n, 1, D, dtype=F64)
+    q[29, 0] = k[10, 0] * 8.0 / k[10, 0].norm() ** 2
+    inside, outside = P.attend(q, k, v, 1.0, 20), P.attend(q, k, v, 1.0, 19)
+    assert float((inside[29] - outside[29]).abs().max()) > 0.5
+    plain = torch.softmax(k[10:30, 0] @ q[29, 0], 0) @ v[10:30, 0]
+    zero = P.attend(torch.zeros_like(q), k, v, 1.0, 1)
+    assert torch.allclose(zero[29, 0], v[29, 0] / 2) and not torch.allclose(inside[29, 0], plain)
+
+
+# ------------------------------------------------------------------ the recurrence
+def recurrence(width, blocks, taps, seed, lam=(-4.0, 2.0)):
+    """Tensors of one mixer by the roles' short names; projections are the identity, so ``proj`` is the input."""
+    n = width // blocks
+    bf = lambda t: t.to(torch.bfloat16)
+    return {"conv": bf(0.3 + randn(width, taps, seed=seed, scale=0.5)), "conv.b": bf(randn(width, seed=seed + 1, scale=0.5)),
+            "ra": bf(randn(blocks, n, n, seed=seed + 2, scale=2.0 / n ** 0.5)), "ra.b": bf(randn(blocks, n, seed=seed + 3)),
+            "ri": bf(randn(blocks, n, n, seed=seed + 4, scale=2.0 / n ** 0.5)), "ri.b": bf(randn(blocks, n, seed=seed + 5)),
+            "lam": bf(lam[0] + lam[1] * randn(width, seed=seed + 6))}
+
+
+def bound(ops, dtype, w, width, blocks, taps, hidden=8):
+    """The part with its tensors laid out, its projections zero (they are not used here)."""
+    names = dict(y_weight="y", y_bias="y.b", x_weight="x", x_bias="x.b", conv="conv", conv_bias="conv.b", r_weight="ra",
+                 r_bias="ra.b", i_weight="ri", i_bias="ri.b", decay="lam", o_weight="o")
+    part = GatedLinearRecurrence(hidden, width, blocks, taps, names)
+    zeros = {"y": (width, hidden), "x": (width, hidden), "y.b": (width,), "x.b": (width,), "o": (hidden, width)}
+    tensors = {k: torch.zeros(s, dtype=torch.bfloat16) for k, s in zeros.items()}
+    tensors.update(w)
+    assert {k: tuple(v.shape) for k, v in tensors.items()} == {k: s.shape for k, s in part.tensor_specs().items()}
+    part.bind({k: (v.to(dtype) if v.dim() > 1 else v).to(ops.device) for k, v in tensors.items()}, ops, dtype)
+    return part
+
+
+def run_recurrence(ops, part, dtype, xs, ys, cuts, slots):
+    """``cuts``: steps, each a list of ``(request, rows)``; -> the outputs of every request."""
+    dev = ops.device
+    parts, n, laid, channels = part.blocks, part.part, part.laid, part.channels
+    lay = lambda t: torch.nn.functional.pad(t.view(-1, parts, n), (0, laid - n)).reshape(-1, channels)
+    state = torch.zeros(max(slots) + 2, channels, device=dev)
+    state[max(slots) + 1] = 7.0                      # (a slot nobody uses stays as it is)
+    ring = torch.zeros(max(slots) + 2, part.taps, channels, device=dev) if part.taps > 1 else None
+    at, out = [0] * len(xs), [[] for _ in xs]
+    for step in cuts:
+        x = torch.cat([lay(xs[b][at[b]:at[b] + c]) for b, c in step])
+        y = torch.cat([lay(ys[b][at[b]:at[b] + c]) for b, c in step])
+        rows = x.shape[0]
+        proj = torch.cat([x, torch.full((rows, 4), 99.0), y], 1).to(dev)
+        q_start, _ = batch([c for _, c in step], dev)
+        pos = ints([p for b, c in step for p in range(at[b], at[b] + c)], dev)
+        mixed = torch.full((rows, channels), float("nan"), dtype=dtype, device=dev)
+        room = [torch.full((rows, channels), float("nan"), device=dev) for _ in range(2)]
+        ops.gated_recurrence(proj, 0, channels + 4, laid, part.conv, part.conv_bias, ring, part.gates, part.r_bias, part.i_bias,
+                             part.decay, state, pos, q_start, ints([slots[b] for b, _ in step], dev), len(step), *room, mixed,
+                             all(c == 1 for _, c in step))
+        got = mixed.view(rows, parts, laid)
+        assert float(got[..., n:].float().abs().sum()) == 0.0        # (the channels behind a part)
+        got, r = got[..., :n].reshape(rows, -1), 0
+        for b, c in step:
+            out[b].append(got[r:r + c].float().cpu())
+            at[b] += c
+            r += c
+    assert float((state[max(slots) + 1] - 7.0).abs().max()) == 0.0
+    return [torch.cat(o) for o in out]
+
+
+def plain_recurrence(w, x, y, dtype):
+    """The branch after its projections, times the gelu branch.  (The gates' products read ``u`` in the compute dtype.)"""
+    u = P.causal_conv(x.to(F64), w["conv"], w["conv.b"])
+    read = u.to(dtype).to(F64)
+    r, i = P.block_gate(read, w["ra"], w["ra.b"]), P.block_gate(read, w["ri"], w["ri.b"])
+    return P.gated_unit(P.decay_logs(r, w["lam"]), i * u) * P.gelu_tanh(y.to(F64))
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("width,blocks,taps", [(64, 2, 4), (40, 1, 3), (36, 3, 2), (96, 3, 1), (160, 5, 6), (320, 1, 4),
+                                               (544, 2, 4), (1280, 20, 4)])
+@pytest.mark.parametrize("how", ["whole", "portions", "decoded", "mixed"])
+def test_recurrence_in_portions_with_states_in_slots(backend, dtype, width, blocks, taps, how):
+    """Portions of every size (tiles of 64 rows and beyond), decoded rows, rows beside other requests' portions:
+    the state and the convolution's inputs are carried in scattered slots; widths of a slab of a part and
+    more, parts that are laid out wider."""
+    if backend == "emu" and width > 320:
+        pytest.skip("the references on the CPU take the small shapes; the kernels all of them")
+    ops = ops_of(backend)
+    lengths = [150, 33, 7] if how != "decoded" else [20, 9, 3]
+    w = recurrence(width, blocks, taps, 1)
+    xs = [randn(n, width, seed=50 + b, scale=1.5) for b, n in enumerate(lengths)]
+    ys = [randn(n, width, seed=60 + b, scale=1.5) for b, n in enumerate(lengths)]
+    cuts = {"whole": [[(0, 150)], [(2, 7), (1, 33)]],
+            "portions": [[(0, 1)], [(0, 2)], [(1, 2), (0, 61)], [(0, 64)], [(1, 31), (0, 22), (2, 3)], [(2, 2)], [(2, 2)]],
+            "decoded": [[(b, 1) for b in range(3) if t < lengths[b]] for t in range(20)],
+            "mixed": [[(1, 2), (2, 1), (0, 130)], [(2, 1), (0, 1), (1, 1)], [(0, 1), (1, 28), (2, 3)], [(2, 1), (1, 1), (0, 1)],
+                      [(0, 17), (1, 1), (2, 1)]]}[how]
+    part = bound(ops, dtype, w, width, blocks, taps)
+    got = run_recurrence(ops, part, dtype, xs, ys, cuts, [3, 0, 2])
+    for b in range(3):
+        want = plain_recurrence(w, xs[b], ys[b], dtype)[:got[b].shape[0]]
+        close(got[b], want, dtype, f"request {b}", f32=2e-5, bf16=1e-2)
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("lam", [(-14.0, 0.5), (6.0, 1.0)])
+def test_decays_near_one_and_near_zero(backend, lam):
+    """Channels that hardly forget (the root of 1 - a^2 for a within 1e-5 of one) and channels that forget
+    within a token (whose decays' product underflows inside a tile)."""
+    ops = ops_of(backend)
+    w = recurrence(64, 2, 4, 5, lam)
+    x, y = randn(300, 64, seed=1, scale=2.0), randn(300, 64, seed=2)
+    part = bound(ops, torch.float32, w, 64, 2, 4)
+    for cuts in ([[(0, 300)]], [[(0, 100)]] + [[(0, 1)]] * 20 + [[(0, 180)]]):
+        got, = run_recurrence(ops, part, torch.float32, [x], [y], cuts, [1])
+        want = plain_recurrence(w, x, y, torch.float32)
+        assert float((got.double() - want).abs().max()) < 2e-5 * float(want.abs().max())
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("cuts", [[[(0, 400)]], [[(0, 2)], [(0, 300)], [(0, 98)]], [[(0, 200)]] + [[(0, 1)]] * 8 + [[(0, 192)]]])
+def test_an_early_input_is_remembered(backend, cuts):
+    """One input hundreds of tokens back, everything behind it zero: it is in the state at the end, by the
+    product of all decays since, whatever tiles and steps lie between."""
+    ops = ops_of(backend)
+    w = recurrence(32, 1, 3, 9, (-7.0, 0.3))
+    w["conv.b"].zero_(), w["ri"].zero_(), w["ra"].zero_()
+    w["conv"].abs_().add_(0.1)
+    x, y = torch.zeros(400, 32), torch.full((400, 32), 3.0)
+    x[1] = 40.0
+    part = bound(ops, torch.float32, w, 32, 1, 3)
+    got, = run_recurrence(ops, part, torch.float32, [x], [y], cuts, [0])
+    want = plain_recurrence(w, x, y, torch.float32)
+    assert float(want[399].abs().min()) > 1e-3
+    assert float(((got[399].double() - want[399]) / want[399]).abs().max()) < 1e-4
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("taps", [2, 4, 7])
+def test_an_input_reaches_exactly_the_taps(backend, taps):
+    """An input that stands out changes the outputs from its own position on (never before), and with a state
+    that forgets at once only as far as the taps reach, over every kind of cut."""
+    ops = ops_of(backend)
+    w = recurrence(32, 1, taps, 3, (12.0, 0.1))
+    w["ra"].zero_(), w["ra.b"].fill_(3.0)
+    x, y = randn(20, 32, seed=1, scale=0.1), torch.full((20, 32), 2.0)
+    other = x.clone()
+    other[9] += 30.0
+    part = bound(ops, torch.float32, w, 32, 1, taps)
+    for cuts in ([[(0, 20)]], [[(0, 1)]] * 20, [[(0, 9)], [(0, 2)], [(0, 9)]], [[(0, 10)], [(0, 1)], [(0, 9)]]):
+        a, = run_recurrence(ops, part, torch.float32, [x], [y], cuts, [0])
+        b, = run_recurrence(ops, part, torch.float32, [other], [y], cuts, [0])
+        moved = (a - b).abs().max(1).values
+        assert [bool(m > 1e-2) for m in moved] == [9 <= t < 9 + taps for t in range(20)], moved
+
+
+# ------------------------------------------------------------------ experts
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("rows", [1, 9, 40, 300])
+@pytest.mark.parametrize("limit", [0.7, 3.0])
+def test_the_clamped_pair_as_the_epilogue_of_a_product(backend, dtype, rows, limit):
+    """Few rows and many (the product kernels differ), both dtypes: gates held from above only, the other
+    factor from both sides."""
+    from llm_inference_lab_amd.parts import interleave_gate_up
+    ops = ops_of(backend)
+    x = randn(rows, 72, seed=5).to(dtype)
+    gate, up = (randn(56, 72, seed=s, scale=0.25).to(dtype) for s in (6, 7))
+    out = torch.full((rows, 56), float("nan"), dtype=dtype, device=ops.device)
+    ops.linear_swiglu(x.to(ops.device), ops.prepare_weight(interleave_gate_up(gate, up).to(ops.device)), out, "clamped",
+                      (limit, 1.702, 1.0))
+    w = {"gate": gate, "up": up, "down": torch.eye(56)}
+    close(out, P.clamped_expert(x.to(F64), w, "", limit), dtype, "g sigmoid(1.702 g) (u + 1)", f32=1e-5)
+    with pytest.raises((TypeError, ValueError)):       # (without its constants)
+        ops.linear_swiglu(x.to(ops.device), ops.prepare_weight(interleave_gate_up(gate, up).to(ops.device)), out, "clamped")
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("experts,groups,keep,top", [(8, 4, 3, 3), (6, 1, 1, 6), (12, 6, 2, 4), (9, 3, 2, 1), (5, 5, 3, 2),
+                                                     (64, 8, 4, 8), (96, 4, 2, 6), (300, 10, 3, 5)])
+def test_the_routers_choice_and_weights(backend, experts, groups, keep, top):
+    """Groups by the sum of their two largest scores (groups of one and of two too), the best of the kept
+    ones, the chosen scores' shares times a constant; routers of one wave and larger."""
+    ops = ops_of(backend)
+    dev = ops.device
+    z = randn(37, experts, seed=8, scale=2.0)
+    router = dict(experts=experts, top=top, scale=2.5, groups=dict(count=groups, keep=keep))
+    want = P.route(z.to(F64), torch.eye(experts), router)
+    chosen = torch.full((37, top), -1, dtype=torch.int32, device=dev)
+    weights = torch.full((37, top), float("nan"), device=dev)
+    ops.moe_select(z.to(dev), torch.zeros(experts, device=dev), groups, keep, 2.5, chosen, weights, scoring="sigmoid",
+                   group_score="top2", share_eps=1e-20)
+    for r in range(37):
+        assert chosen[r].tolist() == [e for e, _ in want[r]], r
+        assert float((weights[r].cpu().double() - torch.tensor([float(s) for _, s in want[r]], dtype=F64)).abs().max()) < 1e-6
+    assert float((weights.sum(1) - 2.5).abs().max()) < 1e-5
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+def test_two_good_scores_beat_one_excellent(backend):
+    """The group of the single best output is dropped where another group's two best sum to more; scores so
+    small that their sum is tiny still share out to the constant."""
+    ops = ops_of(backend)
+    z = torch.tensor([[5.0, -9.0, -9.0, 1.0, 1.0, -9.0], [-30.0, -31.0, -40.0, -30.5, -30.6, -50.0]], device=ops.device)
+    chosen, weights = torch.zeros(2, 2, dtype=torch.int32, device=ops.device), torch.zeros(2, 2, device=ops.device)
+    how = dict(scoring="sigmoid", group_score="top2", share_eps=1e-20)
+    ops.moe_select(z, torch.zeros(6, device=ops.device), 2, 1, 3.0, chosen, weights, **how)
+    assert chosen[0].tolist() == [3, 4] and abs(float(weights[0, 0]) - 1.5) < 1e-6
+    assert chosen[1].tolist() == [0, 1] and abs(float(weights[1].sum()) - 3.0) < 1e-5
+    ops.moe_select(z, torch.zeros(6, device=ops.device), 2, 1, 3.0, chosen, weights, scoring="sigmoid")
+    assert chosen[0].tolist()[0] == 0 and abs(float(weights[0, 0]) - 3.0 / (1.0 + math.exp(-5.0))) < 1e-6
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("rows", [1, 5, 70, 300])
+@pytest.mark.parametrize("shape", [dict(experts=6, top=2, groups=(3, 2), ff=24, width=64, limit=0.6),
+                                   dict(experts=4, top=4, groups=(1, 1), ff=36, width=40, limit=5.0),
+                                   dict(experts=72, top=5, groups=(8, 3), ff=16, width=32, limit=1.0)])
+def test_the_mixture_of_experts_alone(backend, dtype, rows, shape):
+    """The part with its sorting, grouped products and weighted sum, added into a stream and handed over for the
+    norm behind the sum: both the plain mixture."""
+    ops = ops_of(backend)
+    dev = ops.device
+    w, f, n = shape["width"], shape["ff"], shape["experts"]
+    part = RoutedExperts(w, f, n, shape["top"], dict(router="router", expert_gate="e{}.gate", expert_up="e{}.up",
+                                                     expert_down="e{}.down"), scale=1.7, groups=shape["groups"][0],
+                         groups_keep=shape["groups"][1], correction=False, scoring="sigmoid", expert_form="clamped",
+                         expert_constants=(shape["limit"], 1.702, 1.0), group_score="top2", share_eps=1e-20)
+    tensors = {name: randn(*s.shape, seed=i, scale=(2.0 if name == "router" else 1.4) / s.shape[1] ** 0.5).to(torch.bfloat16)
+               for i, (name, s) in enumerate(part.tensor_specs().items())}
+    part.bind({k: v.to(dtype).to(dev) for k, v in tensors.items()}, ops, dtype)
+    h = randn(rows, w, seed=500).to(dtype)
+    mlp = dict(expert=dict(ff=f, limit=shape["limit"]), router=dict(experts=n, top=shape["top"], scale=1.7,
+                                                                    groups=dict(count=shape["groups"][0], keep=shape["groups"][1])))
+    want = P.mixture(h.to(F64), mlp, tensors, "")
+    stream = torch.ones(rows, w, device=dev)
+    part.forward(h.to(dev), stream, Scratch(dev))
+    close(stream, 1.0 + want, dtype, "stream + mixture", bf16=1e-2)
+    out = torch.full((rows, w), float("nan"), device=dev)
+    split = part.forward_split(h.to(dev), out, Scratch(dev))
+    x = randn(rows, w, seed=501).to(dev)
+    g = torch.ones(w, device=dev)
+    normed = P.post_norm(x.cpu().to(F64), want, g.cpu(), 2.0, 1e-5)
+    ops.post_norm(x, 2.0, out if split is None else split, g, 1e-5)
+    close(x, normed, dtype, "norm(2 x + mixture)", bf16=1e-2)
+
+
+# ------------------------------------------------------------------ what is refused
+def test_what_the_parts_refuse():
+    from llm_inference_lab_amd.parts import WindowedSinkAttention
+    names = {k: k for k in ("router", "expert_gate", "expert_up", "expert_down")}
+    for bad in (dict(expert_form="clamped"), dict(expert_constants=(1.0, 1.7, 1.0)), dict(group_score="mean")):
+        with pytest.raises(ValueError):
+            RoutedExperts(16, 16, 4, 2, names, **bad)
+    for bad in (dict(width=30, blocks=4, conv_taps=2), dict(width=32, blocks=2, conv_taps=0)):
+        with pytest.raises(ValueError):
+            GatedLinearRecurrence(16, tensors={}, **bad)
+    with pytest.raises(ValueError):
+        WindowedSinkAttention(16, 2, 1, 8, 8, 1.0, {}, sink=True, plus_one=True)
+    with pytest.raises(ValueError):
+        RotaryEmbedding(16, 1e4, scaling=dict(factor=2.0, low=1.0))
