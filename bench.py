@@ -3,7 +3,7 @@
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--context S]
                     [--shape 0.5b|7b|32b] [--layers L] [--dtype bf16|f32]
     python bench.py --mixed [--shape 7b] [--requests 64] [--chunk 512] [--outputs 64]
-    python bench.py --design vivevik|ruvalorn|minodra|ninisun|mazanex [--size small|medium|large] [--context 2048]
+    python bench.py --design vivevik|ruvalorn|minodra|ninisun|mazanex|molotar [--size small|medium|large] [--context 2048]
 
 Default: the layer sizes of the Qwen2.5-0.5B shape with seeded random weights,
 batch 8, context 4096, bfloat16.  A "step" is one decode step of the whole
@@ -58,6 +58,12 @@ every three) and the Qwen2 decoder.
 sublayers' results, feed-forwards of normed powers; in turn attention over chunks beside time mixing,
 gated linear attention and a matrix memory with exponential gates), beside the Vivevik design of equal
 size (the closest one: the same attention and scan kernels) and the Qwen2 decoder.
+
+``--design molotar``: the same for the Molotar design (norms behind the sums; in threes two recurrences of
+single numbers with block-diagonal gates and windowed attention, every other one of which reads an earlier
+one's keys; clamped experts behind a sigmoid router that chooses among the best groups), beside the Ruvalorn
+design of equal size (the closest one: mixtures of experts behind a grouped router) and the Vivevik design
+(the same attention kernels, a recurrent layer in every three).
 
 ``--mixed``: many requests with prompts of different lengths go through the
 scheduler with a small token budget, so that portions of prompts run beside the
@@ -343,6 +349,50 @@ def mazanex_flops(cfg, tokens):
     return total + 2 * w * cfg.vocab
 
 
+# ``--design molotar``: layers in threes, two recurrences (as many channels as the stream is wide, in parts of
+# 128 or 256, four taps) and windowed attention of 1,024 positions with stretched waves, every other one of
+# which reads the keys and values of the one before; every layer has 32 experts of which a token takes 8,
+# together as wide as the dense feed-forward, out of the best 3 of 4 groups.
+MOLOTAR_PARTS = {"small": 128, "medium": 256, "large": 256}
+
+
+def molotar_config(size):
+    import llm_inference_lab_amd as lab
+    width, heads, kv, dim, ff, layers = DESIGN_SIZES[size]
+    listed = []
+    for i in range(layers):
+        mlp = dict(kind="moe", expert=dict(ff=ff // 8, limit=7.0),
+                   router=dict(experts=32, top=8, scale=2.5, groups=dict(count=4, keep=3)))
+        if i % 3 == 2:
+            mixer = dict(heads=heads, kv_heads=kv, dim=dim, vdim=dim, scale=dim ** -0.5, mask=dict(size=DESIGN_WINDOW),
+                         rot=dict(dims=dim, base=5e5, scaling=dict(factor=4.0, low=1.0, high=4.0, original=1024)))
+            if i % 6 == 5:
+                mixer["kv_from"] = i - 3
+            listed.append(dict(type="attention", mixer=mixer, mlp=mlp))
+        else:
+            listed.append(dict(type="rglru", mixer=dict(width=width, blocks=width // MOLOTAR_PARTS[size], conv=4), mlp=mlp))
+    return lab.MolotarConfig.from_dict(dict(
+        architecture="Molotar", vocab=DESIGN_VOCAB, width=width, norm=dict(eps=1e-6), postln_alpha=2.0, layers=listed,
+        embedding=dict(scale=8.0, bigram=dict(buckets=8191, mul_prev=331, mul_cur=17))))
+
+
+def molotar_flops(cfg, tokens):
+    """Multiply-adds times two of one prompt of ``tokens`` positions (products and attention; a recurrence
+    counts its convolution, its gates' products and its update)."""
+    w, total = cfg.width, 0
+    for l in cfg.layers:
+        m = l.mixer
+        if l.type == "attention":
+            q, k, v = m.heads * m.dim, m.kv_heads * m.dim, m.kv_heads * m.vdim
+            total += tokens * 2 * (w * (q + (k + v if m.kv_from is None else 0) + m.heads) + m.heads * m.vdim * w)
+            total += 2 * sum(min(i + 1, m.window or tokens) for i in range(tokens)) * m.heads * (m.dim + m.vdim)
+        else:
+            total += tokens * (6 * w * m.width + m.width * (4 * (m.width // m.blocks) + 2 * m.conv + 4))
+        if l.mlp is not None:
+            total += tokens * (2 * w * l.mlp.experts + 6 * w * l.mlp.ff * l.mlp.top)
+    return total + 2 * w * cfg.vocab
+
+
 def design_run(args, bracket=None):
     """``--design vivevik``: both models at each size, one after the other on the same GPU.
     ``--only-model``, ``--only-prefill`` / ``--only-decode`` and ``--batch`` narrow the run (for
@@ -363,8 +413,10 @@ def design_run(args, bracket=None):
         record[size] = {"width": width, "heads": heads, "kv_heads": kv, "head_dim": dim, "ff": ff, "layers": layers,
                         "context": context, "window": DESIGN_WINDOW}
         design = {"ruvalorn": ruvalorn_config, "minodra": minodra_config, "vivevik": vivevik_config,
-                  "ninisun": ninisun_config, "mazanex": mazanex_config}[args.design](size)
+                  "ninisun": ninisun_config, "mazanex": mazanex_config, "molotar": molotar_config}[args.design](size)
         beside = [("qwen2", qwen)]
+        if args.design == "molotar":
+            beside = [("ruvalorn", ruvalorn_config(size)), ("vivevik", vivevik_config(size))]
         if args.design in ("ninisun", "mazanex"):         # (the closest design first)
             beside.insert(0, ("vivevik", vivevik_config(size)))
         for label, cfg in [(args.design, design)] + beside:
@@ -386,6 +438,7 @@ def design_run(args, bracket=None):
                      minodra_flops(cfg, args.prefill_tokens) if label == "minodra" else
                      ninisun_flops(cfg, args.prefill_tokens) if label == "ninisun" else
                      mazanex_flops(cfg, args.prefill_tokens) if label == "mazanex" else
+                     molotar_flops(cfg, args.prefill_tokens) if label == "molotar" else
                      prefill_flops(cfg, args.prefill_tokens))
             out = {"weight_bytes_per_step": engine.weight_bytes_per_step()}
             if not args.only_decode:
@@ -407,7 +460,8 @@ def design_run(args, bracket=None):
             torch.cuda.empty_cache()
         print(f"[bench] {size}: {json.dumps(record[size])}", file=sys.stderr, flush=True)
     print(json.dumps({"metric": "design_throughput", "design": args.design,
-                      "beside": "vivevik, qwen2" if args.design in ("ninisun", "mazanex") else "qwen2", "dtype": args.dtype,
+                      "beside": ("ruvalorn, vivevik" if args.design == "molotar" else
+                                 "vivevik, qwen2" if args.design in ("ninisun", "mazanex") else "qwen2"), "dtype": args.dtype,
                       "data": "synthetic", "unit": "tokens/s", "prefill_tokens": args.prefill_tokens,
                       "sizes": record}))
 
@@ -918,10 +972,11 @@ def main():
                     help="fix a choice of the kernels for the whole run, to compare variants: a keyword of "
                          "engine.ops.debug.force, values separated by ':' (attention_splits=64:8, "
                          "attention_merge_kernel=64, gemm_tile=129)")
-    ap.add_argument("--design", choices=["vivevik", "ruvalorn", "minodra", "ninisun", "mazanex"], default=None,
+    ap.add_argument("--design", choices=["vivevik", "ruvalorn", "minodra", "ninisun", "mazanex", "molotar"], default=None,
                     help="throughput of another design beside the Qwen2 decoder of equal size")
     ap.add_argument("--size", choices=sorted(DESIGN_SIZES), default=None, help="--design: one size only")
-    ap.add_argument("--only-model", choices=["vivevik", "ruvalorn", "minodra", "ninisun", "mazanex", "qwen2"], default=None, help="--design: one of the two models only")
+    ap.add_argument("--only-model", choices=["vivevik", "ruvalorn", "minodra", "ninisun", "mazanex", "molotar", "qwen2"], default=None,
+                    help="--design: one of the models only")
     ap.add_argument("--only-decode", action="store_true", help="--design: decode at --batch only, no prefill")
     ap.add_argument("--side", choices=["7b", "32b", "f32", "peaks"], help=argparse.SUPPRESS)
     args = ap.parse_args()

@@ -55,18 +55,24 @@ __device__ __forceinline__ floatx4 multiply(Eight<float>::V w, Eight<float>::V u
   return acc;
 }
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + __expf(-z)); }
+// (reciprocal and square root to a unit in the last place, as the hardware gives them)
+__device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
 // tanh form of gelu, 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))), as z * sigmoid(2 t)
 __device__ __forceinline__ float gelu_f(float z) {
-  return z / (1.0f + __expf(-2.0f * 0.7978845608028654f * (z + 0.044715f * z * z * z)));
+  return z * __builtin_amdgcn_rcpf(1.0f + __expf(-2.0f * 0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
-// sqrt(1 - a^2) for a = exp(l), l <= 0: near a = 1 by the series of 1 - exp(-y), y = -2 l
+// sqrt(1 - a^2) for a = exp(l), l <= 0: near a = 1 by the series of 1 - exp(-y), y = -2 l (the sum of
+// (-1)^k y^(k+1) / (k+1)!)
 __device__ __forceinline__ float complement(float l, float a) {
   const float y = -2.0f * l;
-  float s = 1.0f - y * (1.0f / 9.0f);
-#pragma unroll
-  for (int n = 8; n >= 2; --n) s = 1.0f - y * (1.0f / (float)n) * s;
-  return sqrtf(y < 0.7f ? y * s : 1.0f - a * a);
+  float s = 1.0f / 5040.0f;
+  s = fmaf(s, y, -1.0f / 720.0f);
+  s = fmaf(s, y, 1.0f / 120.0f);
+  s = fmaf(s, y, -1.0f / 24.0f);
+  s = fmaf(s, y, 1.0f / 6.0f);
+  s = fmaf(s, y, -0.5f);
+  s = fmaf(s, y, 1.0f);
+  return __builtin_amdgcn_sqrtf(y < 0.35f ? y * s : fmaf(-a, a, 1.0f));
 }
 
 __device__ __forceinline__ floatx4 load4(const float* p) { return *(const floatx4*)p; }
@@ -103,40 +109,56 @@ __device__ __forceinline__ floatx4 convolve(const Recurrence<T>& a, const float*
 }
 
 // ------------------------------------------------------------------ one row a request
-// A block takes 16 outputs of a part and 16 rows (row r is request r); its four waves share the part's
+// A block takes 16 * STRIPS outputs of a part and 16 rows (row r is request r); its four waves share the part's
 // inputs, each making its operands from the projections and the rings itself.
-template <typename T, int TAPS>
+template <typename T, int TAPS, int STRIPS>
 __global__ __launch_bounds__(256) void recurrence_row_kernel(Recurrence<T> a) {
   typedef typename Eight<T>::V vec8;
-  __shared__ floatx4 sums[4][2][64];
+  __shared__ floatx4 sums[4][STRIPS][2][64];
   const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int taps = TAPS > 0 ? TAPS : a.taps;
   const int strips = a.size >> 4, steps = a.size >> 5;
-  const int part = blockIdx.x / strips, first = part * a.size;
+  const int strip0 = blockIdx.x * STRIPS, first = strip0 / strips * a.size;
   const int r0 = blockIdx.y * 16;
-  // what the block's end needs, asked for first: a thread a row and an output
-  const int er = min(r0 + (int)(threadIdx.x >> 4), a.rows - 1), ec = blockIdx.x * 16 + (threadIdx.x & 15);
+  // what the block's end needs, asked for first: a thread a row and an output of every strip
+  const int er = min(r0 + (int)(threadIdx.x >> 4), a.rows - 1), ec = strip0 * 16 + (threadIdx.x & 15);
   const int e_slot = a.req_rows[er], e_place = a.positions[er] % taps;
   float* e_ring = taps > 1 ? a.ring + (size_t)e_slot * taps * a.channels + ec : nullptr;
-  const float own = a.proj[(size_t)er * a.ld + a.off_x + ec];
-  const float y = a.proj[(size_t)er * a.ld + a.off_y + ec];
+  const float* e_row = a.proj + (size_t)er * a.ld + ec;
   float* s_at = a.state + (size_t)e_slot * a.channels + ec;
-  const float before = *s_at;
-  float u = a.conv_b[ec];
-  for (int k = taps - 1; k > 0; --k)
-    u = fmaf(a.conv[(size_t)(taps - 1 - k) * a.channels + ec],
-             e_ring[(size_t)(e_place - k < 0 ? e_place - k + taps : e_place - k) * a.channels], u);
-  u = fmaf(a.conv[(size_t)(taps - 1) * a.channels + ec], own, u);
-  const float rb = a.rb[ec], ib = a.ib[ec], decay = a.c[ec];
+  float own[STRIPS], y[STRIPS], before[STRIPS], u[STRIPS], rb[STRIPS], ib[STRIPS], decay[STRIPS];
+#pragma unroll
+  for (int n = 0; n < STRIPS; ++n) {
+    own[n] = e_row[a.off_x + 16 * n];
+    y[n] = e_row[a.off_y + 16 * n];
+    before[n] = s_at[16 * n];
+    u[n] = a.conv_b[ec + 16 * n];
+    rb[n] = a.rb[ec + 16 * n], ib[n] = a.ib[ec + 16 * n], decay[n] = a.c[ec + 16 * n];
+  }
+  for (int k = taps - 1; k > 0; --k) {
+    const size_t at = (size_t)(e_place - k < 0 ? e_place - k + taps : e_place - k) * a.channels;
+    const float* w = a.conv + (size_t)(taps - 1 - k) * a.channels + ec;
+#pragma unroll
+    for (int n = 0; n < STRIPS; ++n) u[n] = fmaf(w[16 * n], e_ring[at + 16 * n], u[n]);
+  }
+#pragma unroll
+  for (int n = 0; n < STRIPS; ++n) u[n] = fmaf(a.conv[(size_t)(taps - 1) * a.channels + ec + 16 * n], own[n], u[n]);
 
   const int r = min(r0 + c, a.rows - 1);
   const float* ring = taps > 1 ? a.ring + (size_t)a.req_rows[r] * taps * a.channels : nullptr;
   const int place = a.positions[r] % taps;
-  floatx4 acc[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
-  const vec8* w = (const vec8*)a.gates + (size_t)blockIdx.x * steps * 128 + lane;
+  floatx4 acc[STRIPS][2];
+#pragma unroll
+  for (int n = 0; n < STRIPS; ++n) acc[n][0] = acc[n][1] = floatx4{0.f, 0.f, 0.f, 0.f};
+  const vec8* w = (const vec8*)a.gates + (size_t)strip0 * steps * 128 + lane;
   for (int k = wave; k < steps; k += 4) {
-    const vec8 wr = w[(size_t)k * 128], wi = w[(size_t)k * 128 + 64];
+    vec8 wr[STRIPS], wi[STRIPS];
+#pragma unroll
+    for (int n = 0; n < STRIPS; ++n) {
+      wr[n] = w[((size_t)n * steps + k) * 128];
+      wi[n] = w[((size_t)n * steps + k) * 128 + 64];
+    }
     const int ch = first + 32 * k + 8 * g;
     const floatx4 lo = convolve<T, TAPS>(a, ring, r, 0, place, ch), hi = convolve<T, TAPS>(a, ring, r, 0, place, ch + 4);
     vec8 v;
@@ -145,25 +167,34 @@ __global__ __launch_bounds__(256) void recurrence_row_kernel(Recurrence<T> a) {
       v[j] = from_float<T>(lo[j]);
       v[4 + j] = from_float<T>(hi[j]);
     }
-    acc[0] = multiply(wr, v, acc[0]);
-    acc[1] = multiply(wi, v, acc[1]);
-  }
-  sums[wave][0][lane] = acc[0];
-  sums[wave][1][lane] = acc[1];
-  __syncthreads();
-  const int from = 16 * ((threadIdx.x & 15) >> 2) + (threadIdx.x >> 4), q = threadIdx.x & 3;
-  float zr = rb, zi = ib;
 #pragma unroll
-  for (int n = 0; n < 4; ++n) {
-    zr += sums[n][0][from][q];
-    zi += sums[n][1][from][q];
+    for (int n = 0; n < STRIPS; ++n) {
+      acc[n][0] = multiply(wr[n], v, acc[n][0]);
+      acc[n][1] = multiply(wi[n], v, acc[n][1]);
+    }
   }
+#pragma unroll
+  for (int n = 0; n < STRIPS; ++n) {
+    sums[wave][n][0][lane] = acc[n][0];
+    sums[wave][n][1][lane] = acc[n][1];
+  }
+  __syncthreads();
   if (r0 + (int)(threadIdx.x >> 4) >= a.rows) return;
-  const float l = decay * sigmoid_f(zr), d = __expf(l);
-  const float s = fmaf(d, before, complement(l, d) * sigmoid_f(zi) * u);
-  *s_at = s;
-  if (taps > 1) e_ring[(size_t)e_place * a.channels] = own;
-  a.out[(size_t)er * a.channels + ec] = from_float<T>(s * gelu_f(y));
+  const int from = 16 * ((threadIdx.x & 15) >> 2) + (threadIdx.x >> 4), q = threadIdx.x & 3;
+#pragma unroll
+  for (int n = 0; n < STRIPS; ++n) {
+    float zr = rb[n], zi = ib[n];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      zr += sums[k][n][0][from][q];
+      zi += sums[k][n][1][from][q];
+    }
+    const float l = decay[n] * sigmoid_f(zr), d = __expf(l);
+    const float s = fmaf(d, before[n], complement(l, d) * sigmoid_f(zi) * u[n]);
+    s_at[16 * n] = s;
+    if (taps > 1) e_ring[(size_t)e_place * a.channels + 16 * n] = own[n];
+    a.out[(size_t)er * a.channels + ec + 16 * n] = from_float<T>(s * gelu_f(y[n]));
+  }
 }
 
 // ------------------------------------------------------------------ tiles of rows
@@ -198,22 +229,55 @@ __device__ __forceinline__ bool find_tile(const int* __restrict__ q_start, int n
   return false;
 }
 
-// the value of the lane `n` before within the row of 16 lanes, `other` where there is none
-template <int n>
-__device__ __forceinline__ float lanes_back(float other, float v) {
-  return __int_as_float(__builtin_amdgcn_update_dpp(__float_as_int(other), __float_as_int(v), 0x110 + n, 0xf, 0xf, false));
+// The steps S -> d S + s of four channels: of this lane and of all lanes before it within its row of 16,
+// composed.  A lane takes the composed step of the lane 1, 2, 4, 8 before it in turn; lanes that have none
+// keep theirs (a disabled lane of a shift is not written).  The wait in front: a shift reads a register two
+// instructions after it was written at the earliest; within the block eight lie between.
+#define LLMLAB_COMPOSE(N)                                                                       \
+  "v_fmac_f32_dpp %4, %4, %0 row_shr:" #N " row_mask:0xf bank_mask:0xf\n"                       \
+  "v_fmac_f32_dpp %5, %5, %1 row_shr:" #N " row_mask:0xf bank_mask:0xf\n"                       \
+  "v_fmac_f32_dpp %6, %6, %2 row_shr:" #N " row_mask:0xf bank_mask:0xf\n"                       \
+  "v_fmac_f32_dpp %7, %7, %3 row_shr:" #N " row_mask:0xf bank_mask:0xf\n"                       \
+  "v_mul_f32_dpp %0, %0, %0 row_shr:" #N " row_mask:0xf bank_mask:0xf\n"                        \
+  "v_mul_f32_dpp %1, %1, %1 row_shr:" #N " row_mask:0xf bank_mask:0xf\n"                        \
+  "v_mul_f32_dpp %2, %2, %2 row_shr:" #N " row_mask:0xf bank_mask:0xf\n"                        \
+  "v_mul_f32_dpp %3, %3, %3 row_shr:" #N " row_mask:0xf bank_mask:0xf\n"
+__device__ __forceinline__ void compose(floatx4& d, floatx4& s) {
+  float d0 = d[0], d1 = d[1], d2 = d[2], d3 = d[3], s0 = s[0], s1 = s[1], s2 = s[2], s3 = s[3];
+  asm volatile("s_nop 1\n" LLMLAB_COMPOSE(1) LLMLAB_COMPOSE(2) LLMLAB_COMPOSE(4) LLMLAB_COMPOSE(8) "s_nop 1\n"
+               : "+v"(d0), "+v"(d1), "+v"(d2), "+v"(d3), "+v"(s0), "+v"(s1), "+v"(s2), "+v"(s3));
+  d = floatx4{d0, d1, d2, d3};
+  s = floatx4{s0, s1, s2, s3};
+}
+#undef LLMLAB_COMPOSE
+
+// the value of the last lane of the row of 16 lanes
+__device__ __forceinline__ float last_of_16(float v) {
+  return __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x15f, 0xf, 0xf, true));      // row_newbcast:15
 }
 
-// The composed step (d, s): S -> d S + s of this lane and of all lanes before it within 16
+// the value of the lane `n` before within the row of 16 lanes, round and round
 template <int n>
-__device__ __forceinline__ void compose(float& d, float& s) {
-  const float pd = lanes_back<n>(1.f, d), ps = lanes_back<n>(0.f, s);
-  s = fmaf(d, ps, s);
-  d *= pd;
+__device__ __forceinline__ float lanes_round(float v) {
+  return __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x120 + n, 0xf, 0xf, true));      // row_ror
 }
 
+// x[k] (k >= 1): the inputs k rows before this lane's, the rows of 16 lanes being consecutive rows `cur` and the
+// 16 before them `prev`
+template <int TAPS>
+__device__ __forceinline__ void rows_back(const floatx4& prev, const floatx4& cur, int c, floatx4 (&x)[TAPS > 0 ? TAPS : 1]) {
+  x[0] = cur;
+#pragma unroll
+  for (int q = 0; q < 4; ++q) {
+    if constexpr (TAPS > 1) x[1][q] = lanes_round<1>(c >= 15 ? prev[q] : cur[q]);
+    if constexpr (TAPS > 2) x[2][q] = lanes_round<2>(c >= 14 ? prev[q] : cur[q]);
+    if constexpr (TAPS > 3) x[3][q] = lanes_round<3>(c >= 13 ? prev[q] : cur[q]);
+  }
+}
+
+// A block takes a tile and, a strip a wave, up to blockDim.x / 4 outputs of a part.
 template <typename T, int TAPS>
-__global__ __launch_bounds__(256) void recurrence_tiles_kernel(Recurrence<T> a) {
+__global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(4))) void recurrence_tiles_kernel(Recurrence<T> a) {
   typedef typename Eight<T>::V vec8;
   extern __shared__ __attribute__((aligned(16))) char tile_lds[];
   T* us = (T*)tile_lds;                           // [TILE_ROWS][slab + 8]
@@ -222,8 +286,9 @@ __global__ __launch_bounds__(256) void recurrence_tiles_kernel(Recurrence<T> a) 
   const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int taps = TAPS > 0 ? TAPS : a.taps;
-  const int strips = a.size >> 4, steps = a.size >> 5, groups = (strips + 3) >> 2;
-  const int part = blockIdx.y / groups, strip = (blockIdx.y - part * groups) * 4 + wave;
+  const int threads = blockDim.x, waves = threads >> 6;
+  const int strips = a.size >> 4, steps = a.size >> 5, groups = (strips + waves - 1) / waves;
+  const int part = blockIdx.y / groups, strip = (blockIdx.y - part * groups) * waves + wave;
   const int first = part * a.size;
   const bool works = strip < strips;
   const int row0 = t.index * TILE_ROWS;           // within the request
@@ -232,6 +297,11 @@ __global__ __launch_bounds__(256) void recurrence_tiles_kernel(Recurrence<T> a) 
   const float* ring = taps > 1 ? a.ring + (size_t)slot * taps * a.channels : nullptr;
   const int pos0 = a.positions[t.first] + row0;   // of the tile's first row
   const int slab = a.size < SLAB<T> ? a.size : SLAB<T>, stride = slab + 8;
+  // the input of row j of the request (negative: from before the step), four channels
+  auto input = [&](int j, int ch) {
+    const int place = j < 0 ? (pos0 - row0 + j + taps) % taps : 0;
+    return load4(j >= 0 ? a.proj + ((unsigned)((t.first + j) * a.ld) + a.off_x + ch) : ring + (place * a.channels + ch));
+  };
   floatx4 acc[4][2];
 #pragma unroll
   for (int k = 0; k < 4; ++k) acc[k][0] = acc[k][1] = floatx4{0.f, 0.f, 0.f, 0.f};
@@ -239,30 +309,84 @@ __global__ __launch_bounds__(256) void recurrence_tiles_kernel(Recurrence<T> a) 
   for (int k0 = 0; k0 < a.size; k0 += slab) {
     const int width = a.size - k0 < slab ? a.size - k0 : slab;
     if (k0) __syncthreads();                      // (the slab before has been read)
-    // a thread four channels and every so many rows
-    const int quads = width >> 2, apart = 256 / quads;
-    const int q = threadIdx.x % quads;
-    for (int m = threadIdx.x / quads; m < TILE_ROWS && (int)threadIdx.x < quads * apart; m += apart) {
-      floatx4 v = floatx4{0.f, 0.f, 0.f, 0.f};
-      if (m < n) v = convolve<T, TAPS>(a, ring, t.first + row0 + m, row0 + m, (pos0 + m) % taps, first + k0 + 4 * q);
-      store4(us + m * stride + 4 * q, v);
-    }
-    __syncthreads();
-    if (works)
-      for (int k = 0; k < width >> 5; ++k) {
-        const size_t at = (size_t)((k0 >> 5) + k) * 128;
-        const vec8 wr = w[at], wi = w[at + 64];
+    // a thread four channels and a run of rows, the last inputs in registers
+    const int quads = width >> 2, runs = threads / quads, run = (TILE_ROWS + runs - 1) / runs;
+    const int q = threadIdx.x % quads, m0 = (int)threadIdx.x / quads * run, m1 = min(m0 + run, TILE_ROWS);
+    const int ch = first + k0 + 4 * q;
+    if constexpr (TAPS > 0) {
+      floatx4 w[TAPS], x[TAPS], bias = load4(a.conv_b + ch);
+      if (m0 < n) {
 #pragma unroll
-        for (int m = 0; m < 4; ++m) {
-          const vec8 v = *(const vec8*)(us + (16 * m + c) * stride + 32 * k + 8 * g);
-          acc[m][0] = multiply(wr, v, acc[m][0]);
-          acc[m][1] = multiply(wi, v, acc[m][1]);
+        for (int k = 0; k < TAPS; ++k) w[k] = load4(a.conv + (size_t)(TAPS - 1 - k) * a.channels + ch);
+#pragma unroll
+        for (int k = 1; k < TAPS; ++k) x[k] = input(row0 + m0 - k, ch);
+      }
+      for (int m = m0; m < m1; m += 4) {          // (four rows' loads travel together)
+        floatx4 own[4];
+        if (m < n)
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            own[i] = load4(a.proj + ((unsigned)((t.first + row0 + min(m + i, n - 1)) * a.ld) + a.off_x + ch));
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          if (m + i >= m1) break;
+          floatx4 v = floatx4{0.f, 0.f, 0.f, 0.f};
+          if (m + i < n) {
+            x[0] = own[i];
+            v = bias;
+#pragma unroll
+            for (int k = TAPS - 1; k >= 0; --k) v += w[k] * x[k];
+#pragma unroll
+            for (int k = TAPS - 1; k > 0; --k) x[k] = x[k - 1];
+          }
+          store4(us + (m + i) * stride + 4 * q, v);
         }
       }
+    } else {
+      for (int m = m0; m < m1; ++m) {
+        floatx4 v = floatx4{0.f, 0.f, 0.f, 0.f};
+        if (m < n) v = convolve<T, TAPS>(a, ring, t.first + row0 + m, row0 + m, (pos0 + m) % taps, ch);
+        store4(us + m * stride + 4 * q, v);
+      }
+    }
+    __syncthreads();
+    if (works) {
+      constexpr int AHEAD = sizeof(T) == 4 ? 2 : 4;       // steps whose matrices travel together
+      const int count = width >> 5;
+      for (int k1 = 0; k1 < count; k1 += AHEAD) {
+        vec8 wr[AHEAD], wi[AHEAD];
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) {
+          const int at = ((k0 >> 5) + min(k1 + i, count - 1)) * 128;
+          wr[i] = w[at];
+          wi[i] = w[at + 64];
+        }
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i)
+          if (k1 + i < count) {
+#pragma unroll
+            for (int m = 0; m < 4; ++m) {
+              const vec8 v = *(const vec8*)(us + (16 * m + c) * stride + 32 * (k1 + i) + 8 * g);
+              acc[m][0] = multiply(wr[i], v, acc[m][0]);
+              acc[m][1] = multiply(wi[i], v, acc[m][1]);
+            }
+          }
+      }
+    }
   }
   if (!works) return;
   const int ch = first + 16 * strip + 4 * g;
   const floatx4 rb = load4(a.rb + ch), ib = load4(a.ib + ch), decay = load4(a.c + ch);
+  floatx4 cw[TAPS > 0 ? TAPS : 1], cx[TAPS > 0 ? TAPS : 1], cb, prev, cur[4];
+  if constexpr (TAPS > 0) {
+    cb = load4(a.conv_b + ch);
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) cw[k] = load4(a.conv + (size_t)(TAPS - 1 - k) * a.channels + ch);
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+      cur[m] = load4(a.proj + ((unsigned)((t.first + row0 + min(16 * m + c, n - 1)) * a.ld) + a.off_x + ch));
+    prev = TAPS > 1 ? input(c > 16 - TAPS ? row0 + c - 16 : row0, ch) : cur[0];
+  }
   floatx4 carry_d = floatx4{1.f, 1.f, 1.f, 1.f}, carry_s = floatx4{0.f, 0.f, 0.f, 0.f};
   if (t.index == 0) carry_s = load4(a.state + (size_t)slot * a.channels + ch);
 #pragma unroll
@@ -270,109 +394,145 @@ __global__ __launch_bounds__(256) void recurrence_tiles_kernel(Recurrence<T> a) 
     if (16 * m >= n) break;
     const int k = min(16 * m + c, n - 1);         // (lanes past the last row: that row again, not stored)
     const int r = t.first + row0 + k;
-    const floatx4 u = convolve<T, TAPS>(a, ring, r, row0 + k, (pos0 + k) % taps, ch);
+    floatx4 u;
+    if constexpr (TAPS > 0) {
+      rows_back<TAPS>(prev, cur[m], c, cx);
+      prev = cur[m];
+      u = cb;
+#pragma unroll
+      for (int j = TAPS - 1; j >= 0; --j) u += cw[j] * cx[j];
+    } else {
+      u = convolve<T, TAPS>(a, ring, r, row0 + k, (pos0 + k) % taps, ch);
+    }
     floatx4 d, s;
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
       const float l = decay[q] * sigmoid_f(acc[m][0][q] + rb[q]);
       d[q] = __expf(l);
       s[q] = complement(l, d[q]) * sigmoid_f(acc[m][1][q] + ib[q]) * u[q];
-      float dq = d[q], sq = s[q];
-      compose<1>(dq, sq);
-      compose<2>(dq, sq);
-      compose<4>(dq, sq);
-      compose<8>(dq, sq);
-      s[q] = fmaf(dq, carry_s[q], sq);
-      d[q] = dq * carry_d[q];
     }
+    compose(d, s);
+    s += d * carry_s;
+    d *= carry_d;
     if (16 * m + c < n) {
       store4(a.decays + (size_t)r * a.channels + ch, d);
       store4(a.states + (size_t)r * a.channels + ch, s);
     }
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
-      carry_d[q] = __shfl(d[q], (lane & 48) + 15, WAVE);
-      carry_s[q] = __shfl(s[q], (lane & 48) + 15, WAVE);
+      carry_d[q] = last_of_16(d[q]);
+      carry_s[q] = last_of_16(s[q]);
     }
   }
 }
 
-// A block takes a tile and 256 channels, a lane four of them.  The waves compose the last rows of the tiles
-// before theirs, a run of tiles a wave, and meet in LDS; then each takes 16 of the tile's rows.
-template <typename T>
-__global__ __launch_bounds__(256) void recurrence_carry_kernel(Recurrence<T> a) {
-  __shared__ floatx4 run[4][2][64];
+// A block takes a tile and 256 channels, a lane four of them, a wave a run of the tile's rows, four at a time, of
+// which it asks for the first four at once.  The waves compose the last rows of the tiles before theirs, a
+// run of tiles a wave, and meet in LDS.
+constexpr int CARRY_BATCH = 4;
+template <typename T, int WAVES>
+__global__ __launch_bounds__(64 * WAVES) void recurrence_carry_kernel(Recurrence<T> a) {
+  constexpr int ROWS = TILE_ROWS / WAVES;
+  __shared__ floatx4 run[WAVES][2][64];
   Tile t;
   if (!find_tile(a.q_start, a.n_reqs, blockIdx.x, t)) return;
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int ch = blockIdx.y * 256 + 4 * lane;
-  const bool mine = ch < a.channels;
+  const bool mine = (int)blockIdx.y * 256 + 4 * lane < a.channels;
+  const int ch = mine ? blockIdx.y * 256 + 4 * lane : 0;       // (lanes past the last channel: the first again, dropped)
+  const int row0 = t.index * TILE_ROWS, lo = row0 + ROWS * wave;
+  floatx4 d[CARRY_BATCH], s[CARRY_BATCH], y[CARRY_BATCH];
+  auto ask = [&](int from) {
+#pragma unroll
+    for (int k = 0; k < CARRY_BATCH; ++k) {
+      const int r = t.first + min(from + k, t.n - 1);
+      d[k] = load4(a.decays + (size_t)r * a.channels + ch);
+      s[k] = load4(a.states + (size_t)r * a.channels + ch);
+      y[k] = load4(a.proj + (size_t)r * a.ld + a.off_y + ch);
+    }
+  };
+  ask(lo);
   floatx4 start = floatx4{0.f, 0.f, 0.f, 0.f};
   if (t.index > 0) {                              // (the request's first tile has begun from its state)
-    const int share = (t.index + 3) >> 2, lo = wave * share, hi = min(lo + share, t.index);
-    floatx4 d = floatx4{1.f, 1.f, 1.f, 1.f}, s = start;
-    if (mine)
-      for (int k = lo; k < hi; ++k) {
-        const size_t at = (size_t)(t.first + (k + 1) * TILE_ROWS - 1) * a.channels + ch;
-        const floatx4 dk = load4(a.decays + at), sk = load4(a.states + at);
-        s = dk * s + sk;
-        d *= dk;
-      }
-    run[wave][0][lane] = d;
-    run[wave][1][lane] = s;
+    const int share = (t.index + WAVES - 1) / WAVES, first = wave * share, end = min(first + share, t.index);
+    floatx4 dc = floatx4{1.f, 1.f, 1.f, 1.f}, sc = start;
+#pragma unroll 4
+    for (int k = first; k < end; ++k) {
+      const size_t at = (size_t)(t.first + (k + 1) * TILE_ROWS - 1) * a.channels + ch;
+      const floatx4 dk = load4(a.decays + at), sk = load4(a.states + at);
+      sc = dk * sc + sk;
+      dc *= dk;
+    }
+    run[wave][0][lane] = dc;
+    run[wave][1][lane] = sc;
     __syncthreads();
 #pragma unroll
-    for (int k = 0; k < 4; ++k) start = run[k][0][lane] * start + run[k][1][lane];
+    for (int k = 0; k < WAVES; ++k) start = run[k][0][lane] * start + run[k][1][lane];
   }
   if (!mine) return;
   const int slot = a.req_rows[t.req];
-  const int row0 = t.index * TILE_ROWS;
-  const bool last_tile = row0 + TILE_ROWS >= t.n;
-  const int lo = row0 + 16 * wave, hi = min(lo + 16, t.n);
-#pragma unroll 4
-  for (int k = lo; k < hi; ++k) {
-    const size_t r = (size_t)(t.first + k), at = r * a.channels + ch;
-    const floatx4 s = load4(a.decays + at) * start + load4(a.states + at);
-    const floatx4 y = load4(a.proj + r * a.ld + a.off_y + ch);
-    floatx4 o;
+  for (int from = lo; from < lo + ROWS; from += CARRY_BATCH) {
+    if (from > lo) ask(from);
 #pragma unroll
-    for (int q = 0; q < 4; ++q) o[q] = s[q] * gelu_f(y[q]);
-    store4(a.out + at, o);
-    if (k == t.n - 1) store4(a.state + (size_t)slot * a.channels + ch, s);
+    for (int k = 0; k < CARRY_BATCH; ++k) {
+      if (from + k >= t.n) break;
+      const floatx4 now = d[k] * start + s[k];
+      floatx4 o;
+#pragma unroll
+      for (int q = 0; q < 4; ++q) o[q] = now[q] * gelu_f(y[k][q]);
+      store4(a.out + (size_t)(t.first + from + k) * a.channels + ch, o);
+      if (from + k == t.n - 1) store4(a.state + (size_t)slot * a.channels + ch, now);
+    }
   }
-  if (!last_tile || a.taps <= 1) return;
-  // the ring: the request's last inputs (as many as it brought, at most one a place), a wave every fourth
+  if (row0 + TILE_ROWS < t.n || a.taps <= 1) return;
+  // the request's last tile, the ring: its last inputs (as many as it brought, at most one a place), a row a wave in turn
   const int pos0 = a.positions[t.first];
   float* ring = a.ring + (size_t)slot * a.taps * a.channels + ch;
-  for (int k = t.n - 1 - wave; k >= 0 && k > t.n - 1 - a.taps; k -= 4)
+  for (int k = t.n - 1 - wave; k >= 0 && k > t.n - 1 - a.taps; k -= WAVES)
     store4(ring + (size_t)((pos0 + k) % a.taps) * a.channels, load4(a.proj + (size_t)(t.first + k) * a.ld + a.off_x + ch));
 }
 
 template <typename T>
 static int launch_recurrence(const Recurrence<T>& a, bool one_row_each, hipStream_t stream) {
   const int parts = a.channels / a.size, strips = a.size / 16;
-#define LLMLAB_RECUR(KERNEL, GRID, LDS)                                                                          \
+#define LLMLAB_RECUR(KERNEL, GRID, THREADS, LDS, ...)                                                            \
   switch (a.taps) {                                                                                              \
-    case 1: hipLaunchKernelGGL((KERNEL<T, 1>), GRID, dim3(256), LDS, stream, a); break;                          \
-    case 2: hipLaunchKernelGGL((KERNEL<T, 2>), GRID, dim3(256), LDS, stream, a); break;                          \
-    case 3: hipLaunchKernelGGL((KERNEL<T, 3>), GRID, dim3(256), LDS, stream, a); break;                          \
-    case 4: hipLaunchKernelGGL((KERNEL<T, 4>), GRID, dim3(256), LDS, stream, a); break;                          \
-    default: hipLaunchKernelGGL((KERNEL<T, 0>), GRID, dim3(256), LDS, stream, a); break;                         \
+    case 1: hipLaunchKernelGGL((KERNEL<T, 1 __VA_ARGS__>), GRID, dim3(THREADS), LDS, stream, a); break;          \
+    case 2: hipLaunchKernelGGL((KERNEL<T, 2 __VA_ARGS__>), GRID, dim3(THREADS), LDS, stream, a); break;          \
+    case 3: hipLaunchKernelGGL((KERNEL<T, 3 __VA_ARGS__>), GRID, dim3(THREADS), LDS, stream, a); break;          \
+    case 4: hipLaunchKernelGGL((KERNEL<T, 4 __VA_ARGS__>), GRID, dim3(THREADS), LDS, stream, a); break;          \
+    default: hipLaunchKernelGGL((KERNEL<T, 0 __VA_ARGS__>), GRID, dim3(THREADS), LDS, stream, a); break;         \
   }
   if (one_row_each) {
-    const dim3 grid(parts * strips, (a.rows + 15) / 16);
-    LLMLAB_RECUR(recurrence_row_kernel, grid, 0)
+    // as many outputs a block as leave the chip its blocks: an operand made once serves them all (64 rows of
+    // 3,584 channels in parts of 256: 15.6 us with 16 outputs a block)
+    const int all = parts * strips, groups = (a.rows + 15) / 16;      // (a part has an even number of strips)
+    if (strips % 4 == 0 && all / 4 * groups >= 192) {
+      LLMLAB_RECUR(recurrence_row_kernel, dim3(all / 4, groups), 256, 0, , 4)
+    } else if (all / 2 * groups >= 192) {
+      LLMLAB_RECUR(recurrence_row_kernel, dim3(all / 2, groups), 256, 0, , 2)
+    } else {
+      LLMLAB_RECUR(recurrence_row_kernel, dim3(all, groups), 256, 0, , 1)
+    }
     LLMLAB_LAUNCH_CHECK("gated_recurrence (one row a request)");
     return 0;
   }
   const int tiles = a.rows / TILE_ROWS + a.n_reqs;      // at most so many; blocks past the last leave at once
   const size_t lds = (size_t)TILE_ROWS * ((a.size < SLAB<T> ? a.size : SLAB<T>) + 8) * sizeof(T);
-  const dim3 grid(tiles, parts * ((strips + 3) / 4));
-  LLMLAB_RECUR(recurrence_tiles_kernel, grid, lds)
+  // a part of 128 channels and more: eight waves a block, so that a block's inputs serve more outputs (2,048
+  // rows of 3,584 channels in parts of 256, both launches: 68 us with four waves, 59 with eight)
+  const int waves = strips >= 8 ? 8 : 4;
+  const dim3 grid(tiles, parts * ((strips + waves - 1) / waves));
+  LLMLAB_RECUR(recurrence_tiles_kernel, grid, 64 * waves, lds)
 #undef LLMLAB_RECUR
   LLMLAB_LAUNCH_CHECK("gated_recurrence (tiles)");
-  hipLaunchKernelGGL(recurrence_carry_kernel<T>, dim3(tiles, (a.channels + 255) / 256), dim3(256), 0, stream, a);
+  // few blocks: more waves a block (2,048 rows of 896 channels 13 us with four waves, 9 with sixteen; of 3,584
+  // channels 19 and 24)
+  const dim3 across(tiles, (a.channels + 255) / 256);
+  if ((long)across.x * across.y <= 256)
+    hipLaunchKernelGGL((recurrence_carry_kernel<T, 16>), across, dim3(1024), 0, stream, a);
+  else
+    hipLaunchKernelGGL((recurrence_carry_kernel<T, 4>), across, dim3(256), 0, stream, a);
   LLMLAB_LAUNCH_CHECK("gated_recurrence (carry)");
   return 0;
 }
@@ -395,6 +555,7 @@ extern "C" int llmlab_gated_recurrence(const float* proj, int ld, int off_x, int
                      (taps == 1 || ring), "gated_recurrence: an operand is missing");
   LLMLAB_REQUIRE(one_row_each ? n_reqs == rows : (decays != nullptr && states != nullptr),
                  "gated_recurrence: %d rows of %d requests", rows, n_reqs);
+  LLMLAB_REQUIRE((size_t)rows * ld < ((size_t)1 << 31), "gated_recurrence: %d rows of %d numbers", rows, ld);
   LLMLAB_REQUIRE(channels / 16 <= 65535 && rows / 16 <= 65535, "gated_recurrence: too many channels or rows");
   if (rows == 0 || n_reqs == 0) return 0;
   if (dtype == DT_BF16) {

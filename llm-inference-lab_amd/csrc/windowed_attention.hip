@@ -30,6 +30,100 @@ struct NormWrite {
   const float* freq; int rot_dims, neighbours, page_size; const int* positions; const int* row_req; const int* table;
   int max_pages;
 };
+//
+// QUADS (halves, every size a multiple of 4): a thread takes four channels of a head at a time, loads and
+// stores 16 and 8 bytes wide, the row in registers between the sums and the result.
+__device__ __forceinline__ floatx4 load4(const float* p) { return *(const floatx4*)p; }
+__device__ __forceinline__ void store4(float* p, floatx4 v) { *(floatx4*)p = v; }
+__device__ __forceinline__ void store4(bf16_t* p, floatx4 v) {
+  *(bf16x4*)p = bf16x4{(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
+}
+
+template <typename T>
+__global__ __launch_bounds__(512) void project_norm_write_quads_kernel(NormWrite a, T* __restrict__ q_out,
+                                                                       T* __restrict__ k_cache, T* __restrict__ v_cache) {
+  extern __shared__ __attribute__((aligned(16))) float quad_lds[];     // cos [half], sin [half], the row's q and k
+  __shared__ float red_q[8], red_k[8];
+  const int r = blockIdx.x, lane = threadIdx.x & 63, waves = blockDim.x >> 6, threads = blockDim.x;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const float* src = a.proj + (size_t)r * a.ld;
+  const int q_size = a.n_heads * a.D, k_size = a.own ? a.n_kv * a.D : 0, half = a.rot_dims >> 1;
+  const int turned = q_size + k_size;
+  float* s_cos = quad_lds;
+  float* s_sin = quad_lds + half;
+  float* s_row = quad_lds + 2 * half;
+  const int pos = a.positions ? a.positions[r] : 0;
+  const int page = a.own ? a.table[(size_t)a.row_req[r] * a.max_pages + pos / a.page_size] : 0;
+  const int slot = pos % a.page_size;
+  float sq = 0.f, sk = 0.f;
+  for (int c0 = 4 * threadIdx.x; c0 < turned; c0 += 16 * threads) {    // (four loads travel together)
+    floatx4 v[4];
+#pragma unroll
+    for (int n = 0; n < 4; ++n) v[n] = load4(src + min(c0 + 4 * n * threads, turned - 4));
+#pragma unroll
+    for (int n = 0; n < 4; ++n) {
+      const int c = c0 + 4 * n * threads;
+      if (c >= turned) break;
+      const float s = v[n][0] * v[n][0] + v[n][1] * v[n][1] + v[n][2] * v[n][2] + v[n][3] * v[n][3];
+      if (c < q_size) sq += s;
+      else sk += s;
+      store4(s_row + c, v[n]);
+    }
+  }
+  for (int i = threadIdx.x; i < half; i += threads) {
+    float sn, cs;
+    sincosf((float)pos * a.freq[i], &sn, &cs);
+    s_cos[i] = cs;
+    s_sin[i] = sn;
+  }
+  if (a.norm) {
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if (lane == 0) {
+      red_q[wave] = sq;
+      red_k[wave] = sk;
+    }
+  }
+  __syncthreads();
+  float inv_q = 1.f, inv_k = 1.f;
+  if (a.norm) {
+    sq = sk = 0.f;
+    for (int n = 0; n < waves; ++n) {
+      sq += red_q[n];
+      sk += red_k[n];
+    }
+    inv_q = 1.0f / sqrtf(sq / (float)q_size + a.eps);
+    if (k_size > 0) inv_k = 1.0f / sqrtf(sk / (float)k_size + a.eps);
+  }
+  const int quads = a.DK >> 2, heads = a.n_heads + (a.own ? a.n_kv : 0);
+  for (int i = threadIdx.x; i < heads * quads; i += threads) {
+    const int h = i / quads, d = 4 * (i - h * quads);
+    const bool query = h < a.n_heads;
+    floatx4 v = floatx4{0.f, 0.f, 0.f, 0.f};
+    if (d < a.D) {
+      const float* w = query ? a.q_w + (size_t)h * a.D : a.k_w + (size_t)(h - a.n_heads) * a.D;
+      const float inv = query ? inv_q : inv_k;
+      v = load4(s_row + h * a.D + d);
+      if (a.norm) v *= inv * load4(w + d);
+      if (d < a.rot_dims) {
+        const bool first = d < half;
+        const int o = first ? d + half : d - half, at = first ? d : d - half;
+        floatx4 other = load4(s_row + h * a.D + o);
+        if (a.norm) other *= inv * load4(w + o);
+        const floatx4 cs = load4(s_cos + at), sn = load4(s_sin + at);
+        v = first ? v * cs - other * sn : v * cs + other * sn;
+      }
+    }
+    store4(query ? q_out + ((size_t)r * a.n_heads + h) * a.DK + d
+                 : k_cache + (((size_t)page * a.n_kv + (h - a.n_heads)) * a.page_size + slot) * a.DK + d, v);
+  }
+  if (!a.own) return;
+  for (int c = threadIdx.x; c < a.n_kv * a.E; c += threads) {
+    const int g = c / a.E, e = c - g * a.E;
+    v_cache[((size_t)page * a.n_kv + g) * a.page_size * a.E + value_index(slot, e, a.E)] = from_float<T>(src[turned + c]);
+  }
+}
+
 template <typename T>
 __global__ __launch_bounds__(1024) void project_norm_write_kernel(NormWrite a, T* __restrict__ q_out, T* __restrict__ k_cache,
                                                                   T* __restrict__ v_cache) {
@@ -120,6 +214,19 @@ extern "C" int llmlab_project_norm_write(const float* proj, int ld, int rows, in
   if (rows == 0) return 0;
   const NormWrite a{proj, ld, n_heads, n_kv, D, DK, E, own_kv, norm, eps, q_w, k_w, freq, rot_dims, neighbours, page_size,
                     positions, row_req, table, max_pages};
+  const size_t row_lds = ((size_t)rot_dims + q_size + k_size) * sizeof(float);
+  if (!neighbours && D % 4 == 0 && DK % 4 == 0 && rot_dims % 8 == 0 && ld % 4 == 0 && row_lds <= 56 * 1024 &&
+      (((uintptr_t)proj | (uintptr_t)q_out | (uintptr_t)k_cache | (uintptr_t)q_w | (uintptr_t)k_w) & 15) == 0) {
+    const int threads = rows <= 64 ? 512 : 256;
+    if (dtype == DT_BF16)
+      hipLaunchKernelGGL(project_norm_write_quads_kernel<bf16_t>, dim3(rows), dim3(threads), row_lds, stream, a,
+                         (bf16_t*)q_out, (bf16_t*)k_cache, (bf16_t*)v_cache);
+    else
+      hipLaunchKernelGGL(project_norm_write_quads_kernel<float>, dim3(rows), dim3(threads), row_lds, stream, a,
+                         (float*)q_out, (float*)k_cache, (float*)v_cache);
+    LLMLAB_LAUNCH_CHECK("project_norm_write");
+    return 0;
+  }
   // few rows: more waves, a head a wave
   const int threads = rows <= 64 && n_heads > 4 ? 1024 : 256;
   const size_t lds = (size_t)rot_dims * sizeof(float);
@@ -971,8 +1078,9 @@ __global__ __launch_bounds__(256) void sink_window_attention_mfma_kernel(MfmaArg
   }
 }
 
-// Prompts whose heads read the same keys and values (one key/value head, or groups of a multiple
-// of four heads): a block takes 16 consecutive rows and FOUR heads, a wave a head.  The block
+// Prompts whose heads read the same keys and values (groups of three heads and more): a block takes 16
+// consecutive rows and up to FOUR heads of one key/value head, a wave a head (a group of seven heads: a
+// block of four and one of three, whose last wave only helps to stage).  The block
 // stages every tile of 32 keys and their values in LDS once (each thread asks for its 16-byte
 // pieces two tiles ahead and stores them a tile ahead), and the waves take their fragments from
 // there instead of each from L2.  Key rows lie 16 bytes apart from a
@@ -991,10 +1099,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
   const int tid = threadIdx.x, lane = tid & 63, c = lane & 15, g4 = lane >> 4, wave = tid >> 6;
   const int r0 = blockIdx.x * 16;
   if (r0 >= a.n_rows) return;
-  const int h_raw = blockIdx.y * 4 + wave;
-  const bool head_ok = h_raw < a.n_heads;
-  const int h = head_ok ? h_raw : a.n_heads - 1;
-  const int g = (blockIdx.y * 4) / (a.n_heads / a.n_kv);
+  const int group = a.n_heads / a.n_kv, per_group = (group + 3) >> 2;      // blocks a key/value head's heads take
+  const int g = blockIdx.y / per_group, h_raw = (blockIdx.y - g * per_group) * 4 + wave;
+  const bool head_ok = h_raw < group;
+  const int h = g * group + (head_ok ? h_raw : group - 1);
   const int r = r0 + c;
   const bool row_ok = r < a.n_rows;
   const int pos = row_ok ? a.positions[r] : 0;
@@ -1393,8 +1501,8 @@ extern "C" int llmlab_sink_window_attention(const void* q, int dtype, int rows, 
     if (launches & 2) {
       // heads that read the same keys and values share the tiles a block stages in LDS
       const int group = n_heads / n_kv;
-      if (!g_private_tiles && group >= 3 && (n_kv == 1 || group % 4 == 0))
-        launch_mfma_any(D, E, 2, dim3((rows + 15) / 16, (n_heads + 3) / 4), dim3(256), stream, a);
+      if (!g_private_tiles && group >= 3)
+        launch_mfma_any(D, E, 2, dim3((rows + 15) / 16, n_kv * ((group + 3) / 4)), dim3(256), stream, a);
       else
         launch_mfma_any(D, E, 0, dim3((rows + 63) / 64, n_heads), dim3(256), stream, a);
       LLMLAB_LAUNCH_CHECK("sink_window_attention (prompts)");

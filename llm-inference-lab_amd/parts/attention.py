@@ -405,7 +405,7 @@ class WindowedSinkAttention(Mixer):
         self.hidden_size, self.num_heads, self.num_kv_heads = int(hidden_size), int(num_heads), int(num_kv_heads)
         self.key_dim = int(key_dim)
         self.file_value_dim = int(value_dim)                       # a value head as the model file has it
-        tiled = self.shaped or (self.whole and bool(self.position is not None or output_gate))
+        self.tiled = tiled = self.shaped or (self.whole and bool(self.position is not None or output_gate))
         unit = 16 if tiled else 8
         self.value_dim = (self.file_value_dim + unit - 1) // unit * unit      # and as the kernels and the pages see it
         self.laid_dim = (self.key_dim + 31) // 32 * 32 if tiled else self.key_dim      # a key head in the pages
@@ -432,8 +432,13 @@ class WindowedSinkAttention(Mixer):
         return {None: 0, "sigmoid": self.num_heads, "channels": self.num_heads * self.value_dim}[self.output_gate]
 
     @property
+    def gate_column(self):
+        return self.q_size + (self.k_size + self.v_size if self.own_kv else 0)
+
+    @property
     def in_size(self):
-        return self.q_size + (self.k_size + self.v_size if self.own_kv else 0) + self.gate_size
+        size = self.gate_column + self.gate_size
+        return (size + 3) // 4 * 4 if self.tiled and self.whole else size      # (rows of whole 16-byte pieces)
 
     def tensor_specs(self):
         t, w = self.tensor_names, self.hidden_size
@@ -491,6 +496,9 @@ class WindowedSinkAttention(Mixer):
             rows.append(value_heads(tensors[t["gate_weight"]], self.num_heads))
         elif self.output_gate:
             rows.append(tensors[t["gate_weight"]])
+        more = self.in_size - self.gate_column - self.gate_size
+        if more:
+            rows.append(torch.zeros((more, self.hidden_size), dtype=rows[0].dtype, device=rows[0].device))
         self.w_in = ops.prepare_weight(torch.cat(rows, dim=0).contiguous())       # one product for q (, k, v, gates)
         if self.qkv_bias:
             bias = [tensors[t["q_bias"]].float(), tensors[t["k_bias"]].float(),
@@ -593,7 +601,7 @@ class WindowedSinkAttention(Mixer):
         if self.output_gate == "channels":
             kind["gate"] = (proj, self.q_size + self.k_size + self.v_size)
         elif self.whole and self.output_gate:
-            kind["head_gate"] = (proj, self.in_size - self.gate_size)
+            kind["head_gate"] = (proj, self.gate_column)
         reach = self.window if self.window is not None else self.chunk
 
         def attend():

@@ -144,7 +144,7 @@ def test_whole_norm_rotation_and_the_cache_write(backend, dtype, H_, G, D, E, di
 
 
 # ------------------------------------------------------------------ attention
-SHAPES = [(4, 2, 32, 16), (8, 2, 64, 64), (4, 1, 96, 48), (3, 3, 128, 128), (6, 2, 32, 192)]
+SHAPES = [(4, 2, 32, 16), (8, 2, 64, 64), (4, 1, 96, 48), (3, 3, 128, 128), (6, 2, 32, 192), (14, 2, 64, 64), (10, 2, 32, 32)]
 
 
 @pytest.mark.parametrize("backend", BACKENDS)
@@ -295,6 +295,24 @@ def test_recurrence_in_portions_with_states_in_slots(backend, dtype, width, bloc
     for b in range(3):
         want = plain_recurrence(w, xs[b], ys[b], dtype)[:got[b].shape[0]]
         close(got[b], want, dtype, f"request {b}", f32=2e-5, bf16=1e-2)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_recurrence_of_many_tiles_and_of_many_rows(dtype):
+    """More tiles and channels than a launch of few blocks takes, and a hundred requests of a row each beside
+    each other: the kernels' other block shapes."""
+    ops = ops_of("hip")
+    width, lengths = 1536, [4500, 130] + [3] * 100
+    w = recurrence(width, 6, 4, 21)
+    xs = [randn(n, width, seed=400 + b, scale=1.5) for b, n in enumerate(lengths)]
+    ys = [randn(n, width, seed=600 + b, scale=1.5) for b, n in enumerate(lengths)]
+    part = bound(ops, dtype, w, width, 6, 4)
+    every = range(len(lengths))
+    cuts = [[(b, 1) for b in every], [(0, 4400), (1, 64)] + [(b, 1) for b in every[2:]], [(b, 1) for b in every], [(0, 98), (1, 64)]]
+    got = run_recurrence(ops, part, dtype, xs, ys, cuts, list(reversed(every)))
+    for b in every:
+        close(got[b], plain_recurrence(w, xs[b], ys[b], dtype), dtype, f"request {b}", f32=2e-5, bf16=1e-2)
 
 
 @pytest.mark.parametrize("backend", BACKENDS)
