@@ -537,7 +537,6 @@ static int launch_recurrence(const Recurrence<T>& a, bool one_row_each, hipStrea
   return 0;
 }
 
-extern "C" int llmlab_gated_recurrence_tile_rows() { return TILE_ROWS; }
 
 // proj [rows, ld] float32; gates and out in the compute dtype; q_start [n_reqs + 1]; decays, states (float32
 // [rows, channels]): scratch of steps in which a request brings more than one row.
