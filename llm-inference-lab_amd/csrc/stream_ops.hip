@@ -23,50 +23,91 @@ extern "C" const char* llmlab_last_error() { return g_llmlab_error; }
 // step or, for a request's first row of the step, previous_slot[slot].  The block of a
 // request's first row also stores the request's LAST token of the step there, after it has read
 // the old one (one thread does both, in that order; no other block touches the slot).
-template <typename T>
-__global__ __launch_bounds__(256) void embed_pairs_kernel(
+// A thread takes V neighbouring numbers at a time; the token's are asked for before the pair is
+// known, and what a thread's first EMBED_KEEP trips give stays in registers between the sum of squares and the norm.
+constexpr int EMBED_KEEP = 2;
+template <typename T, int V>
+__global__ __launch_bounds__(1024) void embed_pairs_kernel(
     const T* __restrict__ table, const T* __restrict__ pairs, const int* __restrict__ ids,
     const int* __restrict__ positions, const int* __restrict__ row_req, const int* __restrict__ q_start,
     const int* __restrict__ req_rows, int* __restrict__ previous_slot, float scale, int vocab, int buckets,
     long long mul_prev, long long mul_cur, const void* __restrict__ norm_w, int norm_bf16, float eps,
     float* __restrict__ out, int hidden) {
+  typedef T vec_t __attribute__((ext_vector_type(V)));
+  typedef float fvec_t __attribute__((ext_vector_type(V)));
   __shared__ float red[17];
   __shared__ int s_pair;
-  const int r = blockIdx.x;
+  const int r = blockIdx.x, threads = blockDim.x, units = hidden / V;
   int id = ids[r];
   id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+  const T* t = table + (size_t)id * hidden;
+  vec_t token[EMBED_KEEP];
+#pragma unroll
+  for (int n = 0; n < EMBED_KEEP; ++n) {
+    const int i = threadIdx.x + threads * n;
+    if (i < units) token[n] = *(const vec_t*)(t + (size_t)i * V);
+  }
   if (threadIdx.x == 0) {
     int pair = -1;
     if (buckets > 0) {
-      const int b = row_req[r], first = q_start[b];
+      const int b = row_req[r], at = positions[r], first = q_start[b], last = q_start[b + 1] - 1, slot = req_rows[b];
       long long before = -1;
       if (r > first) {
         before = ids[r - 1];
       } else {
-        const int slot = req_rows[b];
         before = previous_slot[slot];
-        previous_slot[slot] = ids[q_start[b + 1] - 1];
+        previous_slot[slot] = ids[last];
       }
       if (before < 0) before = 0;
-      pair = positions[r] == 0 ? buckets : (int)((before * mul_prev + (long long)id * mul_cur) % buckets);
+      pair = at == 0 ? buckets : (int)((before * mul_prev + (long long)id * mul_cur) % buckets);
     }
     s_pair = pair;
   }
   __syncthreads();
   const int pair = s_pair;
-  const T* t = table + (size_t)id * hidden;
   const T* p = pair >= 0 ? pairs + (size_t)pair * hidden : nullptr;
   float* o = out + (size_t)r * hidden;
+  fvec_t keep[EMBED_KEEP];
   float ss = 0.f;
-  for (int c = threadIdx.x; c < hidden; c += blockDim.x) {
-    float v = to_float(t[c]) * scale;
-    if (p) v += to_float(p[c]);
-    o[c] = v;
-    ss += v * v;
+  auto sum = [&](int i, const vec_t& tok) {
+    fvec_t v;
+#pragma unroll
+    for (int q = 0; q < V; ++q) v[q] = to_float((T)tok[q]) * scale;
+    if (p) {
+      const vec_t e = *(const vec_t*)(p + (size_t)i * V);
+#pragma unroll
+      for (int q = 0; q < V; ++q) v[q] += to_float((T)e[q]);
+    }
+    if (norm_w) {
+#pragma unroll
+      for (int q = 0; q < V; ++q) ss += v[q] * v[q];
+    }
+    return v;
+  };
+#pragma unroll
+  for (int n = 0; n < EMBED_KEEP; ++n) {
+    const int i = threadIdx.x + threads * n;
+    if (i < units) {
+      keep[n] = sum(i, token[n]);
+      if (!norm_w) *(fvec_t*)(o + (size_t)i * V) = keep[n];
+    }
   }
+  for (int i = threadIdx.x + threads * EMBED_KEEP; i < units; i += threads)
+    *(fvec_t*)(o + (size_t)i * V) = sum(i, *(const vec_t*)(t + (size_t)i * V));
   if (!norm_w) return;
   const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)hidden + eps);
-  for (int c = threadIdx.x; c < hidden; c += blockDim.x) o[c] = o[c] * inv * load_vec(norm_w, norm_bf16, c);
+  auto normed = [&](int i, fvec_t v) {
+#pragma unroll
+    for (int q = 0; q < V; ++q) v[q] = v[q] * inv * load_vec(norm_w, norm_bf16, i * V + q);
+    *(fvec_t*)(o + (size_t)i * V) = v;
+  };
+#pragma unroll
+  for (int n = 0; n < EMBED_KEEP; ++n) {
+    const int i = threadIdx.x + threads * n;
+    if (i < units) normed(i, keep[n]);
+  }
+  for (int i = threadIdx.x + threads * EMBED_KEEP; i < units; i += threads)      // (a thread's own numbers)
+    normed(i, *(const fvec_t*)(o + (size_t)i * V));
 }
 
 extern "C" int llmlab_embed_pairs(const void* table, const void* pairs, int dtype, const int* ids, const int* positions,
@@ -79,14 +120,20 @@ extern "C" int llmlab_embed_pairs(const void* table, const void* pairs, int dtyp
   LLMLAB_REQUIRE(buckets == 0 || (pairs && positions && row_req && q_start && req_rows && previous_slot),
                  "embed_pairs: the pairs need their table, the step's description and the slots");
   if (rows == 0) return 0;
-  if (dtype == DT_BF16)
-    hipLaunchKernelGGL(embed_pairs_kernel<bf16_t>, dim3(rows), dim3(256), 0, stream, (const bf16_t*)table,
-                       (const bf16_t*)pairs, ids, positions, row_req, q_start, req_rows, previous_slot, scale, vocab,
-                       buckets, mul_prev, mul_cur, norm_w, norm_dtype == DT_BF16, eps, out, hidden);
-  else
-    hipLaunchKernelGGL(embed_pairs_kernel<float>, dim3(rows), dim3(256), 0, stream, (const float*)table,
-                       (const float*)pairs, ids, positions, row_req, q_start, req_rows, previous_slot, scale, vocab,
-                       buckets, mul_prev, mul_cur, norm_w, norm_dtype == DT_BF16, eps, out, hidden);
+  const bool vec = hidden % 4 == 0 && (((uintptr_t)table | (uintptr_t)pairs | (uintptr_t)out) & 15) == 0;
+  const int units = vec ? hidden / 4 : hidden;
+  int threads = (units + 63) / 64 * 64;
+  if (threads > 1024) threads = 1024;
+#define LLMLAB_EMBED(T, V)                                                                                           \
+  hipLaunchKernelGGL((embed_pairs_kernel<T, V>), dim3(rows), dim3(threads), 0, stream, (const T*)table, (const T*)pairs, \
+                     ids, positions, row_req, q_start, req_rows, previous_slot, scale, vocab, buckets, mul_prev, mul_cur, \
+                     norm_w, norm_dtype == DT_BF16, eps, out, hidden)
+  if (dtype == DT_BF16) {
+    if (vec) LLMLAB_EMBED(bf16_t, 4); else LLMLAB_EMBED(bf16_t, 1);
+  } else {
+    if (vec) LLMLAB_EMBED(float, 4); else LLMLAB_EMBED(float, 1);
+  }
+#undef LLMLAB_EMBED
   LLMLAB_LAUNCH_CHECK("embed_pairs");
   return 0;
 }

@@ -49,7 +49,7 @@ def on(device, *tensors):
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("hidden,vocab,buckets,norm", [(64, 50, 13, True), (100, 300, 1019, True), (24, 9, 1, False),
-                                                       (72, 40, 0, True)])
+                                                       (72, 40, 0, True), (3001, 30, 17, True), (9000, 30, 17, True)])
 def test_embed_pairs_over_steps(ops, emu, dtype, hidden, vocab, buckets, norm):
     """Three steps of three requests in slots 2, 0, 3: portions, single tokens, a request that starts
     in the second step; the slots carry the last token from step to step."""

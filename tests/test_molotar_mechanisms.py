@@ -59,12 +59,13 @@ def test_norm_behind_the_sum(backend, hidden, rows):
 
 
 @pytest.mark.parametrize("backend", BACKENDS)
-def test_pairs_without_a_norm(backend):
+@pytest.mark.parametrize("width", [24, 25, 1030, 3001, 9000])
+def test_pairs_without_a_norm(backend, width):
     """The scaled token vector plus the pair's row, no norm behind; the token before a step's first one
     comes out of the slot; a sequence's first token takes the row behind the buckets."""
     ops = ops_of(backend)
     dev = ops.device
-    vocab, width, buckets, mul_prev, mul_cur = 40, 24, 11, 29, 7
+    vocab, buckets, mul_prev, mul_cur = 40, 11, 29, 7
     table, pairs = randn(vocab, width, seed=1), randn(buckets + 1, width, seed=2)
     cfg = dict(embedding=dict(scale=4.5, bigram=dict(buckets=buckets, mul_prev=mul_prev, mul_cur=mul_cur)))
     ids = torch.randint(0, vocab, (12,), generator=torch.Generator().manual_seed(3)).tolist()
